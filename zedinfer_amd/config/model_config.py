@@ -602,3 +602,94 @@ class KegozenConfig(ModelConfig):
         if self.eos_token_ids:
             d["eos_token_id"] = list(self.eos_token_ids)
         return d
+
+
+@dataclass(frozen=True)
+class KefisunConfig(ModelConfig):
+    """The Kefisun design's config.json: ``width``, ``vocab``, ``norm.eps``, ``canon.taps`` (the convolution in front of
+    every mixer), ``embedding.scale``, ``logit_scale`` and a list ``layers`` whose entries each name a mixer by ``type``
+    ("attention": grouped-query attention under a window with a logarithm of the distance in its scores;
+    "channel_delta": the delta rule with a decay per key channel) with its sizes and constants under ``mixer``, and a
+    feed-forward under ``mlp`` (``kind`` "dense" with ``ff`` and ``limit``; or null for none).  Every size and constant of
+    a model is read from here (the ranks of the low-rank gates are the tensors' own unless ``mixer.decay_rank`` and
+    ``mixer.gate_rank`` name them); the shared keys of ``ModelConfig`` that the format does not have keep their neutral
+    values."""
+
+    layers: Tuple[Any, ...] = ()
+    norm_eps: float = 1e-6
+    canon_taps: int = 1
+    embedding_scale: float = 1.0
+    logit_scale: float = 1.0
+
+    MIXER_KEYS = {"attention": ("heads", "kv_heads", "dim", "vdim", "conv", "scale"),
+                  "channel_delta": ("heads", "kv_heads", "dim", "vdim", "conv")}
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "KefisunConfig":
+        missing = [k for k in ("width", "vocab", "layers", "norm", "canon") if k not in d]
+        if missing:
+            raise ConfigError("config.json lacks required key(s): " + ", ".join(missing))
+        if not isinstance(d["layers"], (list, tuple)) or not d["layers"]:
+            raise ConfigError("config.json: 'layers' must be a non-empty list")
+        for outer, inner in (("norm", "eps"), ("canon", "taps")):
+            if not isinstance(d[outer], Mapping) or inner not in d[outer]:
+                raise ConfigError(f"config.json: '{outer}' must give '{inner}'")
+        eos = d.get("eos_token_id")
+        cfg = cls(architectures=(str(d.get("architecture", "Kefisun")),), model_type="kefisun",
+                  torch_dtype=str(d.get("torch_dtype") or "bfloat16"), hidden_size=_as_int(d, "width"),
+                  vocab_size=_as_int(d, "vocab"), num_hidden_layers=len(d["layers"]), tie_word_embeddings=True,
+                  eos_token_ids=() if eos is None else tuple(int(e) for e in (eos if isinstance(eos, (list, tuple)) else [eos])),
+                  layers=tuple(json.loads(json.dumps(layer)) for layer in d["layers"]), norm_eps=float(d["norm"]["eps"]),
+                  canon_taps=_as_int(d["canon"], "taps"),
+                  embedding_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+                  logit_scale=float(d.get("logit_scale", 1.0)))
+        cfg.validate()
+        return cfg
+
+    def value_mixing_layers(self) -> Tuple[int, ...]:
+        """The layers that mix their values with the first of them."""
+        return tuple(i for i, layer in enumerate(self.layers)
+                     if layer["type"] == "attention" and layer["mixer"].get("v_mix"))
+
+    def validate(self) -> None:
+        if self.hidden_size <= 0 or self.vocab_size <= 0:
+            raise ConfigError("config.json: 'width' and 'vocab' must be positive")
+        if not (self.norm_eps > 0):
+            raise ConfigError(f"config.json: norm.eps must be positive, got {self.norm_eps}")
+        if self.canon_taps <= 0:
+            raise ConfigError(f"config.json: canon.taps must be positive, got {self.canon_taps}")
+        for i, layer in enumerate(self.layers):
+            kind = layer.get("type") if isinstance(layer, Mapping) else None
+            if kind not in self.MIXER_KEYS:
+                raise ConfigError(f"config.json: layer {i} has type {kind!r}; known: {', '.join(sorted(self.MIXER_KEYS))}")
+            m = layer.get("mixer")
+            lacking = [k for k in self.MIXER_KEYS[kind] if not isinstance(m, Mapping) or k not in m]
+            if lacking:
+                raise ConfigError(f"config.json: layer {i} ({kind}) lacks mixer key(s): " + ", ".join(lacking))
+            if any(int(m[k]) <= 0 for k in self.MIXER_KEYS[kind] if k != "scale") or int(m["heads"]) % int(m["kv_heads"]):
+                raise ConfigError(f"config.json: layer {i} ({kind}): sizes must be positive, heads a multiple of kv_heads")
+            if kind == "attention":
+                if not float(m["scale"]) > 0:
+                    raise ConfigError(f"config.json: layer {i}: the scale must be positive")
+                if m.get("mask") is not None and not int(m["mask"].get("size", 0)) > 0:
+                    raise ConfigError(f"config.json: layer {i}: mask.size must be positive")
+            mlp = layer.get("mlp")
+            if mlp is None:
+                continue
+            if mlp.get("kind") != "dense":
+                raise ConfigError(f"config.json: layer {i}: mlp.kind {mlp.get('kind')!r} is not 'dense'")
+            if not int(mlp.get("ff", 0)) > 0 or not float(mlp.get("limit", 0)) > 0:
+                raise ConfigError(f"config.json: layer {i}: a dense mlp needs a positive ff and limit")
+        mixing = self.value_mixing_layers()
+        sizes = {(int(self.layers[i]["mixer"]["kv_heads"]) * int(self.layers[i]["mixer"]["vdim"])) for i in mixing}
+        if len(sizes) > 1:
+            raise ConfigError(f"config.json: layers {', '.join(map(str, mixing))} mix values but differ in their number")
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"architecture": self.architectures[0] if self.architectures else "Kefisun",
+             "canon": {"taps": self.canon_taps}, "embedding": {"scale": self.embedding_scale},
+             "layers": json.loads(json.dumps(list(self.layers))), "logit_scale": self.logit_scale,
+             "norm": {"eps": self.norm_eps}, "vocab": self.vocab_size, "width": self.hidden_size}
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids)
+        return d

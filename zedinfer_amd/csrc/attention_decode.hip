@@ -468,6 +468,8 @@ attention_decode_kernel(zi_bf16* __restrict__ out, int64_t ldo, float* __restric
         float mx = -INFINITY;
         const float inv_cap = (BIASED && ex.softcap > 0.f) ? 1.f / ex.softcap : 0.f;
         const float* brow = (BIASED && ex.bias) ? ex.bias + (int64_t)(kvh * G + (r < G ? r : G - 1)) * ex.bias_len : nullptr;
+        const float slope = (BIASED && ex.slope) ? ex.slope[kvh * G + (r < G ? r : G - 1)] : 0.f;
+        const float rate = (BIASED && ex.slope) ? ex.rate[kvh * G + (r < G ? r : G - 1)] : 0.f;
 #pragma unroll
         for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
@@ -477,6 +479,7 @@ attention_decode_kernel(zi_bf16* __restrict__ out, int64_t ldo, float* __restric
                 if constexpr (BIASED) {
                     sc = s[tt][e] * scale;
                     if (ex.softcap > 0.f) sc = ex.softcap * dec_tanh(sc * inv_cap);
+                    if (ex.slope) sc -= slope * (0.6931471805599453f * __builtin_amdgcn_logf(fmaf(rate, (float)(p - key), 1.f)));      // (NaN for keys ahead of the query, which are masked)
                     if (brow) {
                         int dist = p - key;
                         dist = (int)min((unsigned)dist, (unsigned)(ex.bias_len - 1));      // (a key ahead of the query is masked anyway)
@@ -768,8 +771,9 @@ static int dec_launch(const char* who, void* out, const void* q, int dt, int n_i
                       const int32_t* tok_pos, const int32_t* block_tables, int max_pages, int num_pages, int nh, int nkv,
                       int d, int page_size, int window, float scale, int max_chunks, float* workspace,
                       int64_t workspace_floats, const DecProjection* pj, const float* sinks, hipStream_t stream,
-                      ZiScoreExtras ex = ZiScoreExtras{0.f, nullptr, 0, 0}) {
-    const bool biased = ex.softcap > 0.f || ex.bias != nullptr || ex.keep_first > 0;
+                      ZiScoreExtras ex = ZiScoreExtras{0.f, nullptr, 0, 0, nullptr, nullptr}) {
+    const bool biased = ex.softcap > 0.f || ex.bias != nullptr || ex.keep_first > 0 || ex.slope != nullptr;
+    ZI_REQUIRE((ex.slope == nullptr) == (ex.rate == nullptr), "%s: a slope and a rate, or neither", who);
     ZI_REQUIRE(!(biased && pj), "%s: capped or biased scores come with queries that are made beforehand", who);
     ZI_REQUIRE(ex.softcap >= 0.f && ex.keep_first >= 0 && (!ex.bias || ex.bias_len > 0), "%s: bad cap, bias or kept positions", who);
     ZI_REQUIRE(zi_attention_decode_supported(dt, nh, nkv, d, page_size),
@@ -859,18 +863,19 @@ extern "C" int zi_attention_decode_sink(void* out, const void* q, int dt, int n_
 }
 
 // The same with capped and biased scores and kept first positions (ZiScoreExtras): `softcap` 0 for none, `bias`
-// float32 [nh][bias_len] or null, `keep_first` positions of every sequence stay visible beside the window.
+// float32 [nh][bias_len] or null, `keep_first` positions of every sequence stay visible beside the window; `slope` and
+// `rate` float32 [nh], both or null.  out null (only with a slope): the chunks stay unmerged in the workspace.
 extern "C" int zi_attention_decode_biased(void* out, const void* q, int dt, int n_idx, int64_t ldq, int64_t ldo,
                                           const void* kcache, const void* vcache, const int32_t* tok_index,
                                           const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* block_tables,
                                           int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window,
                                           float scale, int max_chunks, float* workspace, int64_t workspace_floats,
                                           const float* sinks, float softcap, const float* bias, int bias_len,
-                                          int keep_first, hipStream_t stream) {
-    ZI_REQUIRE(out != nullptr, "attention_decode_biased: the chunks are merged here");
+                                          int keep_first, const float* slope, const float* rate, hipStream_t stream) {
+    ZI_REQUIRE(out != nullptr || slope, "attention_decode_biased: the chunks are merged here");
     return dec_launch("attention_decode_biased", out, q, dt, n_idx, ldq, ldo, kcache, vcache, tok_index, tok_seq, tok_pos,
                       block_tables, max_pages, num_pages, nh, nkv, d, page_size, window, scale, max_chunks, workspace,
-                      workspace_floats, nullptr, sinks, stream, ZiScoreExtras{softcap, bias, bias_len, keep_first});
+                      workspace_floats, nullptr, sinks, stream, ZiScoreExtras{softcap, bias, bias_len, keep_first, slope, rate});
 }
 
 // 1 when the fused entry point takes this projection layout, else 0 (then: rotate and store first, and

@@ -33,7 +33,8 @@ attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, int64_t l
                          const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ block_tables,
                          int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window,
                          float scale, const float* __restrict__ sinks, float softcap,
-                         const float* __restrict__ bias, int bias_len, int keep_first) {
+                         const float* __restrict__ bias, int bias_len, int keep_first, const float* __restrict__ slope,
+                         const float* __restrict__ rate) {
     __shared__ float qs[ATTN_MAX_D];
     __shared__ float ps[ZI_WAVE];
     __shared__ int64_t vbase[ZI_WAVE];
@@ -75,6 +76,7 @@ attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, int64_t l
                 for (int x = 0; x < d; ++x) dot += qs[x] * zi_load(kr + x);
                 s = dot * scale;
                 if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+                if (slope) s -= slope[h] * logf(1.f + rate[h] * (float)(p - j));
                 if (brow) s += brow[p - j < bias_len ? p - j : bias_len - 1];
             }
         }
@@ -115,13 +117,16 @@ attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, int64_t l
 
 // `sinks` (float32 [nh], or null): the softmax of head h also counts exp(sinks[h]) in its denominator.  `softcap` > 0
 // caps the scaled scores; `bias` (float32 [nh][bias_len], or null) is added by distance; `keep_first` positions stay
-// visible beside the window.
+// visible beside the window; `slope` and `rate` (float32 [nh], both or null): slope * ln(1 + rate * distance) is taken
+// off the score.
 extern "C" int zi_attention_generic_biased(void* out, const void* q, int dt, int n, int64_t ldq, int64_t ldo,
                                          const void* kcache, const void* vcache, const int32_t* tok_index,
                                          const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* block_tables,
                                          int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window,
                                          float scale, const float* sinks, float softcap, const float* bias,
-                                         int bias_len, int keep_first, hipStream_t stream) {
+                                         int bias_len, int keep_first, const float* slope, const float* rate,
+                                         hipStream_t stream) {
+    ZI_REQUIRE((slope == nullptr) == (rate == nullptr), "attention: a slope and a rate, or neither");
     ZI_REQUIRE(softcap >= 0.f && keep_first >= 0 && (!bias || bias_len > 0), "attention: bad cap, bias or kept positions");
     ZI_REQUIRE(n >= 0 && nh > 0 && nkv > 0 && d > 0 && page_size > 0 && max_pages > 0 && num_pages > 0,
                "attention: bad sizes");
@@ -134,7 +139,8 @@ extern "C" int zi_attention_generic_biased(void* out, const void* q, int dt, int
     ZI_DISPATCH_DTYPE(dt, T, {
         attention_generic_kernel<T><<<dim3(n, nh), ZI_WAVE, 0, stream>>>(
             (T*)out, (const T*)q, ldq, ldo, (const T*)kcache, (const T*)vcache, tok_index, tok_seq, tok_pos, block_tables,
-            max_pages, num_pages, nh, nkv, d, page_size, window, scale, sinks, softcap, bias, bias_len, keep_first);
+            max_pages, num_pages, nh, nkv, d, page_size, window, scale, sinks, softcap, bias, bias_len, keep_first,
+            slope, rate);
     });
     return zi_check_launch("attention_generic");
 }
@@ -146,7 +152,7 @@ extern "C" int zi_attention_generic_sink(void* out, const void* q, int dt, int n
                                          float scale, const float* sinks, hipStream_t stream) {
     return zi_attention_generic_biased(out, q, dt, n, ldq, ldo, kcache, vcache, tok_index, tok_seq, tok_pos, block_tables,
                                        max_pages, num_pages, nh, nkv, d, page_size, window, scale, sinks, 0.f, nullptr, 0,
-                                       0, stream);
+                                       0, nullptr, nullptr, stream);
 }
 
 extern "C" int zi_attention_generic(void* out, const void* q, int dt, int n, int64_t ldq, int64_t ldo,

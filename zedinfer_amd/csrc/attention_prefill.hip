@@ -267,6 +267,7 @@ attention_prefill_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf16* 
             // the wavefront sees whole needs no mask here either
             const float inv_cap = ex.softcap > 0.f ? 1.f / ex.softcap : 0.f;
             const float* brow = ex.bias ? ex.bias + (int64_t)h * ex.bias_len : nullptr;
+            const float slope = ex.slope ? ex.slope[h] * 0.6931471805599453f : 0.f, rate = ex.slope ? ex.rate[h] : 0.f;
             auto transform = [&](auto masked) __attribute__((always_inline)) {
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
@@ -275,6 +276,7 @@ attention_prefill_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf16* 
                         const int key = kb + (t / 2) * 32 + j * 8 + (t % 2) * 4 + x;
                         float sc = s[t][x] * scale;
                         if (ex.softcap > 0.f) sc = ex.softcap * pf_tanh(sc * inv_cap);
+                        if (ex.slope) sc -= slope * __builtin_amdgcn_logf(fmaf(rate, (float)(qpos - key), 1.f));      // (NaN ahead of the query: masked)
                         if (brow) {
                             int dist = qpos - key;
                             dist = (int)min((unsigned)dist, (unsigned)(ex.bias_len - 1));      // (a key ahead of the query is masked anyway)
@@ -469,7 +471,8 @@ __device__ __attribute__((aligned(16))) const unsigned pf_zero16[4] = {0u, 0u, 0
 // workgroups on a compute unit, which are not in step with each other, so that one's matrix instructions run
 // beside the other's softmax and loads; a tile's walk is one wavefront's per query group, so it takes longer:
 // for launches with many tiles).
-template <int D, int QW, int KH>
+// LOGB: slope * ln(1 + rate * distance) is taken off every score, two numbers a head (ZiScoreExtras).
+template <int D, int QW, int KH, bool LOGB>
 __global__ void __launch_bounds__(4 * KH * ZI_WAVE, KH == 1 ? 2 : 1)
 attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf16* __restrict__ q, int64_t ldq,
                              const zi_bf16* __restrict__ kcache, const zi_bf16* __restrict__ vcache,
@@ -478,7 +481,8 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
                              const int32_t* __restrict__ entry_past, const int32_t* __restrict__ block_tables,
                              int max_pages, int num_pages, int nh, int nkv, int ps_shift, int window, float scale,
                              float* __restrict__ part_o, float* __restrict__ part_ml, int max_chunks, int chunk_keys,
-                             const float* __restrict__ sinks) {
+                             const float* __restrict__ sinks, const float* __restrict__ log_slope,
+                             const float* __restrict__ log_rate) {
     static_assert(D == 64 || D == 128, "this variant takes head sizes 64 and 128");
     static_assert(QW == 1 || QW == 2, "16 or 32 queries a wavefront");
     constexpr int BM = PF_BM * QW;                   // queries of a tile
@@ -530,6 +534,9 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
     const int wave_last = pos0 + ((qs * QR + QR - 1 < count) ? qs * QR + QR - 1 : count - 1);
     const float scale_log2 = scale * 1.4426950408889634f;
     const int wave_lo = (window > 0 && pos0 + qs * QR - window + 1 > 0) ? pos0 + qs * QR - window + 1 : 0;
+    // with LOGB the scores leave their loop in base-2 units, else they are scaled where the maximum is taken off
+    const float to_log2 = LOGB ? 1.f : scale_log2;
+    const float neg_slope = LOGB ? -log_slope[h] : 0.f, rate = LOGB ? log_rate[h] : 0.f;
     pf_bf16x8_t qop[QW][DK];
 #pragma unroll
     for (int u = 0; u < QW; ++u) {
@@ -641,6 +648,18 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
 #pragma unroll
         for (int u = 0; u < QW; ++u) {
             float mx = -INFINITY;
+            if constexpr (LOGB) {
+                // 1 + rate * distance of key kb + j * 8 + c is the first key's minus rate * c (c known at compile time);
+                // not above zero for keys ahead of the query, which are masked
+                const float far = fmaf(rate, (float)(qpos[u] - kb - j * 8), 1.f);
+#pragma unroll
+                for (int t = 0; t < 4; ++t)
+#pragma unroll
+                    for (int x = 0; x < 4; ++x) {
+                        const float lg = __builtin_amdgcn_logf(fmaf(-(float)((t / 2) * 32 + (t % 2) * 4 + x), rate, far));
+                        s[u][t][x] = fmaf(neg_slope, lg, s[u][t][x] * scale_log2);
+                    }
+            }
             if (whole) {
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
@@ -660,7 +679,7 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
             }
             mx = fmaxf(mx, __shfl_xor(mx, 16, ZI_WAVE));
             mx = fmaxf(mx, __shfl_xor(mx, 32, ZI_WAVE));
-            const float m_new = fmaxf(m[u], mx * scale_log2);      // the scale is positive
+            const float m_new = fmaxf(m[u], mx * to_log2);      // the scale is positive
             const float m_use = (m_new == -INFINITY) ? 0.f : m_new;
             const float corr = __builtin_amdgcn_exp2f(m[u] - m_use);
             m[u] = m_new;
@@ -669,7 +688,7 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
             for (int t = 0; t < 4; ++t)
 #pragma unroll
                 for (int x = 0; x < 4; ++x) {
-                    s[u][t][x] = __builtin_amdgcn_exp2f(fmaf(s[u][t][x], scale_log2, -m_use));
+                    s[u][t][x] = __builtin_amdgcn_exp2f(fmaf(s[u][t][x], to_log2, -m_use));
                     psum += s[u][t][x];
                 }
 #pragma unroll
@@ -903,8 +922,8 @@ extern "C" int zi_attention_prefill_cuts(int max_keys, int window, int groups, i
 // tiles; a query's keys are then added in another order, so the result differs by rounding.
 // `sinks` (float32 [nh], or null): the softmax of head h also counts exp(sinks[h]) in its denominator, once, whatever
 // the number of cuts of a tile's keys.
-// `softcap`, `bias` (float32 [nh][bias_len]) and `keep_first`: see ZiScoreExtras; with any of them tiles hold 64
-// queries and the kernel that stages through registers runs for every head size.
+// `softcap`, `bias` (float32 [nh][bias_len]), `keep_first`, `slope` and `rate`: see ZiScoreExtras; with any of the first
+// three tiles hold 64 queries and the kernel that stages through registers runs for every head size.
 extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,
                                            const void* kcache, const void* vcache, const int32_t* tile_entry,
                                            const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
@@ -912,11 +931,13 @@ extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int
                                            int num_pages, int nh, int nkv, int d, int page_size, int window, float scale,
                                            int rows, int max_chunks, float* workspace, int64_t workspace_floats, int tile,
                                            int alone, int chunk_keys, const float* sinks, float softcap,
-                                           const float* bias, int bias_len, int keep_first, hipStream_t stream) {
-    const bool biased = softcap > 0.f || bias != nullptr || keep_first > 0;
+                                           const float* bias, int bias_len, int keep_first, const float* slope,
+                                           const float* rate, hipStream_t stream) {
+    const bool tabled = softcap > 0.f || bias != nullptr || keep_first > 0, biased = tabled || slope != nullptr;
+    ZI_REQUIRE((slope == nullptr) == (rate == nullptr), "attention_prefill: a slope and a rate, or neither");
     ZI_REQUIRE(softcap >= 0.f && keep_first >= 0 && (!bias || bias_len > 0), "attention_prefill: bad cap, bias or kept positions");
-    ZI_REQUIRE(!biased || (tile == PF_BM && !alone), "attention_prefill: capped or biased scores and kept positions take tiles of %d queries", PF_BM);
-    const ZiScoreExtras ex = {softcap, bias, bias_len, keep_first};
+    ZI_REQUIRE(!tabled || (tile == PF_BM && !alone), "attention_prefill: capped or biased scores and kept positions take tiles of %d queries", PF_BM);
+    const ZiScoreExtras ex = {softcap, bias, bias_len, keep_first, slope, rate};
     ZI_REQUIRE(tile == PF_BM || (tile == 2 * PF_BM && pf_variant >= 1 && (d == 64 || d == 128)),
                "attention_prefill: tiles of %d queries (64, or 128 for head sizes 64 and 128)", tile);
     ZI_REQUIRE(zi_attention_prefill_supported(dt, nh, nkv, d, page_size),
@@ -955,12 +976,17 @@ extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int
             (zi_bf16*)out, ldo, (const zi_bf16*)q, ldq, (const zi_bf16*)kcache, (const zi_bf16*)vcache, tile_entry, \
             tile_off, entry_start, entry_len, entry_past, block_tables, max_pages, num_pages, nh, nkv, ps_shift, \
             window, scale, po, pml, max_chunks, chunk_keys, sinks, ex)
-#define ZI_PF_DMA(DD, QW, KH)                                                                                  \
-    attention_prefill_dma_kernel<DD, QW, KH><<<grid, 4 * KH * ZI_WAVE, 0, stream>>>(                           \
+#define ZI_PF_DMA2(DD, QW, KH, LOGB)                                                                           \
+    attention_prefill_dma_kernel<DD, QW, KH, LOGB><<<grid, 4 * KH * ZI_WAVE, 0, stream>>>(                     \
         (zi_bf16*)out, ldo, (const zi_bf16*)q, ldq, (const zi_bf16*)kcache, (const zi_bf16*)vcache, tile_entry, \
         tile_off, entry_start, entry_len, entry_past, block_tables, max_pages, num_pages, nh, nkv, ps_shift,   \
-        window, scale, po, pml, max_chunks, chunk_keys, sinks)
-    const bool dma = !biased && pf_variant >= 1 && (d == 64 || d == 128);
+        window, scale, po, pml, max_chunks, chunk_keys, sinks, slope, rate)
+#define ZI_PF_DMA(DD, QW, KH)                              \
+    do {                                                   \
+        if (slope) ZI_PF_DMA2(DD, QW, KH, true);           \
+        else ZI_PF_DMA2(DD, QW, KH, false);                \
+    } while (0)
+    const bool dma = !tabled && pf_variant >= 1 && (d == 64 || d == 128);
     const bool wide = tile == 2 * PF_BM;
     ZI_REQUIRE(!alone || dma, "attention_prefill: workgroups of four wavefronts are for head sizes 64 and 128");
     if (dma && d == 128 && wide && alone) ZI_PF_DMA(128, 2, 1);
@@ -984,6 +1010,7 @@ extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int
     }
 #undef ZI_PF
 #undef ZI_PF_DMA
+#undef ZI_PF_DMA2
     if (max_chunks > 1)
         attention_prefill_merge_kernel<<<dim3(num_tiles * tile, nh), ZI_WAVE, 0, stream>>>(
             (zi_bf16*)out, ldo, po, pml, tile_entry, tile_off, entry_start, entry_len, entry_past, nh, d, window, max_chunks,
@@ -1001,7 +1028,7 @@ extern "C" int zi_attention_prefill_sink(void* out, const void* q, int dt, int n
     return zi_attention_prefill_biased(out, q, dt, num_tiles, ldq, ldo, kcache, vcache, tile_entry, tile_off, entry_start,
                                        entry_len, entry_past, block_tables, max_pages, num_pages, nh, nkv, d, page_size,
                                        window, scale, rows, max_chunks, workspace, workspace_floats, tile, alone,
-                                       chunk_keys, sinks, 0.f, nullptr, 0, 0, stream);
+                                       chunk_keys, sinks, 0.f, nullptr, 0, 0, nullptr, nullptr, stream);
 }
 
 extern "C" int zi_attention_prefill(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,

@@ -5,6 +5,7 @@
 //   y_t[c] = sum_j taps[c][j] * u_(t - (taps-1) + j)[c]                 zeros before the sequence's start
 //   q = y_q / rms(y_q) * w_q,  k = y_k / rms(y_k) * w_k                 one root mean square over ALL heads' channels
 //   the first R dims of every head of q and k turn in pairs (i, i + R/2) by the step's angles
+//   v <- (1 - mix) v + mix * v_other, the same token's values of another layer, where the mixer asks for it
 //   q -> q_out [n][heads * D];  k, v -> the paged cache at the token's slot (heads of D values; a head of fewer
 //   dims is followed by zeros, so that one head size serves keys of `dim` and values of `vdim` dims)
 //
@@ -101,7 +102,8 @@ conv_qkv_kernel(T* __restrict__ q_out, int64_t ldq, T* __restrict__ kcache, T* _
                 const float* __restrict__ k_norm, float eps, const float* __restrict__ table, int rot,
                 const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ entry_start,
                 const int32_t* __restrict__ entry_slot, const int32_t* __restrict__ slots, int64_t cache_slots, int nh,
-                int nkv, int dim, int vdim, int D, int taps, int page_size) {
+                int nkv, int dim, int vdim, int D, int taps, int page_size, float* __restrict__ values_out,
+                const float* __restrict__ mix_values, float mix) {
     extern __shared__ float y[];      // [C] the convolved channels, q and k already times their gains; then [rot] angles
     __shared__ float red[16];
     const int t = blockIdx.x, e = tok_seq[t], local = t - entry_start[e];
@@ -115,10 +117,15 @@ conv_qkv_kernel(T* __restrict__ q_out, int64_t ldq, T* __restrict__ kcache, T* _
     for (int c = threadIdx.x; c < C; c += THREADS) {
         float u[TAPS > 0 ? TAPS : 1];
         const float gain = c < Qd ? q_norm[c] : (c < Qd + Kd ? k_norm[c - Qd] : 1.f);
-        const float v = cq_conv<TP, TAPS>(proj, ld, splits, split_stride, bias, conv_w, tail, t, local, c, C, taps, u);
-        y[c] = v * gain;
+        float v = cq_conv<TP, TAPS>(proj, ld, splits, split_stride, bias, conv_w, tail, t, local, c, C, taps, u);
         if (c < Qd) sq += v * v;
         else if (c < Qd + Kd) sk += v * v;
+        else {
+            const int64_t at = (int64_t)t * Vd + (c - Qd - Kd);
+            if (values_out) values_out[at] = v;
+            if (mix_values) v = (1.f - mix) * v + mix * mix_values[at];
+        }
+        y[c] = v * gain;
         // a step in which every entry brings one token: no other workgroup reads this entry's tail, and this thread
         // alone reads and writes channel c of it, so the tail moves on here (a token without a place in the cache is
         // padding and moves nothing)
@@ -178,14 +185,16 @@ conv_qkv_kernel(T* __restrict__ q_out, int64_t ldq, T* __restrict__ kcache, T* _
 }
 
 // `move_tail` (only for steps in which every entry brings one token): the kernel also writes the new tail, and
-// zi_conv_tail is not needed.  `splits` > 1: proj comes as float32 partial sums [splits][n][ld].
+// zi_conv_tail is not needed.  `splits` > 1: proj comes as float32 partial sums [splits][n][ld].  values_out (float32
+// [n][nkv*vdim], or null) receives the convolved values as they are; with mix_values (the same shape, or null) the
+// values that are cached are (1 - mix) v + mix * mix_values.
 extern "C" int zi_conv_qkv(void* q_out, int dt, int64_t ldq, void* kcache, void* vcache, const void* proj, int proj_dt,
                            int64_t ld, int splits, int64_t split_stride, const float* bias, const float* conv_w,
                            float* state, int64_t state_stride, int move_tail, const float* q_norm, const float* k_norm,
                            float eps, const float* table, int rot, int n,
                            const int32_t* tok_seq, const int32_t* entry_start, const int32_t* entry_slot,
                            const int32_t* slots, int64_t cache_slots, int nh, int nkv, int dim, int vdim, int D, int taps,
-                           int page_size, hipStream_t stream) {
+                           int page_size, float* values_out, const float* mix_values, float mix, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0 && dim > 0 && vdim > 0 && D >= dim && D >= vdim && taps >= 1 &&
                    taps <= CQ_MAX_TAPS && page_size > 0,
                "conv_qkv: bad sizes (heads %d/%d, dim %d, vdim %d, head size %d, taps %d)", nh, nkv, dim, vdim, D, taps);
@@ -209,7 +218,7 @@ extern "C" int zi_conv_qkv(void* q_out, int dt, int64_t ldq, void* kcache, void*
     conv_qkv_kernel<TP, T, TAPS, THREADS><<<n, THREADS, lds, stream>>>(                                                \
         (T*)q_out, ldq, (T*)kcache, (T*)vcache, (const TP*)proj, ld, splits, split_stride, bias, conv_w, state,       \
         state_stride, move_tail, q_norm, k_norm, eps, table, rot, tok_seq, entry_start, entry_slot, slots, cache_slots, \
-        nh, nkv, dim, vdim, D, taps, page_size)
+        nh, nkv, dim, vdim, D, taps, page_size, values_out, mix_values, mix)
 #define ZI_CQ_TAPS(THREADS)                                                 \
     switch (taps) {                                                         \
         case 2: ZI_CQ(2, THREADS); break;                                   \

@@ -3,25 +3,25 @@
 #include "zi_common.h"
 #include "zi_api.h"
 
-// out[i,:] = table[ids[i],:]   (reference: src/backend/ops/embedding/cpu/embedding_cpu.cpp:10-23).
+// out[i,:] = table[ids[i],:] * scale   (scale 1: reference: src/backend/ops/embedding/cpu/embedding_cpu.cpp:10-23).
 // An id outside [0, V) writes NaN into the row so that the fault shows.
 template <typename TW, typename TO>
 __global__ void embedding_kernel(TO* __restrict__ out, const TW* __restrict__ table,
-                                 const int32_t* __restrict__ ids, int H, int V) {
+                                 const int32_t* __restrict__ ids, int H, int V, float scale) {
     const int64_t row = blockIdx.x;
     const int id = ids[row];
     const bool ok = id >= 0 && id < V;
     const TW* src = table + (int64_t)(ok ? id : 0) * H;
     TO* dst = out + row * H;
-    for (int j = threadIdx.x; j < H; j += blockDim.x) zi_store(dst + j, ok ? zi_load(src + j) : NAN);
+    for (int j = threadIdx.x; j < H; j += blockDim.x) zi_store(dst + j, ok ? zi_load(src + j) * scale : NAN);
 }
 
 extern "C" int zi_embedding(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids,
-                            int n, int hidden, int vocab, hipStream_t stream) {
+                            int n, int hidden, int vocab, float scale, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && hidden > 0 && vocab > 0, "embedding: bad sizes n=%d hidden=%d vocab=%d", n, hidden, vocab);
     if (n == 0) return 0;
     ZI_DISPATCH_DTYPE(table_dt, TW, ZI_DISPATCH_DTYPE(out_dt, TO, {
-        embedding_kernel<TW, TO><<<n, 256, 0, stream>>>((TO*)out, (const TW*)table, ids, hidden, vocab);
+        embedding_kernel<TW, TO><<<n, 256, 0, stream>>>((TO*)out, (const TW*)table, ids, hidden, vocab, scale);
     }));
     return zi_check_launch("embedding");
 }
@@ -270,13 +270,21 @@ __global__ void relu_squared_vec_kernel(TO* __restrict__ out, int64_t ldo, const
 
 template <typename T, typename TO>
 __global__ void clamped_glu_vec_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ gate, const T* __restrict__ up,
-                                       int64_t ld_gate, int64_t ld_up, int n, int inter, float limit, float alpha) {
+                                       int64_t ld_gate, int64_t ld_up, int n, int inter, float limit, float alpha,
+                                       const float* __restrict__ gate_bias, const float* __restrict__ up_bias) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     const int q = inter / 4;
     if (i >= (int64_t)n * q) return;
     const int64_t r = i / q, c = (i % q) * 4;
     const float4 g4 = ew_load4(gate + r * ld_gate + c), u4 = ew_load4(up + r * ld_up + c);
-    const float g[4] = {g4.x, g4.y, g4.z, g4.w}, u[4] = {u4.x, u4.y, u4.z, u4.w};
+    float g[4] = {g4.x, g4.y, g4.z, g4.w}, u[4] = {u4.x, u4.y, u4.z, u4.w};
+    if (gate_bias) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            g[k] += gate_bias[c + k];
+            u[k] += up_bias[c + k];
+        }
+    }
     float o[4];
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
@@ -325,7 +333,8 @@ extern "C" int zi_relu_squared(void* out, int out_dt, int64_t ldo, const void* z
 template <typename T, typename TO>
 __global__ void clamped_glu_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ gate, const T* __restrict__ up,
                                    int64_t ld_gate, int64_t ld_up, int splits, int64_t split_stride, int n, int inter,
-                                   float limit, float alpha) {
+                                   float limit, float alpha, const float* __restrict__ gate_bias,
+                                   const float* __restrict__ up_bias) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (int64_t)n * inter) return;
     const int64_t r = i / inter, c = i % inter;
@@ -334,6 +343,10 @@ __global__ void clamped_glu_kernel(TO* __restrict__ out, int64_t ldo, const T* _
         g += zi_load(gate + s * split_stride + r * ld_gate + c);
         u += zi_load(up + s * split_stride + r * ld_up + c);
     }
+    if (gate_bias) {
+        g += gate_bias[c];
+        u += up_bias[c];
+    }
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     zi_store(out + r * ldo + c, g / (1.f + expf(-alpha * g)) * (u + 1.f));
@@ -341,7 +354,8 @@ __global__ void clamped_glu_kernel(TO* __restrict__ out, int64_t ldo, const T* _
 
 extern "C" int zi_clamped_glu(void* out, int out_dt, int64_t ldo, const void* gate, const void* up, int dt, int64_t ld_gate,
                               int64_t ld_up, int splits, int64_t split_stride, int n, int inter, float limit, float alpha,
-                              hipStream_t stream) {
+                              const float* gate_bias, const float* up_bias, hipStream_t stream) {
+    ZI_REQUIRE((gate_bias == nullptr) == (up_bias == nullptr), "clamped_glu: biases of both halves or of neither");
     ZI_REQUIRE(n >= 0 && inter > 0 && ldo >= inter && ld_gate >= inter && ld_up >= inter && splits >= 1,
                "clamped_glu: bad sizes");
     ZI_REQUIRE(limit > 0.f, "clamped_glu: the limit must be positive, got %g", (double)limit);
@@ -350,13 +364,14 @@ extern "C" int zi_clamped_glu(void* out, int out_dt, int64_t ldo, const void* ga
     if (splits == 1 && ew_rows4(gate, ld_gate, inter) && ew_rows4(up, ld_up, inter) && ew_rows4(out, ldo, inter)) {
         ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(out_dt, TO, {
             clamped_glu_vec_kernel<T, TO><<<(unsigned)((total / 4 + 255) / 256), 256, 0, stream>>>(
-                (TO*)out, ldo, (const T*)gate, (const T*)up, ld_gate, ld_up, n, inter, limit, alpha);
+                (TO*)out, ldo, (const T*)gate, (const T*)up, ld_gate, ld_up, n, inter, limit, alpha, gate_bias, up_bias);
         }));
         return zi_check_launch("clamped_glu");
     }
     ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(out_dt, TO, {
         clamped_glu_kernel<T, TO><<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(
-            (TO*)out, ldo, (const T*)gate, (const T*)up, ld_gate, ld_up, splits, split_stride, n, inter, limit, alpha);
+            (TO*)out, ldo, (const T*)gate, (const T*)up, ld_gate, ld_up, splits, split_stride, n, inter, limit, alpha,
+            gate_bias, up_bias);
     }));
     return zi_check_launch("clamped_glu");
 }

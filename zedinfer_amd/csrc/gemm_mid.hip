@@ -76,6 +76,10 @@ __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* _
         const int nb = n0 + j * 4;
         if (nb + 3 < N && vec_out) {
             if (mode == GM_MODE_PARTIAL) {
+                if (bias && split == 0) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) s[e] += zi_load(bias + nb + e);
+                }
                 *reinterpret_cast<gm_f32x4_t*>((float*)out + ((int64_t)split * M + m) * N + nb) = s;
             } else {
                 if (bias) {
@@ -98,7 +102,7 @@ __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* _
             const int n = nb + e;
             if (n >= N) continue;
             if (mode == GM_MODE_PARTIAL) {
-                ((float*)out)[((int64_t)split * M + m) * N + n] = s[e];
+                ((float*)out)[((int64_t)split * M + m) * N + n] = s[e] + ((bias && split == 0) ? zi_load(bias + n) : 0.f);
             } else {
                 const float v = s[e] + (bias ? zi_load(bias + n) : 0.f);
                 if (out_f32) ((float*)out)[(int64_t)m * ldo + n] = v;

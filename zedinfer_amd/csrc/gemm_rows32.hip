@@ -191,6 +191,10 @@ gemm_rows32_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16*
             g32_f32x4_t s = g32_f32x4_t{acc[t][g * 4], acc[t][g * 4 + 1], acc[t][g * 4 + 2], acc[t][g * 4 + 3]};
             if (nb + 3 < N && vec_out) {
                 if (mode == G32_MODE_PARTIAL) {
+                    if (bias && split == 0) {
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) s[e] += zi_load(bias + nb + e);
+                    }
                     *reinterpret_cast<g32_f32x4_t*>((float*)out + ((int64_t)split * M + m) * N + nb) = s;
                 } else {
                     if (bias) {
@@ -213,7 +217,7 @@ gemm_rows32_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16*
                 const int n = nb + e;
                 if (n >= N) continue;
                 if (mode == G32_MODE_PARTIAL) {
-                    ((float*)out)[((int64_t)split * M + m) * N + n] = s[e];
+                    ((float*)out)[((int64_t)split * M + m) * N + n] = s[e] + ((bias && split == 0) ? zi_load(bias + n) : 0.f);
                 } else {
                     const float v = s[e] + (bias ? zi_load(bias + n) : 0.f);
                     if (out_f32) ((float*)out)[(int64_t)m * ldo + n] = v;

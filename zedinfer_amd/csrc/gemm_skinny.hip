@@ -86,7 +86,7 @@ extern "C" int64_t zi_gemm_skinny_workspace(int M, int N, int K) {
 }
 
 // mode 0: out[M,N] (+ bias), reduced through `workspace` when the product is split.
-// mode 1: out = float32 partial sums [splits][M][N] (no bias; splits from zi_gemm_skinny_splits).
+// mode 1: out = float32 partial sums [splits][M][N] (splits from zi_gemm_skinny_splits; the bias, if any, is in the first).
 // mode 2: w holds gate and up rows interleaved in blocks of 8; out[M, N/2] (bfloat16) =
 //         up * silu(gate); only for products that are not split.
 extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M,
@@ -121,7 +121,7 @@ extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, co
         ZI_REQUIRE(N % 16 == 0 && out_dt == ZI_BF16 && ldo >= N / 2,
                    "gemm_skinny: the SwiGLU epilogue needs N %% 16 == 0 and a bfloat16 out of N/2 columns");
     }
-    const zi_bf16* b = kmode == SK_MODE_PLAIN ? (const zi_bf16*)bias : nullptr;
+    const zi_bf16* b = (kmode == SK_MODE_PLAIN || mode == SK_MODE_PARTIAL) ? (const zi_bf16*)bias : nullptr;
     // four columns go out as one store when every row of the destination keeps them aligned
     int vec_out;
     if (kmode == SK_MODE_PARTIAL) vec_out = N % 4 == 0 && ((uintptr_t)dst % 16) == 0;

@@ -364,10 +364,12 @@ extern "C" int zi_linear_attention(float* out, int64_t ldo, const float* q, cons
 template <typename TX, typename TO>
 __global__ void __launch_bounds__(256)
 gate_heads_kernel(TO* __restrict__ out, int64_t ldo, const TX* __restrict__ x, int64_t ldx, int x_head,
-                  const float* __restrict__ gate, int64_t ld_gate, int width, int head, int act, float scale) {
+                  const float* __restrict__ gate, int64_t ld_gate, int splits, int64_t split_stride, int width, int head,
+                  int act, float scale) {
     const int64_t t = blockIdx.x;
     for (int j = threadIdx.x; j < width; j += blockDim.x) {
-        const float g = gate[t * ld_gate + j];
+        float g = gate[t * ld_gate + j];
+        for (int s = 1; s < splits; ++s) g += gate[s * split_stride + t * ld_gate + j];
         const float a = act == GATE_SILU ? la_silu(g) : la_sigmoid(g);
         const float xv = zi_load(x + t * ldx + (int64_t)(j / head) * x_head + j % head);
         zi_store(out + t * ldo + j, xv * a * scale);
@@ -375,17 +377,18 @@ gate_heads_kernel(TO* __restrict__ out, int64_t ldo, const TX* __restrict__ x, i
 }
 
 // out [n][width] = x * act(gate) * scale; x holds heads of x_head >= head values of which the first `head` count
-// (x[t][(j / head) * x_head + j % head]); gate float32 [n][width] (row stride ld_gate).
+// (x[t][(j / head) * x_head + j % head]); gate float32 [n][width] (row stride ld_gate), or `splits` partial sums of it
+// `split_stride` apart, added in rising order.
 extern "C" int zi_gate_heads(void* out, int out_dt, int64_t ldo, const void* x, int x_dt, int64_t ldx, int x_head,
-                             const float* gate, int64_t ld_gate, int n, int width, int head, int act, float scale,
-                             hipStream_t stream) {
-    ZI_REQUIRE(n >= 0 && width > 0 && head > 0 && width % head == 0 && x_head >= head && ldo >= width &&
+                             const float* gate, int64_t ld_gate, int splits, int64_t split_stride, int n, int width,
+                             int head, int act, float scale, hipStream_t stream) {
+    ZI_REQUIRE(splits >= 1 && n >= 0 && width > 0 && head > 0 && width % head == 0 && x_head >= head && ldo >= width &&
                ld_gate >= width && ldx >= (int64_t)(width / head) * x_head, "gate_heads: bad sizes");
     ZI_REQUIRE(act == GATE_SIGMOID || act == GATE_SILU, "gate_heads: unknown activation %d", act);
     if (n == 0) return 0;
     ZI_DISPATCH_DTYPE(x_dt, TX, ZI_DISPATCH_DTYPE(out_dt, TO, {
-        gate_heads_kernel<TX, TO><<<n, 256, 0, stream>>>((TO*)out, ldo, (const TX*)x, ldx, x_head, gate, ld_gate, width,
-                                                         head, act, scale);
+        gate_heads_kernel<TX, TO><<<n, 256, 0, stream>>>((TO*)out, ldo, (const TX*)x, ldx, x_head, gate, ld_gate, splits,
+                                                         split_stride, width, head, act, scale);
     }));
     return zi_check_launch("gate_heads");
 }

@@ -44,7 +44,7 @@ int zi_decode_layer(float* resid, int n, int H, int I, const void* norm1, const 
     max_keys, void* workspace, int64_t workspace_bytes, uint32_t* sync, int* err, int spin_limit, hipStream_t stream);
 // elementwise.hip
 int zi_embedding(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids, int n, int hidden, int
-    vocab, hipStream_t stream);
+    vocab, float scale, hipStream_t stream);
 // elementwise.hip
 int zi_gather_rows(void* out, const void* in, int dt, const int32_t* idx, int n_out, int n_in, int hidden, hipStream_t
     stream);
@@ -122,7 +122,7 @@ int zi_latent_value(void* out, int out_dt, int64_t ldo, const float* o, const vo
 int zi_delta_prepare(float* qk, float* v, float* beta_g, const float* proj, int64_t ld, int n, const void* conv_w, const
     void* a_log, const void* dt_bias, int w_dt, const float* state, int64_t state_stride, int64_t conv_off, const
     int32_t* tok_seq, const int32_t* entry_start, const int32_t* entry_slot, int heads, int kvh, int dim, int vdim, int
-    taps, hipStream_t stream);
+    taps, int b_at, int a_at, hipStream_t stream);
 // delta.hip
 int zi_delta_conv_state(float* state, int64_t state_stride, int64_t conv_off, const float* proj, int64_t ld, const
     int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, int entries, int channels, int taps,
@@ -176,7 +176,7 @@ int zi_conv_qkv(void* q_out, int dt, int64_t ldq, void* kcache, void* vcache, co
     int splits, int64_t split_stride, const float* bias, const float* conv_w, float* state, int64_t state_stride, int
     move_tail, const float* q_norm, const float* k_norm, float eps, const float* table, int rot, int n, const int32_t* tok_seq, const int32_t* entry_start, const
     int32_t* entry_slot, const int32_t* slots, int64_t cache_slots, int nh, int nkv, int dim, int vdim, int D, int taps,
-    int page_size, hipStream_t stream);
+    int page_size, float* values_out, const float* mix_values, float mix, hipStream_t stream);
 // conv_qkv.hip
 int zi_conv_tail(float* state, int64_t state_stride, const void* proj, int proj_dt, int64_t ld, int splits, int64_t
     split_stride, const float* bias, const
@@ -187,7 +187,8 @@ int zi_relu_squared(void* out, int out_dt, int64_t ldo, const void* z, int dt, i
     split_stride, int n, int inter, hipStream_t stream);
 // elementwise.hip
 int zi_clamped_glu(void* out, int out_dt, int64_t ldo, const void* gate, const void* up, int dt, int64_t ld_gate, int64_t
-    ld_up, int splits, int64_t split_stride, int n, int inter, float limit, float alpha, hipStream_t stream);
+    ld_up, int splits, int64_t split_stride, int n, int inter, float limit, float alpha, const float* gate_bias, const float* up_bias,
+    hipStream_t stream);
 // elementwise.hip
 int zi_softcap(float* x, int64_t total, float cap, hipStream_t stream);
 // elementwise.hip
@@ -220,7 +221,8 @@ int zi_linear_attention(float* out, int64_t ldo, const float* q, const float* k,
     heads, int dim, int vdim, int act, float qscale, hipStream_t stream);
 // linear_attention.hip
 int zi_gate_heads(void* out, int out_dt, int64_t ldo, const void* x, int x_dt, int64_t ldx, int x_head, const float*
-    gate, int64_t ld_gate, int n, int width, int head, int act, float scale, hipStream_t stream);
+    gate, int64_t ld_gate, int splits, int64_t split_stride, int n, int width, int head, int act, float scale,
+    hipStream_t stream);
 // delta.hip
 int zi_gated_rmsnorm_act(void* out, int out_dt, int64_t ldo, const float* o, const void* w, int w_dt, const float*
     gate, int64_t ld_gate, int n, int heads, int vdim, float eps, int act, float scale, hipStream_t stream);
@@ -232,20 +234,21 @@ int zi_normed_kv_store(void* q_out, int dt, int64_t ldq, void* kcache, void* vca
 int zi_attention_generic_biased(void* out, const void* q, int dt, int n, int64_t ldq, int64_t ldo, const void* kcache,
     const void* vcache, const int32_t* tok_index, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t*
     block_tables, int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window, float scale, const
-    float* sinks, float softcap, const float* bias, int bias_len, int keep_first, hipStream_t stream);
+    float* sinks, float softcap, const float* bias, int bias_len, int keep_first, const float* slope, const float* rate,
+    hipStream_t stream);
 // attention_prefill.hip
 int zi_attention_prefill_biased(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo, const void*
     kcache, const void* vcache, const int32_t* tile_entry, const int32_t* tile_off, const int32_t* entry_start, const
     int32_t* entry_len, const int32_t* entry_past, const int32_t* block_tables, int max_pages, int num_pages, int nh,
     int nkv, int d, int page_size, int window, float scale, int rows, int max_chunks, float* workspace, int64_t
     workspace_floats, int tile, int alone, int chunk_keys, const float* sinks, float softcap, const float* bias, int
-    bias_len, int keep_first, hipStream_t stream);
+    bias_len, int keep_first, const float* slope, const float* rate, hipStream_t stream);
 // attention_decode.hip
 int zi_attention_decode_biased(void* out, const void* q, int dt, int n_idx, int64_t ldq, int64_t ldo, const void* kcache,
     const void* vcache, const int32_t* tok_index, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t*
     block_tables, int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window, float scale, int
     max_chunks, float* workspace, int64_t workspace_floats, const float* sinks, float softcap, const float* bias, int
-    bias_len, int keep_first, hipStream_t stream);
+    bias_len, int keep_first, const float* slope, const float* rate, hipStream_t stream);
 // moe.hip
 int zi_moe_route_table(int32_t* idx, float* wt, const int32_t* ids, const int32_t* table, int n, int vocab, int
     experts, int top, hipStream_t stream);
@@ -301,6 +304,27 @@ int zi_moe_weighted_glu(void* out, int out_dt, int64_t ldo, const float* gu, int
 // moe.hip
 int zi_moe_sum_shared(float* out, const float* y, const int32_t* place_of, const float* shared, int splits, int64_t
     split_stride, const float* gate, int64_t ld_gate, int n, int top, int hidden, hipStream_t stream);
+// input_conv.hip
+int zi_stream_scale(float* scale, float* resid, const void* delta, int delta_dt, int splits, int64_t split_stride, int n,
+    int hidden, float eps, hipStream_t stream);
+// input_conv.hip
+int zi_input_conv(void* out, int out_dt, int64_t ldo, const void* x, int x_dt, int64_t ldx, const float* scale, const void*
+    gain, int gain_dt, float gain_add, const float* conv_w, float* state, int64_t state_stride, const int32_t* tok_seq,
+    const int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, const int32_t* slots, int n, int
+    hidden, int taps, hipStream_t stream);
+// input_conv.hip
+int zi_norm_input_conv(void* out, int out_dt, float* resid, const void* delta, int delta_dt, int splits, int64_t
+    split_stride, const void* gain, int gain_dt, float gain_add, float eps, const float* conv_w, float* state, int64_t
+    state_stride, const int32_t* tok_seq, const int32_t* entry_slot, const int32_t* slots, int n, int hidden, int taps,
+    hipStream_t stream);
+// delta_channel.hip
+int zi_lowrank_gates(float* out_a, const float* u_a, const void* w_a, int Ca, int Ra, const float* bias, const float*
+    a_log, int dim, float* out_g, const float* u_g, const void* w_g, int Cg, int Rg, int w_dt, int64_t ldu, int n,
+    hipStream_t stream);
+// delta_channel.hip
+int zi_delta_channel(float* out, const float* qk, const float* v, const float* beta, int64_t ld_beta, const float* g, float*
+    state, int64_t state_stride, const int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, int
+    entries, int heads, int kvh, int dim, int vdim, int single_tokens, hipStream_t stream);
 // sampling.hip
 int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int rows, int vocab, const float*
     temperature, const int32_t* top_k, const float* top_p, const float* penalty, const float* uniform, const int32_t*
@@ -383,5 +407,10 @@ int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int ro
     X(zi_moe_route_sigmoid) \
     X(zi_moe_weighted_glu) \
     X(zi_moe_sum_shared) \
+    X(zi_stream_scale) \
+    X(zi_input_conv) \
+    X(zi_norm_input_conv) \
+    X(zi_lowrank_gates) \
+    X(zi_delta_channel) \
     X(zi_argmax) \
     X(zi_sample)

@@ -24,12 +24,15 @@
 // ---- what a softmax mixer may do to a score beside scaling it --------------------------------------
 // score = (q . k) * scale; then softcap * tanh(score / softcap) when softcap > 0; then + bias[head][min(distance,
 // bias_len - 1)] when bias is not null (float32 [heads][bias_len], distance = query position - key position); beside
-// the window, the sequence's first keep_first positions stay visible.
+// the window, the sequence's first keep_first positions stay visible.  With slope and rate (float32 [heads] each, both
+// or neither) slope[head] * ln(1 + rate[head] * distance) is taken off the scaled (and capped) score.
 struct ZiScoreExtras {
     float softcap;
     const float* bias;
     int bias_len;
     int keep_first;
+    const float* slope;
+    const float* rate;
 };
 
 // ---- places in the pool --------------------------------------------------------------------------

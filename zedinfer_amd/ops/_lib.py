@@ -18,7 +18,7 @@ P, I, L, F = c_void_p, c_int, c_int64, c_float
 
 _PROTOTYPES = {
     "zi_abi_version": [],
-    "zi_embedding": [P, I, P, I, P, I, I, I, P],
+    "zi_embedding": [P, I, P, I, P, I, I, I, F, P],
     "zi_gather_rows": [P, P, I, P, I, I, I, P],
     "zi_add": [P, I, P, I, P, I, L, P],
     "zi_swiglu": [P, I, P, P, I, I, I, L, L, I, I, L, P],
@@ -77,7 +77,7 @@ _PROTOTYPES = {
     "zi_headwise_linear_supported": [I, I, L, I],
     "zi_latent_query_rot": [P, P, I, L, P, I, I, I, I, I, P],
     "zi_latent_value": [P, I, L, P, P, I, I, I, I, I, P],
-    "zi_delta_prepare": [P, P, P, P, L, I, P, P, P, I, P, L, L, P, P, P, I, I, I, I, I, P],
+    "zi_delta_prepare": [P, P, P, P, L, I, P, P, P, I, P, L, L, P, P, P, I, I, I, I, I, I, I, P],
     "zi_delta_conv_state": [P, L, L, P, L, P, P, P, I, I, I, P],
     "zi_delta_rule": [P, P, P, P, P, L, P, P, P, I, I, I, I, I, P],
     "zi_gated_rmsnorm": [P, I, P, P, I, P, L, I, I, I, F, P],
@@ -91,10 +91,10 @@ _PROTOTYPES = {
                                   P, P],
     "zi_attention_decode_project_sink": [P, P, L, I, P, I, I, P, I, L, I, I, I, P, P],
     "zi_layer_norm": [P, I, L, P, P, I, I, L, L, P, P, I, I, I, F, P],
-    "zi_conv_qkv": [P, I, L, P, P, P, I, L, I, L, P, P, P, L, I, P, P, F, P, I, I, P, P, P, P, L, I, I, I, I, I, I, I, P],
+    "zi_conv_qkv": [P, I, L, P, P, P, I, L, I, L, P, P, P, L, I, P, P, F, P, I, I, P, P, P, P, L, I, I, I, I, I, I, I, P, P, F, P],
     "zi_conv_tail": [P, L, P, I, L, I, L, P, P, P, P, P, I, I, I, P],
     "zi_relu_squared": [P, I, L, P, I, L, I, L, I, I, P],
-    "zi_clamped_glu": [P, I, L, P, P, I, L, L, I, L, I, I, F, F, P],
+    "zi_clamped_glu": [P, I, L, P, P, I, L, L, I, L, I, I, F, F, P, P, P],
     "zi_softcap": [P, L, F, P],
     "zi_convert": [P, I, P, I, L, P],
     "zi_moe_route_top": [P, P, P, P, I, I, I, P],
@@ -103,13 +103,14 @@ _PROTOTYPES = {
     "zi_stream_reenter": [P, P, I, I, L, P, P, I, I, I, P],
     "zi_lowrank_decay": [P, L, P, L, P, P, I, I, I, I, F, P],
     "zi_linear_attention": [P, L, P, P, P, L, P, L, P, P, L, P, P, P, P, I, I, I, I, I, F, P],
-    "zi_gate_heads": [P, I, L, P, I, L, I, P, L, I, I, I, I, F, P],
+    "zi_gate_heads": [P, I, L, P, I, L, I, P, L, I, L, I, I, I, I, F, P],
     "zi_gated_rmsnorm_act": [P, I, L, P, P, I, P, L, I, I, I, F, I, F, P],
     "zi_normed_kv_store": [P, I, L, P, P, P, L, I, I, I, P, L, I, I, I, I, I, I, I, F, I, P],
-    "zi_attention_generic_biased": [P, P, I, I, L, L, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, F, P, I, I, P],
+    "zi_attention_generic_biased": [P, P, I, I, L, L, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, F, P, I, I, P, P, P],
     "zi_attention_prefill_biased": [P, P, I, I, L, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, L, I, I, I,
-                                    P, F, P, I, I, P],
-    "zi_attention_decode_biased": [P, P, I, I, L, L, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, L, P, F, P, I, I, P],
+                                    P, F, P, I, I, P, P, P],
+    "zi_attention_decode_biased": [P, P, I, I, L, L, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, P, L, P, F, P, I, I, P, P,
+                                   P],
     "zi_moe_route_table": [P, P, P, P, I, I, I, I, P],
     "zi_rope_table_scaled": [P, P, P, I, I, F, P],
     "zi_linear_attention_grouped": [P, L, P, P, P, L, P, L, P, P, L, P, P, P, P, I, I, I, I, I, F, I, I, I, P],
@@ -125,6 +126,12 @@ _PROTOTYPES = {
     "zi_moe_route_sigmoid": [P, P, P, L, I, I, I, P],
     "zi_moe_weighted_glu": [P, I, L, P, L, P, P, I, I, P],
     "zi_moe_sum_shared": [P, P, P, P, I, L, P, L, I, I, I, P],
+    "zi_stream_scale": [P, P, P, I, I, L, I, I, F, P],
+    "zi_input_conv": [P, I, L, P, I, L, P, P, I, F, P, P, L, P, P, P, P, P, I, I, I, P],
+    "zi_norm_input_conv": [P, I, P, P, I, I, L, P, I, F, F, P, P, L, P, P, P, I, I, I, P],
+    "zi_norm_input_conv_supported": [I, I, I],
+    "zi_lowrank_gates": [P, P, P, I, I, P, P, I, P, P, P, I, I, I, L, I, P],
+    "zi_delta_channel": [P, P, P, P, L, P, P, L, P, P, P, I, I, I, I, I, I, P],
     "zi_tape_record": [P, c_char_p, P, I],
     "zi_tape_record_many": [P, c_char_p, P, P, I],
     "zi_tape_run": [P, P],

@@ -75,8 +75,8 @@ def _i32(t: torch.Tensor, what: str, n: Optional[int] = None) -> None:
 
 # ---------------------------------------------------------------------------
 def embedding(ids: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor] = None,
-              out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
-    """out[i,:] = table[ids[i],:] for int32 ids."""
+              out_dtype: Optional[torch.dtype] = None, scale: float = 1.0) -> torch.Tensor:
+    """out[i,:] = table[ids[i],:] * scale for int32 ids."""
     _gpu("embedding", ids, table, out)
     n = ids.numel()
     _i32(ids, "embedding ids")
@@ -88,7 +88,7 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor
     if tuple(out.shape) != (n, H) or not out.is_contiguous():
         raise ValueError(f"embedding: out must be contiguous [{n}, {H}], got {tuple(out.shape)}")
     _lib.call("zi_embedding", _p(out), _code(out, "embedding out"), _p(table), _code(table, "embedding table"),
-              _p(ids), n, H, V, _stream())
+              _p(ids), n, H, V, float(scale), _stream())
     return out
 
 
@@ -411,11 +411,18 @@ def attention_decode_workspace(tokens: int, nh: int, d: int) -> int:
     return int(_lib.load().zi_attention_decode_workspace(int(tokens), int(nh), int(d)))
 
 
-def _score_extras(who: str, nh: int, q: torch.Tensor, softcap: float, bias: Optional[torch.Tensor], keep_first: int):
-    """(softcap, bias pointer, distances of the bias, kept positions) for the entry points that take capped and
-    biased scores; None when none of them is asked for."""
-    if not (softcap and softcap > 0) and bias is None and not keep_first:
+def _score_extras(who: str, nh: int, q: torch.Tensor, softcap: float, bias: Optional[torch.Tensor], keep_first: int,
+                  log_distance=None):
+    """(softcap, bias pointer, distances of the bias, kept positions, slope and rate pointers) for the entry points that
+    take capped and biased scores; None when none of them is asked for."""
+    if not (softcap and softcap > 0) and bias is None and not keep_first and log_distance is None:
         return None
+    slope = rate = None
+    if log_distance is not None:
+        slope, rate = log_distance
+        for t in (slope, rate):
+            if t.dtype != torch.float32 or t.numel() != nh or not t.is_contiguous() or t.device != q.device:
+                raise ValueError(f"{who}: slope and rate must be contiguous float32 [{nh}] tensors on {q.device}")
     L = 0
     if bias is not None:
         if bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[0] != nh or not bias.is_contiguous() \
@@ -424,7 +431,7 @@ def _score_extras(who: str, nh: int, q: torch.Tensor, softcap: float, bias: Opti
         L = int(bias.shape[1])
     if softcap < 0 or keep_first < 0:
         raise ValueError(f"{who}: the cap and the kept positions cannot be negative")
-    return (float(softcap or 0.0), _p(bias), L, int(keep_first))
+    return (float(softcap or 0.0), _p(bias), L, int(keep_first), _p(slope), _p(rate))
 
 
 def attention_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, tok_seq: torch.Tensor,
@@ -432,20 +439,23 @@ def attention_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                      max_keys: int, window: int = 0, out: Optional[torch.Tensor] = None,
                      tok_index: Optional[torch.Tensor] = None, workspace: Optional[torch.Tensor] = None,
                      sinks: Optional[torch.Tensor] = None, leave_chunks: bool = False, softcap: float = 0.0,
-                     bias: Optional[torch.Tensor] = None, keep_first: int = 0) -> Optional[torch.Tensor]:
+                     bias: Optional[torch.Tensor] = None, keep_first: int = 0,
+                     log_distance=None) -> Optional[torch.Tensor]:
     """The same attention for single query tokens, split over the keys, on the matrix cores
     (bfloat16, head_dim a multiple of 16 up to 128, group size <= 16, page size a multiple of 8).
     ``max_keys`` is an upper bound of the keys any listed token sees (its position + 1), known on
-    the host; it only sizes the launch.  ``leave_chunks`` (with ``sinks``, without a token list): nothing is merged
+    the host; it only sizes the launch.  ``leave_chunks`` (with ``sinks`` or ``log_distance``, without a token list): nothing is merged
     or written to ``out``; every token's chunks stay in ``workspace`` for ``attention_decode_project``.
     ``softcap``, ``bias`` (float32 [nh, L]) and ``keep_first``: scores are capped as cap * tanh(score / cap), then
     take ``bias[head, min(distance, L - 1)]``; the sequence's first ``keep_first`` positions stay visible beside the
-    window."""
+    window.  ``log_distance`` (slope, rate), float32 [nh] each: slope * ln(1 + rate * distance) is taken off the score
+    (chunks may be left then too)."""
     out, n, count, ldq, ldo, pages, ps = _attention_args("attention_decode", q, kcache, vcache, tok_seq, tok_pos,
                                                          block_tables, nh, nkv, d, tok_index,
                                                          q if (leave_chunks and out is None) else out)   # (nothing is written there)
-    if leave_chunks and (sinks is None or tok_index is not None or workspace is None):
-        raise ValueError("attention_decode: chunks are left for mixers with sinks, all tokens, in a given workspace")
+    if leave_chunks and ((sinks is None and log_distance is None) or tok_index is not None or workspace is None):
+        raise ValueError("attention_decode: chunks are left for mixers with sinks or a distance's logarithm, all tokens, "
+                         "in a given workspace")
     if window > 0:
         max_keys = min(max_keys, window)
     max_chunks = int(_lib.load().zi_attention_decode_chunks(int(max_keys)))
@@ -459,9 +469,9 @@ def attention_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
             _p(vcache), _p(tok_index), _p(tok_seq), _p(tok_pos), _p(block_tables), block_tables.shape[1], pages,
             nh, nkv, d, ps, int(window), float(scale), max_chunks, _p(workspace),
             workspace.numel() if workspace is not None else 0)
-    extras = _score_extras("attention_decode", nh, q, softcap, bias, keep_first)
+    extras = _score_extras("attention_decode", nh, q, softcap, bias, keep_first, log_distance)
     if extras is not None:
-        if leave_chunks:
+        if leave_chunks and log_distance is None:
             raise ValueError("attention_decode: capped or biased scores are merged here")
         _lib.call("zi_attention_decode_biased", *args,
                   _p(_sinks(sinks, nh, q, "attention_decode") if sinks is not None else None), *extras, _stream())
@@ -763,7 +773,7 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
                       window: int = 0, out: Optional[torch.Tensor] = None, max_keys: int = 0,
                       workspace: Optional[torch.Tensor] = None, tile: int = 0, alone: bool = False,
                       sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
-                      keep_first: int = 0) -> torch.Tensor:
+                      keep_first: int = 0, log_distance=None) -> torch.Tensor:
     """The same attention for portions of prompts, on the matrix cores (bfloat16, head_dim a multiple
     of 16 up to 128, page size a power of two from 8).
 
@@ -776,7 +786,8 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
     entries of float32; allocated here when not given).  A bound that is too low leaves NaN in the rows
     concerned.  ``alone`` (where the head size has tiles of 128): workgroups of four wavefronts, two to a compute
     unit, which pays for launches of many tiles; the result differs by rounding.  ``softcap``, ``bias`` and
-    ``keep_first`` as for ``attention_decode``; with any of them tiles hold ``attention_prefill_tile_min()`` queries."""
+    ``keep_first`` as for ``attention_decode``; with any of them tiles hold ``attention_prefill_tile_min()`` queries.
+    ``log_distance`` as for ``attention_decode``, with every tile."""
     _gpu("attention_prefill", q, kcache, vcache, tile_entry, tile_off, entry_start, entry_len, entry_past,
          block_tables, out)
     ldq, wq = _rows(q, "attention_prefill q")
@@ -819,9 +830,9 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
             _p(block_tables), block_tables.shape[1], pages, nh, nkv, d, ps, int(window), float(scale), n,
             max_chunks, _p(workspace) if need else _p(None), workspace.numel() if need else 0, int(tile), int(bool(alone)),
             chunk_keys)
-    extras = _score_extras("attention_prefill", nh, q, softcap, bias, keep_first)
+    extras = _score_extras("attention_prefill", nh, q, softcap, bias, keep_first, log_distance)
     if extras is not None:
-        if tile != attention_prefill_tile_min() or alone:
+        if (extras[0] > 0 or bias is not None or keep_first) and (tile != attention_prefill_tile_min() or alone):
             raise ValueError("attention_prefill: capped or biased scores take the smallest tiles")
         _lib.call("zi_attention_prefill_biased", *args,
                   _p(_sinks(sinks, nh, q, "attention_prefill") if sinks is not None else None), *extras, _stream())
@@ -991,10 +1002,13 @@ def linear_splits(M: int, N: int, K: int) -> int:
     return int(_lib.load().zi_gemm_skinny_splits(int(M), int(N), int(K)))
 
 
-def linear_sums(x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+def linear_sums(x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Tensor] = None,
+                bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """x[M,K] . weight[N,K]^T for M <= SUMS_MAX_ROWS as float32 partial sums [S, M, N], S =
-    ``linear_splits(M, N, K)``, without bias: the consumer adds them in rising order."""
-    _gpu("linear_sums", x, weight, out)
+    ``linear_splits(M, N, K)``: the consumer adds them in rising order.  A ``bias`` (bfloat16 [N]) is added to the first."""
+    _gpu("linear_sums", x, weight, out, bias)
+    if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != weight.shape[0] or not bias.is_contiguous()):
+        raise ValueError(f"linear_sums: the bias must be a contiguous bfloat16 [{weight.shape[0]}] tensor")
     if not linear_sums_supported(x, weight):
         raise ValueError(f"linear_sums: needs bfloat16 x and weight, at most {SUMS_MAX_ROWS} rows, 16-byte aligned rows")
     M, K = x.shape
@@ -1004,7 +1018,7 @@ def linear_sums(x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Tenso
         out = torch.empty((S, M, N), dtype=torch.float32, device=x.device)
     if tuple(out.shape) != (S, M, N) or out.dtype != torch.float32 or not out.is_contiguous():
         raise ValueError(f"linear_sums: out must be a contiguous float32 [{S}, {M}, {N}] tensor")
-    _lib.call("zi_gemm_skinny", _p(out), F32, 1, _p(x), _p(weight), c_void_p(0), M, N, K, x.stride(0), weight.stride(0),
+    _lib.call("zi_gemm_skinny", _p(out), F32, 1, _p(x), _p(weight), _p(bias), M, N, K, x.stride(0), weight.stride(0),
               N, c_void_p(0), 0, _stream())
     return out
 

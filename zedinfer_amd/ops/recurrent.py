@@ -9,8 +9,9 @@ from typing import Optional
 import torch
 
 from . import _lib
-from .functional import _attention_args, _check_cache, _code, _gpu, _i32, _p, _rows, _sinks, _stream
+from .functional import _attention_args, _check_cache, _code, _gpu, _i32, _p, _rows, _score_extras, _sinks, _stream
 from .mixing import MOE_MAX_EXPERTS, _f32
+from .sublayers import _terms
 
 GATE_ACTIVATIONS = {"sigmoid": 0, "silu": 1}
 
@@ -162,20 +163,21 @@ def linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
 
 def gate_heads(x: torch.Tensor, gate: torch.Tensor, head: int, x_head: int, activation: str, out: torch.Tensor,
                scale: float = 1.0) -> torch.Tensor:
-    """out [n, W] = x * act(gate) * scale, act "sigmoid" or "silu"; gate float32 [n, W]; x holds heads of ``x_head``
-    values of which the first ``head`` count (W = heads * head)."""
+    """out [n, W] = x * act(gate) * scale, act "sigmoid" or "silu"; gate float32 [n, W], or a stack [S, n, W] of partial
+    sums (a column slice is fine); x holds heads of ``x_head`` values of which the first ``head`` count (W = heads *
+    head)."""
     _gpu("gate_heads", x, gate, out)
     ldx, wx = _rows(x, "gate_heads x")
-    ldg, W = _rows(gate, "gate_heads gate")
+    splits, split_stride, ldg, rows, W = _terms(gate, "gate_heads gate", columns=True)
     ldo, wo = _rows(out, "gate_heads out")
     n = x.shape[0]
-    if gate.dtype != torch.float32 or W % head or wx != (W // head) * x_head or wo != W or gate.shape[0] != n \
+    if gate.dtype != torch.float32 or W % head or wx != (W // head) * x_head or wo != W or rows != n \
             or out.shape[0] != n or x_head < head:
         raise ValueError("gate_heads: shapes do not agree")
     if activation not in GATE_ACTIVATIONS:
         raise ValueError(f"gate_heads: unknown activation {activation!r}")
     _lib.call("zi_gate_heads", _p(out), _code(out, "gate_heads out"), ldo, _p(x), _code(x, "gate_heads x"), ldx, x_head,
-              _p(gate), ldg, n, W, head, GATE_ACTIVATIONS[activation], float(scale), _stream())
+              _p(gate), ldg, splits, split_stride, n, W, head, GATE_ACTIVATIONS[activation], float(scale), _stream())
     return out
 
 
@@ -235,22 +237,18 @@ def attention_biased(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                      tok_pos: torch.Tensor, block_tables: torch.Tensor, nh: int, nkv: int, d: int, scale: float,
                      window: int = 0, out: Optional[torch.Tensor] = None, tok_index: Optional[torch.Tensor] = None,
                      sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
-                     keep_first: int = 0) -> torch.Tensor:
+                     keep_first: int = 0, log_distance=None) -> torch.Tensor:
     """The plain attention kernel (``ops.attention``) with its options: scores are (q . k) * scale, then
     ``softcap`` * tanh(score / ``softcap``) when the cap is positive, then plus ``bias[head, min(distance, L - 1)]``
-    (float32 [nh, L]); beside the window the first ``keep_first`` positions of the sequence stay visible."""
+    (float32 [nh, L]); beside the window the first ``keep_first`` positions of the sequence stay visible.
+    ``log_distance`` (slope, rate), float32 [nh] each: slope * ln(1 + rate * distance) is taken off the score."""
     out, n, count, ldq, ldo, pages, ps = _attention_args("attention", q, kcache, vcache, tok_seq, tok_pos,
                                                          block_tables, nh, nkv, d, tok_index, out)
-    L = 0
-    if bias is not None:
-        _f32(bias, "attention bias")
-        if bias.dim() != 2 or bias.shape[0] != nh or bias.device != q.device:
-            raise ValueError(f"attention: the bias must be float32 [{nh}, distances] on {q.device}")
-        L = int(bias.shape[1])
+    extras = _score_extras("attention", nh, q, softcap, bias, keep_first, log_distance) or (0.0, _p(None), 0, 0, _p(None), _p(None))
     _lib.call("zi_attention_generic_biased", _p(out), _p(q), _code(q, "attention"), count, ldq, ldo, _p(kcache), _p(vcache),
               _p(tok_index), _p(tok_seq), _p(tok_pos), _p(block_tables), block_tables.shape[1], pages, nh, nkv, d, ps,
               int(window), float(scale), _p(_sinks(sinks, nh, q, "attention") if sinks is not None else None),
-              float(softcap), _p(bias), L, int(keep_first), _stream())
+              *extras, _stream())
     return out
 
 

@@ -16,12 +16,13 @@ CONV_MAX_TAPS = 16
 CONV_MAX_CHANNELS = 15360
 
 
-def _terms(x: torch.Tensor, what: str):
-    """(splits, stride between splits, row stride, rows, width) of [n, H] rows or a stack [S, n, H] of float32 terms."""
+def _terms(x: torch.Tensor, what: str, columns: bool = False):
+    """(splits, stride between splits, row stride, rows, width) of [n, H] rows or a stack [S, n, H] of float32 terms
+    (``columns``: a column slice of such a stack is fine)."""
     if x.dim() == 3:
-        if x.dtype != torch.float32 or not x.is_contiguous():
+        if x.dtype != torch.float32 or not (x.is_contiguous() or (columns and x.stride(2) == 1)):
             raise ValueError(f"{what}: a stack of terms must be contiguous float32 [S, n, width]")
-        return int(x.shape[0]), int(x.shape[1] * x.shape[2]), int(x.shape[2]), int(x.shape[1]), int(x.shape[2])
+        return int(x.shape[0]), int(x.stride(0)), int(x.stride(1)), int(x.shape[1]), int(x.shape[2])
     ld, width = _rows(x, what)
     return 1, 0, ld, int(x.shape[0]), width
 
@@ -65,7 +66,9 @@ def conv_qkv(proj: torch.Tensor, bias: Optional[torch.Tensor], conv_w: torch.Ten
              q_norm: torch.Tensor, k_norm: torch.Tensor, eps: float, table: Optional[torch.Tensor], tok_seq: torch.Tensor,
              entry_start: torch.Tensor, entry_slot: torch.Tensor, slots: Optional[torch.Tensor],
              kcache: Optional[torch.Tensor], vcache: Optional[torch.Tensor], nh: int, nkv: int, dim: int, vdim: int,
-             head: int, taps: int, q_out: torch.Tensor, move_tail: bool = False) -> torch.Tensor:
+             head: int, taps: int, q_out: torch.Tensor, move_tail: bool = False,
+             values_out: Optional[torch.Tensor] = None, mix_values: Optional[torch.Tensor] = None,
+             mix: float = 0.0) -> torch.Tensor:
     """Rows of proj [n, nh*dim + nkv*dim + nkv*vdim] (q | k | v, any storage type, or a stack [S, n, ...] of float32
     partial sums) plus ``bias`` pass, per channel, a
     causal convolution of ``taps`` taps (``conv_w`` [channels, taps]; rows before the step come from the request's
@@ -74,10 +77,12 @@ def conv_qkv(proj: torch.Tensor, bias: Optional[torch.Tensor], conv_w: torch.Ten
     The queries go to ``q_out`` [n, nh*head]; keys and values, where the caches are given, into the paged cache at
     ``slots`` (a token whose slot is negative stores nothing), whose heads hold ``head`` >= dim, vdim values (the
     rest zero).  ``move_tail`` (only when every entry brings one token): the new tails are written here too, for
-    tokens that have a slot, and ``conv_tail`` is not needed.  Everything float32 but the stores."""
-    _gpu("conv_qkv", proj, bias, conv_w, state, q_norm, k_norm, table, tok_seq, entry_start, entry_slot, slots, kcache,
+    tokens that have a slot, and ``conv_tail`` is not needed.  ``values_out`` (float32 [n, nkv*vdim]) receives the
+    convolved values; with ``mix_values`` (the same shape) what is cached is (1 - mix) v + mix * mix_values.  Everything
+    float32 but the stores."""
+    _gpu("conv_qkv", values_out, mix_values, proj, bias, conv_w, state, q_norm, k_norm, table, tok_seq, entry_start, entry_slot, slots, kcache,
          vcache, q_out)
-    splits, split_stride, ld, n, width = _terms(proj, "conv_qkv proj")
+    splits, split_stride, ld, n, width = _terms(proj, "conv_qkv proj", columns=True)
     Qd, Kd, Vd = nh * dim, nkv * dim, nkv * vdim
     C = Qd + Kd + Vd
     if width != C:
@@ -89,8 +94,11 @@ def conv_qkv(proj: torch.Tensor, bias: Optional[torch.Tensor], conv_w: torch.Ten
     _f32(k_norm, "conv_qkv k_norm", (Kd,))
     if bias is not None:
         _f32(bias, "conv_qkv bias", (C,))
-    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or state.shape[1] < (taps - 1) * C:
-        raise ValueError(f"conv_qkv: state must be contiguous float32 [slots, >= {(taps - 1) * C}]")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < (taps - 1) * C:
+        raise ValueError(f"conv_qkv: state must be float32 [slots, >= {(taps - 1) * C}] with dense rows")
+    for t in (values_out, mix_values):
+        if t is not None:
+            _f32(t, "conv_qkv values", (n, Vd))
     rot = 0
     if table is not None:
         _f32(table, "conv_qkv table")
@@ -116,7 +124,8 @@ def conv_qkv(proj: torch.Tensor, bias: Optional[torch.Tensor], conv_w: torch.Ten
               _p(vcache if kcache is not None else None), _p(proj), _code(proj, "conv_qkv proj"), ld, splits, split_stride,
               _p(bias), _p(conv_w), _p(state), int(state.stride(0)), int(bool(move_tail)), _p(q_norm), _p(k_norm),
               float(eps), _p(table), rot, n, _p(tok_seq),
-              _p(entry_start), _p(entry_slot), _p(slots), pages * ps, nh, nkv, dim, vdim, head, taps, max(ps, 1), _stream())
+              _p(entry_start), _p(entry_slot), _p(slots), pages * ps, nh, nkv, dim, vdim, head, taps, max(ps, 1),
+              _p(values_out), _p(mix_values), float(mix), _stream())
     return q_out
 
 
@@ -127,11 +136,11 @@ def conv_tail(state: torch.Tensor, proj: torch.Tensor, bias: Optional[torch.Tens
     that have none (negative; they stand behind an entry's own) do not count, and an entry without any token of its
     own leaves its slot's tail as it is."""
     _gpu("conv_tail", state, proj, bias, entry_start, entry_len, entry_slot, slots)
-    splits, split_stride, ld, n, C = _terms(proj, "conv_tail proj")
+    splits, split_stride, ld, n, C = _terms(proj, "conv_tail proj", columns=True)
     if slots is not None:
         _i32(slots, "conv_tail slots", n)
-    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or state.shape[1] < (taps - 1) * C:
-        raise ValueError(f"conv_tail: state must be contiguous float32 [slots, >= {(taps - 1) * C}]")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < (taps - 1) * C:
+        raise ValueError(f"conv_tail: state must be float32 [slots, >= {(taps - 1) * C}] with dense rows")
     if bias is not None:
         _f32(bias, "conv_tail bias", (C,))
     E = entry_start.numel()
@@ -156,11 +165,13 @@ def relu_squared(z: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     return out
 
 
-def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, out: torch.Tensor, alpha: float = 1.702) -> torch.Tensor:
+def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, out: torch.Tensor, alpha: float = 1.702,
+                gate_bias: Optional[torch.Tensor] = None, up_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out = g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit); gate and up [n, I]
     with dense rows (column slices of one product are fine), or the same slices [S, n, I] of a stack of float32 partial
-    sums, which are added first."""
-    _gpu("clamped_glu", gate, up, out)
+    sums, which are added first.  ``gate_bias`` and ``up_bias`` (float32 [I], both or neither) are added to gate and up
+    before anything else is done with them."""
+    _gpu("clamped_glu", gate, up, out, gate_bias, up_bias)
     splits, split_stride = 1, 0
     if gate.dim() == 3:
         if gate.dtype != torch.float32 or up.dtype != torch.float32 or gate.shape != up.shape or gate.stride() != up.stride() \
@@ -176,8 +187,14 @@ def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, out: torch.T
         raise ValueError("clamped_glu: gate, up and out must agree in shape, gate and up in type")
     if not limit > 0:
         raise ValueError("clamped_glu: the limit must be positive")
+    if (gate_bias is None) != (up_bias is None):
+        raise ValueError("clamped_glu: biases of both halves or of neither")
+    for t in (gate_bias, up_bias):
+        if t is not None:
+            _f32(t, "clamped_glu bias", (I,))
     _lib.call("zi_clamped_glu", _p(out), _code(out, "clamped_glu out"), ldo, _p(gate), _p(up), _code(gate, "clamped_glu"),
-              ldg, ldu, splits, split_stride, n, I, float(limit), float(alpha), _stream())
+              ldg, ldu, splits, split_stride, n, I, float(limit), float(alpha), _p(gate_bias), _p(up_bias),
+              _stream())
     return out
 
 

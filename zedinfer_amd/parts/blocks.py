@@ -14,7 +14,8 @@ from .base import Block, LayerMemory, Runtime, register_block
 class PreNormBlock(Block):
     """h += mixer(norm_in(h)); h += feed_forward(norm_post(h))
     (reference: src/frontend/models/transformer_forward.cpp:63-149).  The residual stream is
-    float32 and every add into it happens inside the norm that follows it."""
+    float32 and every add into it happens inside the norm that follows it.  A mixer that offers
+    ``forward_from_stream(norm, resid, delta, batch, memory)`` is given the norm and the stream instead of normed rows."""
 
     graph_safe = True
     tape_safe = True
@@ -27,11 +28,15 @@ class PreNormBlock(Block):
         self.mixer = mixer
         self.feed_forward = feed_forward
         self.has_ff = getattr(feed_forward, "kind", "") != "none"      # without one the mixer's addition is handed on
+        self.from_stream = getattr(mixer, "forward_from_stream", None)
         self.rt = rt
 
     def forward(self, resid: torch.Tensor, delta: Optional[torch.Tensor], batch, memory: LayerMemory):
-        x = self.norm_in.add_forward(resid, delta) if delta is not None else self.norm_in.forward(resid)
-        a = self.mixer.forward(x, batch, memory)
+        if self.from_stream is not None:
+            a = self.from_stream(self.norm_in, resid, delta, batch, memory)
+        else:
+            x = self.norm_in.add_forward(resid, delta) if delta is not None else self.norm_in.forward(resid)
+            a = self.mixer.forward(x, batch, memory)
         if not self.has_ff:
             return a
         y = self.norm_post.add_forward(resid, a)

@@ -15,7 +15,7 @@ from .base import Part, Runtime, register_embedding, register_head
 class TokenEmbedding(Part):
     """h[i,:] = table[ids[i],:], unscaled, widened into the float32 residual stream
     (reference: src/frontend/models/transformer_forward.cpp:54-60).  With ``norm_eps`` the rows are then RMS-normed
-    in place, in float32, with the gain ``norm`` [hidden_size].
+    in place, in float32, with the gain ``norm`` [hidden_size].  ``scale`` multiplies every row of the table, in float32.
 
     Two more terms can be added to the row, in the same kernel: with ``pair`` ({"buckets", "mul_prev", "mul_cur"}) the
     row (previous id * mul_prev + id * mul_cur) mod buckets of a second table ``pair`` [buckets + 1, hidden_size] (its
@@ -24,7 +24,7 @@ class TokenEmbedding(Part):
     padded.  With ``sinusoid`` (a base, 10000 in the classic form) the fixed position vector whose entries 2i and
     2i+1 are sin and cos of position * base^(-2i/hidden_size); the frequencies are made in double precision on the
     host and the angle and its sine in double on the device.
-    params: vocab_size, hidden_size, norm_eps (None), pair (None), sinusoid (None)."""
+    params: vocab_size, hidden_size, norm_eps (None), pair (None), sinusoid (None), scale (1)."""
 
     graph_safe = True
     tape_safe = True
@@ -57,6 +57,9 @@ class TokenEmbedding(Part):
             self.freq = torch.tensor(f, dtype=torch.float64, device=self.weight.device)
         # the step's entries and positions are read when there is more than the table
         self.reads_batch = self.pair is not None or self.freq is not None
+        self.scale = float(spec.params.get("scale", 1.0))
+        if self.scale != 1.0 and self.reads_batch:
+            raise ValueError("embedding: a scale of the table's rows alone, without further terms")
         self.padding_safe = self.pair is None      # a padding entry would rewrite the slot it names
 
     def state_request(self):
@@ -75,7 +78,7 @@ class TokenEmbedding(Part):
                               entry_start=batch.entry_start, entry_len=batch.entry_len, entry_slot=batch.entry_slot,
                               freq=self.freq)
         else:
-            ops.embedding(ids, self.weight, out=out)
+            ops.embedding(ids, self.weight, out=out, scale=self.scale)
         if self.norm is not None:
             ops.rms_norm(out, self.norm, float(self.norm_eps), out=out)      # a thread rewrites what it read itself
         return out

@@ -2,7 +2,7 @@
 from __future__ import annotations
 
 import os
-from typing import Dict
+from typing import Dict, Optional
 
 import torch
 
@@ -338,15 +338,20 @@ class ReluSquaredMLP(FeedForward):
 
 class _ClampedGated:
     """One feed-forward of the clamped gated form, down(g sigmoid(1.702 g) (u + 1)) with g = min(gate x, limit) and
-    u = clamp(up x, -limit, limit): gate and up stacked into one product (the up rows begin at a multiple of 8)."""
+    u = clamp(up x, -limit, limit): gate and up stacked into one product (the up rows begin at a multiple of 8).  With
+    biases (``gate_bias``, ``up_bias``) they are added to the product's float32 results before the clamps."""
 
-    def __init__(self, gate: torch.Tensor, up: torch.Tensor, down: torch.Tensor, limit: float):
+    def __init__(self, gate: torch.Tensor, up: torch.Tensor, down: torch.Tensor, limit: float,
+                 gate_bias: Optional[torch.Tensor] = None, up_bias: Optional[torch.Tensor] = None):
         self.inter, self.hidden = int(gate.shape[0]), int(gate.shape[1])
         self.up_at = -(-self.inter // 8) * 8
         stacked = torch.zeros((self.up_at + self.inter, self.hidden), dtype=gate.dtype, device=gate.device)
         stacked[:self.inter] = gate
         stacked[self.up_at:] = up.to(gate.dtype)
         self.gate_up, self.down, self.limit = stacked, down, float(limit)
+        self.biases = {}
+        if gate_bias is not None:
+            self.biases = {"gate_bias": gate_bias.float().contiguous(), "up_bias": up_bias.float().contiguous()}
 
     def forward(self, rt: Runtime, x: torch.Tensor, name: str) -> torch.Tensor:
         n, I = x.shape[0], self.inter
@@ -354,11 +359,57 @@ class _ClampedGated:
         if ops.linear_sums_supported(x, self.gate_up):
             S = ops.linear_splits(n, self.up_at + I, self.hidden)
             gu = ops.linear_sums(x, self.gate_up, out=rt.buffer(name + "_gate_up_sums", (S, n, self.up_at + I), torch.float32))
-            ops.clamped_glu(gu[:, :, :I], gu[:, :, self.up_at:], self.limit, out=act)
+            ops.clamped_glu(gu[:, :, :I], gu[:, :, self.up_at:], self.limit, out=act, **self.biases)
         else:
             gu = ops.linear(x, self.gate_up, out=rt.buffer(name + "_gate_up", (n, self.up_at + I), torch.float32))
-            ops.clamped_glu(gu[:, :I], gu[:, self.up_at:], self.limit, out=act)
+            ops.clamped_glu(gu[:, :I], gu[:, self.up_at:], self.limit, out=act, **self.biases)
         return act
+
+
+@register_feed_forward("clamped_mlp")
+class ClampedMLP(FeedForward):
+    """A dense feed-forward of the clamped gated form, down(g sigmoid(1.702 g) (u + 1)) with g = min(gate x, limit) and
+    u = clamp(up x, -limit, limit); with ``bias`` all three projections have one (``gate_bias``, ``up_bias``,
+    ``down_bias``).  The gate/up product leaves float32 results (partial sums for few rows), the activation's kernel
+    adds the biases; the down product of few rows leaves partial sums whose first holds its bias.
+    params: hidden_size, intermediate_size, limit, bias (False)."""
+
+    graph_safe = True
+    tape_safe = True
+
+    @staticmethod
+    def weight_specs(spec: PartSpec) -> Dict[str, WeightSpec]:
+        H, I = int(spec.params["hidden_size"]), int(spec.params["intermediate_size"])
+        w = {"gate": WeightSpec((I, H)), "up": WeightSpec((I, H)), "down": WeightSpec((H, I))}
+        if spec.params.get("bias", False):
+            w.update({"gate_bias": WeightSpec((I,)), "up_bias": WeightSpec((I,)), "down_bias": WeightSpec((H,))})
+        return w
+
+    def __init__(self, spec: PartSpec, weights: Dict[str, torch.Tensor], rt: Runtime):
+        super().__init__(spec, weights, rt)
+        p = spec.params
+        self.hidden, self.inter = int(p["hidden_size"]), int(p["intermediate_size"])
+        self.half = _ClampedGated(weights["gate"], weights["up"], weights["down"], float(p["limit"]),
+                                  weights.get("gate_bias"), weights.get("up_bias"))
+        self.down = weights["down"]
+        self.down_bias = weights["down_bias"].to(self.down.dtype).contiguous() if p.get("bias", False) else None
+
+    def step_rows(self, rows: int, kind: str) -> int:
+        return ProductRows.step_rows(rows, kind)
+
+    def tune(self, num_tokens: int) -> None:
+        n = int(num_tokens)
+        self.rt.tune_linear(self.rt.buffer("norm_out", (n, self.hidden)), self.half.gate_up, out_dtype=torch.float32)
+        self.rt.tune_linear(self.rt.buffer("ffn_act", (n, self.inter)), self.down, self.down_bias)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        n, rt = x.shape[0], self.rt
+        act = self.half.forward(rt, x, "ffn")
+        if ops.linear_sums_supported(act, self.down):
+            S = ops.linear_splits(n, self.hidden, self.inter)
+            return ops.linear_sums(act, self.down, bias=self.down_bias,
+                                   out=rt.buffer("ffn_out_sums", (S, n, self.hidden), torch.float32))
+        return ops.linear(act, self.down, self.down_bias, out=rt.buffer("ffn_out", (n, self.hidden)))
 
 
 @register_feed_forward("clamped_experts")

@@ -161,6 +161,8 @@ class Attention(Mixer):
     PROJECT_FROM_CHUNKS_MAX_BYTES = 8 << 20
     # float32 [heads] in mixers whose softmax counts exp(sink) of a learned number per head in its denominator
     sinks: Optional[torch.Tensor] = None
+    # (slope, rate), float32 [heads] each, in mixers that take slope * ln(1 + rate * distance) off every score
+    log_distance: Optional[tuple] = None
 
     @staticmethod
     def weight_specs(spec: PartSpec) -> Dict[str, WeightSpec]:
@@ -219,6 +221,8 @@ class Attention(Mixer):
         not take goes to the plain one."""
         kc, vc = memory.tensors["k"], memory.tensors["v"]
         args = (kc, vc, batch.tok_seq, batch.positions, view.block_tables, self.nh, self.nkv, self.d, self.scale)
+        extras = {} if self.log_distance is None else {"log_distance": self.log_distance}
+        plain = ops.attention if self.log_distance is None else ops.attention_biased
         plan = batch.plans[self.plan_key]
         n_short, n_long, N = plan.sizes["num_short"], plan.sizes["num_long"], batch.num_tokens
         if n_short:
@@ -227,11 +231,11 @@ class Attention(Mixer):
                                     torch.float32)
                 ops.attention_decode(q, *args, plan.sizes["max_short_keys"], self.window, out=att,
                                      tok_index=plan.dev["short_idx"] if n_short < N else None, workspace=ws,
-                                     sinks=self.sinks)
+                                     sinks=self.sinks, **extras)
             else:
                 n_long = -1      # everything through the plain kernel
         if n_long < 0:
-            ops.attention(q, *args, self.window, out=att, sinks=self.sinks)
+            plain(q, *args, self.window, out=att, sinks=self.sinks, **extras)
         elif n_long > 0:
             if ops.attention_prefill_supported(q.dtype, self.nh, self.nkv, self.d, kc.shape[2]):
                 max_keys = plan.sizes["max_long_keys"]
@@ -241,10 +245,11 @@ class Attention(Mixer):
                 ops.attention_prefill(q, kc, vc, plan.dev["tile_entry"], plan.dev["tile_off"],
                                       batch.entry_start, batch.entry_len, batch.entry_past, view.block_tables, self.nh,
                                       self.nkv, self.d, self.scale, self.window, out=att, max_keys=max_keys,
-                                      workspace=ws, tile=plan.sizes["tile"], alone=plan.sizes["alone"], sinks=self.sinks)
+                                      workspace=ws, tile=plan.sizes["tile"], alone=plan.sizes["alone"], sinks=self.sinks,
+                                      **extras)
             else:
-                ops.attention(q, *args, self.window, out=att, tok_index=plan.dev["long_idx"] if n_long < N else None,
-                              sinks=self.sinks)
+                plain(q, *args, self.window, out=att, tok_index=plan.dev["long_idx"] if n_long < N else None,
+                      sinks=self.sinks, **extras)
 
     def planner(self) -> StepPlanner:
         return attention_planner(self.wide_tile, self.nh)
@@ -399,6 +404,13 @@ class ConvAttention(Attention):
     softmax's denominator also holds exp(sink_h), a learned number per head without key or value; W_o on the
     concatenated heads.  Keys have ``head_dim`` values a head, values ``value_dim``.
 
+    What the part's options change (by default biases and sinks are there and the rest is not): ``bias`` and ``sink``
+    False leave them out; ``log_distance``: r1 ln(1 + r2 distance) is taken off every score, two learned numbers a head
+    (``r1``, ``r2``); ``gate``: the concatenated heads are multiplied by sigmoid(W_g x) before W_o; ``value_mix`` "first":
+    the step's values (after the convolution) are kept for later layers, "mix": v <- (1 - a) v + a v_kept of the same
+    token, a the number ``vmix``, and the mixed values are what is cached (layers that mix must agree in the values'
+    sizes).
+
     The cache holds heads of one size, the larger of the two rounded up to what the matrix-core kernels take (a
     multiple of 16 up to 128 in bfloat16); the shorter kind is followed by zeros, which change no score and no
     output, and W_o gets zero columns where the padding stands.  A request's state is the last conv - 1 rows that
@@ -408,7 +420,8 @@ class ConvAttention(Attention):
     writes the new tail counts only the tokens that have one, and an entry of no request leaves the tail of the slot
     it names alone.
 
-    params: hidden_size, num_heads, num_kv_heads, head_dim, value_dim, conv, scale, window (0), eps, position."""
+    params: hidden_size, num_heads, num_kv_heads, head_dim, value_dim, conv, scale, window (0), eps, position, bias (True),
+    sink (True), log_distance (False), gate (False), value_mix (None)."""
 
     padding_safe = True
 
@@ -417,12 +430,22 @@ class ConvAttention(Attention):
         p = spec.params
         H, nh, nkv, d, dv, taps = (int(p[k]) for k in ("hidden_size", "num_heads", "num_kv_heads", "head_dim",
                                                       "value_dim", "conv"))
-        return {"q": WeightSpec((nh * d, H)), "k": WeightSpec((nkv * d, H)), "v": WeightSpec((nkv * dv, H)),
-                "q_bias": WeightSpec((nh * d,)), "k_bias": WeightSpec((nkv * d,)), "v_bias": WeightSpec((nkv * dv,)),
-                "q_conv": WeightSpec((nh * d, taps)), "k_conv": WeightSpec((nkv * d, taps)),
-                "v_conv": WeightSpec((nkv * dv, taps)),
-                "q_norm": WeightSpec((nh * d,), init="ones"), "k_norm": WeightSpec((nkv * d,), init="ones"),
-                "sink": WeightSpec((nh,), init="zeros"), "o": WeightSpec((H, nh * dv))}
+        w = {"q": WeightSpec((nh * d, H)), "k": WeightSpec((nkv * d, H)), "v": WeightSpec((nkv * dv, H)),
+             "q_conv": WeightSpec((nh * d, taps)), "k_conv": WeightSpec((nkv * d, taps)),
+             "v_conv": WeightSpec((nkv * dv, taps)),
+             "q_norm": WeightSpec((nh * d,), init="ones"), "k_norm": WeightSpec((nkv * d,), init="ones"),
+             "o": WeightSpec((H, nh * dv))}
+        if p.get("bias", True):
+            w.update({"q_bias": WeightSpec((nh * d,)), "k_bias": WeightSpec((nkv * d,)), "v_bias": WeightSpec((nkv * dv,))})
+        if p.get("sink", True):
+            w["sink"] = WeightSpec((nh,), init="zeros")
+        if p.get("log_distance", False):
+            w.update({"r1": WeightSpec((nh,), init="ones"), "r2": WeightSpec((nh,), init="ones")})
+        if p.get("gate", False):
+            w["g"] = WeightSpec((nh * dv, H))
+        if p.get("value_mix") == "mix":
+            w["vmix"] = WeightSpec((), init="zeros")
+        return w
 
     def __init__(self, spec: PartSpec, weights: Dict[str, torch.Tensor], rt: Runtime):
         Mixer.__init__(self, spec, weights, rt)
@@ -447,13 +470,29 @@ class ConvAttention(Attention):
         pos_spec: PartSpec = p["position"]
         self.position = POSITION_ENCODINGS.get(pos_spec.kind)(pos_spec, {}, rt)
         mats = [weights["q"], weights["k"], weights["v"]]
+        self.gated = bool(p.get("gate", False))
+        self.gate_at = self.channels
+        if self.gated:      # the gate's rows begin at a multiple of 8 of the stacked product
+            self.gate_at = -(-self.channels // 8) * 8
+            if self.gate_at > self.channels:
+                mats.append(torch.zeros((self.gate_at - self.channels, self.hidden), dtype=mats[0].dtype, device=mats[0].device))
+            mats.append(weights["g"])
         self.qkv = torch.cat([m.to(mats[0].dtype) for m in mats], dim=0).contiguous()
-        self.bias = torch.cat([weights[k].float() for k in ("q_bias", "k_bias", "v_bias")]).contiguous()
+        self.bias = None
+        if p.get("bias", True):
+            self.bias = torch.cat([weights[k].float() for k in ("q_bias", "k_bias", "v_bias")]).contiguous()
+        self.value_mix = p.get("value_mix")
+        if self.value_mix not in (None, "first", "mix"):
+            raise ValueError(f"conv_attention: unknown value_mix {self.value_mix!r}")
+        self.mix = float(weights["vmix"].float().reshape(()).item()) if self.value_mix == "mix" else 0.0
+        self.log_distance = None
+        if p.get("log_distance", False):
+            self.log_distance = (weights["r1"].float().contiguous(), weights["r2"].float().contiguous())
         self.conv_w = torch.cat([weights[k].float() for k in ("q_conv", "k_conv", "v_conv")]).contiguous()
         self.q_norm, self.k_norm = weights["q_norm"].float().contiguous(), weights["k_norm"].float().contiguous()
-        self.sinks = weights["sink"].float().contiguous()
+        self.sinks = weights["sink"].float().contiguous() if p.get("sink", True) else None
         o = weights["o"]
-        if self.d != self.vdim:        # zero columns where the heads' padding stands
+        if self.d != self.vdim and not self.gated:        # zero columns where the heads' padding stands (the gate drops it)
             wide = torch.zeros((self.hidden, self.nh, self.d), dtype=o.dtype, device=o.device)
             wide[:, :, :self.vdim] = o.view(self.hidden, self.nh, self.vdim)
             o = wide.view(self.hidden, self.qd).contiguous()
@@ -468,12 +507,12 @@ class ConvAttention(Attention):
     def tune(self, num_tokens: int) -> None:
         n = int(num_tokens)
         self.rt.tune_linear(self.rt.buffer("resid_copy", (n, self.hidden)), self.qkv, out_dtype=torch.float32)
-        self.rt.tune_linear(self.rt.buffer("attn_out", (n, self.qd)), self.o, out_dtype=torch.float32)
+        self.rt.tune_linear(self.rt.buffer("attn_out", (n, self.o.shape[1])), self.o, out_dtype=torch.float32)
 
     def project(self, att: torch.Tensor, n: int) -> torch.Tensor:
         """W_o with float32 results (a norm reads them): partial sums for few rows, else one product."""
         if ops.linear_sums_supported(att, self.o):
-            S = ops.linear_splits(n, self.hidden, self.qd)
+            S = ops.linear_splits(n, self.hidden, self.o.shape[1])
             return ops.linear_sums(att, self.o, out=self.rt.buffer("attn_proj_sums", (S, n, self.hidden), torch.float32))
         return ops.linear(att, self.o, out=self.rt.buffer("attn_proj_f32", (n, self.hidden), torch.float32))
 
@@ -485,10 +524,12 @@ class ConvAttention(Attention):
             raise ValueError("conv_attention: the position encoding must hand over a table of split-half angles")
         if ops.linear_sums_supported(x, self.qkv):
             # few rows: the projection leaves float32 partial sums, which the next kernel adds as it reads them
-            S = ops.linear_splits(n, self.channels, self.hidden)
-            proj = ops.linear_sums(x, self.qkv, out=rt.buffer("conv_attn_sums", (S, n, self.channels), torch.float32))
+            S = ops.linear_splits(n, self.qkv.shape[0], self.hidden)
+            full = ops.linear_sums(x, self.qkv, out=rt.buffer("conv_attn_sums", (S, n, self.qkv.shape[0]), torch.float32))
         else:
-            proj = ops.linear(x, self.qkv, out=rt.buffer("conv_attn_proj", (n, self.channels), torch.float32))
+            full = ops.linear(x, self.qkv, out=rt.buffer("conv_attn_proj", (n, self.qkv.shape[0]), torch.float32))
+        proj = full[..., :self.channels] if self.gated else full
+        gate = full[..., self.gate_at:] if self.gated else None
         q = rt.buffer("attn_q", (n, self.qd))
         writes = memory.writes
         # when every entry brings one token, the kernel that reads a tail is the only one that does, and moves it on
@@ -496,16 +537,35 @@ class ConvAttention(Attention):
         ops.conv_qkv(proj, self.bias, self.conv_w, memory.state, self.q_norm, self.k_norm, self.eps,
                      None if isinstance(table, str) else table, batch.tok_seq, batch.entry_start, batch.entry_slot,
                      view.slots, memory.tensors["k"] if writes else None, memory.tensors["v"] if writes else None,
-                     self.nh, self.nkv, self.dim, self.vdim, self.d, self.taps, q, move_tail=single)
+                     self.nh, self.nkv, self.dim, self.vdim, self.d, self.taps, q, move_tail=single,
+                     **self.mixed_values(n, batch))
         if not single:
             ops.conv_tail(memory.state, proj, self.bias, batch.entry_start, batch.entry_len, batch.entry_slot, self.taps,
                           slots=view.slots)
-        out = self.decode_and_project(q, batch, view, memory) if single else None
+        out = self.decode_and_project(q, batch, view, memory) if single and not self.gated else None
         if out is not None:
             return out
         att = rt.buffer("attn_out", (n, self.qd))
         self.attend(q, att, batch, view, memory)
+        if self.gated:
+            att = ops.gate_heads(att, gate, self.vdim, self.d, "sigmoid", out=rt.buffer("attn_gated", (n, self.nh * self.vdim)))
         return self.project(att, n)
+
+    FIRST_VALUES = "conv_attention.first_values"
+
+    def mixed_values(self, n: int, batch) -> Dict[str, object]:
+        """What ``ops.conv_qkv`` is told about the values that layers share: where the first such layer leaves the
+        step's (``batch.shared`` holds for one run of the model), or which to mix in."""
+        if self.value_mix is None:
+            return {}
+        shape = (n, self.nkv * self.vdim)
+        if self.value_mix == "first":
+            batch.shared[self.FIRST_VALUES] = kept = self.rt.buffer("first_values", shape, torch.float32)
+            return {"values_out": kept}
+        kept = batch.shared.get(self.FIRST_VALUES)
+        if kept is None or tuple(kept.shape) != shape:
+            raise ValueError("conv_attention: no earlier layer kept values of this layer's sizes")
+        return {"mix_values": kept, "mix": self.mix}
 
     def decode_and_project(self, q, batch, view, memory: LayerMemory) -> Optional[torch.Tensor]:
         """A pure decode step of few tokens: the attention kernel leaves every token's chunks of keys unmerged and

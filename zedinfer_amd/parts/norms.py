@@ -18,7 +18,9 @@ class RMSNorm(Norm):
     With ``scalar`` the checkpoint holds ONE number (a tensor without axes) that multiplies every coordinate; it is
     spread over ``dim`` values at load, so the kernels are the same.  ``out_dtype`` "float32": the normed rows leave
     in float32 whatever the engine's activation type (for a reader that works on them in float32 before any product).
-    params: dim, eps, add_one (default False), scalar (False), out_dtype (None)."""
+    ``gain_scale`` multiplies every gain (a constant of a linear reader, logits times a number for instance, costs nothing
+    there).
+    params: dim, eps, add_one (default False), scalar (False), out_dtype (None), gain_scale (1)."""
 
     graph_safe = True
     tape_safe = True
@@ -37,6 +39,10 @@ class RMSNorm(Norm):
         self.weight = weights["weight"]
         if spec.params.get("scalar", False):
             self.weight = self.weight.reshape(1).expand(self.dim).contiguous()
+        gain_scale = float(spec.params.get("gain_scale", 1.0))
+        if gain_scale != 1.0:      # the gains themselves, in float32
+            self.weight = ((self.weight.float() + (1.0 if self.add_one else 0.0)) * gain_scale).contiguous()
+            self.add_one = False
         self.out_dtype = torch.float32 if spec.params.get("out_dtype") == "float32" else None
 
     def forward(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
