@@ -481,13 +481,32 @@ def kegozen_shape(size, layers, vocab):
     return dict(architecture="Kegozen", width=z["width"], vocab=vocab, norm=dict(eps=1e-6), layers=out)
 
 
+def kefisun_shape(size, layers, vocab):
+    """Layer sizes that resemble a real model's, for the Kefisun design: layers of the delta rule with a decay per key
+    channel (as many heads as the Qwen2 model beside it, on half as many q/k heads, 128 x 128, gates of rank 128)
+    alternate with windowed attention (heads of 128 on the Qwen2 model's key/value heads, a window of 1,024 positions,
+    mixed values), four taps everywhere; every feed-forward is dense, of the Qwen2 model's width."""
+    z = DESIGN_SIZES[size]
+    out = []
+    for i in range(layers):
+        if i % 2 == 0:
+            kind, mixer = "channel_delta", dict(heads=z["heads"], kv_heads=z["heads"] // 2, dim=128, vdim=128, conv=4,
+                                                decay_rank=128, gate_rank=128)
+        else:
+            kind, mixer = "attention", dict(heads=z["heads"], kv_heads=max(2, z["heads"] // 7), dim=128, vdim=128, conv=4,
+                                            scale=128 ** -0.5, mask=dict(size=1024), v_mix=True)
+        out.append(dict(type=kind, mixer=mixer, mlp=dict(kind="dense", ff=z["ff"], limit=7.0)))
+    return dict(architecture="Kefisun", width=z["width"], vocab=vocab, norm=dict(eps=1e-6), canon=dict(taps=4),
+                embedding=dict(scale=16.0), logit_scale=0.5, layers=out)
+
+
 def design_comparison(args):
     """Prefill and decode of a model of the design at a real model's layer sizes, and of the benchmark's own
     architecture (Qwen2 dense) at the same width, layers, heads and dense feed-forward, one after the other; for
-    Tilivik and Kegozen also of Dedelorn, the nearest design the engine has (recurrent layers, latent attention,
-    experts)."""
+    Tilivik, Kegozen and Kefisun also of Dedelorn, the nearest design the engine has (recurrent layers, latent
+    attention, experts), and for Kefisun of Tosisun (convolved projections)."""
     import torch
-    from zedinfer_amd.config import DedelornConfig, KegozenConfig, Qwen2Config, SchedulerConfig, TilivikConfig, TosisunConfig
+    from zedinfer_amd.config import DedelornConfig, KefisunConfig, KegozenConfig, Qwen2Config, SchedulerConfig, TilivikConfig, TosisunConfig
     from zedinfer_amd.engine import Engine
     layers = args.layers if args.layers != FULL_LAYERS else 8
     vocab, prompt = 32000, args.prompt_len
@@ -498,7 +517,8 @@ def design_comparison(args):
         design = {"dedelorn": lambda: (DedelornConfig.from_dict(dedelorn_shape(size, layers, vocab)), "Dedelorn"),
                   "tosisun": lambda: (TosisunConfig.from_dict(tosisun_shape(size, layers, vocab)), "Tosisun"),
                   "tilivik": lambda: (TilivikConfig.from_dict(tilivik_shape(size, layers, vocab)), "Tilivik"),
-                  "kegozen": lambda: (KegozenConfig.from_dict(kegozen_shape(size, layers, vocab)), "Kegozen")}[args.design]
+                  "kegozen": lambda: (KegozenConfig.from_dict(kegozen_shape(size, layers, vocab)), "Kegozen"),
+                  "kefisun": lambda: (KefisunConfig.from_dict(kefisun_shape(size, layers, vocab)), "Kefisun")}[args.design]
         models = {
             args.design: design(),
             "qwen2": (Qwen2Config.from_dict(dict(SHAPE, hidden_size=z["width"], intermediate_size=z["ff"], vocab_size=vocab,
@@ -506,8 +526,10 @@ def design_comparison(args):
                                                  num_key_value_heads=max(2, z["heads"] // 7), tie_word_embeddings=False)),
                       "Qwen2ForCausalLM"),
         }
-        if args.design in ("tilivik", "kegozen"):
+        if args.design in ("tilivik", "kegozen", "kefisun"):
             models["dedelorn"] = (DedelornConfig.from_dict(dedelorn_shape(size, layers, vocab)), "Dedelorn")
+        if args.design == "kefisun":
+            models["tosisun"] = (TosisunConfig.from_dict(tosisun_shape(size, layers, vocab)), "Tosisun")
         if args.design_only:
             models = {args.design: models[args.design]}
         rec = {}
@@ -563,7 +585,7 @@ def main():
                     help="run only the 2,048-token prefill (for profiling) and print its figures")
     ap.add_argument("--resident-layer", action="store_true",
                     help="instead: time the one-launch decoder layer (ops.decode_layer) alone, --layers launches a step")
-    ap.add_argument("--design", default="", choices=["", "dedelorn", "tosisun", "tilivik", "kegozen"],
+    ap.add_argument("--design", default="", choices=["", "dedelorn", "tosisun", "tilivik", "kegozen", "kefisun"],
                     help="instead: prefill and decode of a model of this design at a real model's layer sizes, beside "
                          "Qwen2 dense of equal sizes (8 layers unless --layers says otherwise)")
     ap.add_argument("--design-sizes", default="", help="with --design: layer sizes, of " + ", ".join(sorted(DESIGN_SIZES)) +
