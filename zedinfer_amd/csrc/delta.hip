@@ -16,8 +16,7 @@
 __device__ __forceinline__ float delta_silu(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float delta_softplus(float z) { return z > 30.f ? z : log1pf(expf(z)); }
 
-// proj [n][ld]: columns [q (kvh*dim) | k (kvh*dim) | v (heads*vdim) | ...], beta's heads at column b_at, the decay's at
-// a_at (negative: no decay is made here).
+// proj [n][ld]: columns [q (kvh*dim) | k (kvh*dim) | v (heads*vdim) | gate (heads*vdim) | b (heads) | a (heads)].
 // One workgroup per (token, unit): a unit is one head of q or k (its dim channels, and their unit length), or 256
 // channels of v; the first unit of a token also makes its beta and g.
 #define DELTA_UNIT 256
@@ -39,7 +38,7 @@ delta_prepare_kernel(float* __restrict__ qk, float* __restrict__ v, float* __res
                      const float* __restrict__ a_log, const float* __restrict__ dt_bias, const float* __restrict__ state,
                      int64_t state_stride, int64_t conv_off, const int32_t* __restrict__ tok_seq,
                      const int32_t* __restrict__ entry_start, const int32_t* __restrict__ entry_slot, int heads,
-                     int kvh, int dim, int vdim, int taps, int b_at, int a_at) {
+                     int kvh, int dim, int vdim, int taps) {
     __shared__ float red[16];
     const int t = blockIdx.x, unit = blockIdx.y, e = tok_seq[t];
     const int local = t - entry_start[e];
@@ -66,11 +65,10 @@ delta_prepare_kernel(float* __restrict__ qk, float* __restrict__ v, float* __res
         if (c < heads * vdim) v[(int64_t)t * heads * vdim + c] = delta_conv(proj, ld, conv_w, tail, t, local, qkc + c, C, taps);
     }
     if (unit == 0) {
-        const float* row = proj + (int64_t)t * ld;
+        const float* row = proj + (int64_t)t * ld + C + heads * vdim;      // b, then a
         for (int h = threadIdx.x; h < heads; h += blockDim.x) {
-            beta_g[(int64_t)t * 2 * heads + h] = 1.f / (1.f + expf(-row[b_at + h]));
-            if (a_at < 0) continue;
-            const float step = delta_softplus(row[a_at + h] + dt_bias[h]);
+            beta_g[(int64_t)t * 2 * heads + h] = 1.f / (1.f + expf(-row[h]));
+            const float step = delta_softplus(row[heads + h] + dt_bias[h]);
             beta_g[(int64_t)t * 2 * heads + heads + h] = expf(-expf(a_log[h]) * step);
         }
     }
@@ -79,22 +77,21 @@ delta_prepare_kernel(float* __restrict__ qk, float* __restrict__ v, float* __res
 extern "C" int zi_delta_prepare(float* qk, float* v, float* beta_g, const float* proj, int64_t ld, int n,
                                 const void* conv_w, const void* a_log, const void* dt_bias, int w_dt, const float* state,
                                 int64_t state_stride, int64_t conv_off, const int32_t* tok_seq, const int32_t* entry_start,
-                                const int32_t* entry_slot, int heads, int kvh, int dim, int vdim, int taps, int b_at,
-                                int a_at, hipStream_t stream) {
+                                const int32_t* entry_slot, int heads, int kvh, int dim, int vdim, int taps,
+                                hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && heads > 0 && kvh > 0 && heads % kvh == 0 && dim > 0 && vdim > 0 && taps >= 1,
                "delta_prepare: bad sizes");
     ZI_REQUIRE(w_dt == ZI_F32, "delta_prepare: the convolution's taps, A_log and dt_bias are float32");
     ZI_REQUIRE(dim <= 2 * DELTA_UNIT, "delta_prepare: dim %d is more than %d", dim, 2 * DELTA_UNIT);
     const int64_t C = 2LL * kvh * dim + (int64_t)heads * vdim;
-    ZI_REQUIRE(b_at >= C && ld >= b_at + heads && (a_at < 0 || (a_at >= C && ld >= a_at + heads && a_log && dt_bias)),
-               "delta_prepare: the columns do not fit the rows");
+    ZI_REQUIRE(ld >= C + (int64_t)heads * vdim + 2 * heads, "delta_prepare: row stride too small");
     ZI_REQUIRE(state_stride >= conv_off + (int64_t)(taps - 1) * C, "delta_prepare: the state row is too short");
     const int units = 2 * kvh + (heads * vdim + DELTA_UNIT - 1) / DELTA_UNIT;
     ZI_REQUIRE(units <= 65535, "delta_prepare: too many channels");
     if (n == 0) return 0;
     delta_prepare_kernel<<<dim3(n, units), DELTA_UNIT, 0, stream>>>(
         qk, v, beta_g, proj, ld, (const float*)conv_w, (const float*)a_log, (const float*)dt_bias, state, state_stride,
-        conv_off, tok_seq, entry_start, entry_slot, heads, kvh, dim, vdim, taps, b_at, a_at);
+        conv_off, tok_seq, entry_start, entry_slot, heads, kvh, dim, vdim, taps);
     return zi_check_launch("delta_prepare");
 }
 

@@ -4,6 +4,7 @@
 //
 // q and k as in delta.hip (zi_delta_prepare makes them, v and beta), g [heads][dim] in (0, 1) per token.
 //
+//   zi_channel_inputs    from the stacked projection: convolution, SiLU, unit vectors, beta, and the convolution's tail
 //   zi_lowrank_gates     two low-rank projections of float32 rows at once: the decays
 //                        g = exp(-exp(a_log_h) * softplus(W_a u_a + bias)) and, as they are, the output gate's W_g u_g
 //   zi_delta_channel     the recurrence over the tokens of every entry, state in the request's slot
@@ -25,11 +26,184 @@ __device__ __forceinline__ float dc_decay(float z, float a) {      // a = exp(a_
     return expf(-a * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
 }
 
+// ---- what the recurrence reads -----------------------------------------------------------------------------------------
+// From the stacked projection (float32 rows, or partial sums of them): q, k and v pass a causal convolution over time
+// per channel (K taps, the last one the present token's, zeros before the start) and SiLU; every head of q and k
+// becomes a unit vector, q also times dim^-1/2; beta = sigmoid.  The convolution's new tail is written here too: the
+// first K - 1 tokens of an entry, which reach into the request's tail, all belong to the wavefront that has the entry's
+// first token.  A wavefront takes one unit (a head of q or k, 64 I channels of v, or, from partial sums, 64 I of the
+// columns that the low-rank gates read, which are only added up) of `per` consecutive tokens, the rows before the
+// present one in registers; lane l holds channels l, l + 64, ...
+template <int I, int K>
+__global__ void __launch_bounds__(256)
+channel_inputs_kernel(float* __restrict__ qk, float* __restrict__ v, float* __restrict__ beta, int64_t ld_beta,
+                      float* __restrict__ rest, const float* __restrict__ proj, int64_t ld, int splits, int64_t split_stride,
+                      const float* __restrict__ conv_w, float* __restrict__ tails, int64_t state_stride,
+                      const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ entry_start,
+                      const int32_t* __restrict__ entry_len, const int32_t* __restrict__ entry_slot, int n, int heads, int kvh,
+                      int dim, int vdim, int taps_rt, int b_at, int rest_at, int rest_cols, int per) {
+    const int lane = threadIdx.x & (ZI_WAVE - 1), unit = blockIdx.y * 4 + threadIdx.x / ZI_WAVE;
+    const int taps = K > 0 ? K : taps_rt;
+    const int qkc = 2 * kvh * dim, Vd = heads * vdim, C = qkc + Vd;
+    const int v_units = (Vd + 64 * I - 1) / (64 * I), r_units = (rest_cols + 64 * I - 1) / (64 * I);
+    if (unit >= 2 * kvh + v_units + r_units) return;
+    const bool is_qk = unit < 2 * kvh, is_rest = unit >= 2 * kvh + v_units;
+    // the unit's first channel (column, for the gates' columns) and how many it has
+    const int at = is_qk ? unit * dim : (is_rest ? (unit - 2 * kvh - v_units) * 64 * I : qkc + (unit - 2 * kvh) * 64 * I);
+    const int count = is_qk ? dim : (is_rest ? rest_cols - at : C - at);
+    const int col = is_rest ? rest_at + at : at;
+    const int t0 = blockIdx.x * per, t1 = t0 + per < n ? t0 + per : n;
+    auto value = [&](int64_t t, int c) __attribute__((always_inline)) {
+        const float* p = proj + t * ld + c;
+        float x = *p;
+        int s = 1;
+        for (; s + 4 <= splits; s += 4) {      // four loads in flight; the additions keep their order
+            const float a = p[s * split_stride], b = p[(s + 1) * split_stride], d = p[(s + 2) * split_stride], e = p[(s + 3) * split_stride];
+            x += a; x += b; x += d; x += e;
+        }
+        for (; s < splits; ++s) x += p[s * split_stride];
+        return x;
+    };
+    if (is_rest) {
+        for (int t = t0; t < t1; ++t)
+#pragma unroll
+            for (int i = 0; i < I; ++i)
+                if (lane + 64 * i < count) rest[(int64_t)t * rest_cols + at + lane + 64 * i] = value(t, col + lane + 64 * i);
+        return;
+    }
+    const float unit_scale = unit < kvh ? 1.f / sqrtf((float)dim) : 1.f;
+    auto finish = [&](int64_t t, const float* y) __attribute__((always_inline)) {
+        float r = 1.f;
+        if (is_qk) {
+            float ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < I; ++i) ss += y[i] * y[i];
+            r = unit_scale / sqrtf(zi_wave_sum(ss) + 1e-6f);
+        }
+        float* dst = is_qk ? qk + t * qkc + at : v + t * Vd + (at - qkc);
+#pragma unroll
+        for (int i = 0; i < I; ++i)
+            if (lane + 64 * i < count) dst[lane + 64 * i] = y[i] * r;
+        if (unit == 0)
+            for (int h = lane; h < heads; h += ZI_WAVE) beta[t * ld_beta + h] = 1.f / (1.f + expf(-value(t, b_at + h)));
+    };
+    constexpr int W = K > 1 ? K - 1 : 1;
+    float win[W][I], wt[K > 0 ? K : 1][I];
+    int ch[I];
+#pragma unroll
+    for (int i = 0; i < I; ++i) ch[i] = at + (lane + 64 * i < count ? lane + 64 * i : 0);
+    if constexpr (K > 0) {
+#pragma unroll
+        for (int j = 0; j < K; ++j)
+#pragma unroll
+            for (int i = 0; i < I; ++i) wt[j][i] = conv_w[(int64_t)ch[i] * K + j];
+    }
+    if constexpr (K > 1) {
+        if (per > 1) {
+#pragma unroll
+            for (int k = 0; k < K - 1; ++k) {
+                const int t = t0 - (K - 1) + k;
+#pragma unroll
+                for (int i = 0; i < I; ++i) win[k][i] = value(t > 0 ? t : 0, ch[i]);      // (of another entry, or none: never used)
+            }
+        }
+    }
+    for (int t = t0; t < t1; ++t) {
+        const int e = tok_seq[t], start = entry_start[e], local = t - start;
+        float cur[I], y[I];
+#pragma unroll
+        for (int i = 0; i < I; ++i) cur[i] = value(t, ch[i]);
+        if (local >= taps - 1) {
+#pragma unroll
+            for (int i = 0; i < I; ++i) {
+                float a = 0.f;
+                if constexpr (K > 0) {
+                    if constexpr (K > 1) {
+#pragma unroll
+                        for (int k = 0; k < K - 1; ++k) a += wt[k][i] * (per > 1 ? win[k][i] : value(t - (K - 1) + k, ch[i]));
+                    }
+                    a += wt[K - 1][i] * cur[i];
+                } else {
+                    for (int j = 0; j < taps; ++j) a += conv_w[(int64_t)ch[i] * taps + j] * value(t - (taps - 1) + j, ch[i]);
+                }
+                y[i] = lane + 64 * i < count ? a / (1.f + expf(-a)) : 0.f;
+            }
+            finish(t, y);
+        } else if (local == 0) {
+            float* tail = tails + (int64_t)entry_slot[e] * state_stride;
+            const int len = entry_len[e], m = len < taps - 1 ? len : taps - 1;
+            auto row = [&](int li, int i) __attribute__((always_inline)) {
+                return li >= 0 ? value(start + li, ch[i]) : tail[(int64_t)(li + taps - 1) * C + ch[i]];
+            };
+            for (int i0 = 0; i0 < m; ++i0) {
+#pragma unroll
+                for (int i = 0; i < I; ++i) {
+                    float a = 0.f;
+                    for (int j = 0; j < taps; ++j) a += conv_w[(int64_t)ch[i] * taps + j] * row(i0 - (taps - 1) + j, i);
+                    y[i] = lane + 64 * i < count ? a / (1.f + expf(-a)) : 0.f;
+                }
+                finish(start + i0, y);
+            }
+            // in rising order: row k of the new tail comes from row len + k of the old one or later
+#pragma unroll
+            for (int i = 0; i < I; ++i)
+                if (lane + 64 * i < count)
+                    for (int k = 0; k < taps - 1; ++k) tail[(int64_t)k * C + ch[i]] = row(len - (taps - 1) + k, i);
+        }
+        if constexpr (K > 1) {
+#pragma unroll
+            for (int i = 0; i < I; ++i) {
+#pragma unroll
+                for (int k = 0; k + 1 < K - 1; ++k) win[k][i] = win[k + 1][i];
+                win[K - 2][i] = cur[i];
+            }
+        }
+    }
+}
+
+// proj: float32 [n] rows of stride ld, columns [q | k | v | ...], beta's heads at b_at; or `splits` partial sums of such
+// rows, `split_stride` apart.  rest (float32 [n][rest_cols], or null with rest_cols 0): the sums of the columns
+// rest_at ... + rest_cols - 1.  tails: the place of [taps - 1][channels] in the slot's row.
+extern "C" int zi_channel_inputs(float* qk, float* v, float* beta, int64_t ld_beta, float* rest, const float* proj, int64_t ld,
+                                 int splits, int64_t split_stride, const float* conv_w, float* tails, int64_t state_stride,
+                                 const int32_t* tok_seq, const int32_t* entry_start, const int32_t* entry_len,
+                                 const int32_t* entry_slot, int n, int heads, int kvh, int dim, int vdim, int taps, int b_at,
+                                 int rest_at, int rest_cols, hipStream_t stream) {
+    ZI_REQUIRE(n >= 0 && heads > 0 && kvh > 0 && heads % kvh == 0 && dim > 0 && dim <= 256 && vdim > 0 && taps >= 1 &&
+               ld_beta >= heads && splits >= 1, "channel_inputs: bad sizes");
+    const int64_t C = 2LL * kvh * dim + (int64_t)heads * vdim;
+    ZI_REQUIRE(b_at >= C && ld >= b_at + heads && rest_cols >= 0 && (!rest_cols || (rest && rest_at >= C && ld >= rest_at + rest_cols)),
+               "channel_inputs: the columns do not fit the rows");
+    ZI_REQUIRE(taps == 1 || (tails && state_stride >= (int64_t)(taps - 1) * C), "channel_inputs: the state row is too short");
+    if (n == 0) return 0;
+    const int per = n >= 2048 ? 8 : (n >= 512 ? 4 : (n >= 128 ? 2 : 1));
+    const int wide = dim <= 64 ? 1 : (dim <= 128 ? 2 : 4);
+    const int units = 2 * kvh + (heads * vdim + 64 * wide - 1) / (64 * wide) + (rest_cols + 64 * wide - 1) / (64 * wide);
+    ZI_REQUIRE((units + 3) / 4 <= 65535, "channel_inputs: too many channels");
+    const dim3 grid((n + per - 1) / per, (units + 3) / 4);
+#define ZI_CI(I, K)                                                                                                        \
+    channel_inputs_kernel<I, K><<<grid, 256, 0, stream>>>(qk, v, beta, ld_beta, rest, proj, ld, splits, split_stride, conv_w, \
+        tails, state_stride, tok_seq, entry_start, entry_len, entry_slot, n, heads, kvh, dim, vdim, taps, b_at, rest_at,    \
+        rest_cols, per)
+#define ZI_CI_K(I)                          \
+    switch (taps) {                         \
+        case 1: ZI_CI(I, 1); break;         \
+        case 2: ZI_CI(I, 2); break;         \
+        case 3: ZI_CI(I, 3); break;         \
+        case 4: ZI_CI(I, 4); break;         \
+        default: ZI_CI(I, 0); break;        \
+    }
+    if (wide == 1) { ZI_CI_K(1) } else if (wide == 2) { ZI_CI_K(2) } else { ZI_CI_K(4) }
+#undef ZI_CI_K
+#undef ZI_CI
+    return zi_check_launch("channel_inputs");
+}
+
 // ---- low-rank gates -------------------------------------------------------------------------------------------------
 // Matrix cores: the float32 rows u are split into two bfloat16 parts (u = hi + lo within 2^-17 of u), so that the
 // product with bfloat16 weights is float32 but for that; ranks are padded to multiples of 32 (zero columns of W).  A
-// wavefront makes 16 channels of TM * 16 tokens.
-template <int TM>
+// wavefront makes CT * 16 channels of TM * 16 tokens (CT = 4 for many tokens: u is then split a quarter as often).
+template <int TM, int CT>
 __global__ void __launch_bounds__(256)
 lowrank_gates_cores_kernel(float* __restrict__ out_a, const float* __restrict__ u_a, const zi_bf16* __restrict__ w_a, int Ca,
                            int Ra, const float* __restrict__ bias, const float* __restrict__ a_log, int dim,
@@ -38,17 +212,22 @@ lowrank_gates_cores_kernel(float* __restrict__ out_a, const float* __restrict__ 
     const int lane = threadIdx.x & (ZI_WAVE - 1), wave = threadIdx.x / ZI_WAVE, r = lane & 15, j = lane >> 4;
     const bool decays = (int)blockIdx.x < blocks_a;
     const int C = decays ? Ca : Cg, R = decays ? Ra : Rg;
-    const int c0 = ((decays ? blockIdx.x : blockIdx.x - blocks_a) * 4 + wave) * 16;
+    const int c0 = ((decays ? blockIdx.x : blockIdx.x - blocks_a) * 4 + wave) * (16 * CT);
     if (c0 >= C) return;
-    const zi_bf16* w = (decays ? w_a : w_g) + (int64_t)(c0 + r < C ? c0 + r : C - 1) * R;
+    const zi_bf16* w[CT];
+#pragma unroll
+    for (int q = 0; q < CT; ++q) w[q] = (decays ? w_a : w_g) + (int64_t)(c0 + q * 16 + r < C ? c0 + q * 16 + r : C - 1) * R;
     const float* u = decays ? u_a : u_g;
     const int t0 = blockIdx.y * (TM * 16);
-    dc_f32x4_t acc[TM];
+    dc_f32x4_t acc[CT][TM];
 #pragma unroll
-    for (int m = 0; m < TM; ++m) acc[m] = dc_f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int q = 0; q < CT; ++q)
+#pragma unroll
+        for (int m = 0; m < TM; ++m) acc[q][m] = dc_f32x4_t{0.f, 0.f, 0.f, 0.f};
     for (int k0 = 0; k0 < R; k0 += 32) {
-        dc_pack a;
-        a.u = *reinterpret_cast<const uint4*>(w + k0 + j * 8);
+        dc_pack a[CT];
+#pragma unroll
+        for (int q = 0; q < CT; ++q) a[q].u = *reinterpret_cast<const uint4*>(w[q] + k0 + j * 8);
 #pragma unroll
         for (int m = 0; m < TM; ++m) {
             const int t = t0 + m * 16 + r;
@@ -64,34 +243,42 @@ lowrank_gates_cores_kernel(float* __restrict__ out_a, const float* __restrict__ 
             }
             hi.u = make_uint4(h[0], h[1], h[2], h[3]);
             lo.u = make_uint4(l[0], l[1], l[2], l[3]);
-            acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, hi.b, acc[m], 0, 0, 0);
-            acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, lo.b, acc[m], 0, 0, 0);
+#pragma unroll
+            for (int q = 0; q < CT; ++q) {
+                acc[q][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[q].b, hi.b, acc[q][m], 0, 0, 0);
+                acc[q][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[q].b, lo.b, acc[q][m], 0, 0, 0);
+            }
         }
     }
-    // lane (r, j): channels c0 + 4j .. + 3 of token r of each tile
+    // lane (r, j): channels 4j .. + 3 of every 16, of token r of each tile
+    float* out = decays ? out_a : out_g;
+#pragma unroll
+    for (int q = 0; q < CT; ++q) {
+    const int cq = c0 + q * 16 + j * 4;
+    if (cq >= C) continue;
     float ba[4], ea[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-        const int c = c0 + j * 4 + e < C ? c0 + j * 4 + e : C - 1;
+        const int c = cq + e < C ? cq + e : C - 1;
         ba[e] = decays ? bias[c] : 0.f;
         ea[e] = decays ? expf(a_log[c / dim]) : 0.f;
     }
-    float* out = decays ? out_a : out_g;
 #pragma unroll
     for (int m = 0; m < TM; ++m) {
         const int t = t0 + m * 16 + r;
         if (t >= n) continue;
         float v[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = decays ? dc_decay(acc[m][e] + ba[e], ea[e]) : acc[m][e];
-        float* dst = out + (int64_t)t * C + c0 + j * 4;
-        if (C % 4 == 0 && c0 + j * 4 + 3 < C) {
+        for (int e = 0; e < 4; ++e) v[e] = decays ? dc_decay(acc[q][m][e] + ba[e], ea[e]) : acc[q][m][e];
+        float* dst = out + (int64_t)t * C + cq;
+        if (C % 4 == 0 && cq + 3 < C) {
             *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
         } else {
 #pragma unroll
             for (int e = 0; e < 4; ++e)
-                if (c0 + j * 4 + e < C) dst[e] = v[e];
+                if (cq + e < C) dst[e] = v[e];
         }
+    }
     }
 }
 
@@ -129,14 +316,14 @@ extern "C" int zi_lowrank_gates(float* out_a, const float* u_a, const void* w_a,
                        ((uintptr_t)u_g % 16) == 0 && ((uintptr_t)w_a % 16) == 0 && ((uintptr_t)w_g % 16) == 0 &&
                        ((uintptr_t)out_a % 16) == 0 && ((uintptr_t)out_g % 16) == 0;
     if (cores) {
-        const int blocks_a = (Ca + 63) / 64, blocks = blocks_a + (Cg + 63) / 64;
-        const int tm = n > 128 ? 4 : 1;
-        ZI_REQUIRE((n + 16 * tm - 1) / (16 * tm) <= 65535, "lowrank_gates: too many tokens");
-        if (tm == 4)
-            lowrank_gates_cores_kernel<4><<<dim3(blocks, (n + 63) / 64), 256, 0, stream>>>(
+        const bool many = n > 256;
+        const int per = many ? 256 : 64, blocks_a = (Ca + per - 1) / per, blocks = blocks_a + (Cg + per - 1) / per;
+        ZI_REQUIRE((n + 15) / 16 <= 65535, "lowrank_gates: too many tokens");
+        if (many)
+            lowrank_gates_cores_kernel<2, 4><<<dim3(blocks, (n + 31) / 32), 256, 0, stream>>>(
                 out_a, u_a, (const zi_bf16*)w_a, Ca, Ra, bias, a_log, dim, out_g, u_g, (const zi_bf16*)w_g, Cg, Rg, ldu, n, blocks_a);
         else
-            lowrank_gates_cores_kernel<1><<<dim3(blocks, (n + 15) / 16), 256, 0, stream>>>(
+            lowrank_gates_cores_kernel<1, 1><<<dim3(blocks, (n + 15) / 16), 256, 0, stream>>>(
                 out_a, u_a, (const zi_bf16*)w_a, Ca, Ra, bias, a_log, dim, out_g, u_g, (const zi_bf16*)w_g, Cg, Rg, ldu, n, blocks_a);
         return zi_check_launch("lowrank_gates");
     }
@@ -148,45 +335,52 @@ extern "C" int zi_lowrank_gates(float* out_a, const float* u_a, const void* w_a,
 }
 
 // ---- the recurrence over portions -----------------------------------------------------------------------------------
-// A workgroup per (entry, head, 4 * WAVES columns of S); a wavefront holds 4 columns, lane (c, p) of it the R rows
-// 64 i + 4 p .. + 3 (i < R / 4) of column c, so that the sixteen lanes of a column read 256 consecutive bytes of a
-// staged row.  k, q and g of TOKS tokens at a time lie in LDS; the next TOKS tokens' are requested before the present
+// A workgroup per (entry, head, WAVES * 64 / PARTS columns of S); a wavefront holds 64 / PARTS columns, lane (c, p) of it
+// the R rows 4 PARTS i + 4 p .. + 3 (i < R / 4) of column c, so that the lanes of a column read consecutive bytes of a
+// staged row.  (One wavefront a SIMD is all a layer of twelve heads of 128 columns gives the chip, so a token costs what
+// its instructions cost one wavefront: 32 lanes a column with 4 rows each, in workgroups that stage 16 tokens at a time,
+// take 283 us for 2,048 tokens, 16 lanes with 8 rows and 8 tokens at a time 365; loads two stages ahead changed nothing.)
+//  k, q and g of TOKS tokens at a time lie in LDS; the next TOKS tokens' are requested before the present
 // ones are worked on.  Tokens past the entry's end stand there with k = q = 0, g = 1 and beta = 0, which leaves S as it
 // is to the bit, so the walk has no branch and every token's instructions are the same ones wherever it stands.
-// Per token only S^T k is summed over the lanes (four in-row lane moves); the read-outs' sums over the lanes are made
+// Per token only S^T k is summed over the lanes (in-row lane moves and a swap of rows); the read-outs' sums over the lanes are made
 // together after the TOKS tokens.
-#define DC_TOKS 8
-#define DC_PARTS 16
-
 template <int CTRL>
 __device__ __forceinline__ float dc_dpp(float x) {
     return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
 }
-__device__ __forceinline__ float dc_row_sum(float x) {      // over the 16 lanes of a row, in every one of them
+template <int PARTS>
+__device__ __forceinline__ float dc_row_sum(float x) {      // over 16 or 32 neighbouring lanes, in every one of them
     x += dc_dpp<0xB1>(x);       // quad_perm [1, 0, 3, 2]
     x += dc_dpp<0x4E>(x);       // quad_perm [2, 3, 0, 1]
     x += dc_dpp<0x141>(x);      // row_half_mirror
     x += dc_dpp<0x140>(x);      // row_mirror
+    if constexpr (PARTS == 32) {      // the sums of rows 0 and 1 (2 and 3) meet in both
+        const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+        x = __uint_as_float(r[0]) + __uint_as_float(r[1]);
+    }
     return x;
 }
 
-template <int R, int WAVES, int VL>
+template <int R, int DC_PARTS, int WAVES, int DC_TOKS, int VL>
 __global__ void __launch_bounds__(WAVES* ZI_WAVE)
 delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, const float* __restrict__ v,
                      const float* __restrict__ beta, int64_t ld_beta, const float* __restrict__ g, float* __restrict__ state,
                      int64_t state_stride, const int32_t* __restrict__ entry_start, const int32_t* __restrict__ entry_len,
                      const int32_t* __restrict__ entry_slot, int heads, int kvh, int dim, int vdim) {
-    constexpr int D = DC_PARTS * R, COLS = 4 * WAVES, THREADS = WAVES * ZI_WAVE;
+    static_assert(DC_PARTS == 16 || DC_PARTS == 32, "a column lies in one row of lanes or in two");
+    constexpr int CPW = ZI_WAVE / DC_PARTS;              // columns of a wavefront
+    constexpr int D = DC_PARTS * R, COLS = CPW * WAVES, THREADS = WAVES * ZI_WAVE;
     constexpr int PER = DC_TOKS * D / VL / THREADS;      // pieces of VL values of k (or q, or g) of a chunk a thread stages
     static_assert(PER * THREADS * VL == DC_TOKS * D && PER >= 1, "a chunk's rows divide evenly over the threads");
-    static_assert(DC_TOKS * COLS <= 2 * THREADS && R % 4 == 0, "values of a chunk: at most two a thread");
+    static_assert(DC_TOKS * COLS <= 2 * THREADS && R % 4 == 0 && DC_TOKS <= DC_PARTS, "values of a chunk: at most two a thread");
     __shared__ __attribute__((aligned(16))) float rows[2][DC_TOKS][3][D];      // k, q, g
     __shared__ float vs[2][DC_TOKS][COLS];
     __shared__ float bs[2][DC_TOKS];
     const int tid = threadIdx.x, lane = tid & (ZI_WAVE - 1), wave = tid / ZI_WAVE;
     const int c = lane / DC_PARTS, p = lane % DC_PARTS;
     const int h = blockIdx.y, e = blockIdx.z;
-    const int col0 = blockIdx.x * COLS, col = col0 + wave * 4 + c;
+    const int col0 = blockIdx.x * COLS, col = col0 + wave * CPW + c;
     const bool live = col < vdim;
     const int start = entry_start[e], len = entry_len[e];
     if (len <= 0) return;
@@ -195,7 +389,7 @@ delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, cons
     float S[R];
 #pragma unroll
     for (int i = 0; i < R; ++i) {
-        const int d = (i / 4) * 64 + p * 4 + i % 4;
+        const int d = (i / 4) * (4 * DC_PARTS) + p * 4 + i % 4;
         S[i] = (live && d < dim) ? S_[(int64_t)d * vdim + col] : 0.f;
     }
     float pk[PER][VL], pq[PER][VL], pg[PER][VL], pv[2], pb;
@@ -253,11 +447,11 @@ delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, cons
     auto fetch = [&](Tok& x, int b, int tt) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < R / 4; ++i) {
-            x.k[i] = *reinterpret_cast<const float4*>(&rows[b][tt][0][i * 64 + p * 4]);
-            x.q[i] = *reinterpret_cast<const float4*>(&rows[b][tt][1][i * 64 + p * 4]);
-            x.g[i] = *reinterpret_cast<const float4*>(&rows[b][tt][2][i * 64 + p * 4]);
+            x.k[i] = *reinterpret_cast<const float4*>(&rows[b][tt][0][i * (4 * DC_PARTS) + p * 4]);
+            x.q[i] = *reinterpret_cast<const float4*>(&rows[b][tt][1][i * (4 * DC_PARTS) + p * 4]);
+            x.g[i] = *reinterpret_cast<const float4*>(&rows[b][tt][2][i * (4 * DC_PARTS) + p * 4]);
         }
-        x.v = vs[b][tt][wave * 4 + c];
+        x.v = vs[b][tt][wave * CPW + c];
         x.beta = bs[b][tt];
     };
     auto work = [&](const Tok& x) __attribute__((always_inline)) {
@@ -273,7 +467,7 @@ delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, cons
             a2 = fmaf(S[4 * i + 2], x.k[i].z, a2);
             a3 = fmaf(S[4 * i + 3], x.k[i].w, a3);
         }
-        const float a = dc_row_sum((a0 + a1) + (a2 + a3));
+        const float a = dc_row_sum<DC_PARTS>((a0 + a1) + (a2 + a3));
         const float u = x.beta * (x.v - a);
         float o0 = 0.f, o1 = 0.f;
 #pragma unroll
@@ -308,7 +502,7 @@ delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, cons
         float mine = 0.f;
 #pragma unroll
         for (int tt = 0; tt < DC_TOKS; ++tt) {
-            const float total = dc_row_sum(read[tt]);
+            const float total = dc_row_sum<DC_PARTS>(read[tt]);
             if (p == tt) mine = total;
         }
         // lane (c, p) writes token p's read-out of column c
@@ -319,30 +513,32 @@ delta_channel_kernel(float* __restrict__ out, const float* __restrict__ qk, cons
     if (live) {
 #pragma unroll
         for (int i = 0; i < R; ++i) {
-            const int d = (i / 4) * 64 + p * 4 + i % 4;
+            const int d = (i / 4) * (4 * DC_PARTS) + p * 4 + i % 4;
             if (d < dim) S_[(int64_t)d * vdim + col] = S[i];
         }
     }
 }
 
 // ---- steps in which every entry brings one token --------------------------------------------------------------------
-// A workgroup per (entry, head, 64 columns) takes the head's rows through registers once: a load instruction of a
-// wavefront covers four rows x 64 columns (lane: row l / 16, columns 4 (l % 16) .. + 3), all loads issued before the
-// first is used.  S^T k and S^T q of the decayed state are summed over rows together, and the read-out of the updated
-// state is (S^T q) + (k . q) u.
-template <int P>      // passes of 16 rows: dim <= 16 P
-__global__ void __launch_bounds__(256)
-delta_channel_step_kernel(float* __restrict__ out, const float* __restrict__ qk, const float* __restrict__ v,
+// A workgroup per (entry, head, 64 CB columns; four wavefronts for every 64) takes the head's rows through registers
+// once: a load instruction of a wavefront covers four rows x 64 columns (lane: row l / 16, columns 4 (l % 16) .. + 3),
+// all loads issued before the first is used.  S^T k and S^T q of the decayed state are summed over rows together, and the read-out of the updated
+// state is (S^T q) + (k . q) u.  Where a workgroup holds the whole head it can finish it: y = o / rms(o) * w *
+// sigmoid(gate), and o itself is then not written.
+template <typename TY, int P, int CB>      // passes of 16 rows: dim <= 16 P
+__global__ void __launch_bounds__(256 * CB)
+delta_channel_step_kernel(TY* __restrict__ y, const float* __restrict__ norm, const float* __restrict__ gate, float eps,
+                          float* __restrict__ out, const float* __restrict__ qk, const float* __restrict__ v,
                           const float* __restrict__ beta, int64_t ld_beta, const float* __restrict__ g,
                           float* __restrict__ state, int64_t state_stride, const int32_t* __restrict__ entry_start,
                           const int32_t* __restrict__ entry_len, const int32_t* __restrict__ entry_slot, int heads, int kvh,
                           int dim, int vdim) {
     __shared__ float ks[16 * P], qs[16 * P], gs[16 * P];
-    __shared__ float4 pa[4][16], pb[4][16];
+    __shared__ float4 pa[CB][4][16], pb[CB][4][16];
     __shared__ float red[16];
-    const int h = blockIdx.y, e = blockIdx.z, tid = threadIdx.x, lane = tid & (ZI_WAVE - 1), wave = tid / ZI_WAVE;
+    const int h = blockIdx.y, e = blockIdx.z, tid = threadIdx.x, lane = tid & (ZI_WAVE - 1), cb = tid / 256, wave = (tid / ZI_WAVE) % 4;
     if (entry_len[e] != 1) return;
-    const int rr = lane / 16, cc = blockIdx.x * 64 + (lane % 16) * 4;
+    const int rr = lane / 16, cc = (blockIdx.x * CB + cb) * 64 + (lane % 16) * 4;
     const bool live = cc < vdim;      // vdim is a multiple of 4
     const int64_t t = entry_start[e];
     const int kh = h / (heads / kvh), qkc = 2 * kvh * dim;
@@ -357,7 +553,7 @@ delta_channel_step_kernel(float* __restrict__ out, const float* __restrict__ qk,
     const float4 vv = *reinterpret_cast<const float4*>(v + (t * heads + h) * vdim + (live ? cc : 0));
     const float bt = beta[t * ld_beta + h];
     float kq = 0.f;
-    for (int d = tid; d < 16 * P; d += 256) {
+    for (int d = tid; d < 16 * P; d += 256 * CB) {
         const bool in = d < dim;
         const float kk = in ? qk[t * qkc + (int64_t)(kvh + kh) * dim + d] : 0.f, qq = in ? qk[t * qkc + (int64_t)kh * dim + d] : 0.f;
         ks[d] = kk;
@@ -384,23 +580,35 @@ delta_channel_step_kernel(float* __restrict__ out, const float* __restrict__ qk,
         b.z += __shfl_xor(b.z, o, ZI_WAVE); b.w += __shfl_xor(b.w, o, ZI_WAVE);
     }
     if (rr == 0) {
-        pa[wave][lane] = a;
-        pb[wave][lane] = b;
+        pa[cb][wave][lane] = a;
+        pb[cb][wave][lane] = b;
     }
     __syncthreads();
-    a = pa[0][lane % 16];
-    b = pb[0][lane % 16];
+    a = pa[cb][0][lane % 16];
+    b = pb[cb][0][lane % 16];
 #pragma unroll
     for (int w = 1; w < 4; ++w) {
-        const float4 x = pa[w][lane % 16], y = pb[w][lane % 16];
+        const float4 x = pa[cb][w][lane % 16], z = pb[cb][w][lane % 16];
         a.x += x.x; a.y += x.y; a.z += x.z; a.w += x.w;
-        b.x += y.x; b.y += y.y; b.z += y.z; b.w += y.w;
+        b.x += z.x; b.y += z.y; b.z += z.z; b.w += z.w;
     }
     const float4 u = make_float4(bt * (vv.x - a.x), bt * (vv.y - a.y), bt * (vv.z - a.z), bt * (vv.w - a.w));
+    const float4 o = make_float4(fmaf(kq, u.x, b.x), fmaf(kq, u.y, b.y), fmaf(kq, u.z, b.z), fmaf(kq, u.w, b.w));
+    if (y) {      // the workgroup holds the whole head
+        const bool one = wave == 0 && rr == 0 && live;
+        const float ss = zi_block_sum(one ? o.x * o.x + o.y * o.y + o.z * o.z + o.w * o.w : 0.f, red);
+        if (one) {
+            const float rstd = 1.f / sqrtf(ss / (float)vdim + eps);
+            const float* gr = gate + (t * heads + h) * vdim + cc;
+            TY* dst = y + (t * heads + h) * vdim + cc;
+            const float ov[4] = {o.x, o.y, o.z, o.w};
+#pragma unroll
+            for (int i = 0; i < 4; ++i) zi_store(dst + i, ov[i] * rstd * norm[cc + i] / (1.f + expf(-gr[i])));
+        }
+    } else if (wave == 0 && rr == 0 && live) {
+        *reinterpret_cast<float4*>(out + (t * heads + h) * vdim + cc) = o;
+    }
     if (!live) return;
-    if (wave == 0 && rr == 0)
-        *reinterpret_cast<float4*>(out + (t * heads + h) * vdim + cc) =
-            make_float4(fmaf(kq, u.x, b.x), fmaf(kq, u.y, b.y), fmaf(kq, u.z, b.z), fmaf(kq, u.w, b.w));
 #pragma unroll
     for (int i = 0; i < P; ++i) {
         const int row = i * 16 + wave * 4 + rr;
@@ -413,11 +621,18 @@ delta_channel_step_kernel(float* __restrict__ out, const float* __restrict__ qk,
 
 // qk [n][2][kvh*dim] (q, then k), v [n][heads*vdim], beta [n] rows of stride ld_beta (heads first), g [n][heads*dim],
 // out [n][heads*vdim], all float32.  state: the matrices' place in the slot's row.  single_tokens: the caller says that
-// every entry brings one token (entries that do not are then left alone by the kernel for such steps).
+// every entry brings one token (entries that do not are then left alone by the kernel for such steps).  y (type y_dt,
+// [n][heads*vdim], or null; only for such steps, see zi_delta_channel_finishes): the read-outs normed with the gain
+// norm [vdim], times sigmoid(gate), and out is not written.
+extern "C" int zi_delta_channel_finishes(int vdim, int64_t state_stride) {
+    return vdim > 0 && vdim % 4 == 0 && vdim <= 128 && state_stride % 4 == 0;
+}
+
 extern "C" int zi_delta_channel(float* out, const float* qk, const float* v, const float* beta, int64_t ld_beta,
                                 const float* g, float* state, int64_t state_stride, const int32_t* entry_start,
                                 const int32_t* entry_len, const int32_t* entry_slot, int entries, int heads, int kvh, int dim,
-                                int vdim, int single_tokens, hipStream_t stream) {
+                                int vdim, int single_tokens, void* y, int y_dt, const float* norm, const float* gate, float eps,
+                                hipStream_t stream) {
     ZI_REQUIRE(entries >= 0 && entries <= 65535 && heads > 0 && heads <= 65535 && kvh > 0 && heads % kvh == 0 && dim > 0 &&
                vdim > 0 && ld_beta >= heads, "delta_channel: bad sizes");
     ZI_REQUIRE(dim <= 256, "delta_channel: dim %d is more than the 256 rows a wavefront holds", dim);
@@ -426,24 +641,41 @@ extern "C" int zi_delta_channel(float* out, const float* qk, const float* v, con
     const bool a16 = ((uintptr_t)qk % 16) == 0 && ((uintptr_t)g % 16) == 0;
     if (single_tokens && vdim % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)state % 16) == 0 && ((uintptr_t)v % 16) == 0 &&
         ((uintptr_t)out % 16) == 0) {
-        const dim3 grid((vdim + 63) / 64, heads, entries);
-#define ZI_DCS(P)                                                                                                     \
-    delta_channel_step_kernel<P><<<grid, 256, 0, stream>>>(out, qk, v, beta, ld_beta, g, state, state_stride, entry_start, \
-                                                           entry_len, entry_slot, heads, kvh, dim, vdim)
-        if (dim <= 32) ZI_DCS(2);
-        else if (dim <= 64) ZI_DCS(4);
-        else if (dim <= 128) ZI_DCS(8);
-        else ZI_DCS(16);
+        const int cb = y && vdim > 64 ? 2 : 1;
+        const dim3 grid((vdim + 64 * cb - 1) / (64 * cb), heads, entries);
+        ZI_REQUIRE(!y || (grid.x == 1 && norm && gate && eps > 0.f), "delta_channel: a head of %d values is not finished here", vdim);
+#define ZI_DCS2(P, CB)                                                                                                 \
+    delta_channel_step_kernel<TY, P, CB><<<grid, 256 * CB, 0, stream>>>((TY*)y, norm, gate, eps, out, qk, v, beta, ld_beta, g, \
+        state, state_stride, entry_start, entry_len, entry_slot, heads, kvh, dim, vdim)
+#define ZI_DCS(P)                  \
+    do {                           \
+        if (cb == 2) ZI_DCS2(P, 2); \
+        else ZI_DCS2(P, 1);        \
+    } while (0)
+        ZI_DISPATCH_DTYPE(y ? y_dt : ZI_F32, TY, {
+            if (dim <= 32) ZI_DCS(2);
+            else if (dim <= 64) ZI_DCS(4);
+            else if (dim <= 128) ZI_DCS(8);
+            else ZI_DCS(16);
+        });
 #undef ZI_DCS
+#undef ZI_DCS2
         return zi_check_launch("delta_channel_step");
     }
-#define ZI_DC(R, WAVES, VL)                                                                                             \
-    delta_channel_kernel<R, WAVES, VL><<<dim3((vdim + 4 * WAVES - 1) / (4 * WAVES), heads, entries), WAVES * ZI_WAVE, 0, stream>>>( \
+    ZI_REQUIRE(!y, "delta_channel: heads are finished in steps of single tokens only");
+#define ZI_DC2(R, PARTS, TOKS, VL)                                                                                      \
+    delta_channel_kernel<R, PARTS, 4, TOKS, VL><<<dim3((vdim + 256 / PARTS - 1) / (256 / PARTS), heads, entries), 256, 0, stream>>>( \
         out, qk, v, beta, ld_beta, g, state, state_stride, entry_start, entry_len, entry_slot, heads, kvh, dim, vdim)
     const bool v4 = dim % 4 == 0 && a16;
-    if (dim <= 64) { if (v4) ZI_DC(4, 2, 4); else ZI_DC(4, 2, 1); }
-    else if (dim <= 128) { if (v4) ZI_DC(8, 2, 4); else ZI_DC(8, 2, 1); }
-    else { if (v4) ZI_DC(16, 2, 4); else ZI_DC(16, 2, 1); }
+#define ZI_DC(R, PARTS, TOKS)                  \
+    do {                                       \
+        if (v4) ZI_DC2(R, PARTS, TOKS, 4);     \
+        else ZI_DC2(R, PARTS, TOKS, 1);        \
+    } while (0)
+    if (dim <= 64) ZI_DC(4, 16, 16);
+    else if (dim <= 128) ZI_DC(4, 32, 16);
+    else ZI_DC(8, 32, 8);
 #undef ZI_DC
+#undef ZI_DC2
     return zi_check_launch("delta_channel");
 }

@@ -16,14 +16,19 @@ __global__ void embedding_kernel(TO* __restrict__ out, const TW* __restrict__ ta
     for (int j = threadIdx.x; j < H; j += blockDim.x) zi_store(dst + j, ok ? zi_load(src + j) * scale : NAN);
 }
 
-extern "C" int zi_embedding(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids,
-                            int n, int hidden, int vocab, float scale, hipStream_t stream) {
+extern "C" int zi_embedding_scaled(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids,
+                                   int n, int hidden, int vocab, float scale, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && hidden > 0 && vocab > 0, "embedding: bad sizes n=%d hidden=%d vocab=%d", n, hidden, vocab);
     if (n == 0) return 0;
     ZI_DISPATCH_DTYPE(table_dt, TW, ZI_DISPATCH_DTYPE(out_dt, TO, {
         embedding_kernel<TW, TO><<<n, 256, 0, stream>>>((TO*)out, (const TW*)table, ids, hidden, vocab, scale);
     }));
     return zi_check_launch("embedding");
+}
+
+extern "C" int zi_embedding(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids,
+                            int n, int hidden, int vocab, hipStream_t stream) {
+    return zi_embedding_scaled(out, out_dt, table, table_dt, ids, n, hidden, vocab, 1.f, stream);
 }
 
 // out[i,:] = in[idx[i],:]

@@ -14,6 +14,7 @@
 #include "zi_api.h"
 
 #define IC_MAX_TAPS 16
+#define IC_RUN 4          // rows of a workgroup in long steps
 
 template <int V>
 struct ic_vec {
@@ -182,6 +183,33 @@ input_conv_kernel(TO* __restrict__ out, int64_t ldo, const TX* __restrict__ x, i
             }
         }
     }
+    if constexpr (K > 1) {
+        // a run of rows of one entry that do not reach into the tail: every row's load issued before the first is used
+        if (per == IC_RUN && t1 - t0 == IC_RUN) {
+            const int e = tok_seq[t0];
+            if (tok_seq[t1 - 1] == e && t0 - entry_start[e] >= K - 1) {
+                ic_vec<V> h[IC_RUN];
+#pragma unroll
+                for (int u = 0; u < IC_RUN; ++u) h[u] = h_at(t0 + u);
+#pragma unroll
+                for (int u = 0; u < IC_RUN; ++u) {
+                    ic_vec<V> y = h[u];
+#pragma unroll
+                    for (int i = 0; i < V; ++i) {
+                        float a = 0.f;
+#pragma unroll
+                        for (int k = 0; k < K; ++k) {
+                            const int r = u - (K - 1) + k;      // (known when the loops are unrolled)
+                            a += wt[k].x[i] * (r >= 0 ? h[r >= 0 ? r : 0].x[i] : win[r < 0 ? r + K - 1 : 0].x[i]);
+                        }
+                        y.x[i] += a;
+                    }
+                    ic_store<V>(out + (int64_t)(t0 + u) * ldo + c, y);
+                }
+                return;
+            }
+        }
+    }
     for (int t = t0; t < t1; ++t) {
         const int e = tok_seq[t], start = entry_start[e], local = t - start;
         const ic_vec<V> cur = h_at(t);
@@ -267,7 +295,7 @@ extern "C" int zi_input_conv(void* out, int out_dt, int64_t ldo, const void* x, 
     const int xe = x_dt == ZI_F32 ? 16 : 8, ge = gain_dt == ZI_F32 ? 16 : 8, oe = out_dt == ZI_F32 ? 16 : 8;
     const bool v4 = hidden % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && state_stride % 4 == 0 && ic_aligned(x, xe) &&
                     ic_aligned(out, oe) && ic_aligned(conv_w, 16) && ic_aligned(state, 16) && (!scale || ic_aligned(gain, ge));
-    const int per = n >= 2048 ? 8 : (n >= 512 ? 4 : (n >= 128 ? 2 : 1));
+    const int per = n >= 512 ? IC_RUN : (n >= 128 ? 2 : 1);
     const int lanes = v4 ? 4 : 1;
     const dim3 grid((n + per - 1) / per, (hidden + 128 * lanes - 1) / (128 * lanes));
 #define ZI_IC(V, K)                                                                                                     \

@@ -44,6 +44,9 @@ int zi_decode_layer(float* resid, int n, int H, int I, const void* norm1, const 
     max_keys, void* workspace, int64_t workspace_bytes, uint32_t* sync, int* err, int spin_limit, hipStream_t stream);
 // elementwise.hip
 int zi_embedding(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids, int n, int hidden, int
+    vocab, hipStream_t stream);
+// elementwise.hip
+int zi_embedding_scaled(void* out, int out_dt, const void* table, int table_dt, const int32_t* ids, int n, int hidden, int
     vocab, float scale, hipStream_t stream);
 // elementwise.hip
 int zi_gather_rows(void* out, const void* in, int dt, const int32_t* idx, int n_out, int n_in, int hidden, hipStream_t
@@ -122,7 +125,7 @@ int zi_latent_value(void* out, int out_dt, int64_t ldo, const float* o, const vo
 int zi_delta_prepare(float* qk, float* v, float* beta_g, const float* proj, int64_t ld, int n, const void* conv_w, const
     void* a_log, const void* dt_bias, int w_dt, const float* state, int64_t state_stride, int64_t conv_off, const
     int32_t* tok_seq, const int32_t* entry_start, const int32_t* entry_slot, int heads, int kvh, int dim, int vdim, int
-    taps, int b_at, int a_at, hipStream_t stream);
+    taps, hipStream_t stream);
 // delta.hip
 int zi_delta_conv_state(float* state, int64_t state_stride, int64_t conv_off, const float* proj, int64_t ld, const
     int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, int entries, int channels, int taps,
@@ -324,7 +327,13 @@ int zi_lowrank_gates(float* out_a, const float* u_a, const void* w_a, int Ca, in
 // delta_channel.hip
 int zi_delta_channel(float* out, const float* qk, const float* v, const float* beta, int64_t ld_beta, const float* g, float*
     state, int64_t state_stride, const int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, int
-    entries, int heads, int kvh, int dim, int vdim, int single_tokens, hipStream_t stream);
+    entries, int heads, int kvh, int dim, int vdim, int single_tokens, void* y, int y_dt, const float* norm, const float*
+    gate, float eps, hipStream_t stream);
+// delta_channel.hip
+int zi_channel_inputs(float* qk, float* v, float* beta, int64_t ld_beta, float* rest, const float* proj, int64_t ld, int
+    splits, int64_t split_stride, const float* conv_w, float* tails, int64_t state_stride, const int32_t* tok_seq, const
+    int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_slot, int n, int heads, int kvh, int dim, int vdim,
+    int taps, int b_at, int rest_at, int rest_cols, hipStream_t stream);
 // sampling.hip
 int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int rows, int vocab, const float*
     temperature, const int32_t* top_k, const float* top_p, const float* penalty, const float* uniform, const int32_t*
@@ -407,7 +416,9 @@ int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int ro
     X(zi_moe_route_sigmoid) \
     X(zi_moe_weighted_glu) \
     X(zi_moe_sum_shared) \
+    X(zi_embedding_scaled) \
     X(zi_stream_scale) \
+    X(zi_channel_inputs) \
     X(zi_input_conv) \
     X(zi_norm_input_conv) \
     X(zi_lowrank_gates) \

@@ -27,7 +27,7 @@ from .sublayers import (clamped_glu, conv_qkv, conv_state_floats, conv_tail, con
 from .recurrent import (attention_biased, embedding_sum, gate_heads, gated_rms_norm_act, linear_attention,
                         linear_attention_state_floats, lowrank_decay, moe_route_table, normed_kv_store, stream_reenter,
                         token_shift)
-from .convolved import (channel_state_floats, delta_channel, input_conv, lowrank_gates, norm_input_conv,
+from .convolved import (channel_inputs, channel_state_floats, delta_channel, delta_channel_finishes, input_conv, lowrank_gates, norm_input_conv,
                         norm_input_conv_supported, stream_scale)
 from . import hybrid
 from .hybrid import (linear_attention_grouped, moe_route_sigmoid, moe_sum_shared, moe_weighted_glu, norm_rope_store,
@@ -58,7 +58,7 @@ __all__ = [
     "linear_attention_state_floats", "lowrank_decay", "moe_route_table", "normed_kv_store", "stream_reenter", "token_shift",
     "linear_attention_grouped", "moe_route_sigmoid", "moe_sum_shared", "moe_weighted_glu", "norm_rope_store",
     "normed_add_norm", "pool_blocks", "pooled_attention", "pooled_attention_cores", "pooled_attention_cores_cut", "pooled_attention_cores_supported", "pooled_attention_cores_workspace", "rope_table_scaled", "ssm_finish", "ssm_prepare", "ssm_state_floats",
-    "channel_state_floats", "delta_channel", "input_conv", "lowrank_gates", "norm_input_conv", "norm_input_conv_supported",
+    "channel_inputs", "channel_state_floats", "delta_channel", "delta_channel_finishes", "input_conv", "lowrank_gates", "norm_input_conv", "norm_input_conv_supported",
     "stream_scale",
     "KernelLibraryError", "library_path", "load", "FEW_ROWS", "SUMS_MAX_ROWS",
 ]

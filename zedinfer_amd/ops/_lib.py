@@ -18,7 +18,8 @@ P, I, L, F = c_void_p, c_int, c_int64, c_float
 
 _PROTOTYPES = {
     "zi_abi_version": [],
-    "zi_embedding": [P, I, P, I, P, I, I, I, F, P],
+    "zi_embedding": [P, I, P, I, P, I, I, I, P],
+    "zi_embedding_scaled": [P, I, P, I, P, I, I, I, F, P],
     "zi_gather_rows": [P, P, I, P, I, I, I, P],
     "zi_add": [P, I, P, I, P, I, L, P],
     "zi_swiglu": [P, I, P, P, I, I, I, L, L, I, I, L, P],
@@ -77,7 +78,7 @@ _PROTOTYPES = {
     "zi_headwise_linear_supported": [I, I, L, I],
     "zi_latent_query_rot": [P, P, I, L, P, I, I, I, I, I, P],
     "zi_latent_value": [P, I, L, P, P, I, I, I, I, I, P],
-    "zi_delta_prepare": [P, P, P, P, L, I, P, P, P, I, P, L, L, P, P, P, I, I, I, I, I, I, I, P],
+    "zi_delta_prepare": [P, P, P, P, L, I, P, P, P, I, P, L, L, P, P, P, I, I, I, I, I, P],
     "zi_delta_conv_state": [P, L, L, P, L, P, P, P, I, I, I, P],
     "zi_delta_rule": [P, P, P, P, P, L, P, P, P, I, I, I, I, I, P],
     "zi_gated_rmsnorm": [P, I, P, P, I, P, L, I, I, I, F, P],
@@ -131,7 +132,9 @@ _PROTOTYPES = {
     "zi_norm_input_conv": [P, I, P, P, I, I, L, P, I, F, F, P, P, L, P, P, P, I, I, I, P],
     "zi_norm_input_conv_supported": [I, I, I],
     "zi_lowrank_gates": [P, P, P, I, I, P, P, I, P, P, P, I, I, I, L, I, P],
-    "zi_delta_channel": [P, P, P, P, L, P, P, L, P, P, P, I, I, I, I, I, I, P],
+    "zi_delta_channel": [P, P, P, P, L, P, P, L, P, P, P, I, I, I, I, I, I, P, I, P, P, F, P],
+    "zi_delta_channel_finishes": [I, L],
+    "zi_channel_inputs": [P, P, P, L, P, P, L, I, L, P, P, L, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
     "zi_tape_record": [P, c_char_p, P, I],
     "zi_tape_record_many": [P, c_char_p, P, P, I],
     "zi_tape_run": [P, P],

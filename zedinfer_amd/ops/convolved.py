@@ -8,7 +8,7 @@ import torch
 
 from . import _lib
 from .functional import F32, _code, _gpu, _i32, _p, _rows, _stream
-from .mixing import _f32, delta_state_floats as channel_state_floats      # the same row: matrices, then the convolution's tail
+from .mixing import DELTA_MAX_TAPS, _f32, delta_state_floats as channel_state_floats      # the same row: matrices, then the convolution's tail
 from .sublayers import CONV_MAX_TAPS, _terms
 
 
@@ -148,13 +148,62 @@ def lowrank_gates(u_a: torch.Tensor, w_a: torch.Tensor, bias: torch.Tensor, a_lo
               _p(u_g), _p(w_g), Cg, Rg, _code(w_a, "lowrank_gates w"), max(lda, ldg), n, _stream())
 
 
+def channel_inputs(proj: torch.Tensor, conv_w: torch.Tensor, tails: Optional[torch.Tensor], tok_seq: torch.Tensor,
+                   entry_start: torch.Tensor, entry_len: torch.Tensor, entry_slot: torch.Tensor, heads: int, kv_heads: int,
+                   dim: int, vdim: int, taps: int, beta_at: int, qk: torch.Tensor, v: torch.Tensor, beta: torch.Tensor,
+                   rest_at: int = 0, rest: Optional[torch.Tensor] = None) -> None:
+    """From rows proj [n, q | k | v | ...] (float32), or a stack [S, n, ...] of partial sums of them: the short convolution
+    (``conv_w`` [channels, taps]) and SiLU of q, k and v, q and k made unit vectors per head (q also times dim^-1/2) into
+    ``qk`` [n, 2 kv_heads dim], v into ``v`` [n, heads vdim], beta = sigmoid(b) with b at column ``beta_at`` into the
+    first ``heads`` columns of ``beta``'s rows (row stride free); the sums of the columns ``rest_at`` ... into ``rest``
+    [n, columns], if given.  Rows before an entry's first one come from ``tails`` [slots, >= (taps - 1) channels] (dense
+    rows) at the entry's slot, which then takes the entry's last taps - 1 rows."""
+    _gpu("channel_inputs", proj, conv_w, tails, tok_seq, entry_start, entry_len, entry_slot, qk, v, beta, rest)
+    splits, split_stride, ld, n, width = _terms(proj, "channel_inputs proj", columns=True)
+    C = 2 * kv_heads * dim + heads * vdim
+    if proj.dtype != torch.float32 or not (C <= beta_at <= width - heads):
+        raise ValueError(f"channel_inputs: proj must be float32 with the {C} channels first and beta behind them")
+    _f32(conv_w, "channel_inputs conv_w", (C, taps))
+    _f32(qk, "channel_inputs qk", (n, 2 * kv_heads * dim))
+    _f32(v, "channel_inputs v", (n, heads * vdim))
+    if beta.dtype != torch.float32 or beta.shape[0] != n or beta.stride(-1) != 1 or beta[0].numel() < heads:
+        raise ValueError(f"channel_inputs: beta must be float32 [n, >= {heads}]")
+    cols = 0
+    if rest is not None:
+        cols = int(rest.shape[1])
+        _f32(rest, "channel_inputs rest", (n, cols))
+        if not (C <= rest_at <= width - cols):
+            raise ValueError("channel_inputs: the columns to be added up lie outside the rows")
+    if not (1 <= taps <= DELTA_MAX_TAPS) or dim > 256:
+        raise ValueError(f"channel_inputs: at most {DELTA_MAX_TAPS} taps and heads of 256 channels")
+    stride = 0
+    if taps > 1:
+        if tails is None or tails.dtype != torch.float32 or tails.dim() != 2 or tails.stride(1) != 1 or tails.shape[1] < (taps - 1) * C:
+            raise ValueError(f"channel_inputs: tails must be float32 [slots, >= {(taps - 1) * C}] with dense rows")
+        stride = int(tails.stride(0))
+    _i32(tok_seq, "channel_inputs tok_seq", n)
+    E = entry_start.numel()
+    for t in (entry_start, entry_len, entry_slot):
+        _i32(t, "channel_inputs entries", E)
+    _lib.call("zi_channel_inputs", _p(qk), _p(v), _p(beta), int(beta.stride(0)), _p(rest), _p(proj), ld, splits, split_stride,
+              _p(conv_w), _p(tails if taps > 1 else None), stride, _p(tok_seq), _p(entry_start), _p(entry_len), _p(entry_slot), n,
+              heads, kv_heads, dim, vdim, taps, int(beta_at), int(rest_at), cols, _stream())
+
+
+def delta_channel_finishes(vdim: int, state: torch.Tensor) -> bool:
+    """Whether ``delta_channel`` can norm and gate the read-outs of single tokens itself (``finish``)."""
+    return bool(_lib.load().zi_delta_channel_finishes(int(vdim), int(state.stride(0)))) and state.data_ptr() % 16 == 0
+
+
 def delta_channel(qk: torch.Tensor, v: torch.Tensor, beta_g: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
                   entry_start: torch.Tensor, entry_len: torch.Tensor, entry_slot: torch.Tensor, heads: int, kv_heads: int,
-                  dim: int, vdim: int, out: torch.Tensor, single_tokens: bool = False) -> torch.Tensor:
+                  dim: int, vdim: int, out: torch.Tensor, single_tokens: bool = False, finish=None) -> torch.Tensor:
     """Every entry's tokens in order, per head: S <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, with
     S read from and left in ``state`` [slots, >= heads*dim*vdim] float32 (dense rows); qk [n, 2 kv_heads dim] (q, then
     k), v [n, heads vdim], ``beta_g`` [n, 2, heads] (beta first; the rest is not read), decay [n, heads dim], out
-    [n, heads vdim], all float32.  ``single_tokens``: every entry brings one token."""
+    [n, heads vdim], all float32.  ``single_tokens``: every entry brings one token.  ``finish`` (y, norm, gate, eps; only
+    then, and where ``delta_channel_finishes``): y [n, heads vdim] = o / rms(o over a head) * norm [vdim] * sigmoid(gate)
+    is written instead of o."""
     _gpu("delta_channel", qk, v, beta_g, decay, state, entry_start, entry_len, entry_slot, out)
     n = qk.shape[0]
     _f32(qk, "delta_channel qk", (n, 2 * kv_heads * dim))
@@ -166,9 +215,20 @@ def delta_channel(qk: torch.Tensor, v: torch.Tensor, beta_g: torch.Tensor, decay
         raise ValueError(f"delta_channel: the state must be float32 [slots, >= {heads * dim * vdim}] with dense rows")
     if dim > 256:
         raise ValueError(f"delta_channel: dim {dim} is more than the kernel's 256")
+    last = (_p(None), F32, _p(None), _p(None), 0.0)
+    if finish is not None:
+        y, norm, gate, eps = finish
+        _gpu("delta_channel finish", y, norm, gate)
+        if not single_tokens or not delta_channel_finishes(vdim, state):
+            raise ValueError("delta_channel: heads are finished in steps of single tokens, where the kernel holds them whole")
+        if tuple(y.shape) != (n, heads * vdim) or not y.is_contiguous():
+            raise ValueError("delta_channel: y must be contiguous [n, heads * vdim]")
+        _f32(norm, "delta_channel norm", (vdim,))
+        _f32(gate, "delta_channel gate", (n, heads * vdim))
+        last = (_p(y), _code(y, "delta_channel y"), _p(norm), _p(gate), float(eps))
     E = entry_start.numel()
     for t in (entry_start, entry_len, entry_slot):
         _i32(t, "delta_channel entries", E)
     _lib.call("zi_delta_channel", _p(out), _p(qk), _p(v), _p(beta_g), 2 * heads, _p(decay), _p(state), int(state.stride(0)),
-              _p(entry_start), _p(entry_len), _p(entry_slot), E, heads, kv_heads, dim, vdim, int(bool(single_tokens)), _stream())
-    return out
+              _p(entry_start), _p(entry_len), _p(entry_slot), E, heads, kv_heads, dim, vdim, int(bool(single_tokens)), *last, _stream())
+    return out if finish is None else finish[0]

@@ -87,8 +87,11 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor
         out = torch.empty((n, H), dtype=out_dtype or table.dtype, device=table.device)
     if tuple(out.shape) != (n, H) or not out.is_contiguous():
         raise ValueError(f"embedding: out must be contiguous [{n}, {H}], got {tuple(out.shape)}")
-    _lib.call("zi_embedding", _p(out), _code(out, "embedding out"), _p(table), _code(table, "embedding table"),
-              _p(ids), n, H, V, float(scale), _stream())
+    args = (_p(out), _code(out, "embedding out"), _p(table), _code(table, "embedding table"), _p(ids), n, H, V)
+    if scale != 1.0:
+        _lib.call("zi_embedding_scaled", *args, float(scale), _stream())
+    else:
+        _lib.call("zi_embedding", *args, _stream())
     return out
 
 

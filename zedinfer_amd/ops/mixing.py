@@ -247,40 +247,31 @@ def delta_state_floats(heads: int, dim: int, vdim: int, kv_heads: int, taps: int
 def delta_prepare(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
                   state: torch.Tensor, tok_seq: torch.Tensor, entry_start: torch.Tensor, entry_slot: torch.Tensor,
                   heads: int, kv_heads: int, dim: int, vdim: int, taps: int, qk: torch.Tensor, v: torch.Tensor,
-                  beta_g: torch.Tensor, beta_at: Optional[int] = None) -> None:
+                  beta_g: torch.Tensor) -> None:
     """From the stacked projection proj [n, q | k | v | gate | b | a] (float32): the short convolution and SiLU of
     q, k, v (rows before an entry's first come from the tail kept in ``state``), q and k made unit vectors per
     head (q also times dim^-1/2) into ``qk`` [n, 2 kv_heads dim], v into ``v`` [n, heads vdim], and into
-    ``beta_g`` [n, 2, heads] beta = sigmoid(b) and the decay g = exp(-exp(a_log) softplus(a + dt_bias)).  With
-    ``beta_at`` proj is [n, q | k | v | ...] with b at that column and no decay is made (``a_log`` and ``dt_bias`` None;
-    ``beta_g``'s second half is left alone)."""
+    ``beta_g`` [n, 2, heads] beta = sigmoid(b) and the decay g = exp(-exp(a_log) softplus(a + dt_bias))."""
     _gpu("delta_prepare", proj, conv_w, a_log, dt_bias, state, tok_seq, entry_start, entry_slot, qk, v, beta_g)
     n = proj.shape[0]
     C = 2 * kv_heads * dim + heads * vdim
     ld, width = _rows(proj, "delta_prepare proj")
-    if beta_at is None:
-        if proj.dtype != torch.float32 or width != C + heads * vdim + 2 * heads:
-            raise ValueError(f"delta_prepare: proj must be float32 [n, {C + heads * vdim + 2 * heads}]")
-        _f32(a_log, "delta_prepare a_log", (heads,))
-        _f32(dt_bias, "delta_prepare dt_bias", (heads,))
-        b_at, a_at = C + heads * vdim, C + heads * vdim + heads
-    else:
-        b_at, a_at = int(beta_at), -1
-        if proj.dtype != torch.float32 or b_at < C or width < b_at + heads or a_log is not None or dt_bias is not None:
-            raise ValueError(f"delta_prepare: proj must be float32 with the {C} channels first and beta behind them")
-    _f32(conv_w, "delta_prepare conv_w", (C, taps))
+    if proj.dtype != torch.float32 or width != C + heads * vdim + 2 * heads:
+        raise ValueError(f"delta_prepare: proj must be float32 [n, {C + heads * vdim + 2 * heads}]")
+    for t, shape, what in ((conv_w, (C, taps), "conv_w"), (a_log, (heads,), "a_log"), (dt_bias, (heads,), "dt_bias")):
+        _f32(t, f"delta_prepare {what}", shape)
     _f32(qk, "delta_prepare qk", (n, 2 * kv_heads * dim))
     _f32(v, "delta_prepare v", (n, heads * vdim))
     _f32(beta_g, "delta_prepare beta_g", (n, 2, heads))
-    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 \
-            or state.shape[1] < delta_state_floats(heads, dim, vdim, kv_heads, taps):
+    _f32(state, "delta_prepare state")
+    if state.dim() != 2 or state.shape[1] < delta_state_floats(heads, dim, vdim, kv_heads, taps):
         raise ValueError("delta_prepare: the state must be [slots, floats of one request's state]")
     _i32(tok_seq, "delta_prepare tok_seq", n)
     _i32(entry_start, "delta_prepare entry_start")
     _i32(entry_slot, "delta_prepare entry_slot", entry_start.numel())
     _lib.call("zi_delta_prepare", _p(qk), _p(v), _p(beta_g), _p(proj), ld, n, _p(conv_w), _p(a_log), _p(dt_bias), 0,
-              _p(state), int(state.stride(0)), heads * dim * vdim, _p(tok_seq), _p(entry_start), _p(entry_slot), heads,
-              kv_heads, dim, vdim, taps, b_at, a_at, _stream())
+              _p(state), int(state.shape[1]), heads * dim * vdim, _p(tok_seq), _p(entry_start), _p(entry_slot), heads,
+              kv_heads, dim, vdim, taps, _stream())
 
 
 def delta_conv_state(state: torch.Tensor, proj: torch.Tensor, entry_start: torch.Tensor, entry_len: torch.Tensor,
@@ -291,14 +282,13 @@ def delta_conv_state(state: torch.Tensor, proj: torch.Tensor, entry_start: torch
     ld, width = _rows(proj, "delta_conv_state proj")
     if proj.dtype != torch.float32 or width < C:
         raise ValueError("delta_conv_state: proj must be float32 and hold the convolution's channels first")
-    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1:
-        raise ValueError("delta_conv_state: the state must be float32 [slots, ...] with dense rows")
+    _f32(state, "delta_conv_state state")
     if taps > DELTA_MAX_TAPS:
         raise ValueError(f"delta_conv_state: at most {DELTA_MAX_TAPS} taps")
     E = entry_start.numel()
     for t in (entry_start, entry_len, entry_slot):
         _i32(t, "delta_conv_state entries", E)
-    _lib.call("zi_delta_conv_state", _p(state), int(state.stride(0)), heads * dim * vdim, _p(proj), ld, _p(entry_start),
+    _lib.call("zi_delta_conv_state", _p(state), int(state.shape[1]), heads * dim * vdim, _p(proj), ld, _p(entry_start),
               _p(entry_len), _p(entry_slot), E, C, taps, _stream())
 
 

@@ -191,22 +191,32 @@ class ChannelDeltaRule(Mixer):
     def forward(self, x: torch.Tensor, batch, memory: LayerMemory) -> torch.Tensor:
         n, rt, nh, kvh, dim, vdim = x.shape[0], self.rt, self.nh, self.kvh, self.dim, self.vdim
         state = memory.state
-        proj = ops.linear(x, self.w_in, out=rt.buffer("delta_proj", (n, self.width), torch.float32))
+        matrices, tails = state[:, :nh * dim * vdim], state[:, nh * dim * vdim:]
+        rest = None
+        if ops.linear_sums_supported(x, self.w_in):      # few rows: the kernel that convolves adds the partial sums
+            S = ops.linear_splits(n, self.width, self.hidden)
+            proj = ops.linear_sums(x, self.w_in, out=rt.buffer("delta_proj_sums", (S, n, self.width), torch.float32))
+            rest = gates = rt.buffer("delta_lowrank", (n, self.b_at - self.a_at), torch.float32)
+        else:
+            proj = ops.linear(x, self.w_in, out=rt.buffer("delta_proj", (n, self.width), torch.float32))
+            gates = proj[:, self.a_at:self.b_at]
         qk = rt.buffer("delta_qk", (n, 2 * kvh * dim), torch.float32)
         v = rt.buffer("delta_v", (n, nh * vdim), torch.float32)
         beta = rt.buffer("delta_beta_g", (n, 2, nh), torch.float32)
-        ops.delta_prepare(proj, self.conv_w, None, None, state, batch.tok_seq, batch.entry_start, batch.entry_slot, nh, kvh,
-                          dim, vdim, self.taps, qk, v, beta, beta_at=self.b_at)
-        ops.delta_conv_state(state, proj, batch.entry_start, batch.entry_len, batch.entry_slot, nh, kvh, dim, vdim,
-                             self.taps)
+        ops.channel_inputs(proj, self.conv_w, tails, batch.tok_seq, batch.entry_start, batch.entry_len, batch.entry_slot, nh,
+                           kvh, dim, vdim, self.taps, self.b_at, qk, v, beta.view(n, 2 * nh), rest_at=self.a_at, rest=rest)
         decay = rt.buffer("delta_decay", (n, nh * dim), torch.float32)
         gate = rt.buffer("delta_gate", (n, nh * vdim), torch.float32)
-        ops.lowrank_gates(proj[:, self.a_at:self.g_at], self.second["a2"], self.dt_bias, self.a_log,
-                          proj[:, self.g_at:self.b_at], self.second["g2"], decay, gate)
+        ranks = self.g_at - self.a_at
+        ops.lowrank_gates(gates[:, :ranks], self.second["a2"], self.dt_bias, self.a_log, gates[:, ranks:], self.second["g2"],
+                          decay, gate)
         o = rt.buffer("delta_read", (n, nh * vdim), torch.float32)
-        ops.delta_channel(qk, v, beta, decay, state, batch.entry_start, batch.entry_len, batch.entry_slot, nh, kvh, dim, vdim,
-                          out=o, single_tokens=bool(batch.single_tokens))
-        y = ops.gated_rms_norm_act(o, self.norm, gate, nh, vdim, self.eps, "sigmoid", out=rt.buffer("delta_heads", (n, nh * vdim)))
+        y, single = rt.buffer("delta_heads", (n, nh * vdim)), bool(batch.single_tokens)
+        finish = (y, self.norm, gate, self.eps) if single and ops.delta_channel_finishes(vdim, matrices) else None
+        ops.delta_channel(qk, v, beta, decay, matrices, batch.entry_start, batch.entry_len, batch.entry_slot, nh, kvh, dim, vdim,
+                          out=o, single_tokens=single, finish=finish)
+        if finish is None:
+            ops.gated_rms_norm_act(o, self.norm, gate, nh, vdim, self.eps, "sigmoid", out=y)
         if ops.linear_sums_supported(y, self.o):      # few rows: the partial sums go to the norm that follows
             S = ops.linear_splits(n, self.hidden, nh * vdim)
             return ops.linear_sums(y, self.o, out=rt.buffer("delta_out_sums", (S, n, self.hidden), torch.float32))
