@@ -326,6 +326,35 @@ def test_attention_with_a_logarithm_of_the_distance_through_every_kernel(case, d
         att2 = torch.zeros(T, H * d, dtype=dtype, device=DEV)
         ops.attention_decode(qd, kc, vc, seq0, pos, tab, H, G, d, scale, T, window, out=att2, tok_index=some, **extras)
         assert torch.equal(att2[some.long()], att[some.long()]) and float(att2[6].abs().max()) == 0.0
+        # the same behind a gate: chunks left, merged and gated by a kernel, or by the output projection for few tokens
+        head = d - 3                                       # (heads padded in the cache: only their first values count)
+        rows = torch.cat([torch.arange(T - 9, T), torch.tensor([0, 5, W - 1, T // 2])]).clamp(0, T - 1)
+        n, ws = rows.numel(), torch.full((ops.attention_decode_workspace(rows.numel(), H, d),), float("nan"), device=DEV)
+        gate = 2 * torch.randn(3, n, H * head + 6, generator=g)
+        args = (qd[rows.to(DEV)].contiguous(), kc, vc, seq0[:n], pos[rows.to(DEV)].contiguous(), tab, H, G, d, scale, T, window)
+        sinks = torch.randn(H, generator=g).to(DEV) if G > 1 else None
+        merged = want[rows].view(n, H, d)
+        if sinks is not None:                              # (a sink rescales a head: the sums of its softmax, from the scores)
+            merged = torch.zeros_like(merged)
+            for i, t in enumerate(rows.tolist()):
+                lo = max(0, t - window + 1) if window else 0
+                for h in range(H):
+                    dist = torch.arange(t - lo, -1, -1).double()
+                    sc = k[lo:t + 1, h // (H // G)].double() @ q[t, h].double() * scale - r1[h].double() * torch.log(1 + r2[h].double() * dist)
+                    wgt = torch.softmax(torch.cat([sc, sinks[h:h + 1].cpu().double()]), dim=0)[:-1]
+                    merged[i, h] = wgt @ v[lo:t + 1, h // (H // G)].double()
+        ops.attention_decode(*args, workspace=ws, sinks=sinks, leave_chunks=True, **extras)
+        y = torch.zeros(n, H * head, dtype=BF, device=DEV)
+        ops.attention_decode_merge_gated(ws, args[4], H, d, head, T, gate.to(DEV)[:, :, 6:], y, window=window, sinks=sinks)
+        _close(y, (merged[:, :, :head].reshape(n, -1) * torch.sigmoid(gate[:, :, 6:].double().sum(0))), 2.5e-2, "merged and gated")
+        wo = (torch.randn(40, H * d, generator=g) / (H * d) ** 0.5).to(BF)
+        gate = 2 * torch.randn(6, n, H * d + 4, generator=g)
+        for gt in (gate[:, :, 4:], gate[0, :, 4:]):
+            if not ops.attention_decode_project_supported(wo.to(DEV), n, H, d):
+                continue
+            sums = ops.attention_decode_project(ws, wo.to(DEV), args[4], H, d, T, window, sinks=sinks, gate=gt.to(DEV))
+            gated = merged.reshape(n, -1) * torch.sigmoid(gt.double().sum(0) if gt.dim() == 3 else gt.double())
+            _close(sums.sum(0), gated @ wo.double().T, 2.5e-2, "projected behind the gate")
     if not ops.attention_prefill_supported(dtype, H, G, d, ps):
         return
     least, most = ops.attention_prefill_tile_min(), ops.attention_prefill_tile(dtype, d)
@@ -340,7 +369,7 @@ def test_attention_with_a_logarithm_of_the_distance_through_every_kernel(case, d
 
 
 # ---- the smaller pieces ---------------------------------------------------------------------------------------------------------
-@pytest.mark.parametrize("inter, n, dtype", [(64, 5, BF), (62, 130, torch.float32), (300, 70, BF)])
+@pytest.mark.parametrize("inter, n, dtype", [(64, 5, BF), (62, 130, torch.float32), (300, 70, BF), (296, 70, BF), (1500, 64, BF), (37, 9, BF)])
 def test_the_clamped_feed_forward_with_biases(inter, n, dtype):
     from zedinfer_amd.config import PartSpec
     from zedinfer_amd.parts import FEED_FORWARDS, Runtime
@@ -364,6 +393,27 @@ def test_the_clamped_feed_forward_with_biases(inter, n, dtype):
     y = part.forward(x.to(DEV))
     want = plain.clamped_glu(x.double() @ p["f.gate"].T, x.double() @ p["f.up"].T, limit) @ p["f.down"].T
     _close(y.float().sum(0) if y.dim() == 3 else y, want, 1e-5 if dtype == torch.float32 else 2e-2, "no biases")
+
+
+@pytest.mark.parametrize("M, I, K", [(1, 88, 64), (17, 1504, 320), (64, 8192, 1024), (33, 6400, 264), (250, 24, 8)])
+@pytest.mark.parametrize("biased", [True, False])
+def test_the_clamped_activation_over_rows_that_alternate_in_blocks(M, I, K, biased):
+    g = torch.Generator().manual_seed(I)
+    x, w = torch.randn(M, K, generator=g).to(BF), (2 * torch.randn(2 * I, K, generator=g) / K ** 0.5).to(BF)
+    b = torch.randn(2 * I, generator=g).to(BF) if biased else None
+    full = x.double() @ w.double().T + (b.double() if biased else 0.0)
+    blocks = full.view(M, I // 8, 2, 8)
+    want = plain.clamped_glu(blocks[:, :, 0].reshape(M, I), blocks[:, :, 1].reshape(M, I), 1.1)
+    rows = full.to(BF).to(DEV)
+    wide = torch.zeros(M, I + 16, dtype=BF, device=DEV)
+    _close(ops.clamped_glu_il8(rows, 1.1, out=wide[:, 8:8 + I]), want, 2e-2, "rows")
+    assert float(wide[:, :8].abs().max()) == 0.0 and float(wide[:, 8 + I:].abs().max()) == 0.0
+    xd, wd, bd = x.to(DEV), w.to(DEV), (b.to(DEV) if biased else None)
+    if M <= ops.FEW_ROWS and ops.linear_swiglu_supported(xd, wd):
+        _close(ops.linear_clamped_glu(xd, wd, bd, 1.1), want, 1e-2, "epilogue")
+    else:
+        with pytest.raises(ValueError):
+            ops.linear_clamped_glu(xd, wd, bd, 1.1)
 
 
 @pytest.mark.parametrize("M, N, K", [(1, 96, 512), (7, 1536, 1536), (70, 260, 768), (128, 90, 256), (200, 4096, 8192)])

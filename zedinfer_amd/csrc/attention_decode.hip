@@ -572,16 +572,47 @@ attention_decode_kernel(zi_bf16* __restrict__ out, int64_t ldo, float* __restric
     }
 }
 
-// Merge the chunks of one (token, head): out = sum_c e^(m_c - M) o_c / sum_c e^(m_c - M) l_c.
+// A gate of the merged heads: sigmoid(g), g the sum of `splits` float32 terms `stride` apart at [token][head * vd + dim].
+struct DecGate {
+    const float* g;      // null: none
+    int64_t ld, stride;
+    int splits, vd;
+};
+
+__device__ __forceinline__ float dec_gate(const DecGate& gt, int64_t at) {
+    float v = gt.g[at];
+    int s = 1;
+    for (; s + 4 <= gt.splits; s += 4) {      // four terms in flight; the additions keep their order
+        const float a = gt.g[s * gt.stride + at], b = gt.g[(s + 1) * gt.stride + at], c = gt.g[(s + 2) * gt.stride + at],
+                    d = gt.g[(s + 3) * gt.stride + at];
+        v += a; v += b; v += c; v += d;
+    }
+    for (; s < gt.splits; ++s) v += gt.g[s * gt.stride + at];
+    return 1.f / (1.f + expf(-v));
+}
+
+// Merge the chunks of one (token, head): out = sum_c e^(m_c - M) o_c / sum_c e^(m_c - M) l_c.  With a gate every token's
+// chunks are in the workspace (also where there is one) and the first gt.vd values of every head, gated, are written
+// side by side.
 __global__ void __launch_bounds__(ZI_WAVE)
 attention_decode_merge_kernel(zi_bf16* __restrict__ out, int64_t ldo, const float* __restrict__ part_o,
                               const float* __restrict__ part_ml, const int32_t* __restrict__ tok_index,
                               const int32_t* __restrict__ tok_pos, int nh, int D, int window, int max_chunks,
-                              const float* __restrict__ sinks) {
+                              const float* __restrict__ sinks, DecGate gt) {
     const int x = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int t = tok_index ? tok_index[x] : x;
     const DecSplit sp = dec_split(tok_pos[t], window);
-    if (sp.count == 1 || sp.count > max_chunks) return;
+    if (!gt.g && (sp.count == 1 || sp.count > max_chunks)) return;
+    float gate[2] = {1.f, 1.f};
+    if (gt.g) {
+#pragma unroll
+        for (int v = 0; v < 2; ++v)
+            if (lane + v * ZI_WAVE < gt.vd) gate[v] = dec_gate(gt, (int64_t)t * gt.ld + (int64_t)h * gt.vd + lane + v * ZI_WAVE);
+        if (sp.count > max_chunks) {      // chunks the launch did not cover: it shows
+            for (int v = lane; v < gt.vd; v += ZI_WAVE) zi_store(out + (int64_t)t * ldo + (int64_t)h * gt.vd + v, NAN);
+            return;
+        }
+    }
     const int64_t slot0 = zi_dec_part_slot(x, nh, h, 0);
     // chunk c's (m, l) sit in lane c
     const float mc = lane < sp.count ? part_ml[(slot0 + lane) * 2] : -INFINITY;
@@ -607,9 +638,11 @@ attention_decode_merge_kernel(zi_bf16* __restrict__ out, int64_t ldo, const floa
     }
     if (sinks) L += __builtin_amdgcn_exp2f(sinks[h] * 1.4426950408889634f - M);
     const float inv = 1.f / L;
+    const int vd = gt.g ? gt.vd : D;
 #pragma unroll
     for (int v = 0; v < 2; ++v)
-        if (lane + v * ZI_WAVE < D) zi_store(out + (int64_t)t * ldo + (int64_t)h * D + lane + v * ZI_WAVE, acc[v] * inv);
+        if (lane + v * ZI_WAVE < vd)
+            zi_store(out + (int64_t)t * ldo + (int64_t)h * vd + lane + v * ZI_WAVE, acc[v] * inv * gate[v]);
 }
 
 // The output projection straight from the chunks: sums[s][t][:] = W[:, heads of split s] . merged
@@ -626,7 +659,7 @@ __global__ void __launch_bounds__(256)
 attention_decode_project_kernel(float* __restrict__ sums, const float* __restrict__ part_o,
                                 const float* __restrict__ part_ml, const int32_t* __restrict__ tok_pos, int n, int nh,
                                 int window, int max_chunks, const zi_bf16* __restrict__ w, int64_t ldw, int N, int hg,
-                                const float* __restrict__ sinks) {
+                                const float* __restrict__ sinks, DecGate gt) {
     constexpr int DK = (D + 31) / 32;
     constexpr int XS = DK * 32 + 8;     // row stride of the merged head in LDS, in elements (16-byte rows, no bank repeat)
     __shared__ __attribute__((aligned(16))) uint16_t sx[16][XS];
@@ -654,6 +687,18 @@ attention_decode_project_kernel(float* __restrict__ sums, const float* __restric
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[e] = 0.f;
         const int q = tid & 15, mtc = mt < n ? mt : n - 1;
+        float gsum[8];
+        if (gt.g) {      // (gt.vd == D here; rows of the gate are aligned to 16 bytes)
+            const float* gp = gt.g + (int64_t)mtc * gt.ld + (int64_t)h * D + (d0 < D ? d0 : 0);
+            float4 g0 = *reinterpret_cast<const float4*>(gp), g1 = *reinterpret_cast<const float4*>(gp + 4);
+            for (int s = 1; s < gt.splits; ++s) {
+                const float4 x0 = *reinterpret_cast<const float4*>(gp + s * gt.stride), x1 = *reinterpret_cast<const float4*>(gp + s * gt.stride + 4);
+                g0.x += x0.x; g0.y += x0.y; g0.z += x0.z; g0.w += x0.w;
+                g1.x += x1.x; g1.y += x1.y; g1.z += x1.z; g1.w += x1.w;
+            }
+            gsum[0] = g0.x; gsum[1] = g0.y; gsum[2] = g0.z; gsum[3] = g0.w;
+            gsum[4] = g1.x; gsum[5] = g1.y; gsum[6] = g1.z; gsum[7] = g1.w;
+        }
         const int count = dec_split(tok_pos[mtc], window).count;
         const int64_t slot0 = zi_dec_part_slot(mtc, nh, h, 0);
         const float2* ml = reinterpret_cast<const float2*>(part_ml) + slot0;
@@ -710,6 +755,10 @@ attention_decode_project_kernel(float* __restrict__ sums, const float* __restric
             const float inv = count > max_chunks ? NAN : 1.f / L;      // chunks the launch did not cover: it shows
 #pragma unroll
             for (int e = 0; e < 8; ++e) v[e] *= inv;
+            if (gt.g) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[e] *= 1.f / (1.f + expf(-gsum[e]));
+            }
         }
 #pragma unroll
         for (int dk = 0; dk < DK; ++dk) {     // the padding of the last k-step is zero on both sides
@@ -832,7 +881,8 @@ static int dec_launch(const char* who, void* out, const void* q, int dt, int n_i
 #undef ZI_DEC
     if (max_chunks > 1 && !leave_parts)
         attention_decode_merge_kernel<<<dim3(n_idx, nh), ZI_WAVE, 0, stream>>>((zi_bf16*)out, ldo, po, pml, tok_index,
-                                                                              tok_pos, nh, d, window, max_chunks, sinks);
+                                                                              tok_pos, nh, d, window, max_chunks, sinks,
+                                                                              DecGate{nullptr, 0, 0, 1, 0});
     return zi_check_launch(who);
 }
 
@@ -939,11 +989,15 @@ extern "C" int zi_attention_decode_project_supported(int dt, int n, int nh, int 
 // max_chunks (and without tok_index): sums[s][t][:] = W[:, columns of the heads of group s] . attention
 // of token t, float32, s < ceil(nh / zi_attention_decode_project_heads(nh)), rows of `sums` N long.
 // W is [N, nh * d] bfloat16 with row stride ldw.
-// `sinks` (float32 [nh], or null): exp(sinks[h]) counts once in the denominator of head h's merge.
-extern "C" int zi_attention_decode_project_sink(float* sums, const float* workspace, int64_t workspace_floats, int n,
+// `sinks` (float32 [nh], or null): exp(sinks[h]) counts once in the denominator of head h's merge.  `gate` (float32, or
+// null): the merged heads are multiplied by sigmoid(gate[t][head * d + dim]), the gate the sum of `gate_splits` terms
+// `gate_stride` apart with rows of stride ld_gate.
+extern "C" int zi_attention_decode_project_gated(float* sums, const float* workspace, int64_t workspace_floats, int n,
                                                 const int32_t* tok_pos, int window, int max_chunks, const void* w, int dt,
-                                                int64_t ldw, int N, int nh, int d, const float* sinks,
-                                                hipStream_t stream) {
+                                                int64_t ldw, int N, int nh, int d, const float* sinks, const float* gate,
+                                                int64_t ld_gate, int gate_splits, int64_t gate_stride, hipStream_t stream) {
+    ZI_REQUIRE(!gate || (ld_gate >= (int64_t)nh * d && ld_gate % 4 == 0 && gate_splits >= 1 && gate_stride % 4 == 0 && ((uintptr_t)gate % 16) == 0),
+               "attention_decode_project: the gate's rows must be aligned to 16 bytes");
     ZI_REQUIRE(zi_attention_decode_project_supported(dt, n, nh, d, ldw),
                "attention_decode_project: unsupported shape (bfloat16, 1..16 tokens, head_dim a multiple of 16 up to "
                "128, row stride a multiple of 8): dtype %d tokens %d heads %d head_dim %d stride %lld", dt, n, nh, d,
@@ -958,9 +1012,10 @@ extern "C" int zi_attention_decode_project_sink(float* sums, const float* worksp
     const int hg = zi_attention_decode_project_heads(nh);
     const dim3 grid((N + DPJ_ROWS - 1) / DPJ_ROWS, (nh + hg - 1) / hg);
     ZI_REQUIRE(grid.y <= 65535, "attention_decode_project: too many heads");
+    const DecGate gt = {gate, ld_gate, gate_stride, gate_splits, d};
 #define ZI_DPJ(DD)                                                                                                    \
     attention_decode_project_kernel<DD><<<grid, 256, 0, stream>>>(sums, po, pml, tok_pos, n, nh, window, max_chunks,   \
-                                                                  (const zi_bf16*)w, ldw, N, hg, sinks)
+                                                                  (const zi_bf16*)w, ldw, N, hg, sinks, gt)
     switch (d) {
         case 16: ZI_DPJ(16); break;
         case 32: ZI_DPJ(32); break;
@@ -973,6 +1028,32 @@ extern "C" int zi_attention_decode_project_sink(float* sums, const float* worksp
     }
 #undef ZI_DPJ
     return zi_check_launch("attention_decode_project");
+}
+
+// The chunks that zi_attention_decode_biased left in `workspace` (out == nullptr) for the same n, nh, d, tok_pos, window
+// and max_chunks, merged and gated: y[t][head * vd + dim] = o * sigmoid(gate[t][head * vd + dim]) for the first vd <= d
+// values of every head, bfloat16, rows of stride ldy.
+extern "C" int zi_attention_decode_merge_gated(void* y, int64_t ldy, const float* workspace, int64_t workspace_floats, int n,
+                                               const int32_t* tok_pos, int window, int max_chunks, int nh, int d, int vd,
+                                               const float* sinks, const float* gate, int64_t ld_gate, int gate_splits,
+                                               int64_t gate_stride, hipStream_t stream) {
+    ZI_REQUIRE(n >= 0 && n <= 65535 && nh > 0 && nh <= 65535 && d >= 16 && d <= 128 && vd > 0 && vd <= d && window >= 0 &&
+                   max_chunks >= 1 && max_chunks <= DEC_MAXC && ldy >= (int64_t)nh * vd, "attention_decode_merge_gated: bad sizes");
+    ZI_REQUIRE(gate && gate_splits >= 1 && ld_gate >= (int64_t)nh * vd, "attention_decode_merge_gated: a gate is needed");
+    ZI_REQUIRE(workspace && workspace_floats >= zi_attention_decode_workspace(n, nh, d) && ((uintptr_t)workspace % 16) == 0,
+               "attention_decode_merge_gated: workspace of %lld floats is too small or not aligned", (long long)workspace_floats);
+    if (n == 0) return 0;
+    attention_decode_merge_kernel<<<dim3(n, nh), ZI_WAVE, 0, stream>>>((zi_bf16*)y, ldy, workspace, workspace + (int64_t)n * nh * DEC_MAXC * d,
+                                                                      nullptr, tok_pos, nh, d, window, max_chunks, sinks,
+                                                                      DecGate{gate, ld_gate, gate_stride, gate_splits, vd});
+    return zi_check_launch("attention_decode_merge_gated");
+}
+
+extern "C" int zi_attention_decode_project_sink(float* sums, const float* workspace, int64_t workspace_floats, int n,
+                                                const int32_t* tok_pos, int window, int max_chunks, const void* w, int dt,
+                                                int64_t ldw, int N, int nh, int d, const float* sinks, hipStream_t stream) {
+    return zi_attention_decode_project_gated(sums, workspace, workspace_floats, n, tok_pos, window, max_chunks, w, dt, ldw, N,
+                                             nh, d, sinks, nullptr, 0, 1, 0, stream);
 }
 
 extern "C" int zi_attention_decode_project(float* sums, const float* workspace, int64_t workspace_floats, int n,

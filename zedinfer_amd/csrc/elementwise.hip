@@ -381,6 +381,42 @@ extern "C" int zi_clamped_glu(void* out, int out_dt, int64_t ldo, const void* ga
     return zi_check_launch("clamped_glu");
 }
 
+// The same over rows [n][2 inter] (bfloat16) whose gate and up columns alternate in blocks of 8: eight results a thread.
+__global__ void __launch_bounds__(256)
+clamped_glu_il8_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf16* __restrict__ gu, int64_t ld, int n, int inter,
+                       float limit, float alpha) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const int blocks = inter / 8;
+    if (i >= (int64_t)n * blocks) return;
+    const int64_t r = i / blocks, b = i % blocks;
+    const uint4 g4 = *reinterpret_cast<const uint4*>(gu + r * ld + b * 16), u4 = *reinterpret_cast<const uint4*>(gu + r * ld + b * 16 + 8);
+    const uint32_t gw[4] = {g4.x, g4.y, g4.z, g4.w}, uw[4] = {u4.x, u4.y, u4.z, u4.w};
+    uint32_t o[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        float y[2];
+#pragma unroll
+        for (int z = 0; z < 2; ++z) {
+            const float g = fminf(__uint_as_float(z ? gw[k] & 0xffff0000u : gw[k] << 16), limit);
+            const float u = fminf(fmaxf(__uint_as_float(z ? uw[k] & 0xffff0000u : uw[k] << 16), -limit), limit);
+            y[z] = g / (1.f + expf(-alpha * g)) * (u + 1.f);
+        }
+        o[k] = zi_pack_bf16x2(y[0], y[1]);
+    }
+    *reinterpret_cast<uint4*>(out + r * ldo + b * 8) = make_uint4(o[0], o[1], o[2], o[3]);
+}
+
+extern "C" int zi_clamped_glu_il8(void* out, int64_t ldo, const void* gu, int64_t ld, int n, int inter, float limit,
+                                  float alpha, hipStream_t stream) {
+    ZI_REQUIRE(n >= 0 && inter > 0 && inter % 8 == 0 && ldo >= inter && ld >= 2LL * inter && ld % 8 == 0 && ldo % 8 == 0 &&
+                   ((uintptr_t)gu % 16) == 0 && ((uintptr_t)out % 16) == 0 && limit > 0.f, "clamped_glu_il8: bad sizes or alignment");
+    if (n == 0) return 0;
+    const int64_t total = (int64_t)n * (inter / 8);
+    clamped_glu_il8_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>((zi_bf16*)out, ldo, (const zi_bf16*)gu, ld, n,
+                                                                               inter, limit, alpha);
+    return zi_check_launch("clamped_glu_il8");
+}
+
 // x <- cap * tanh(x / cap), float32, in place (the soft cap of logits).
 __global__ void softcap_kernel(float* __restrict__ x, int64_t total, float cap) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;

@@ -28,6 +28,7 @@ typedef __attribute__((ext_vector_type(4))) unsigned gm_u32x4_t;
 #define GM_MODE_PLAIN 0
 #define GM_MODE_PARTIAL 1
 #define GM_MODE_SWIGLU 2
+#define GM_MODE_CLAMPED 3      // like SWIGLU, with biases: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1)
 
 union gm_pack {
     gm_u32x4_t u;
@@ -45,12 +46,16 @@ __device__ __forceinline__ gm_u32x4_t gm_keep(gm_u32x4_t v, bool keep) {
 template <int MT>
 __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* __restrict__ out, int mode, int out_f32,
                                             const zi_bf16* __restrict__ bias, int M, int N, int64_t ldo, int split,
-                                            int n0, int r, int j, int vec_out) {
+                                            int n0, int r, int j, int vec_out, float limit) {
 #pragma unroll
     for (int t = 0; t < MT; ++t) {
         gm_f32x4_t s = acc[t];
         const int m = t * 16 + r;
-        if (mode == GM_MODE_SWIGLU) {
+        if (mode == GM_MODE_SWIGLU || mode == GM_MODE_CLAMPED) {
+            if (mode == GM_MODE_CLAMPED && bias && n0 < N) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) s[e] += zi_load(bias + n0 + j * 4 + e);
+            }
             // lanes j = 0,1 hold gate rows j*4 + e, lanes j = 2,3 the up rows of the same columns
             gm_f32x4_t up;
             up[0] = __shfl_xor(s[0], 32, ZI_WAVE); up[1] = __shfl_xor(s[1], 32, ZI_WAVE);
@@ -59,7 +64,14 @@ __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* _
             const int col = (n0 / 16) * 8 + j * 4;     // N / 2 columns of output; N % 16 == 0
             float act[4];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) act[e] = up[e] * (s[e] / (1.f + expf(-s[e])));
+            for (int e = 0; e < 4; ++e) {
+                if (mode == GM_MODE_SWIGLU) {
+                    act[e] = up[e] * (s[e] / (1.f + expf(-s[e])));
+                } else {
+                    const float g = fminf(s[e], limit), u = fminf(fmaxf(up[e], -limit), limit);
+                    act[e] = g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+                }
+            }
             zi_bf16* dst = (zi_bf16*)out + (int64_t)m * ldo + col;
             if (vec_out) {
                 uint2 pk;
@@ -116,7 +128,7 @@ template <int MT, int GM_RING, int GM_WAVES>
 __global__ void __launch_bounds__(GM_WAVES* ZI_WAVE)
 gemm_mid_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16* __restrict__ x,
                 const zi_bf16* __restrict__ w, const zi_bf16* __restrict__ bias, int M, int N, int K, int64_t ldx,
-                int64_t ldw, int64_t ldo, int kb_per_split, int vec_out) {
+                int64_t ldw, int64_t ldo, int kb_per_split, int vec_out, float limit) {
     __shared__ __attribute__((aligned(16))) uint16_t xs[2][MT * 16 * GM_XS];
     __shared__ __attribute__((aligned(16))) uint16_t wt[GM_WAVES][16 * GM_XS];   // a wavefront's weight tile
     const int tid = threadIdx.x, lane = tid & (ZI_WAVE - 1), wave = tid / ZI_WAVE;
@@ -245,7 +257,7 @@ gemm_mid_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16* __
             default: if (GM_RING > 3) ending(std::integral_constant<int, 3>{}, kb0); break;
         }
     }
-    gm_epilogue<MT>(acc, out, mode, out_f32, bias, M, N, ldo, split, n0, r, j, vec_out);
+    gm_epilogue<MT>(acc, out, mode, out_f32, bias, M, N, ldo, split, n0, r, j, vec_out, limit);
 }
 
 // The same product for 65 .. 128 rows of x (MT = 5 .. 8 tiles of 16 rows): one pass over the weights where two
@@ -260,7 +272,7 @@ template <int MT, int GM_WAVES>
 __global__ void __launch_bounds__(GM_WAVES* ZI_WAVE)
 gemm_wide_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16* __restrict__ x,
                  const zi_bf16* __restrict__ w, const zi_bf16* __restrict__ bias, int M, int N, int K, int64_t ldx,
-                 int64_t ldw, int64_t ldo, int kb_per_split, int vec_out) {
+                 int64_t ldw, int64_t ldo, int kb_per_split, int vec_out, float limit) {
     constexpr int RING = 3;
     __shared__ __attribute__((aligned(16))) uint16_t xs[MT * 16 * GM_XS];
     __shared__ __attribute__((aligned(16))) uint16_t wt[GM_WAVES][16 * GM_XS];
@@ -363,7 +375,7 @@ gemm_wide_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16* _
             default: ending(std::integral_constant<int, 2>{}, kb0); break;
         }
     }
-    gm_epilogue<MT>(acc, out, mode, out_f32, bias, M, N, ldo, split, n0, r, j, vec_out);
+    gm_epilogue<MT>(acc, out, mode, out_f32, bias, M, N, ldo, split, n0, r, j, vec_out, limit);
 }
 
 // How the product with a weight matrix [N, K] is cut: wavefronts a workgroup (16 weight rows each), splits
@@ -406,7 +418,7 @@ void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves) 
 
 // The launch; the checks are the caller's (zi_gemm_skinny).
 int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
-                       int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, hipStream_t stream) {
+                       int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream) {
     int splits, per, waves;
     zi_gemm_mid_plan(N, K, &splits, &per, &waves);
     const int tiles = (N + 15) / 16;
@@ -414,7 +426,7 @@ int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const
     const int mt = (M + 15) / 16;
 #define ZI_GM2(MT, WV)                                                                                            \
     gemm_mid_kernel<MT, 3, WV><<<grid, WV * ZI_WAVE, 0, stream>>>(out, mode, out_f32, x, w, bias, M, N, K, ldx, ldw, \
-                                                                  ldo, per, vec_out)
+                                                                  ldo, per, vec_out, limit)
 #define ZI_GM(MT)                               \
     switch (waves) {                            \
         case 4: ZI_GM2(MT, 4); break;           \
@@ -425,7 +437,7 @@ int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const
     }
 #define ZI_GW2(MT, WV)                                                                                         \
     gemm_wide_kernel<MT, WV><<<grid, WV * ZI_WAVE, 0, stream>>>(out, mode, out_f32, x, w, bias, M, N, K, ldx, ldw, ldo, \
-                                                               per, vec_out)
+                                                               per, vec_out, limit)
 #define ZI_GW(MT)                               \
     switch (waves) {                            \
         case 4: ZI_GW2(MT, 4); break;           \

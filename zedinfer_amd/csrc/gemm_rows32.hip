@@ -261,7 +261,8 @@ void zi_gemm_rows32_plan(int N, int K, int many_rows, int whole, int* splits, in
 
 // The launch; the checks are the caller's (zi_gemm_skinny).  M is 1 .. 256.
 int zi_gemm_rows32_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
-                          int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, hipStream_t stream) {
+                          int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream) {
+    (void)limit;      // (these products have no clamped epilogue)
     int splits, per, waves;
     zi_gemm_rows32_plan(N, K, M > 128, mode == G32_MODE_SWIGLU, &splits, &per, &waves);
     const int tiles = (N + 31) / 32;

@@ -23,6 +23,7 @@
 #define SK_MODE_PLAIN 0
 #define SK_MODE_PARTIAL 1
 #define SK_MODE_SWIGLU 2
+#define SK_MODE_CLAMPED 3
 
 // out[m,n] = sum_s partial[s,m,n] + bias[n], splits added in rising order.
 __global__ void gemm_skinny_reduce_kernel(void* __restrict__ out, int out_f32, const float* __restrict__ partial,
@@ -62,13 +63,13 @@ extern "C" int zi_gemm_skinny_pays(int M, int N, int K) {
 // The product kernel (gemm_mid.hip): its cut and its launch.
 void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves);
 int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
-                       int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, hipStream_t stream);
+                       int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream);
 
 void zi_gemm_rows32_plan(int N, int K, int many_rows, int whole, int* splits, int* kb_per_split, int* waves);
 int zi_gemm_rows32_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
-                          int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, hipStream_t stream);
+                          int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream);
 
-static bool sk_rows32(int M, int mode) { return M > (mode == SK_MODE_SWIGLU ? SK_MID_MAX_ROWS_SWIGLU : SK_MID_MAX_ROWS); }
+static bool sk_rows32(int M, int mode) { return M > (mode >= SK_MODE_SWIGLU ? SK_MID_MAX_ROWS_SWIGLU : SK_MID_MAX_ROWS); }
 
 // Splits of k for a weight matrix [N, K]: the leading dimension of the partial sums.  A function of N and K and
 // of which of the two kernels the rows go to (up to 128, or more).
@@ -89,13 +90,16 @@ extern "C" int64_t zi_gemm_skinny_workspace(int M, int N, int K) {
 // mode 1: out = float32 partial sums [splits][M][N] (splits from zi_gemm_skinny_splits; the bias, if any, is in the first).
 // mode 2: w holds gate and up rows interleaved in blocks of 8; out[M, N/2] (bfloat16) =
 //         up * silu(gate); only for products that are not split.
-extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M,
-                              int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace,
-                              int64_t workspace_floats, hipStream_t stream) {
+// mode 3: the same with g = min(gate + bias, limit), u = clamp(up + bias, -limit, limit), g sigmoid(1.702 g) (u + 1), the
+//         bias [N] (or null) interleaved as the rows are; up to 64 rows.
+extern "C" int zi_gemm_skinny_act(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M,
+                                  int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace,
+                                  int64_t workspace_floats, float limit, hipStream_t stream) {
     ZI_REQUIRE(zi_gemm_skinny_supported(M, N, K, ldx, ldw),
                "gemm_skinny: unsupported sizes M=%d N=%d K=%d (1 <= M <= 256, K and row strides multiples of 8)", M, N, K);
     ZI_REQUIRE(out_dt == ZI_F32 || out_dt == ZI_BF16, "gemm_skinny: unknown output dtype %d", out_dt);
-    ZI_REQUIRE(mode >= 0 && mode <= 2, "gemm_skinny: unknown mode %d", mode);
+    ZI_REQUIRE(mode >= 0 && mode <= 3, "gemm_skinny: unknown mode %d", mode);
+    ZI_REQUIRE(mode != SK_MODE_CLAMPED || (limit > 0.f && M <= SK_MID_MAX_ROWS_SWIGLU), "gemm_skinny: the clamped epilogue takes up to %d rows and a positive limit", SK_MID_MAX_ROWS_SWIGLU);
     ZI_REQUIRE(ldx >= K && ldw >= K, "gemm_skinny: leading dimension too small");
     ZI_REQUIRE(((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0, "gemm_skinny: x and w must be 16-byte aligned");
     int splits, per, waves;
@@ -121,15 +125,15 @@ extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, co
         ZI_REQUIRE(N % 16 == 0 && out_dt == ZI_BF16 && ldo >= N / 2,
                    "gemm_skinny: the SwiGLU epilogue needs N %% 16 == 0 and a bfloat16 out of N/2 columns");
     }
-    const zi_bf16* b = (kmode == SK_MODE_PLAIN || mode == SK_MODE_PARTIAL) ? (const zi_bf16*)bias : nullptr;
+    const zi_bf16* b = (kmode == SK_MODE_PLAIN || mode == SK_MODE_PARTIAL || mode == SK_MODE_CLAMPED) ? (const zi_bf16*)bias : nullptr;
     // four columns go out as one store when every row of the destination keeps them aligned
     int vec_out;
     if (kmode == SK_MODE_PARTIAL) vec_out = N % 4 == 0 && ((uintptr_t)dst % 16) == 0;
-    else if (kmode == SK_MODE_SWIGLU) vec_out = ldo % 4 == 0 && ((uintptr_t)dst % 8) == 0;
+    else if (kmode >= SK_MODE_SWIGLU) vec_out = ldo % 4 == 0 && ((uintptr_t)dst % 8) == 0;
     else vec_out = ldo % 4 == 0 && ((uintptr_t)dst % (out_dt == ZI_F32 ? 16 : 8)) == 0;
     const int of32 = out_dt == ZI_F32;
     const int rc = (rows32 ? zi_gemm_rows32_launch : zi_gemm_mid_launch)(dst, of32, kmode, (const zi_bf16*)x, (const zi_bf16*)w, b,
-                                                                         M, N, K, ldx, ldw, ldo, vec_out, stream);
+                                                                         M, N, K, ldx, ldw, ldo, vec_out, limit, stream);
     if (rc) return rc;
     if (mode == SK_MODE_PLAIN && splits > 1) {
         const int64_t total = (int64_t)M * N;
@@ -137,6 +141,13 @@ extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, co
                                                                                   (const zi_bf16*)bias, M, N, ldo, splits);
     }
     return zi_check_launch("gemm_skinny");
+}
+
+extern "C" int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M,
+                              int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace,
+                              int64_t workspace_floats, hipStream_t stream) {
+    ZI_REQUIRE(mode >= 0 && mode <= 2, "gemm_skinny: unknown mode %d", mode);
+    return zi_gemm_skinny_act(out, out_dt, mode, x, w, bias, M, N, K, ldx, ldw, ldo, workspace, workspace_floats, 0.f, stream);
 }
 
 // out[m,n] = sum_s sums[s,m,n] + bias[n] for float32 sums [splits][M][N], added in rising order.

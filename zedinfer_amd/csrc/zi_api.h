@@ -69,6 +69,12 @@ int zi_gemm_lt(void* out, int out_dt, const void* x, const void* weight, const v
 int zi_gemm_skinny(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M, int N, int
     K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace, int64_t workspace_floats, hipStream_t stream);
 // gemm_skinny.hip
+int zi_gemm_skinny_act(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M, int N, int
+    K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace, int64_t workspace_floats, float limit, hipStream_t stream);
+// elementwise.hip
+int zi_clamped_glu_il8(void* out, int64_t ldo, const void* gu, int64_t ld, int n, int inter, float limit, float alpha,
+    hipStream_t stream);
+// gemm_skinny.hip
 int zi_reduce_splits(void* out, int out_dt, const float* sums, const void* bias, int M, int N, int64_t ldo, int
     splits, hipStream_t stream);
 // norm.hip
@@ -170,6 +176,14 @@ int zi_attention_prefill_sink(void* out, const void* q, int dt, int num_tiles, i
 int zi_attention_decode_project_sink(float* sums, const float* workspace, int64_t workspace_floats, int n, const int32_t*
     tok_pos, int window, int max_chunks, const void* w, int dt, int64_t ldw, int N, int nh, int d, const float* sinks,
     hipStream_t stream);
+// attention_decode.hip
+int zi_attention_decode_project_gated(float* sums, const float* workspace, int64_t workspace_floats, int n, const int32_t*
+    tok_pos, int window, int max_chunks, const void* w, int dt, int64_t ldw, int N, int nh, int d, const float* sinks, const
+    float* gate, int64_t ld_gate, int gate_splits, int64_t gate_stride, hipStream_t stream);
+// attention_decode.hip
+int zi_attention_decode_merge_gated(void* y, int64_t ldy, const float* workspace, int64_t workspace_floats, int n, const
+    int32_t* tok_pos, int window, int max_chunks, int nh, int d, int vd, const float* sinks, const float* gate, int64_t
+    ld_gate, int gate_splits, int64_t gate_stride, hipStream_t stream);
 // layer_norm.hip
 int zi_layer_norm(void* out, int out_dt, int64_t ldo, float* resid, const void* x, int x_dt, int splits, int64_t
     split_stride, int64_t ldx, const void* w, const void* b, int w_dt, int n, int hidden, float eps, hipStream_t
@@ -417,6 +431,10 @@ int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int ro
     X(zi_moe_weighted_glu) \
     X(zi_moe_sum_shared) \
     X(zi_embedding_scaled) \
+    X(zi_attention_decode_project_gated) \
+    X(zi_attention_decode_merge_gated) \
+    X(zi_gemm_skinny_act) \
+    X(zi_clamped_glu_il8) \
     X(zi_stream_scale) \
     X(zi_channel_inputs) \
     X(zi_input_conv) \

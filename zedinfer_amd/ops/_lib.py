@@ -57,6 +57,8 @@ _PROTOTYPES = {
     "zi_attention_prefill_chunk_keys": [],
     "zi_gemm_generic": [P, I, P, I, P, I, P, I, I, I, I, L, L, L, P],
     "zi_gemm_skinny": [P, I, I, P, P, P, I, I, I, L, L, L, P, L, P],
+    "zi_gemm_skinny_act": [P, I, I, P, P, P, I, I, I, L, L, L, P, L, F, P],
+    "zi_clamped_glu_il8": [P, L, P, L, I, I, F, F, P],
     "zi_gemm_skinny_splits": [I, I, I],
     "zi_gemm_lt": [P, I, P, P, P, I, L, L, L, L, L, L, P, L, P],
     "zi_gemm_lt_tune": [P, I, P, P, P, I, L, L, L, L, L, L, P, L, I, I, P, P, P, P],
@@ -91,6 +93,8 @@ _PROTOTYPES = {
     "zi_attention_prefill_sink": [P, P, I, I, L, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, L, I, I, I,
                                   P, P],
     "zi_attention_decode_project_sink": [P, P, L, I, P, I, I, P, I, L, I, I, I, P, P],
+    "zi_attention_decode_project_gated": [P, P, L, I, P, I, I, P, I, L, I, I, I, P, P, L, I, L, P],
+    "zi_attention_decode_merge_gated": [P, L, P, L, I, P, I, I, I, I, I, P, P, L, I, L, P],
     "zi_layer_norm": [P, I, L, P, P, I, I, L, L, P, P, I, I, I, F, P],
     "zi_conv_qkv": [P, I, L, P, P, P, I, L, I, L, P, P, P, L, I, P, P, F, P, I, I, P, P, P, P, L, I, I, I, I, I, I, I, P, P, F, P],
     "zi_conv_tail": [P, L, P, I, L, I, L, P, P, P, P, P, I, I, I, P],

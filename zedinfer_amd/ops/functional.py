@@ -596,11 +596,13 @@ def attention_decode_project_splits(nh: int) -> int:
 
 def attention_decode_project(workspace: torch.Tensor, weight: torch.Tensor, tok_pos: torch.Tensor, nh: int, d: int,
                              max_keys: int, window: int = 0, out: Optional[torch.Tensor] = None,
-                             sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                             sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The output projection of decoded tokens straight from the chunks that ``attention_decode_fused(...,
     leave_chunks=True)`` left in ``workspace`` (same tokens, heads, ``max_keys`` and ``window``): float32
-    partial sums [splits, n, N] over groups of heads, to be added in rising order.  ``weight`` is [N, nh*d]."""
-    _gpu("attention_decode_project", workspace, weight, tok_pos, out)
+    partial sums [splits, n, N] over groups of heads, to be added in rising order.  ``weight`` is [N, nh*d].  ``gate``
+    (float32 [n, nh*d] or a stack [S, n, nh*d] of partial sums, rows aligned to 16 bytes): the merged heads are multiplied
+    by its sigmoid first."""
+    _gpu("attention_decode_project", workspace, weight, tok_pos, out, gate)
     n = tok_pos.numel()
     _i32(tok_pos, "attention_decode_project tok_pos", n)
     if not attention_decode_project_supported(weight, n, nh, d):
@@ -620,10 +622,46 @@ def attention_decode_project(workspace: torch.Tensor, weight: torch.Tensor, tok_
     max_chunks = int(_lib.load().zi_attention_decode_chunks(int(max_keys)))
     args = (_p(out), _p(workspace), workspace.numel(), n, _p(tok_pos), int(window), max_chunks, _p(weight),
             _code(weight, "attention_decode_project"), weight.stride(0), N, nh, d)
-    if sinks is not None:      # (float32 [nh]: exp(sinks[h]) counts once in the denominator of head h's merge)
+    if gate is not None:
+        ldg, gsplits, gstride = _gate_terms(gate, n, nh * d, "attention_decode_project")
+        _lib.call("zi_attention_decode_project_gated", *args, _p(_sinks(sinks, nh, weight, "attention_decode_project") if sinks is not None else None),
+                  _p(gate), ldg, gsplits, gstride, _stream())
+    elif sinks is not None:      # (float32 [nh]: exp(sinks[h]) counts once in the denominator of head h's merge)
         _lib.call("zi_attention_decode_project_sink", *args, _p(_sinks(sinks, nh, weight, "attention_decode_project")), _stream())
     else:
         _lib.call("zi_attention_decode_project", *args, _stream())
+    return out
+
+
+def _gate_terms(gate: torch.Tensor, n: int, width: int, what: str):
+    """(row stride, splits, stride between splits) of a gate [n, width] or a stack [S, n, width] of partial sums of it."""
+    if gate.dtype != torch.float32 or gate.dim() not in (2, 3) or tuple(gate.shape[-2:]) != (n, width) or gate.stride(-1) != 1:
+        raise ValueError(f"{what}: the gate must be float32 [{n}, {width}] or a stack of such rows")
+    return int(gate.stride(-2)), (int(gate.shape[0]) if gate.dim() == 3 else 1), (int(gate.stride(0)) if gate.dim() == 3 else 0)
+
+
+def attention_decode_merge_gated(workspace: torch.Tensor, tok_pos: torch.Tensor, nh: int, d: int, head: int, max_keys: int,
+                                 gate: torch.Tensor, out: torch.Tensor, window: int = 0,
+                                 sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The chunks that ``attention_decode(..., leave_chunks=True)`` left in ``workspace`` (same tokens, heads, ``max_keys``
+    and ``window``), merged, the first ``head`` values of every head of ``d`` times sigmoid(gate): out bfloat16
+    [n, nh*head]; gate float32 [n, nh*head] or a stack [S, n, nh*head] of partial sums (column slices are fine)."""
+    _gpu("attention_decode_merge_gated", workspace, tok_pos, gate, out)
+    n = tok_pos.numel()
+    _i32(tok_pos, "attention_decode_merge_gated tok_pos", n)
+    ldy, width = _rows(out, "attention_decode_merge_gated out")
+    if tuple(out.shape) != (n, nh * head) or out.dtype != torch.bfloat16 or head > d:
+        raise ValueError(f"attention_decode_merge_gated: out must be bfloat16 [{n}, {nh * head}] with heads within {d}")
+    ldg, splits, stride = _gate_terms(gate, n, nh * head, "attention_decode_merge_gated")
+    need = attention_decode_workspace(n, nh, d)
+    if workspace.dtype != torch.float32 or workspace.numel() < need or not workspace.is_contiguous():
+        raise ValueError(f"attention_decode_merge_gated: workspace must be a contiguous float32 buffer of {need} entries")
+    if window > 0:
+        max_keys = min(max_keys, window)
+    _lib.call("zi_attention_decode_merge_gated", _p(out), ldy, _p(workspace), workspace.numel(), n, _p(tok_pos), int(window),
+              int(_lib.load().zi_attention_decode_chunks(int(max_keys))), nh, d, head,
+              _p(_sinks(sinks, nh, out, "attention_decode_merge_gated") if sinks is not None else None), _p(gate), ldg, splits,
+              stride, _stream())
     return out
 
 
@@ -1047,6 +1085,28 @@ def linear_swiglu(x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Ten
         raise ValueError(f"linear_swiglu: out must be bfloat16 [{M}, {N // 2}]")
     _lib.call("zi_gemm_skinny", _p(out), BF16, 2, _p(x), _p(weight), c_void_p(0), M, N, K, x.stride(0), weight.stride(0),
               ldo, c_void_p(0), 0, _stream())
+    return out
+
+
+def linear_clamped_glu(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], limit: float,
+                       out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit) of x . weight^T + bias in one
+    kernel, for a weight [2I, K] (and a bias [2I], bfloat16) whose rows alternate between gate and up in blocks of 8; out
+    [M, I] bfloat16.  Taken where ``linear_swiglu_supported``."""
+    _gpu("linear_clamped_glu", x, weight, bias, out)
+    if not linear_swiglu_supported(x, weight) or x.shape[0] > FEW_ROWS:
+        raise ValueError("linear_clamped_glu: needs an unsplit bfloat16 few-rows product with 2I a multiple of 16")
+    M, K = x.shape
+    N = weight.shape[0]
+    if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != N or not bias.is_contiguous()):
+        raise ValueError(f"linear_clamped_glu: the bias must be a contiguous bfloat16 [{N}] tensor")
+    if out is None:
+        out = torch.empty((M, N // 2), dtype=torch.bfloat16, device=x.device)
+    ldo, wo = _rows(out, "linear_clamped_glu out")
+    if tuple(out.shape) != (M, N // 2) or out.dtype != torch.bfloat16 or not limit > 0:
+        raise ValueError(f"linear_clamped_glu: out must be bfloat16 [{M}, {N // 2}], the limit positive")
+    _lib.call("zi_gemm_skinny_act", _p(out), BF16, 3, _p(x), _p(weight), _p(bias), M, N, K, x.stride(0), weight.stride(0),
+              ldo, c_void_p(0), 0, float(limit), _stream())
     return out
 
 

@@ -198,6 +198,17 @@ def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, out: torch.T
     return out
 
 
+def clamped_glu_il8(gate_up: torch.Tensor, limit: float, out: torch.Tensor, alpha: float = 1.702) -> torch.Tensor:
+    """``clamped_glu`` over bfloat16 rows [n, 2I] whose gate and up columns alternate in blocks of 8."""
+    _gpu("clamped_glu_il8", gate_up, out)
+    ld, width = _rows(gate_up, "clamped_glu_il8 gate_up")
+    ldo, I = _rows(out, "clamped_glu_il8 out")
+    if gate_up.dtype != torch.bfloat16 or out.dtype != torch.bfloat16 or width != 2 * I or out.shape[0] != gate_up.shape[0]:
+        raise ValueError("clamped_glu_il8: bfloat16 rows [n, 2I] and out [n, I] are needed")
+    _lib.call("zi_clamped_glu_il8", _p(out), ldo, _p(gate_up), ld, gate_up.shape[0], I, float(limit), float(alpha), _stream())
+    return out
+
+
 def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
     """In place: x <- cap * tanh(x / cap) for a contiguous float32 tensor."""
     _gpu("softcap", x)

@@ -370,8 +370,10 @@ class _ClampedGated:
 class ClampedMLP(FeedForward):
     """A dense feed-forward of the clamped gated form, down(g sigmoid(1.702 g) (u + 1)) with g = min(gate x, limit) and
     u = clamp(up x, -limit, limit); with ``bias`` all three projections have one (``gate_bias``, ``up_bias``,
-    ``down_bias``).  The gate/up product leaves float32 results (partial sums for few rows), the activation's kernel
-    adds the biases; the down product of few rows leaves partial sums whose first holds its bias.
+    ``down_bias``).  In bfloat16 (and with I a multiple of 8) gate and up rows alternate in blocks of 8, so that the
+    few-rows product applies biases and activation in its epilogue; for many rows the library's product adds the biases
+    and leaves bfloat16 results.  Otherwise the product leaves float32 results (partial sums for few rows) and the
+    activation's kernel adds the biases.  The down product of few rows leaves partial sums whose first holds its bias.
     params: hidden_size, intermediate_size, limit, bias (False)."""
 
     graph_safe = True
@@ -389,22 +391,44 @@ class ClampedMLP(FeedForward):
         super().__init__(spec, weights, rt)
         p = spec.params
         self.hidden, self.inter = int(p["hidden_size"]), int(p["intermediate_size"])
-        self.half = _ClampedGated(weights["gate"], weights["up"], weights["down"], float(p["limit"]),
-                                  weights.get("gate_bias"), weights.get("up_bias"))
+        self.limit, gate, up = float(p["limit"]), weights["gate"], weights["up"]
+        self.interleaved = self.half = None
+        bf = torch.bfloat16
+        biased = bool(p.get("bias", False))
+        if rt.dtype == bf and gate.dtype == bf and up.dtype == bf and self.inter % GATE_UP_BLOCK == 0 \
+                and (not biased or (weights["gate_bias"].dtype == bf and weights["up_bias"].dtype == bf)):
+            self.interleaved = interleave_rows(gate, up, GATE_UP_BLOCK)
+            self.gate_up_bias = None
+            if biased:
+                self.gate_up_bias = interleave_rows(weights["gate_bias"].view(-1, 1), weights["up_bias"].view(-1, 1), GATE_UP_BLOCK).view(-1)
+        else:
+            self.half = _ClampedGated(gate, up, weights["down"], self.limit, weights.get("gate_bias"), weights.get("up_bias"))
         self.down = weights["down"]
-        self.down_bias = weights["down_bias"].to(self.down.dtype).contiguous() if p.get("bias", False) else None
+        self.down_bias = weights["down_bias"].to(self.down.dtype).contiguous() if biased else None
 
     def step_rows(self, rows: int, kind: str) -> int:
         return ProductRows.step_rows(rows, kind)
 
     def tune(self, num_tokens: int) -> None:
         n = int(num_tokens)
-        self.rt.tune_linear(self.rt.buffer("norm_out", (n, self.hidden)), self.half.gate_up, out_dtype=torch.float32)
+        x = self.rt.buffer("norm_out", (n, self.hidden))
+        if self.interleaved is not None:
+            self.rt.tune_linear(x, self.interleaved, self.gate_up_bias)
+        else:
+            self.rt.tune_linear(x, self.half.gate_up, out_dtype=torch.float32)
         self.rt.tune_linear(self.rt.buffer("ffn_act", (n, self.inter)), self.down, self.down_bias)
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         n, rt = x.shape[0], self.rt
-        act = self.half.forward(rt, x, "ffn")
+        if self.interleaved is None:
+            act = self.half.forward(rt, x, "ffn")
+        else:
+            act = rt.buffer("ffn_act", (n, self.inter))
+            if n <= ops.FEW_ROWS and ops.linear_swiglu_supported(x, self.interleaved):
+                ops.linear_clamped_glu(x, self.interleaved, self.gate_up_bias, self.limit, out=act)
+            else:
+                gu = ops.linear(x, self.interleaved, self.gate_up_bias, out=rt.buffer("ffn_gate_up", (n, 2 * self.inter)))
+                ops.clamped_glu_il8(gu, self.limit, out=act)
         if ops.linear_sums_supported(act, self.down):
             S = ops.linear_splits(n, self.hidden, self.inter)
             return ops.linear_sums(act, self.down, bias=self.down_bias,

@@ -542,7 +542,9 @@ class ConvAttention(Attention):
         if not single:
             ops.conv_tail(memory.state, proj, self.bias, batch.entry_start, batch.entry_len, batch.entry_slot, self.taps,
                           slots=view.slots)
-        out = self.decode_and_project(q, batch, view, memory) if single and not self.gated else None
+        out = None
+        if single:
+            out = self.decode_and_gate(q, gate, batch, view, memory) if self.gated else self.decode_and_project(q, batch, view, memory)
         if out is not None:
             return out
         att = rt.buffer("attn_out", (n, self.qd))
@@ -566,6 +568,30 @@ class ConvAttention(Attention):
         if kept is None or tuple(kept.shape) != shape:
             raise ValueError("conv_attention: no earlier layer kept values of this layer's sizes")
         return {"mix_values": kept, "mix": self.mix}
+
+    def decode_and_gate(self, q, gate, batch, view, memory: LayerMemory) -> Optional[torch.Tensor]:
+        """A pure decode step of a gated mixer: the attention kernel leaves every token's chunks of keys unmerged; for
+        few tokens the output projection merges and gates them as it loads its operand, else the merge's kernel gates.
+        None: the shape is not taken, nothing was done."""
+        n = q.shape[0]
+        kc, vc = memory.tensors["k"], memory.tensors["v"]
+        if (self.log_distance is None and self.sinks is None) or not ops.attention_decode_supported(q.dtype, self.nh, self.nkv, self.d,
+                                                                                                   kc.shape[2]):
+            return None
+        max_keys = batch.plans[self.plan_key].sizes["max_short_keys"]
+        extras = {} if self.log_distance is None else {"log_distance": self.log_distance}
+        ws = self.rt.buffer("attn_split", (ops.attention_decode_workspace(n, self.nh, self.d),), torch.float32)
+        ops.attention_decode(q, kc, vc, batch.tok_seq, batch.positions, view.block_tables, self.nh, self.nkv, self.d,
+                             self.scale, max_keys, self.window, workspace=ws, sinks=self.sinks, leave_chunks=True, **extras)
+        if (n <= self.FUSED_DECODE_MAX_TOKENS and self.d == self.vdim and gate.stride(-2) % 4 == 0 and self.gate_at % 4 == 0
+                and self.o.numel() * self.o.element_size() <= self.PROJECT_FROM_CHUNKS_MAX_BYTES
+                and ops.attention_decode_project_supported(self.o, n, self.nh, self.d)):
+            out = self.rt.buffer("attn_proj_heads", (ops.attention_decode_project_splits(self.nh), n, self.hidden), torch.float32)
+            return ops.attention_decode_project(ws, self.o, batch.positions, self.nh, self.d, max_keys, self.window, out=out,
+                                                sinks=self.sinks, gate=gate)
+        y = ops.attention_decode_merge_gated(ws, batch.positions, self.nh, self.d, self.vdim, max_keys, gate, window=self.window,
+                                             sinks=self.sinks, out=self.rt.buffer("attn_gated", (n, self.nh * self.vdim)))
+        return self.project(y, n)
 
     def decode_and_project(self, q, batch, view, memory: LayerMemory) -> Optional[torch.Tensor]:
         """A pure decode step of few tokens: the attention kernel leaves every token's chunks of keys unmerged and
