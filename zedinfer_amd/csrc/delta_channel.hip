@@ -21,9 +21,12 @@ union dc_pack {
     dc_bf16x8_t b;
 };
 
-__device__ __forceinline__ float dc_decay(float z, float a) {      // a = exp(a_log)
-    // softplus(z) = max(z, 0) + log1p(exp(-|z|)), exact for large |z| too
-    return expf(-a * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
+__device__ __forceinline__ float dc_decay(float z, float a) {      // exp(-a softplus(z)), a = exp(a_log)
+    // softplus(z) = max(z, 0) + ln(1 + e), e = exp(-|z|), in units of ln 2; where 1 + e would drop digits of e the
+    // series' first two terms are exact to 32 bits
+    const float e = __builtin_amdgcn_exp2f(-fabsf(z) * 1.4426950408889634f);
+    const float l = e < 0x1p-11f ? e * fmaf(-0.5f, e, 1.f) * 1.4426950408889634f : __builtin_amdgcn_logf(1.f + e);
+    return __builtin_amdgcn_exp2f(-a * fmaf(fmaxf(z, 0.f), 1.4426950408889634f, l));
 }
 
 // ---- what the recurrence reads -----------------------------------------------------------------------------------------
