@@ -2,7 +2,7 @@
 //
 //   for every token:  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
-// q and k as in delta.hip (zi_delta_prepare makes them, v and beta), g [heads][dim] in (0, 1) per token.
+// q and k unit vectors per head (q times dim^-1/2), beta in (0, 1) per head, g [heads][dim] in (0, 1), per token.
 //
 //   zi_channel_inputs    from the stacked projection: convolution, SiLU, unit vectors, beta, and the convolution's tail
 //   zi_lowrank_gates     two low-rank projections of float32 rows at once: the decays
