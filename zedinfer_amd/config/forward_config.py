@@ -38,6 +38,8 @@ class LayerSpec:
     mixer: PartSpec
     feed_forward: PartSpec
     norms: Dict[str, PartSpec]      # arrangement-specific names, e.g. "input", "post_mixer"
+    # how each sublayer reads the residual streams and writes its result back, for arrangements that name any
+    connections: Dict[str, PartSpec] = field(default_factory=dict)
 
 
 @dataclass(frozen=True)
@@ -72,6 +74,9 @@ class ModelForwardConfig:
     final_norm: PartSpec
     lm_head: PartSpec
     tie_word_embeddings: bool = False
+    # residual streams a token (all equal to the embedding's output at the start, added up before the final norm); 0: the one
+    # stream that blocks change in place.  With streams every block must be one that has connections.
+    streams: int = 0
     eos_token_ids: Tuple[int, ...] = ()
     max_position_embeddings: int = 0
     # What the architecture wants to say about itself, for whoever inspects a model (the reference keeps family
@@ -83,6 +88,10 @@ class ModelForwardConfig:
 
     def validate(self) -> None:
         n = len(self.layers)
+        if self.streams < 0 or any(bool(layer.connections) != (self.streams > 0) for layer in self.layers):
+            raise ValueError("layers name connections exactly where the model has residual streams for them")
+        if self.streams and any(st.enter is not None for st in self.schedule):
+            raise ValueError("a stream step between layers changes the one residual stream; this model has several")
         writers: Dict[int, int] = {}
         for i, st in enumerate(self.schedule):
             if not (0 <= st.layer < n):

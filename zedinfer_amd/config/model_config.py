@@ -693,3 +693,104 @@ class KefisunConfig(ModelConfig):
         if self.eos_token_ids:
             d["eos_token_id"] = list(self.eos_token_ids)
         return d
+
+
+@dataclass(frozen=True)
+class FovenexConfig(ModelConfig):
+    """The Fovenex design's config.json: ``width``, ``vocab``, ``norm.eps``, ``streams`` (residual streams a token),
+    ``residual_mult`` (what every sublayer's result is multiplied by) and a list ``layers`` whose entries each name a mixer by
+    ``type`` ("attention": heads that are differences of two softmax maps; "latent_attention": windowed attention over latents
+    that a later layer may read, ``kv_from``) with its sizes and constants under ``mixer``, and a feed-forward under ``mlp``
+    (``kind`` "dense" with ``ff``; or null for none).  Every size and constant of a model is read from here (``q_rank`` is the
+    tensor's own unless it is given); the shared keys of ``ModelConfig`` that the format does not have keep their neutral
+    values."""
+
+    layers: Tuple[Any, ...] = ()
+    norm_eps: float = 1e-6
+    streams: int = 1
+    residual_mult: float = 1.0
+
+    MIXER_KEYS = {"attention": ("heads", "kv_heads", "dim", "vdim", "scale", "diff"),
+                  "latent_attention": ("heads", "dim", "rot_dim", "vdim", "kv_rank", "scale", "rot")}
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "FovenexConfig":
+        missing = [k for k in ("width", "vocab", "layers", "norm", "streams") if k not in d]
+        if missing:
+            raise ConfigError("config.json lacks required key(s): " + ", ".join(missing))
+        if not isinstance(d["layers"], (list, tuple)) or not d["layers"]:
+            raise ConfigError("config.json: 'layers' must be a non-empty list")
+        if not isinstance(d["norm"], Mapping) or "eps" not in d["norm"]:
+            raise ConfigError("config.json: 'norm' must give 'eps'")
+        eos = d.get("eos_token_id")
+        cfg = cls(architectures=(str(d.get("architecture", "Fovenex")),), model_type="fovenex",
+                  torch_dtype=str(d.get("torch_dtype") or "bfloat16"), hidden_size=_as_int(d, "width"),
+                  vocab_size=_as_int(d, "vocab"), num_hidden_layers=len(d["layers"]),
+                  eos_token_ids=() if eos is None else tuple(int(e) for e in (eos if isinstance(eos, (list, tuple)) else [eos])),
+                  layers=tuple(json.loads(json.dumps(layer)) for layer in d["layers"]), norm_eps=float(d["norm"]["eps"]),
+                  streams=_as_int(d, "streams"), residual_mult=float(d.get("residual_mult", 1.0)))
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.hidden_size <= 0 or self.vocab_size <= 0:
+            raise ConfigError("config.json: 'width' and 'vocab' must be positive")
+        if not (self.norm_eps > 0):
+            raise ConfigError(f"config.json: norm.eps must be positive, got {self.norm_eps}")
+        if not (1 <= self.streams <= 16):
+            raise ConfigError(f"config.json: streams must lie in 1..16, got {self.streams}")
+        for i, layer in enumerate(self.layers):
+            kind = layer.get("type") if isinstance(layer, Mapping) else None
+            if kind not in self.MIXER_KEYS:
+                raise ConfigError(f"config.json: layer {i} has type {kind!r}; known: {', '.join(sorted(self.MIXER_KEYS))}")
+            m = layer.get("mixer")
+            lacking = [k for k in self.MIXER_KEYS[kind] if not isinstance(m, Mapping) or k not in m]
+            if lacking:
+                raise ConfigError(f"config.json: layer {i} ({kind}) lacks mixer key(s): " + ", ".join(lacking))
+            if any(int(m[k]) <= 0 for k in self.MIXER_KEYS[kind] if k not in ("scale", "diff", "rot")) or not float(m["scale"]) > 0:
+                raise ConfigError(f"config.json: layer {i} ({kind}): sizes and the scale must be positive")
+            rot = m.get("rot")
+            if rot is not None:
+                if not isinstance(rot, Mapping) or "base" not in rot or "dims" not in rot or int(rot["dims"]) % 2 \
+                        or int(rot["dims"]) <= 0 or not float(rot["base"]) > 1:
+                    raise ConfigError(f"config.json: layer {i}: rot needs a base above 1 and an even, positive dims")
+                sc = rot.get("scaling")
+                if sc is not None and (not isinstance(sc, Mapping) or any(k not in sc for k in ("factor", "original", "fast", "slow"))):
+                    raise ConfigError(f"config.json: layer {i}: rot.scaling needs factor, original, fast and slow")
+            if m.get("mask") is not None and not int(m["mask"].get("size", 0)) > 0:
+                raise ConfigError(f"config.json: layer {i}: mask.size must be positive")
+            if kind == "attention":
+                if int(m["heads"]) % int(m["kv_heads"]):
+                    raise ConfigError(f"config.json: layer {i}: heads must be a multiple of kv_heads")
+                if rot is not None and int(rot["dims"]) > int(m["dim"]):
+                    raise ConfigError(f"config.json: layer {i}: rot.dims must lie within dim")
+            else:
+                if rot is None or int(rot["dims"]) != int(m["rot_dim"]):
+                    raise ConfigError(f"config.json: layer {i}: rot.dims must be rot_dim")
+                if m.get("q_rank") is not None and int(m["q_rank"]) <= 0:
+                    raise ConfigError(f"config.json: layer {i}: q_rank must be positive")
+                src = m.get("kv_from")
+                if src is not None:
+                    ok = isinstance(src, int) and not isinstance(src, bool) and 0 <= src < i \
+                        and self.layers[src].get("type") == "latent_attention" and self.layers[src]["mixer"].get("kv_from") is None
+                    if ok:
+                        o = self.layers[src]["mixer"]
+                        ok = (o["kv_rank"], o["rot_dim"], o["rot"]) == (m["kv_rank"], m["rot_dim"], m["rot"])
+                    if not ok:
+                        raise ConfigError(f"config.json: layer {i}: kv_from must name an earlier latent_attention layer with "
+                                          "a projection of its own and the same kv_rank, rot_dim and rot")
+            mlp = layer.get("mlp")
+            if mlp is None:
+                continue
+            if mlp.get("kind") != "dense":
+                raise ConfigError(f"config.json: layer {i}: mlp.kind {mlp.get('kind')!r} is not 'dense'")
+            if not int(mlp.get("ff", 0)) > 0:
+                raise ConfigError(f"config.json: layer {i}: a dense mlp needs a positive ff")
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"architecture": self.architectures[0] if self.architectures else "Fovenex",
+             "layers": json.loads(json.dumps(list(self.layers))), "norm": {"eps": self.norm_eps},
+             "residual_mult": self.residual_mult, "streams": self.streams, "vocab": self.vocab_size, "width": self.hidden_size}
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids)
+        return d

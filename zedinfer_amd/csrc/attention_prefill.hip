@@ -472,7 +472,9 @@ __device__ __attribute__((aligned(16))) const unsigned pf_zero16[4] = {0u, 0u, 0
 // beside the other's softmax and loads; a tile's walk is one wavefront's per query group, so it takes longer:
 // for launches with many tiles).
 // LOGB: slope * ln(1 + rate * distance) is taken off every score, two numbers a head (ZiScoreExtras).
-template <int D, int QW, int KH, bool LOGB>
+// MAPS: several softmax maps over the same values: a key row holds MAPS keys of D / MAPS values side by side, head h
+// reads the (h mod MAPS)-th of them, and only that part of its query row (the rest of the row is not read).
+template <int D, int QW, int KH, bool LOGB, int MAPS>
 __global__ void __launch_bounds__(4 * KH * ZI_WAVE, KH == 1 ? 2 : 1)
 attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf16* __restrict__ q, int64_t ldq,
                              const zi_bf16* __restrict__ kcache, const zi_bf16* __restrict__ vcache,
@@ -487,8 +489,10 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
     static_assert(QW == 1 || QW == 2, "16 or 32 queries a wavefront");
     constexpr int BM = PF_BM * QW;                   // queries of a tile
     constexpr int QR = 16 * QW;                      // queries of a wavefront
-    constexpr int DK = D / 32, DT = D / 16;
-    constexpr int KC = D / 8;                        // 16-byte pieces of a key row
+    static_assert((D / MAPS) % 32 == 0, "a map's key is whole k-steps");
+    constexpr int DQ = D / MAPS;                     // values of a key that a head multiplies
+    constexpr int DK = DQ / 32, DT = D / 16;
+    constexpr int KC = DQ / 8;                       // 16-byte pieces of such a key
     static_assert(KH == 1 || KH == 2, "one or two wavefronts a query group");
     constexpr int WAVES = 4 * KH;
     constexpr int BS = PF_BN * KH;                   // keys of a block
@@ -507,7 +511,7 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
     __shared__ int32_t bt_lds[ZI_PF_CHUNK_LONG / 8 + 8];     // the pages of this workgroup's keys (page size >= 8)
 
     const int tile = blockIdx.x / nh, h = blockIdx.x % nh;
-    const int g = h / (nh / nkv);
+    const int g = h / (nh / nkv), map_off = MAPS > 1 ? (h % MAPS) * DQ : 0;
     const int e = tile_entry[tile], off = tile_off[tile];
     const int start = entry_start[e], len = entry_len[e], past = entry_past[e];
     const int count = (len - off < BM) ? len - off : BM;
@@ -540,7 +544,7 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
     pf_bf16x8_t qop[QW][DK];
 #pragma unroll
     for (int u = 0; u < QW; ++u) {
-        const zi_bf16* qr = q + (int64_t)(start + off + (qvalid[u] ? row[u] : count - 1)) * ldq + (int64_t)h * D + j * 8;
+        const zi_bf16* qr = q + (int64_t)(start + off + (qvalid[u] ? row[u] : count - 1)) * ldq + (int64_t)h * D + map_off + j * 8;
 #pragma unroll
         for (int dk = 0; dk < DK; ++dk) {
             pf_pack p;
@@ -581,7 +585,7 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
         v_dim[i] = L / VC;
         v_key[i] = ((L % VC) ^ ((v_dim[i] / VSW) & (VC - 1))) * 8;
     }
-    const zi_bf16* kbase = kcache + (int64_t)g * ps * D;
+    const zi_bf16* kbase = kcache + (int64_t)g * ps * D + map_off;
     const zi_bf16* vbase = vcache + (int64_t)g * D * ps;
     const int64_t page_stride = (int64_t)nkv * ps * D;
     const int khi8 = khi & ~7;
@@ -750,9 +754,10 @@ attention_prefill_dma_kernel(zi_bf16* __restrict__ out, int64_t ldo, const zi_bf
     if constexpr (KH > 1) {
         // the two wavefronts of a query group merge their (maximum, sum, output) through LDS; nobody reads
         // the tiles any more
-        float* mo = reinterpret_cast<float*>(k_ab);                  // [qs][QW][DT][64][4]: within the two key tiles
-        float* ml = reinterpret_cast<float*>(v_ab);                  // [qs][QW][64][2]
-        static_assert(sizeof(float) * 4 * QW * DT * ZI_WAVE * 4 <= sizeof(uint4) * 2 * KCH, "the key tiles hold the merge");
+        // (the tiles of keys are the smaller ones where a key row holds several maps)
+        float* mo = reinterpret_cast<float*>(MAPS == 1 ? k_ab : v_ab);      // [qs][QW][DT][64][4]: within two tiles
+        float* ml = reinterpret_cast<float*>(MAPS == 1 ? v_ab : k_ab);      // [qs][QW][64][2]
+        static_assert(sizeof(float) * 4 * QW * DT * ZI_WAVE * 4 <= sizeof(uint4) * 2 * (MAPS == 1 ? KCH : VCH), "the tiles hold the merge");
         if (kh > 0) {
 #pragma unroll
             for (int u = 0; u < QW; ++u) {
@@ -915,29 +920,27 @@ extern "C" int zi_attention_prefill_cuts(int max_keys, int window, int groups, i
     return (max_keys + chunk - 1) / chunk;
 }
 
-// Tile i covers the queries [tile_off[i], tile_off[i] + tile) of entry tile_entry[i] (fewer at the
-// entry's end; `tile` is 64, or 128 for head sizes 64 and 128); entry e brings entry_len[e] tokens that start at row entry_start[e] of q and at
-// position entry_past[e] of its sequence, whose block table is row e of block_tables.  `alone` (head sizes 64 and
-// 128): workgroups of four wavefronts that walk blocks of 64 keys, two to a compute unit, for launches of many
-// tiles; a query's keys are then added in another order, so the result differs by rounding.
-// `sinks` (float32 [nh], or null): the softmax of head h also counts exp(sinks[h]) in its denominator, once, whatever
-// the number of cuts of a tile's keys.
-// `softcap`, `bias` (float32 [nh][bias_len]), `keep_first`, `slope` and `rate`: see ZiScoreExtras; with any of the first
-// three tiles hold 64 queries and the kernel that stages through registers runs for every head size.
-extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,
-                                           const void* kcache, const void* vcache, const int32_t* tile_entry,
-                                           const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
-                                           const int32_t* entry_past, const int32_t* block_tables, int max_pages,
-                                           int num_pages, int nh, int nkv, int d, int page_size, int window, float scale,
-                                           int rows, int max_chunks, float* workspace, int64_t workspace_floats, int tile,
-                                           int alone, int chunk_keys, const float* sinks, float softcap,
-                                           const float* bias, int bias_len, int keep_first, const float* slope,
-                                           const float* rate, hipStream_t stream) {
+// 1 when heads that hold `maps` keys in a row of d values (and one value) are taken by zi_attention_prefill_maps.
+extern "C" int zi_attention_prefill_maps_supported(int dt, int nh, int nkv, int d, int page_size, int maps) {
+    if (maps == 1) return zi_attention_prefill_supported(dt, nh, nkv, d, page_size);
+    return zi_attention_prefill_supported(dt, nh, nkv, d, page_size) && pf_variant >= 1 && (d == 64 || d == 128) && maps == 2 &&
+           nh % (maps * nkv) == 0;
+}
+
+// Checks and launches shared by the entry points below.
+static int pf_launch(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo, const void* kcache, const void* vcache,
+                     const int32_t* tile_entry, const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
+                     const int32_t* entry_past, const int32_t* block_tables, int max_pages, int num_pages, int nh, int nkv, int d,
+                     int page_size, int window, float scale, int rows, int max_chunks, float* workspace, int64_t workspace_floats,
+                     int tile, int alone, int chunk_keys, const float* sinks, float softcap, const float* bias, int bias_len,
+                     int keep_first, const float* slope, const float* rate, int maps, hipStream_t stream) {
     const bool tabled = softcap > 0.f || bias != nullptr || keep_first > 0, biased = tabled || slope != nullptr;
     ZI_REQUIRE((slope == nullptr) == (rate == nullptr), "attention_prefill: a slope and a rate, or neither");
     ZI_REQUIRE(softcap >= 0.f && keep_first >= 0 && (!bias || bias_len > 0), "attention_prefill: bad cap, bias or kept positions");
     ZI_REQUIRE(!tabled || (tile == PF_BM && !alone), "attention_prefill: capped or biased scores and kept positions take tiles of %d queries", PF_BM);
     const ZiScoreExtras ex = {softcap, bias, bias_len, keep_first, slope, rate};
+    ZI_REQUIRE(maps == 1 || (!biased && zi_attention_prefill_maps_supported(dt, nh, nkv, d, page_size, maps)),
+               "attention_prefill: %d maps a key row of %d values are not taken", maps, d);
     ZI_REQUIRE(tile == PF_BM || (tile == 2 * PF_BM && pf_variant >= 1 && (d == 64 || d == 128)),
                "attention_prefill: tiles of %d queries (64, or 128 for head sizes 64 and 128)", tile);
     ZI_REQUIRE(zi_attention_prefill_supported(dt, nh, nkv, d, page_size),
@@ -976,15 +979,16 @@ extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int
             (zi_bf16*)out, ldo, (const zi_bf16*)q, ldq, (const zi_bf16*)kcache, (const zi_bf16*)vcache, tile_entry, \
             tile_off, entry_start, entry_len, entry_past, block_tables, max_pages, num_pages, nh, nkv, ps_shift, \
             window, scale, po, pml, max_chunks, chunk_keys, sinks, ex)
-#define ZI_PF_DMA2(DD, QW, KH, LOGB)                                                                           \
-    attention_prefill_dma_kernel<DD, QW, KH, LOGB><<<grid, 4 * KH * ZI_WAVE, 0, stream>>>(                     \
+#define ZI_PF_DMA2(DD, QW, KH, LOGB, MAPS)                                                                     \
+    attention_prefill_dma_kernel<DD, QW, KH, LOGB, MAPS><<<grid, 4 * KH * ZI_WAVE, 0, stream>>>(                     \
         (zi_bf16*)out, ldo, (const zi_bf16*)q, ldq, (const zi_bf16*)kcache, (const zi_bf16*)vcache, tile_entry, \
         tile_off, entry_start, entry_len, entry_past, block_tables, max_pages, num_pages, nh, nkv, ps_shift,   \
         window, scale, po, pml, max_chunks, chunk_keys, sinks, slope, rate)
 #define ZI_PF_DMA(DD, QW, KH)                              \
     do {                                                   \
-        if (slope) ZI_PF_DMA2(DD, QW, KH, true);           \
-        else ZI_PF_DMA2(DD, QW, KH, false);                \
+        if (maps == 2) ZI_PF_DMA2(DD, QW, KH, false, 2);   \
+        else if (slope) ZI_PF_DMA2(DD, QW, KH, true, 1);   \
+        else ZI_PF_DMA2(DD, QW, KH, false, 1);             \
     } while (0)
     const bool dma = !tabled && pf_variant >= 1 && (d == 64 || d == 128);
     const bool wide = tile == 2 * PF_BM;
@@ -1016,6 +1020,43 @@ extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int
             (zi_bf16*)out, ldo, po, pml, tile_entry, tile_off, entry_start, entry_len, entry_past, nh, d, window, max_chunks,
             tile, chunk_keys, sinks);
     return zi_check_launch("attention_prefill");
+}
+
+// Tile i covers the queries [tile_off[i], tile_off[i] + tile) of entry tile_entry[i] (fewer at the
+// entry's end; `tile` is 64, or 128 for head sizes 64 and 128); entry e brings entry_len[e] tokens that start at row entry_start[e] of q and at
+// position entry_past[e] of its sequence, whose block table is row e of block_tables.  `alone` (head sizes 64 and
+// 128): workgroups of four wavefronts that walk blocks of 64 keys, two to a compute unit, for launches of many
+// tiles; a query's keys are then added in another order, so the result differs by rounding.
+// `sinks` (float32 [nh], or null): the softmax of head h also counts exp(sinks[h]) in its denominator, once, whatever
+// the number of cuts of a tile's keys.
+// `softcap`, `bias` (float32 [nh][bias_len]), `keep_first`, `slope` and `rate`: see ZiScoreExtras; with any of the first
+// three tiles hold 64 queries and the kernel that stages through registers runs for every head size.
+extern "C" int zi_attention_prefill_biased(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,
+                                           const void* kcache, const void* vcache, const int32_t* tile_entry,
+                                           const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
+                                           const int32_t* entry_past, const int32_t* block_tables, int max_pages,
+                                           int num_pages, int nh, int nkv, int d, int page_size, int window, float scale,
+                                           int rows, int max_chunks, float* workspace, int64_t workspace_floats, int tile,
+                                           int alone, int chunk_keys, const float* sinks, float softcap,
+                                           const float* bias, int bias_len, int keep_first, const float* slope,
+                                           const float* rate, hipStream_t stream) {
+    return pf_launch(out, q, dt, num_tiles, ldq, ldo, kcache, vcache, tile_entry, tile_off, entry_start, entry_len, entry_past,
+                     block_tables, max_pages, num_pages, nh, nkv, d, page_size, window, scale, rows, max_chunks, workspace,
+                     workspace_floats, tile, alone, chunk_keys, sinks, softcap, bias, bias_len, keep_first, slope, rate, 1, stream);
+}
+// The same for heads that are softmax maps over shared values: `maps` (2) keys of d / maps values lie side by side in a
+// key row, query head h (of nh = heads * maps, head-major) reads map h % maps and only that part of its query row.
+extern "C" int zi_attention_prefill_maps(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,
+                                         const void* kcache, const void* vcache, const int32_t* tile_entry,
+                                         const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
+                                         const int32_t* entry_past, const int32_t* block_tables, int max_pages,
+                                         int num_pages, int nh, int nkv, int d, int page_size, int window, float scale,
+                                         int rows, int max_chunks, float* workspace, int64_t workspace_floats, int tile,
+                                         int alone, int chunk_keys, int maps, hipStream_t stream) {
+    ZI_REQUIRE(maps >= 1, "attention_prefill: %d maps", maps);
+    return pf_launch(out, q, dt, num_tiles, ldq, ldo, kcache, vcache, tile_entry, tile_off, entry_start, entry_len, entry_past,
+                     block_tables, max_pages, num_pages, nh, nkv, d, page_size, window, scale, rows, max_chunks, workspace,
+                     workspace_floats, tile, alone, chunk_keys, nullptr, 0.f, nullptr, 0, 0, nullptr, nullptr, maps, stream);
 }
 
 extern "C" int zi_attention_prefill_sink(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo,

@@ -332,6 +332,78 @@ extern "C" int zi_relu_squared(void* out, int out_dt, int64_t ldo, const void* z
     return zi_check_launch("relu_squared");
 }
 
+// An activation alone: out = act(z), z [n][inter] with dense rows, possibly as `splits` float32 partial sums.  act: 0 SiLU,
+// 1 GELU in its tanh form, 2 GELU with the error function, 3 relu(z)^2.  The tanh form as z / (1 + e^(-2u)), u = sqrt(2 / pi)
+// (z + 0.044715 z^3), which is the same and loses nothing to cancellation; for bfloat16 results by the chip's exponential and
+// reciprocal.
+#define ZI_ACT_RELU2 3
+template <bool ROUGH>
+__device__ __forceinline__ float ew_activate(float z, int act) {
+    if (act == ZI_ACT_GELU_TANH) {
+        const float w = -2.f * 0.7978845608028654f * z * fmaf(0.044715f * z, z, 1.f);
+        return ROUGH ? z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(w * 1.4426950408889634f)) : z / (1.f + expf(w));
+    }
+    if (act == ZI_ACT_RELU2) {
+        const float p = fmaxf(z, 0.f);
+        return p * p;
+    }
+    return zi_activation(z, act);
+}
+
+template <typename T, typename TO>
+__global__ void activate_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ z, int64_t ldz, int splits,
+                                int64_t split_stride, int n, int inter, int act) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= (int64_t)n * inter) return;
+    const int64_t r = i / inter, c = i % inter;
+    float v = zi_load(z + r * ldz + c);
+    for (int s = 1; s < splits; ++s) v += zi_load(z + s * split_stride + r * ldz + c);
+    zi_store(out + r * ldo + c, ew_activate<sizeof(TO) == 2>(v, act));
+}
+
+// Four values a thread, the loads of up to SP terms in flight.
+template <typename T, typename TO, int SP>
+__global__ void __launch_bounds__(256)
+activate_vec_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ z, int64_t ldz, int splits, int64_t split_stride,
+                    int inter, int act) {
+    const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
+    const int64_t r = blockIdx.y;
+    if (c >= inter) return;
+    float4 t[SP];
+#pragma unroll
+    for (int s = 0; s < SP; ++s) t[s] = s < splits ? ew_load4(z + s * split_stride + r * ldz + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 v = t[0];
+#pragma unroll
+    for (int s = 1; s < SP; ++s) { v.x += t[s].x; v.y += t[s].y; v.z += t[s].z; v.w += t[s].w; }
+    constexpr bool rough = sizeof(TO) == 2;
+    ew_store4(out + r * ldo + c, make_float4(ew_activate<rough>(v.x, act), ew_activate<rough>(v.y, act), ew_activate<rough>(v.z, act),
+                                             ew_activate<rough>(v.w, act)));
+}
+
+extern "C" int zi_activate(void* out, int out_dt, int64_t ldo, const void* z, int dt, int64_t ldz, int splits,
+                           int64_t split_stride, int n, int inter, int act, hipStream_t stream) {
+    ZI_REQUIRE(n >= 0 && inter > 0 && ldo >= inter && ldz >= inter && splits >= 1 && (splits == 1 || dt == ZI_F32), "activate: bad sizes");
+    ZI_REQUIRE(act >= ZI_ACT_SILU && act <= ZI_ACT_RELU2, "activate: unknown activation %d", act);
+    if (n == 0) return 0;
+    if (splits <= 16 && n <= 65535 && split_stride % 4 == 0 && ew_rows4(z, ldz, inter) && ew_rows4(out, ldo, inter)) {
+        const dim3 grid((inter / 4 + 255) / 256, n);
+#define ZI_ACTV(SP) activate_vec_kernel<T, TO, SP><<<grid, 256, 0, stream>>>((TO*)out, ldo, (const T*)z, ldz, splits, split_stride, inter, act)
+        ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(out_dt, TO, {
+            if (splits == 1) ZI_ACTV(1);
+            else if (splits <= 4) ZI_ACTV(4);
+            else ZI_ACTV(16);
+        }));
+#undef ZI_ACTV
+        return zi_check_launch("activate");
+    }
+    const int64_t total = (int64_t)n * inter;
+    ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(out_dt, TO, {
+        activate_kernel<T, TO><<<(unsigned)((total + 255) / 256), 256, 0, stream>>>((TO*)out, ldo, (const T*)z, ldz, splits,
+                                                                                    split_stride, n, inter, act);
+    }));
+    return zi_check_launch("activate");
+}
+
 // The clamped gated activation: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1).
 // gate and up are [n][inter] with dense rows (column slices of one product are fine), possibly as `splits` float32
 // partial sums.

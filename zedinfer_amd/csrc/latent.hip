@@ -84,6 +84,73 @@ extern "C" int zi_latent_store(const float* dkv, int dt, int64_t ld, int n, cons
     return zi_check_launch("latent_store");
 }
 
+// ---- the inputs of a layer whose queries come through a latent, from one product -----------------------------
+// Rows of proj hold the query latent (q_rank values) from column 0 and, where the layer writes a cache, the token's latent and
+// key part (rank + rot values) from column dkv_at; any storage type, or `splits` float32 partial sums.  Workgroup (token, 0):
+// cq = rms_norm(query latent) * q_norm; workgroup (token, 1): what latent_store does.
+template <typename T, typename TP, typename TW>
+__global__ void __launch_bounds__(256)
+latent_inputs_kernel(T* __restrict__ cq, int64_t ld_cq, const TP* __restrict__ proj, int64_t ld, int splits, int64_t split_stride,
+                     const TW* __restrict__ q_norm, const TW* __restrict__ c_norm, float eps, int q_rank, int dkv_at,
+                     const float* __restrict__ table, const int32_t* __restrict__ slots, T* __restrict__ c_cache,
+                     T* __restrict__ kr_cache, int64_t cache_slots, int rank, int rot) {
+    extern __shared__ float xs[];      // [max(q_rank, rank + rot)]
+    __shared__ float red[16];
+    const int t = blockIdx.x;
+    const bool query = blockIdx.y == 0;
+    const int slot = query ? 0 : slots[t];
+    if (slot < 0 || slot >= cache_slots) return;      // a token without a place (padding): the whole workgroup leaves
+    const TP* row = proj + (int64_t)t * ld + (query ? 0 : dkv_at);
+    const int normed = query ? q_rank : rank, width = query ? q_rank : rank + rot;
+    float ss = 0.f;
+    for (int j = threadIdx.x; j < width; j += blockDim.x) {
+        float v = zi_load(row + j);
+        int s = 1;
+        for (; s + 3 < splits; s += 4) {      // four terms' loads in flight, added in their order
+            const float a = zi_load(row + s * split_stride + j), b = zi_load(row + (s + 1) * split_stride + j);
+            const float c = zi_load(row + (s + 2) * split_stride + j), d = zi_load(row + (s + 3) * split_stride + j);
+            v += a; v += b; v += c; v += d;
+        }
+        for (; s < splits; ++s) v += zi_load(row + s * split_stride + j);
+        xs[j] = v;
+        if (j < normed) ss += v * v;
+    }
+    ss = zi_block_sum(ss, red);      // (its barriers also make xs visible to all)
+    const float rstd = 1.0f / sqrtf(ss / (float)normed + eps);
+    if (query) {
+        for (int j = threadIdx.x; j < q_rank; j += blockDim.x) zi_store(cq + (int64_t)t * ld_cq + j, xs[j] * rstd * zi_load(q_norm + j));
+        return;
+    }
+    for (int j = threadIdx.x; j < rank; j += blockDim.x) zi_store(c_cache + (int64_t)slot * rank + j, xs[j] * rstd * zi_load(c_norm + j));
+    const float* tab = table + (int64_t)t * rot;      // [rot / 2][2]
+    for (int i = threadIdx.x; i < rot / 2; i += blockDim.x) {
+        const float u = xs[rank + 2 * i], v = xs[rank + 2 * i + 1], c = tab[2 * i], s = tab[2 * i + 1];
+        zi_store(kr_cache + (int64_t)slot * rot + 2 * i, u * c - v * s);
+        zi_store(kr_cache + (int64_t)slot * rot + 2 * i + 1, v * c + u * s);
+    }
+}
+
+// c_cache null: the query latents alone.
+extern "C" int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* proj, int p_dt, int64_t ld, int splits,
+                                int64_t split_stride, int n, const void* q_norm, const void* c_norm, int w_dt, float eps,
+                                int q_rank, int dkv_at, const float* table, const int32_t* slots, void* c_cache,
+                                void* kr_cache, int64_t cache_slots, int rank, int rot, hipStream_t stream) {
+    const int width = c_cache ? rank + rot : 0, most = q_rank > width ? q_rank : width;
+    ZI_REQUIRE(n >= 0 && q_rank > 0 && rank >= 0 && rot >= 0 && rot % 2 == 0 && eps > 0.f && ld_cq >= q_rank && ld >= q_rank &&
+                   splits >= 1 && (splits == 1 || p_dt == ZI_F32), "latent_inputs: bad sizes");
+    ZI_REQUIRE(!c_cache || (rank > 0 && dkv_at >= q_rank && ld >= (int64_t)dkv_at + width && kr_cache && slots && c_norm && cache_slots > 0 &&
+                            (rot == 0 || table)), "latent_inputs: a cache without slots, norm or angles");
+    ZI_REQUIRE((size_t)most * sizeof(float) <= 60 * 1024, "latent_inputs: latents of %d values are too large", most);
+    if (n == 0) return 0;
+    const dim3 grid(n, c_cache ? 2 : 1);
+    ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(p_dt, TP, ZI_DISPATCH_DTYPE(w_dt, TW, {
+        latent_inputs_kernel<T, TP, TW><<<grid, 256, most * sizeof(float), stream>>>(
+            (T*)cq, ld_cq, (const TP*)proj, ld, splits, split_stride, (const TW*)q_norm, (const TW*)c_norm, eps, q_rank, dkv_at, table,
+            slots, (T*)c_cache, (T*)kr_cache, c_cache ? cache_slots : 1, rank, rot);
+    })));
+    return zi_check_launch("latent_inputs");
+}
+
 // ---- queries: qa[t][h] = (W_uk[h]^T q_plain[t][h], turn(q_rot[t][h])), float32 ------------------------------
 // One workgroup per (tile of QT tokens, head).  W_uk is [heads * dim][rank], row h * dim + d the d-th unrotated
 // dimension of head h: for a fixed d the threads read neighbouring ranks.

@@ -314,15 +314,32 @@ extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t par
 // ldx and head stride xs (rounded to bfloat16 as it is loaded), out float32 or bfloat16 with row stride ldo and head
 // stride os.  One wavefront per (16 tokens, head, 16 outputs); operands straight from memory.  It carries the
 // queries through W_uk (w = W_uk of the head, transposed at load) and the attended latents through W_uv.
-template <typename TO>
+// GATED: out *= sigmoid(gate[t][h * N + i]), the gate bfloat16 or the sum of `splits` float32 terms.
+struct LaGate {
+    const void* g;
+    int f32, splits;
+    int64_t ld, stride;
+};
+
+template <typename TO, bool GATED>
 __global__ void __launch_bounds__(ZI_WAVE)
 headwise_linear_cores_kernel(TO* __restrict__ out, int64_t ldo, int os, const float* __restrict__ x, int64_t ldx, int xs,
-                             const zi_bf16* __restrict__ w, int n, int N, int K) {
+                             const zi_bf16* __restrict__ w, int n, int N, int K, LaGate gt) {
     const int t0 = blockIdx.x * 16, h = blockIdx.y, n0 = blockIdx.z * 16;
     const int lane = threadIdx.x, r = lane % 16, j = lane / 16;
     const zi_bf16* wrow = w + ((int64_t)h * N + (n0 + r < N ? n0 + r : N - 1)) * K;
     const float* xrow = x + (int64_t)(t0 + r < n ? t0 + r : n - 1) * ldx + (int64_t)h * xs;
     la_f32x4_t acc = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float gate[4];
+    if constexpr (GATED) {      // asked for before the product, used after it
+        const int64_t at = (int64_t)(t0 + r < n ? t0 + r : n - 1) * gt.ld + (int64_t)h * N;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int col = n0 + 4 * j + i < N ? n0 + 4 * j + i : N - 1;
+            gate[i] = gt.f32 ? ((const float*)gt.g)[at + col] : zi_load((const zi_bf16*)gt.g + at + col);
+            for (int s = 1; s < gt.splits; ++s) gate[i] += ((const float*)gt.g)[s * gt.stride + at + col];
+        }
+    }
 #pragma unroll 4
     for (int k0 = 0; k0 < K; k0 += 32) {
         const int k = k0 + 8 * j;
@@ -342,26 +359,38 @@ headwise_linear_cores_kernel(TO* __restrict__ out, int64_t ldo, int os, const fl
     TO* orow = out + (int64_t)(t0 + r) * ldo + (int64_t)h * os + n0 + 4 * j;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-        if (n0 + 4 * j + i < N) zi_store(orow + i, acc[i]);
+        if (n0 + 4 * j + i < N) zi_store(orow + i, GATED ? acc[i] / (1.f + expf(-gate[i])) : acc[i]);
 }
 
 extern "C" int zi_headwise_linear_supported(int w_dt, int K, int64_t ldx, int xs) {
     return w_dt == ZI_BF16 && K > 0 && K % 8 == 0 && ldx % 4 == 0 && xs % 4 == 0;
 }
 
-extern "C" int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs,
-                                  const void* w, int n, int heads, int N, int K, hipStream_t stream) {
+extern "C" int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs,
+                                        const void* w, int n, int heads, int N, int K, const void* gate, int g_dt,
+                                        int64_t ld_gate, int g_splits, int64_t g_stride, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && heads > 0 && heads <= 65535 && N > 0 && (N + 15) / 16 <= 65535, "headwise_linear: bad sizes");
     ZI_REQUIRE(zi_headwise_linear_supported(ZI_BF16, K, ldx, xs) && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0,
                "headwise_linear: K %d, row stride %lld, head stride %d or an address is not aligned", K, (long long)ldx, xs);
     ZI_REQUIRE(xs >= K && os >= N && ldx >= (int64_t)(heads - 1) * xs + K && ldo >= (int64_t)(heads - 1) * os + N,
                "headwise_linear: strides too small");
+    ZI_REQUIRE(!gate || (ld_gate >= (int64_t)heads * N && g_splits >= 1 && (g_dt == ZI_F32 || (g_dt == ZI_BF16 && g_splits == 1))),
+               "headwise_linear: bad gate");
     if (n == 0) return 0;
     const dim3 grid((n + 15) / 16, heads, (N + 15) / 16);
+    const LaGate gt = {gate, g_dt == ZI_F32, g_splits, ld_gate, g_stride};
     ZI_DISPATCH_DTYPE(out_dt, TO, {
-        headwise_linear_cores_kernel<TO><<<grid, ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, x, ldx, xs, (const zi_bf16*)w, n, N, K);
+        if (gate)
+            headwise_linear_cores_kernel<TO, true><<<grid, ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, x, ldx, xs, (const zi_bf16*)w, n, N, K, gt);
+        else
+            headwise_linear_cores_kernel<TO, false><<<grid, ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, x, ldx, xs, (const zi_bf16*)w, n, N, K, gt);
     });
     return zi_check_launch("headwise_linear");
+}
+
+extern "C" int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs,
+                                  const void* w, int n, int heads, int N, int K, hipStream_t stream) {
+    return zi_headwise_linear_gated(out, out_dt, ldo, os, x, ldx, xs, w, n, heads, N, K, nullptr, ZI_F32, 0, 1, 0, stream);
 }
 
 // qa[t][h][rank + ...] = the rotated part of every head's query, turned in neighbouring pairs.

@@ -30,6 +30,38 @@ int zi_attention_generic(void* out, const void* q, int dt, int n, int64_t ldq, i
     block_tables, int max_pages, int num_pages, int nh, int nkv, int d, int page_size, int window, float scale,
     hipStream_t stream);
 // attention_prefill.hip
+int zi_attention_prefill_maps(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo, const void* kcache,
+    const void* vcache, const int32_t* tile_entry, const int32_t* tile_off, const int32_t* entry_start, const int32_t* entry_len,
+    const int32_t* entry_past, const int32_t* block_tables, int max_pages, int num_pages, int nh, int nkv, int d, int page_size,
+    int window, float scale, int rows, int max_chunks, float* workspace, int64_t workspace_floats, int tile, int alone,
+    int chunk_keys, int maps, hipStream_t stream);
+// stream_mix.hip
+int zi_stream_mix(void* out, int out_dt, const float* in, int64_t in_stride, float* keep, int64_t keep_stride, const void* y,
+    int y_dt, int splits, int64_t split_stride, const float* scale, const float* write, const float* read, const float* gain,
+    const int32_t* rows, int n, int total_rows, int streams, int hidden, float eps, int centered, hipStream_t stream);
+// difference.hip
+int zi_head_norm_store(void* q_out, int dt, int64_t ldq, void* kcache, void* vcache, const void* proj, int p_dt, int64_t ld,
+    int splits, int64_t split_stride, const float* q_gain, const float* k_gain, float eps, const float* table, int rot,
+    const int32_t* slots, int64_t cache_slots, int n, int nh, int nkv, int maps, int dim, int vdim, int d, int page_size, int pad,
+    hipStream_t stream);
+int zi_difference_heads(void* out, int dt, int64_t ldo, const void* att, int64_t lda, int n, int heads, int d, int vdim,
+    float lam, float factor, float eps, const void* gate, int g_dt, int64_t ld_gate, int g_splits, int64_t g_stride,
+    hipStream_t stream);
+int zi_difference_merge(void* out, int64_t ldo, const float* workspace, int64_t workspace_floats, int n, const int32_t* tok_pos,
+    int window, int max_chunks, int heads, int d, int vdim, float lam, float factor, float eps, const void* gate, int g_dt,
+    int64_t ld_gate, int g_splits, int64_t g_stride, hipStream_t stream);
+// elementwise.hip
+int zi_activate(void* out, int out_dt, int64_t ldo, const void* z, int dt, int64_t ldz, int splits, int64_t split_stride,
+    int n, int inter, int act, hipStream_t stream);
+// latent.hip
+int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* proj, int p_dt, int64_t ld, int splits, int64_t split_stride,
+    int n, const void* q_norm, const void* c_norm, int w_dt, float eps, int q_rank, int dkv_at, const float* table,
+    const int32_t* slots, void* c_cache, void* kr_cache, int64_t cache_slots, int rank, int rot, hipStream_t stream);
+// latent_cores.hip
+int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs, const void* w,
+    int n, int heads, int N, int K, const void* gate, int g_dt, int64_t ld_gate, int g_splits, int64_t g_stride,
+    hipStream_t stream);
+// attention_prefill.hip
 int zi_attention_prefill(void* out, const void* q, int dt, int num_tiles, int64_t ldq, int64_t ldo, const void*
     kcache, const void* vcache, const int32_t* tile_entry, const int32_t* tile_off, const int32_t* entry_start, const
     int32_t* entry_len, const int32_t* entry_past, const int32_t* block_tables, int max_pages, int num_pages, int nh,
@@ -441,5 +473,13 @@ int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int ro
     X(zi_norm_input_conv) \
     X(zi_lowrank_gates) \
     X(zi_delta_channel) \
+    X(zi_attention_prefill_maps) \
+    X(zi_stream_mix) \
+    X(zi_head_norm_store) \
+    X(zi_difference_heads) \
+    X(zi_difference_merge) \
+    X(zi_activate) \
+    X(zi_latent_inputs) \
+    X(zi_headwise_linear_gated) \
     X(zi_argmax) \
     X(zi_sample)

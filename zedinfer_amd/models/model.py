@@ -14,8 +14,9 @@ import torch
 from .. import ops
 from ..config.forward_config import ModelForwardConfig, PartSpec
 from ..cache.manager import EMBEDDING_CACHE
-from ..parts import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, STREAM_STEPS, KVCacheRequest, LayerMemory,
+from ..parts import (BLOCKS, CONNECTIONS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, STREAM_STEPS, KVCacheRequest, LayerMemory,
                      Part, Runtime, StateRequest)
+from ..parts.connections import Streams
 from ..weights.loader import WeightSpec
 
 
@@ -47,6 +48,8 @@ def expected_weights(fc: ModelForwardConfig) -> Dict[str, WeightSpec]:
         merge(_part_weights(FEED_FORWARDS, layer.feed_forward))
         for n in layer.norms.values():
             merge(_part_weights(NORMS, n))
+        for c in layer.connections.values():
+            merge(_part_weights(CONNECTIONS, c))
     for st in fc.schedule:
         if st.enter is not None:
             merge(_part_weights(STREAM_STEPS, st.enter))
@@ -77,9 +80,14 @@ class DecoderModel:
             norms = {n: _build(NORMS, layer.norms[n], weights, rt) for n in block_cls.norm_names}
             mixer = _build(MIXERS, layer.mixer, weights, rt)
             ffn = _build(FEED_FORWARDS, layer.feed_forward, weights, rt)
-            self.blocks.append(block_cls(norms, mixer, ffn, rt))
+            missing = [n for n in block_cls.connection_names if n not in layer.connections]
+            if missing or (fc.streams > 0 and not block_cls.connection_names):
+                raise ValueError(f"block '{layer.block}' needs connections {missing}" if missing else
+                                 f"block '{layer.block}' works on one residual stream; this model has {fc.streams}")
+            connections = {n: _build(CONNECTIONS, layer.connections[n], weights, rt) for n in block_cls.connection_names}
+            self.blocks.append(block_cls(norms, mixer, ffn, rt, **({"connections": connections} if connections else {})))
             # a mixer's position encoding is a part of its own
-            self.parts += [self.blocks[-1], mixer, ffn, *norms.values()]
+            self.parts += [self.blocks[-1], mixer, ffn, *norms.values(), *connections.values()]
             self.parts += [p for p in vars(mixer).values() if isinstance(p, Part)]
         # what a schedule step does to the stream before its layer runs
         self.enters = [(_build(STREAM_STEPS, st.enter, weights, rt) if st.enter is not None else None) for st in fc.schedule]
@@ -95,6 +103,9 @@ class DecoderModel:
         self.keeps_embedded = any(getattr(e, "needs_embedded", False) for e in self.enters if e is not None)
         self.final_norm = _build(NORMS, fc.final_norm, weights, rt)
         self.lm_head = _build(HEADS, fc.lm_head, weights, rt)
+        if fc.streams > 0:      # the streams are added up in the launch that makes the final norm
+            self.final_row_norm = self.final_norm.row_norm()
+            self.all_streams = torch.ones((fc.streams,), dtype=torch.float32, device=rt.device)
         self.parts += [self.embedding, self.final_norm, self.lm_head]
         self.vocab_size = fc.vocab_size
         self.hidden_size = fc.hidden_size
@@ -204,6 +215,8 @@ class DecoderModel:
         if self.keeps_embedded:
             embedded = ops.convert(resid, self.rt.buffer("embedded", tuple(resid.shape), torch.float32))
         delta = None
+        if self.fc.streams > 0:
+            resid = Streams(self.rt, resid, self.fc.streams)
         for st, mem, enter, next_norm in zip(self.fc.schedule, memories, self.enters, self.next_input_norms):
             if enter is not None:
                 delta = enter.forward(resid, delta, embedded)
@@ -215,6 +228,10 @@ class DecoderModel:
                 pass  # the last feed-forward's output is not needed when no logits are
             return None
         rows = batch.logit_rows
+        if self.fc.streams > 0:
+            x = resid.finish(delta, self.all_streams, self.final_row_norm,
+                             rows=None if getattr(batch, "all_rows_wanted", False) else rows)
+            return self.lm_head.forward(x)
         if delta is not None and delta.dim() == 3:
             # float32 partial sums (few tokens): norm every row, then pick the wanted ones
             x_all = self.final_norm.add_forward(resid, delta)

@@ -139,6 +139,16 @@ _PROTOTYPES = {
     "zi_delta_channel": [P, P, P, P, L, P, P, L, P, P, P, I, I, I, I, I, I, P, I, P, P, F, P],
     "zi_delta_channel_finishes": [I, L],
     "zi_channel_inputs": [P, P, P, L, P, P, L, I, L, P, P, L, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
+    "zi_attention_prefill_maps": [P, P, I, I, L, L, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, L, I, I, I, I, P],
+    "zi_attention_prefill_maps_supported": [I, I, I, I, I, I],
+    "zi_stream_mix": [P, I, P, L, P, L, P, I, I, L, P, P, P, P, P, I, I, I, I, F, I, P],
+    "zi_stream_mix_max_streams": [],
+    "zi_head_norm_store": [P, I, L, P, P, P, I, L, I, L, P, P, F, P, I, P, L, I, I, I, I, I, I, I, I, I, P],
+    "zi_difference_heads": [P, I, L, P, L, I, I, I, I, F, F, F, P, I, L, I, L, P],
+    "zi_difference_merge": [P, L, P, L, I, P, I, I, I, I, I, F, F, F, P, I, L, I, L, P],
+    "zi_activate": [P, I, L, P, I, L, I, L, I, I, I, P],
+    "zi_latent_inputs": [P, I, L, P, I, L, I, L, I, P, P, I, F, I, I, P, P, P, P, L, I, I, P],
+    "zi_headwise_linear_gated": [P, I, L, I, P, L, I, P, I, I, I, I, P, I, L, I, L, P],
     "zi_tape_record": [P, c_char_p, P, I],
     "zi_tape_record_many": [P, c_char_p, P, P, I],
     "zi_tape_run": [P, P],

@@ -447,7 +447,7 @@ def attention_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
     """The same attention for single query tokens, split over the keys, on the matrix cores
     (bfloat16, head_dim a multiple of 16 up to 128, group size <= 16, page size a multiple of 8).
     ``max_keys`` is an upper bound of the keys any listed token sees (its position + 1), known on
-    the host; it only sizes the launch.  ``leave_chunks`` (with ``sinks`` or ``log_distance``, without a token list): nothing is merged
+    the host; it only sizes the launch.  ``leave_chunks`` (without a token list): nothing is merged
     or written to ``out``; every token's chunks stay in ``workspace`` for ``attention_decode_project``.
     ``softcap``, ``bias`` (float32 [nh, L]) and ``keep_first``: scores are capped as cap * tanh(score / cap), then
     take ``bias[head, min(distance, L - 1)]``; the sequence's first ``keep_first`` positions stay visible beside the
@@ -456,9 +456,8 @@ def attention_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
     out, n, count, ldq, ldo, pages, ps = _attention_args("attention_decode", q, kcache, vcache, tok_seq, tok_pos,
                                                          block_tables, nh, nkv, d, tok_index,
                                                          q if (leave_chunks and out is None) else out)   # (nothing is written there)
-    if leave_chunks and ((sinks is None and log_distance is None) or tok_index is not None or workspace is None):
-        raise ValueError("attention_decode: chunks are left for mixers with sinks or a distance's logarithm, all tokens, "
-                         "in a given workspace")
+    if leave_chunks and (tok_index is not None or workspace is None):
+        raise ValueError("attention_decode: chunks are left of all tokens, in a given workspace")
     if window > 0:
         max_keys = min(max_keys, window)
     max_chunks = int(_lib.load().zi_attention_decode_chunks(int(max_keys)))
@@ -792,6 +791,11 @@ def attention_prefill_supported(dtype: torch.dtype, nh: int, nkv: int, d: int, p
     return bool(_lib.load().zi_attention_prefill_supported(_CODES[dtype], nh, nkv, d, page_size))
 
 
+def attention_prefill_maps_supported(dtype: torch.dtype, nh: int, nkv: int, d: int, page_size: int, maps: int) -> bool:
+    """Whether ``attention_prefill`` takes heads that are ``maps`` softmax maps with keys side by side in rows of ``d`` values."""
+    return dtype == torch.bfloat16 and bool(_lib.load().zi_attention_prefill_maps_supported(BF16, nh, nkv, d, page_size, int(maps)))
+
+
 def attention_prefill_workspace(rows: int, nh: int, d: int, max_keys: int, window: int = 0, num_tiles: int = 0) -> int:
     """float32 entries of workspace ``attention_prefill`` needs for ``rows`` query rows in ``num_tiles`` tiles of
     which none sees more than ``max_keys`` keys (0: none)."""
@@ -814,7 +818,7 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
                       window: int = 0, out: Optional[torch.Tensor] = None, max_keys: int = 0,
                       workspace: Optional[torch.Tensor] = None, tile: int = 0, alone: bool = False,
                       sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
-                      keep_first: int = 0, log_distance=None) -> torch.Tensor:
+                      keep_first: int = 0, log_distance=None, maps: int = 1) -> torch.Tensor:
     """The same attention for portions of prompts, on the matrix cores (bfloat16, head_dim a multiple
     of 16 up to 128, page size a power of two from 8).
 
@@ -828,7 +832,10 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
     concerned.  ``alone`` (where the head size has tiles of 128): workgroups of four wavefronts, two to a compute
     unit, which pays for launches of many tiles; the result differs by rounding.  ``softcap``, ``bias`` and
     ``keep_first`` as for ``attention_decode``; with any of them tiles hold ``attention_prefill_tile_min()`` queries.
-    ``log_distance`` as for ``attention_decode``, with every tile."""
+    ``log_distance`` as for ``attention_decode``, with every tile.  ``maps`` > 1 (where ``attention_prefill_maps_supported``;
+    without sinks and the options of the scores): head h is one of ``maps`` softmax maps over the same values, a key row
+    holds their keys of d / maps values side by side, and head h multiplies the (h mod maps)-th part of its query row with
+    that part of the keys; the rest of the query row is not read."""
     _gpu("attention_prefill", q, kcache, vcache, tile_entry, tile_off, entry_start, entry_len, entry_past,
          block_tables, out)
     ldq, wq = _rows(q, "attention_prefill q")
@@ -872,7 +879,11 @@ def attention_prefill(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tenso
             max_chunks, _p(workspace) if need else _p(None), workspace.numel() if need else 0, int(tile), int(bool(alone)),
             chunk_keys)
     extras = _score_extras("attention_prefill", nh, q, softcap, bias, keep_first, log_distance)
-    if extras is not None:
+    if maps != 1:
+        if extras is not None or sinks is not None:
+            raise ValueError("attention_prefill: several maps a key row have plain scores")
+        _lib.call("zi_attention_prefill_maps", *args, int(maps), _stream())
+    elif extras is not None:
         if (extras[0] > 0 or bias is not None or keep_first) and (tile != attention_prefill_tile_min() or alone):
             raise ValueError("attention_prefill: capped or biased scores take the smallest tiles")
         _lib.call("zi_attention_prefill_biased", *args,

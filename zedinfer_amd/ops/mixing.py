@@ -84,6 +84,34 @@ def latent_store(dkv: torch.Tensor, norm_w: torch.Tensor, eps: float, table: Opt
               float(eps), _p(table), _p(slots), _p(c_cache), _p(kr_cache), pages * ps, rank, rot, _stream())
 
 
+def latent_inputs(proj: torch.Tensor, q_norm: torch.Tensor, eps: float, cq: torch.Tensor, dkv_at: int = 0,
+                  c_norm: Optional[torch.Tensor] = None, table: Optional[torch.Tensor] = None, slots: Optional[torch.Tensor] = None,
+                  c_cache: Optional[torch.Tensor] = None, kr_cache: Optional[torch.Tensor] = None, rank: int = 0, rot: int = 0) -> None:
+    """From rows of one product, proj [n, ...] (any storage type, dense rows; or a stack of float32 partial sums): cq [n, q_rank] =
+    the first q_rank columns RMS-normed with ``q_norm``; with the caches, columns dkv_at .. dkv_at + rank + rot go where
+    ``latent_store`` puts them (``c_norm``, ``table``, ``slots``)."""
+    _gpu("latent_inputs", proj, q_norm, cq, c_norm, table, slots, c_cache, kr_cache)
+    from .sublayers import _terms
+    splits, split_stride, ld, n, width = _terms(proj, "latent_inputs proj", columns=True)
+    ldc, q_rank = _rows(cq, "latent_inputs cq")
+    if cq.shape[0] != n or width < q_rank or q_norm.numel() != q_rank or not q_norm.is_contiguous():
+        raise ValueError("latent_inputs: cq, its norm and proj do not agree")
+    rows = 0
+    if c_cache is not None:
+        pages, ps = _latent_caches(c_cache, kr_cache, rank, rot, "latent_inputs")
+        rows = pages * ps
+        if not (q_rank <= dkv_at <= width - rank - rot) or c_norm is None or c_norm.numel() != rank or not c_norm.is_contiguous() \
+                or c_norm.dtype != q_norm.dtype or c_cache.dtype != cq.dtype:
+            raise ValueError("latent_inputs: the latents' columns, norm or caches do not agree")
+        _i32(slots, "latent_inputs slots", n)
+        if rot:
+            _f32(table, "latent_inputs table", (n, rot // 2, 2))
+    _lib.call("zi_latent_inputs", _p(cq), _code(cq, "latent_inputs cq"), ldc, _p(proj), _code(proj, "latent_inputs proj"), ld, splits,
+              split_stride, n, _p(q_norm), _p(c_norm if c_cache is not None else None), _code(q_norm, "latent_inputs q_norm"), float(eps),
+              q_rank, int(dkv_at), _p(table), _p(slots if c_cache is not None else None), _p(c_cache),
+              _p(kr_cache if c_cache is not None else None), rows, int(rank), int(rot), _stream())
+
+
 def latent_query(q: torch.Tensor, w_uk: torch.Tensor, table: Optional[torch.Tensor], heads: int, dim: int, rank: int,
                  rot: int, out: torch.Tensor, w_uk_t: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out [n, heads, rank + rot] float32: every head's unrotated query part carried through its block of
@@ -216,10 +244,17 @@ def latent_attention_cores(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: to
     return out
 
 
-def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tensor) -> torch.Tensor:
+def latent_value_gates(w_uv: torch.Tensor, heads: int, rank: int) -> bool:
+    """Whether ``latent_value`` takes a gate itself (else: ``gate_heads`` on its result)."""
+    return w_uv.dtype == torch.bfloat16 and w_uv.data_ptr() % 16 == 0 \
+        and bool(_lib.load().zi_headwise_linear_supported(1, rank, heads * rank, rank))
+
+
+def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out [n, heads * vdim] = every head's attended latent o [n, heads, rank] through its block of ``w_uv``
-    [heads * vdim, rank]."""
-    _gpu("latent_value", o, w_uv, out)
+    [heads * vdim, rank]; with ``gate`` ([n, heads * vdim] bfloat16 or float32 with dense rows, or a stack of float32 terms;
+    where ``latent_value_gates``) times sigmoid(gate)."""
+    _gpu("latent_value", o, w_uv, out, gate)
     _f32(o, "latent_value o")
     n, heads, rank = o.shape
     if tuple(w_uv.shape) != (heads * vdim, rank) or not w_uv.is_contiguous():
@@ -227,11 +262,20 @@ def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tens
     ldo, width = _rows(out, "latent_value out")
     if tuple(out.shape) != (n, heads * vdim):
         raise ValueError(f"latent_value: out must be [{n}, {heads * vdim}]")
-    if w_uv.dtype == torch.bfloat16 and _lib.load().zi_headwise_linear_supported(1, rank, heads * rank, rank) \
-            and w_uv.data_ptr() % 16 == 0:
-        _lib.call("zi_headwise_linear", _p(out), _code(out, "latent_value out"), ldo, vdim, _p(o), heads * rank, rank,
-                  _p(w_uv), n, heads, vdim, rank, _stream())
+    if latent_value_gates(w_uv, heads, rank):
+        args = (_p(out), _code(out, "latent_value out"), ldo, vdim, _p(o), heads * rank, rank, _p(w_uv), n, heads, vdim, rank)
+        if gate is None:
+            _lib.call("zi_headwise_linear", *args, _stream())
+            return out
+        if gate.dim() not in (2, 3) or tuple(gate.shape[-2:]) != (n, heads * vdim) or gate.stride(-1) != 1 \
+                or (gate.dim() == 3 and gate.dtype != torch.float32):
+            raise ValueError(f"latent_value: the gate must be [{n}, {heads * vdim}] or a float32 stack of such rows")
+        stack = gate.dim() == 3
+        _lib.call("zi_headwise_linear_gated", *args, _p(gate), _code(gate, "latent_value gate"), int(gate.stride(-2)),
+                  int(gate.shape[0]) if stack else 1, int(gate.stride(0)) if stack else 0, _stream())
         return out
+    if gate is not None:
+        raise ValueError("latent_value: a gate is not taken with these sizes")
     _lib.call("zi_latent_value", _p(out), _code(out, "latent_value out"), ldo, _p(o), _p(w_uv), _code(w_uv, "latent_value w_uv"),
               n, heads, vdim, rank, _stream())
     return out

@@ -128,6 +128,7 @@ BLOCKS = Registry("block arrangement")
 EMBEDDINGS = Registry("embedding")
 HEADS = Registry("output head")
 STREAM_STEPS = Registry("stream step")
+CONNECTIONS = Registry("connection")
 
 register_mixer = MIXERS.register
 register_feed_forward = FEED_FORWARDS.register
@@ -137,6 +138,7 @@ register_block = BLOCKS.register
 register_embedding = EMBEDDINGS.register
 register_head = HEADS.register
 register_stream_step = STREAM_STEPS.register
+register_connection = CONNECTIONS.register
 
 
 PAGE = -1      # in the shape of a page tensor: where the number of tokens a page holds goes
@@ -425,9 +427,14 @@ class Block:
     ``forward(resid, delta, batch, memory)``: ``resid`` is the float32 residual stream
     [n, hidden], ``delta`` a pending addition to it (or None; [n, hidden] or a stack
     [S, n, hidden] of float32 partial sums); returns the next pending addition.  The add is
-    folded into the following norm."""
+    folded into the following norm.
+
+    An arrangement for several residual streams names its sublayers' connections in ``connection_names`` and is
+    built with them as well; ``resid`` is then the step's ``parts.connections.Streams`` and ``delta`` a pending pair of
+    (connection, result)."""
 
     norm_names: Tuple[str, ...] = ()
+    connection_names: Tuple[str, ...] = ()
 
     def forward(self, resid, delta, batch, memory: LayerMemory):
         raise NotImplementedError

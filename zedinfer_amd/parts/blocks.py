@@ -190,3 +190,34 @@ class SandwichBlock(Block):
         return (type(norm) is type(last) and getattr(norm, "add_one", None) == getattr(last, "add_one", None)
                 and getattr(norm, "weight", None) is not None and norm.weight.dtype == last.weight.dtype
                 and getattr(norm, "out_dtype", None) is None)
+
+
+@register_block("connected")
+class ConnectedBlock(Block):
+    """Pre-norm sublayers over several residual streams: each reads the row its connection makes of the streams, normed, and
+    its result is written back by the same connection.  ``resid`` is the step's ``Streams``; a result is handed on as a pending
+    (connection, result), written by the launch that reads and norms the next sublayer's row.  The feed-forward may be the
+    kind "none" (its norm and connection are then the kind "none" too)."""
+
+    graph_safe = True
+    tape_safe = True
+
+    norm_names = ("input", "post_mixer")
+    connection_names = ("mixer", "feed_forward")
+
+    def __init__(self, norms, mixer, feed_forward, rt: Runtime, connections=None):
+        self.mixer, self.feed_forward = mixer, feed_forward
+        self.has_ff = getattr(feed_forward, "kind", "") != "none"
+        self.connections = connections
+        self.mixer_norm = norms["input"].row_norm()
+        self.ff_norm = norms["post_mixer"].row_norm() if self.has_ff else None
+        self.rt = rt
+
+    def forward(self, resid, delta, batch, memory: LayerMemory):
+        con = self.connections["mixer"]
+        a = self.mixer.forward(resid.read(delta, con, self.mixer_norm), batch, memory)
+        if not self.has_ff:
+            return con, a
+        x = resid.read((con, a), self.connections["feed_forward"], self.ff_norm)
+        f = self.feed_forward.forward(x, batch=batch) if self.feed_forward.reads_batch else self.feed_forward.forward(x)
+        return self.connections["feed_forward"], f

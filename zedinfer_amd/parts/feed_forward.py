@@ -336,6 +336,52 @@ class ReluSquaredMLP(FeedForward):
         return _float_result(rt, "ffn_out_f32", act, self.down)
 
 
+@register_feed_forward("activated_mlp")
+class ActivatedMLP(FeedForward):
+    """down(act(up(x))), no gate, no biases, the activation one of ``ops.ACTIVATIONS`` ("gelu_tanh", "gelu_erf", "silu",
+    "relu2").  Few rows: the up product leaves partial sums, which the activation's kernel adds; the down product leaves its own
+    for the norm that follows.  params: hidden_size, intermediate_size, activation."""
+
+    graph_safe = True
+    tape_safe = True
+
+    @staticmethod
+    def weight_specs(spec: PartSpec) -> Dict[str, WeightSpec]:
+        H, I = int(spec.params["hidden_size"]), int(spec.params["intermediate_size"])
+        return {"up": WeightSpec((I, H)), "down": WeightSpec((H, I))}
+
+    def __init__(self, spec: PartSpec, weights: Dict[str, torch.Tensor], rt: Runtime):
+        super().__init__(spec, weights, rt)
+        self.hidden = int(spec.params["hidden_size"])
+        self.inter = int(spec.params["intermediate_size"])
+        self.activation = str(spec.params["activation"])
+        if self.activation not in ops.ACTIVATIONS:
+            raise ValueError(f"activated_mlp: unknown activation {self.activation!r}")
+        self.up, self.down = weights["up"], weights["down"]
+
+    def step_rows(self, rows: int, kind: str) -> int:
+        return ProductRows.step_rows(rows, kind)
+
+    def tune(self, num_tokens: int) -> None:
+        n = int(num_tokens)
+        self.rt.tune_linear(self.rt.buffer("norm_out", (n, self.hidden)), self.up)
+        self.rt.tune_linear(self.rt.buffer("ffn_act", (n, self.inter)), self.down)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        n, I, rt = x.shape[0], self.inter, self.rt
+        act = rt.buffer("ffn_act", (n, I))
+        if ops.linear_sums_supported(x, self.up):
+            S = ops.linear_splits(n, I, self.hidden)
+            z = ops.linear_sums(x, self.up, out=rt.buffer("ffn_up_sums", (S, n, I), torch.float32))
+        else:
+            z = ops.linear(x, self.up, out=rt.buffer("ffn_up", (n, I)))
+        ops.activate(z, self.activation, out=act)
+        if ops.linear_sums_supported(act, self.down):
+            S = ops.linear_splits(n, self.hidden, I)
+            return ops.linear_sums(act, self.down, out=rt.buffer("ffn_out_sums", (S, n, self.hidden), torch.float32))
+        return ops.linear(act, self.down, out=rt.buffer("ffn_out", (n, self.hidden)))
+
+
 class _ClampedGated:
     """One feed-forward of the clamped gated form, down(g sigmoid(1.702 g) (u + 1)) with g = min(gate x, limit) and
     u = clamp(up x, -limit, limit): gate and up stacked into one product (the up rows begin at a multiple of 8).  With

@@ -36,14 +36,18 @@ class LatentAttention(Mixer):
     latents it reads (``ScheduleStep.writes_cache`` False), and it brings its own W_uk, W_uv, queries, window.
 
     With ``q_rank`` the queries come through a latent of their own: c_q = rms_norm(W_dq x) * g_q, q = W_uq c_q
-    (two products and a norm instead of the one product W_q x).
+    (two products and a norm instead of the one product W_q x); -1 takes the checkpoint's own size.
+
+    With ``gate`` the heads side by side are multiplied by sigmoid(W_g x) before W_o.  A gated layer with query latents makes
+    everything that reads x (query latent, the token's latent and key part, gate) in one product; the kernel that norms both
+    latents adds its partial sums (``ops.latent_inputs``), the gate is applied where the values are made.
 
     ``pairing`` says which of the rot_dim dims a checkpoint pairs: "interleaved" (2i with 2i + 1, what the kernels
     turn; the default) or "halves" (i with i + rot_dim / 2: the turned rows of the query and key projections are
     reordered at load, the same way in both, which changes no score).
 
     params: hidden_size, heads, dim, rot_dim, vdim, kv_rank, scale, window (0: all keys), eps, shares_cache, q_rank
-    (0: none), pairing, position (a PartSpec of an encoding that hands over ``pair_table``: neighbouring pairs turn)."""
+    (0: none), gate (False), pairing, position (a PartSpec of an encoding that hands over ``pair_table``: neighbouring pairs turn)."""
 
     graph_safe = True
     tape_safe = True
@@ -64,6 +68,8 @@ class LatentAttention(Mixer):
         if not p.get("shares_cache", False):
             w["dkv"] = WeightSpec((rank + rot, H))
             w["dkv_norm"] = WeightSpec((rank,), init="ones")
+        if p.get("gate", False):
+            w["g"] = WeightSpec((nh * vdim, H))
         return w
 
     def __init__(self, spec: PartSpec, weights: Dict[str, torch.Tensor], rt: Runtime):
@@ -99,6 +105,7 @@ class LatentAttention(Mixer):
         self.q = q_w
         if self.q_rank:
             self.dq, self.dq_norm = weights["dq"], weights["dq_norm"]
+            self.q_rank = int(self.dq.shape[0])
         # a bfloat16 cache of sizes the matrix-core kernel takes goes there; everything else to the plain kernel
         self.cores = (rt.device.type == "cuda" and rt.dtype == torch.bfloat16
                       and ops.latent_attention_cores_supported(rt.dtype, self.rank, self.rot))
@@ -112,6 +119,25 @@ class LatentAttention(Mixer):
             if order is not None:
                 self.dkv = torch.cat([self.dkv[:self.rank], self.dkv[self.rank:][order]]).contiguous()
             self.dkv_norm = weights["dkv_norm"]
+        self.gate = weights["g"] if p.get("gate", False) else None
+        self.inputs = None
+        if self.gate is not None and self.q_rank:
+            # one product of everything that reads x; its parts begin at multiples of 8 columns
+            mats, at = [], 0
+            for name, m in (("query", self.dq), ("dkv", None if self.shares_cache else self.dkv), ("gate", self.gate)):
+                if m is None:
+                    continue
+                if name == "dkv":
+                    self.dkv_at = at
+                elif name == "gate":
+                    self.gate_at = at
+                mats.append(m.to(self.dq.dtype))
+                at += int(m.shape[0])
+                if at % 8:
+                    mats.append(torch.zeros((-at % 8, self.hidden), dtype=self.dq.dtype, device=self.dq.device))
+                    at += -at % 8
+            self.inputs = torch.cat(mats).contiguous()
+        self.value_gates = self.gate is not None and rt.device.type == "cuda" and ops.latent_value_gates(self.uv, self.nh, self.rank)
 
     def cache_request(self) -> Optional[KVCacheRequest]:
         return latent_cache_request("window" if self.window > 0 else "full", self.rank, self.rot, self.window)
@@ -123,17 +149,49 @@ class LatentAttention(Mixer):
         """Without a window the cut of a tile's keys over workgroups is sized by the most keys a token sees."""
         return KEY_BOUND_PLANNER if self.window <= 0 else None
 
+    def tune(self, num_tokens: int) -> None:
+        n = int(num_tokens)
+        if self.inputs is not None:
+            self.rt.tune_linear(self.rt.buffer("norm_out", (n, self.hidden)), self.inputs, out_dtype=self.inputs_dtype())
+            self.rt.tune_linear(self.rt.buffer("latent_cq_normed", (n, self.q_rank)), self.q, out_dtype=torch.float32)
+            self.rt.tune_linear(self.rt.buffer("latent_heads", (n, self.nh * self.vdim)), self.o)
+
+    def inputs_dtype(self) -> torch.dtype:
+        """Of the one product's result for many rows: the activation type, float32 where the gate is a kernel of its own."""
+        return self.rt.dtype if self.value_gates else torch.float32
+
+    def gated_inputs(self, x, batch, view, memory: LayerMemory, table):
+        """The one product and what is made of it: (normed query latents, gate); the token's latent goes into the cache."""
+        n, rt, rows = x.shape[0], self.rt, self.inputs.shape[0]
+        if ops.linear_sums_supported(x, self.inputs):
+            S = ops.linear_splits(n, rows, self.hidden)
+            full = ops.linear_sums(x, self.inputs, out=rt.buffer("latent_inputs_sums", (S, n, rows), torch.float32))
+        else:
+            full = ops.linear(x, self.inputs, out=rt.buffer("latent_inputs", (n, rows), self.inputs_dtype()))
+        cq = rt.buffer("latent_cq_normed", (n, self.q_rank))
+        if memory.writes:
+            ops.latent_inputs(full, self.dq_norm, self.eps, cq, self.dkv_at, self.dkv_norm, table, view.slots,
+                              memory.tensors["latent"], memory.tensors["key_part"], self.rank, self.rot)
+        else:
+            ops.latent_inputs(full, self.dq_norm, self.eps, cq)
+        return cq, full[..., self.gate_at:self.gate_at + self.nh * self.vdim]
+
     def forward(self, x: torch.Tensor, batch, memory: LayerMemory, out=None) -> torch.Tensor:
         n, rt = x.shape[0], self.rt
         view = batch.groups[memory.group]
         table = self.position.pair_table(batch) if self.rot else None
         c_cache, kr_cache = memory.tensors["latent"], memory.tensors["key_part"]
-        if memory.writes:
-            if self.shares_cache:
-                raise ValueError("latent_attention: a layer without W_dkv cannot write a cache")
+        if memory.writes and self.shares_cache:
+            raise ValueError("latent_attention: a layer without W_dkv cannot write a cache")
+        gate = None
+        if self.inputs is not None:
+            x, gate = self.gated_inputs(x, batch, view, memory, table)
+        elif self.gate is not None:
+            gate = ops.linear(x, self.gate, out=rt.buffer("latent_gate", (n, self.nh * self.vdim), torch.float32))
+        if memory.writes and self.inputs is None:
             dkv = ops.linear(x, self.dkv, out=rt.buffer("latent_dkv", (n, self.rank + self.rot), torch.float32))
             ops.latent_store(dkv, self.dkv_norm, self.eps, table, view.slots, c_cache, kr_cache, self.rank, self.rot)
-        if self.q_rank:
+        if self.q_rank and self.inputs is None:
             cq = ops.linear(x, self.dq, out=rt.buffer("latent_cq", (n, self.q_rank), torch.float32))
             x = ops.rms_norm(cq, self.dq_norm, self.eps, out=rt.buffer("latent_cq_normed", (n, self.q_rank)))
         q = ops.linear(x, self.q, out=rt.buffer("latent_q", (n, self.nh * (self.dim + self.rot)), torch.float32))
@@ -152,7 +210,10 @@ class LatentAttention(Mixer):
         else:
             ops.latent_attention(qa, c_cache, kr_cache, batch.tok_seq, batch.positions, view.block_tables, self.scale,
                                  self.window, out=o)
-        heads = ops.latent_value(o, self.uv, self.vdim, out=rt.buffer("latent_heads", (n, self.nh * self.vdim)))
+        heads = ops.latent_value(o, self.uv, self.vdim, out=rt.buffer("latent_heads", (n, self.nh * self.vdim)),
+                                 gate=gate if self.value_gates else None)
+        if gate is not None and not self.value_gates:
+            heads = ops.gate_heads(heads, gate, self.vdim, self.vdim, "sigmoid", out=rt.buffer("latent_gated", (n, self.nh * self.vdim)))
         if out is None:
             if ops.linear_sums_supported(heads, self.o):      # few rows: the partial sums go to the norm that follows
                 S = ops.linear_splits(n, self.hidden, self.nh * self.vdim)

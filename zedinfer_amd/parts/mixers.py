@@ -163,6 +163,8 @@ class Attention(Mixer):
     sinks: Optional[torch.Tensor] = None
     # (slope, rate), float32 [heads] each, in mixers that take slope * ln(1 + rate * distance) off every score
     log_distance: Optional[tuple] = None
+    # in mixers whose heads are several softmax maps over the same values (a key row holds their keys side by side)
+    maps: int = 1
 
     @staticmethod
     def weight_specs(spec: PartSpec) -> Dict[str, WeightSpec]:
@@ -242,6 +244,8 @@ class Attention(Mixer):
                 need = ops.attention_prefill_workspace(q.shape[0], self.nh, self.d, max_keys, self.window,
                                                        plan.sizes["num_tiles"])
                 ws = self.rt.buffer("attn_prompt_split", (need,), torch.float32) if need else None
+                if self.prompt_reads_parts(q.dtype, kc.shape[2]):
+                    extras = {"maps": self.maps}
                 ops.attention_prefill(q, kc, vc, plan.dev["tile_entry"], plan.dev["tile_off"],
                                       batch.entry_start, batch.entry_len, batch.entry_past, view.block_tables, self.nh,
                                       self.nkv, self.d, self.scale, self.window, out=att, max_keys=max_keys,
@@ -250,6 +254,11 @@ class Attention(Mixer):
             else:
                 plain(q, *args, self.window, out=att, tok_index=plan.dev["long_idx"] if n_long < N else None,
                       sinks=self.sinks, **extras)
+
+    def prompt_reads_parts(self, dtype: torch.dtype, page_size: int) -> bool:
+        """Whether the prompt kernel multiplies a map's part of a query and key row alone (else a query row is zero outside
+        its map's part and the whole rows are multiplied)."""
+        return self.maps > 1 and ops.attention_prefill_maps_supported(dtype, self.nh, self.nkv, self.d, page_size, self.maps)
 
     def planner(self) -> StepPlanner:
         return attention_planner(self.wide_tile, self.nh)

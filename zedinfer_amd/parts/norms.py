@@ -45,6 +45,10 @@ class RMSNorm(Norm):
             self.add_one = False
         self.out_dtype = torch.float32 if spec.params.get("out_dtype") == "float32" else None
 
+    def row_norm(self):
+        """(gains float32 [dim], eps, whether the mean is taken off) for a kernel that makes this norm itself."""
+        return (self.weight.float() + (1.0 if self.add_one else 0.0)).contiguous(), self.eps, False
+
     def forward(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
         out = self.rt.buffer("norm_out", (x.shape[0], self.dim), out_dtype or self.out_dtype or self.rt.dtype)
         return ops.rms_norm(x, self.weight, self.eps, out=out, add_one=self.add_one)
@@ -84,7 +88,7 @@ class NoNorm(Norm):
 @register_norm("layernorm")
 class LayerNorm(Norm):
     """y = (x - mean) / sqrt(var + eps) * w + b, var the mean of the squared deviations, all in float32.
-    params: dim, eps.  Beside the norm's two usual forms it has a third, ``add_normed(resid, y)``: the norm sits on a
+    params: dim, eps, bias (True; False: no b).  Beside the norm's two usual forms it has a third, ``add_normed(resid, y)``: the norm sits on a
     sublayer's OUTPUT, resid += norm(y), and the new residual rows come back in the activation type (what the next
     sublayer's products read)."""
 
@@ -94,14 +98,24 @@ class LayerNorm(Norm):
     @staticmethod
     def weight_specs(spec: PartSpec) -> Dict[str, WeightSpec]:
         dim = int(spec.params["dim"])
-        return {"weight": WeightSpec((dim,), init="ones"), "bias": WeightSpec((dim,), init="zeros")}
+        w = {"weight": WeightSpec((dim,), init="ones")}
+        if spec.params.get("bias", True):
+            w["bias"] = WeightSpec((dim,), init="zeros")
+        return w
 
     def __init__(self, spec: PartSpec, weights: Dict[str, torch.Tensor], rt: Runtime):
         super().__init__(spec, weights, rt)
         self.dim = int(spec.params["dim"])
         self.eps = float(spec.params["eps"])
         self.weight = weights["weight"]
-        self.bias = weights["bias"].to(self.weight.dtype)
+        self.has_bias = bool(spec.params.get("bias", True))
+        self.bias = weights["bias"].to(self.weight.dtype) if self.has_bias else torch.zeros_like(self.weight)
+
+    def row_norm(self):
+        """See ``RMSNorm.row_norm``."""
+        if self.has_bias:
+            raise ValueError("layernorm: a norm folded into another kernel has no bias")
+        return self.weight.float().contiguous(), self.eps, True
 
     def forward(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
         out = self.rt.buffer("norm_out", (x.shape[-2], self.dim), out_dtype or self.rt.dtype)

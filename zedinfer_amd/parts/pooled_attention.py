@@ -1,43 +1,16 @@
 """Windowed softmax attention that sees the positions before its window as means of blocks."""
 from __future__ import annotations
 
-import math
 from typing import Dict, Optional
 
-import numpy as np
 import torch
 
 from .. import ops
 from ..config.forward_config import PartSpec
 from ..weights.loader import WeightSpec
 from .base import KEY_BOUND_PLANNER, PAGE, KVCacheRequest, LayerMemory, Mixer, PageTensor, Runtime, StepPlanner, register_mixer
+from .positions import ramped_frequencies
 from .rows import ProductRows
-
-
-def ramped_frequencies(dims: int, base: float, scaling) -> tuple:
-    """(f_i for the dims / 2 pairs as float32, the magnitude of cos and sin).  f_i = base^(-2i / dims); with
-    ``scaling`` (factor, original, fast, slow) the pairs that turn few times within ``original`` positions are slowed
-    by ``factor``, those that turn many times are kept, with a linear ramp over the pair index between the two: with
-    dim(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(dim(fast)), 0), hi = min(ceil(dim(slow)),
-    dims - 1), ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), f_i <- f_i / factor * ramp_i + f_i (1 - ramp_i);
-    the magnitude is 0.1 ln(factor) + 1.  Computed in double precision, rounded once."""
-    i = np.arange(dims // 2, dtype=np.float64)
-    f = np.power(float(base), -2.0 * i / dims)
-    if not scaling:
-        return f.astype(np.float32), 1.0
-    missing = [k for k in ("factor", "original", "fast", "slow") if k not in scaling]
-    if missing:
-        raise ValueError("rotation scaling lacks " + ", ".join(missing))
-    factor, orig, fast, slow = (float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
-    if not (factor > 0 and orig > 0 and fast > 0 and slow > 0 and base > 1):
-        raise ValueError("rotation scaling: factor, original, fast and slow must be positive")
-
-    def dim_of(turns: float) -> float:
-        return dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
-    lo = max(math.floor(dim_of(fast)), 0)
-    hi = min(math.ceil(dim_of(slow)), dims - 1)
-    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
-    return (f / factor * ramp + f * (1.0 - ramp)).astype(np.float32), 0.1 * math.log(factor) + 1.0
 
 
 def halves_order(size: int, turned: int) -> torch.Tensor:

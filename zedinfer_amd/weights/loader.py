@@ -41,7 +41,7 @@ class WeightSpec:
     kind: str = "float"              # "float" or "int"
     fallback: Optional[str] = None   # tensor to alias when this one is absent (tied head)
     # what the random-weights mode fills it with: "normal" (N(0, std)), "ones" (a gain: 1, or 1 + N(0, std)
-    # with noisy gains) or "zeros"
+    # with noisy gains), "zeros" or "eye" (a matrix with ones on the diagonal)
     init: str = "normal"
     # for "int" tensors in the random-weights mode: every row holds distinct values below ``high`` (0: zeros)
     high: int = 0

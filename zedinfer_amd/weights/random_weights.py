@@ -58,10 +58,14 @@ def random_weights(expected: Mapping[str, WeightSpec], seed: int, dtype: torch.d
             t = torch.zeros(spec.shape, dtype=torch.float32, device=device)
             if noisy_norms:
                 t += torch.randn(spec.shape, generator=g, dtype=torch.float32, device=device) * std
+        elif spec.init == "eye":
+            t = torch.eye(spec.shape[0], spec.shape[1], dtype=torch.float32, device=device)
+            if noisy_norms:
+                t += torch.randn(spec.shape, generator=g, dtype=torch.float32, device=device) * std
         elif spec.init == "normal":
             t = torch.randn(spec.shape, generator=g, dtype=torch.float32, device=device) * std
         else:
-            raise ValueError(f"tensor '{name}': unknown init '{spec.init}' (normal, ones, zeros)")
+            raise ValueError(f"tensor '{name}': unknown init '{spec.init}' (normal, ones, zeros, eye)")
         out[name] = t.to(dtype)
     for name, spec in expected.items():
         if name not in out:
