@@ -138,7 +138,7 @@ extern "C" int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* pro
     const int width = c_cache ? rank + rot : 0, most = q_rank > width ? q_rank : width;
     ZI_REQUIRE(n >= 0 && q_rank > 0 && rank >= 0 && rot >= 0 && rot % 2 == 0 && eps > 0.f && ld_cq >= q_rank && ld >= q_rank &&
                    splits >= 1 && (splits == 1 || p_dt == ZI_F32), "latent_inputs: bad sizes");
-    ZI_REQUIRE(!c_cache || (rank > 0 && dkv_at >= q_rank && ld >= (int64_t)dkv_at + width && kr_cache && slots && c_norm && cache_slots > 0 &&
+    ZI_REQUIRE(!c_cache || (rank > 0 && dkv_at >= q_rank && ld >= (int64_t)dkv_at + width && (rot == 0 || kr_cache) && slots && c_norm && cache_slots > 0 &&
                             (rot == 0 || table)), "latent_inputs: a cache without slots, norm or angles");
     ZI_REQUIRE((size_t)most * sizeof(float) <= 60 * 1024, "latent_inputs: latents of %d values are too large", most);
     if (n == 0) return 0;

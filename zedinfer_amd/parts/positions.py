@@ -62,6 +62,8 @@ def angle_table(positions, inv_freq, magnitude: float = 1.0, out=None):
     """(cos, sin) of every position and frequency, float32 [n, R/2, 2], times the magnitude."""
     if magnitude == 1.0:
         return ops.rope_table(positions, inv_freq, out=out)
+    if out is None:
+        out = torch.empty((positions.numel(), inv_freq.numel(), 2), dtype=torch.float32, device=inv_freq.device)
     return ops.rope_table_scaled(positions, inv_freq, magnitude, out=out)
 
 
