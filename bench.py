@@ -500,13 +500,35 @@ def kefisun_shape(size, layers, vocab):
                 embedding=dict(scale=16.0), logit_scale=0.5, layers=out)
 
 
+def fovenex_shape(size, layers, vocab):
+    """Layer sizes that resemble a real model's, for the Fovenex design: two layers of latent attention (the heads of the Qwen2
+    model beside it, latents of 512 for keys and values and of half the width for queries, a window of 1,024 positions; the
+    second reads the first's latents), then two whose heads are differences of two maps of 64 over values of 128 on the Qwen2
+    model's key/value heads (projections of the Qwen2 model's sizes), half of every map turned with slowed frequencies; two
+    residual streams; every feed-forward is dense, of the Qwen2 model's width."""
+    z = DESIGN_SIZES[size]
+    out = []
+    for i in range(layers):
+        if i % 4 < 2:
+            kind, mixer = "latent_attention", dict(heads=z["heads"], dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=z["width"] // 2,
+                                                   scale=192 ** -0.5, mask=dict(size=1024), rot=dict(base=10000.0, dims=64))
+            if i % 4 == 1:
+                mixer["kv_from"] = i - 1
+        else:
+            kind, mixer = "attention", dict(heads=z["heads"], kv_heads=max(2, z["heads"] // 7), dim=64, vdim=128, scale=0.125, diff=0.5,
+                                            rot=dict(base=1000000.0, dims=32, scaling=dict(factor=4.0, original=8192, fast=32.0, slow=1.0)))
+        out.append(dict(type=kind, mixer=mixer, mlp=dict(kind="dense", ff=z["ff"])))
+    return dict(architecture="Fovenex", width=z["width"], vocab=vocab, norm=dict(eps=1e-6), streams=2, residual_mult=0.5, layers=out)
+
+
 def design_comparison(args):
     """Prefill and decode of a model of the design at a real model's layer sizes, and of the benchmark's own
     architecture (Qwen2 dense) at the same width, layers, heads and dense feed-forward, one after the other; for
     Tilivik, Kegozen and Kefisun also of Dedelorn, the nearest design the engine has (recurrent layers, latent
-    attention, experts), and for Kefisun of Tosisun (convolved projections)."""
+    attention, experts), for Kefisun of Tosisun (convolved projections), and for Fovenex of Kegozen (latent attention with query
+    latents)."""
     import torch
-    from zedinfer_amd.config import DedelornConfig, KefisunConfig, KegozenConfig, Qwen2Config, SchedulerConfig, TilivikConfig, TosisunConfig
+    from zedinfer_amd.config import DedelornConfig, FovenexConfig, KefisunConfig, KegozenConfig, Qwen2Config, SchedulerConfig, TilivikConfig, TosisunConfig
     from zedinfer_amd.engine import Engine
     layers = args.layers if args.layers != FULL_LAYERS else 8
     vocab, prompt = 32000, args.prompt_len
@@ -518,7 +540,8 @@ def design_comparison(args):
                   "tosisun": lambda: (TosisunConfig.from_dict(tosisun_shape(size, layers, vocab)), "Tosisun"),
                   "tilivik": lambda: (TilivikConfig.from_dict(tilivik_shape(size, layers, vocab)), "Tilivik"),
                   "kegozen": lambda: (KegozenConfig.from_dict(kegozen_shape(size, layers, vocab)), "Kegozen"),
-                  "kefisun": lambda: (KefisunConfig.from_dict(kefisun_shape(size, layers, vocab)), "Kefisun")}[args.design]
+                  "kefisun": lambda: (KefisunConfig.from_dict(kefisun_shape(size, layers, vocab)), "Kefisun"),
+                  "fovenex": lambda: (FovenexConfig.from_dict(fovenex_shape(size, layers, vocab)), "Fovenex")}[args.design]
         models = {
             args.design: design(),
             "qwen2": (Qwen2Config.from_dict(dict(SHAPE, hidden_size=z["width"], intermediate_size=z["ff"], vocab_size=vocab,
@@ -530,6 +553,8 @@ def design_comparison(args):
             models["dedelorn"] = (DedelornConfig.from_dict(dedelorn_shape(size, layers, vocab)), "Dedelorn")
         if args.design == "kefisun":
             models["tosisun"] = (TosisunConfig.from_dict(tosisun_shape(size, layers, vocab)), "Tosisun")
+        if args.design == "fovenex":
+            models["kegozen"] = (KegozenConfig.from_dict(kegozen_shape(size, layers, vocab)), "Kegozen")
         if args.design_only:
             models = {args.design: models[args.design]}
         rec = {}
@@ -585,7 +610,7 @@ def main():
                     help="run only the 2,048-token prefill (for profiling) and print its figures")
     ap.add_argument("--resident-layer", action="store_true",
                     help="instead: time the one-launch decoder layer (ops.decode_layer) alone, --layers launches a step")
-    ap.add_argument("--design", default="", choices=["", "dedelorn", "tosisun", "tilivik", "kegozen", "kefisun"],
+    ap.add_argument("--design", default="", choices=["", "dedelorn", "tosisun", "tilivik", "kegozen", "kefisun", "fovenex"],
                     help="instead: prefill and decode of a model of this design at a real model's layer sizes, beside "
                          "Qwen2 dense of equal sizes (8 layers unless --layers says otherwise)")
     ap.add_argument("--design-sizes", default="", help="with --design: layer sizes, of " + ", ".join(sorted(DESIGN_SIZES)) +
