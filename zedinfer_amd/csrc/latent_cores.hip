@@ -3,18 +3,21 @@
 // nearly the same, so a workgroup takes 16 rows a wavefront of ONE entry (rows in the order token, head) and walks
 // the keys its rows see in blocks of 32:
 //
-//   stage    the block's latents and key parts, [32][rank + rot], from the pages into LDS, rows padded by 16
-//            bytes; the latents once more transposed, [rank][32], for the second product.  Neighbouring lanes take
-//            neighbouring keys, so that the transposed copy's 2-byte stores fall into neighbouring LDS banks (with
-//            neighbouring pieces of one key a lane, all 64 stores of an instruction met in one bank: 694 against
-//            381 us for a layer's 2,048 tokens)
+//   stage    the block's latents and key parts, [32][rank + rot], from the pages straight into LDS
+//            (global_load_lds_dwordx4), one block ahead, in one of two buffers; where its keys lie in the pool is asked for
+//            two blocks ahead, a lane a key, and traded between lanes.  Rows are not padded but swizzled: the 16-byte
+//            piece c of row k sits at place c xor (k / 2 mod 8), so that neither product's reads meet in a bank
 //   scores   S[key][row] = K . Q^T   v_mfma_f32_16x16x32_bf16: first operand the keys' rows from LDS, second the
 //            queries, held in registers for the whole walk (KS operands a lane)
 //   softmax  a lane holds 8 of a row's 32 scores, the row's other 24 are in 3 lanes: two lane exchanges; running
-//            maximum and sum in float32, base e
+//            maximum and sum in float32, base 2; a block that all rows of the wavefront see whole needs no mask
 //   values   O[dim][row] += C^T . P   the same instruction, contraction over the block's keys in the order in
-//            which the lanes hold P (keys 4j..4j+3 and 16+4j..16+4j+3 for lane group j), the transposed latents
-//            read in that order: no exchange of P between lanes
+//            which the lanes hold P (keys 4j..4j+3 and 16+4j..16+4j+3 for lane group j): the latents are read
+//            transposed from the same rows (ds_read_b64_tr_b16: sixteen lanes read four keys x sixteen dims and each
+//            gets one dim of the four keys), so no second copy of them is made
+//
+// (Staged through registers, with a transposed copy of the latents written by 2-byte stores, the same walk took 381 us
+// for the 2,048 tokens of a layer with 12 heads, rank 512 and a window of 1,024 keys.)
 //
 // A tile's keys can be cut into chunks over blockIdx.y (decoded tokens: few rows, many keys); the chunks leave
 // (maximum, sum, unnormalised O) per row and a second kernel merges them.  The cut is a launch parameter that
@@ -26,32 +29,41 @@
 typedef __attribute__((ext_vector_type(8))) __bf16 la_bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float la_f32x4_t;
 typedef __attribute__((ext_vector_type(4))) unsigned la_u32x4_t;
-typedef __attribute__((ext_vector_type(2))) unsigned la_u32x2_t;
+typedef __attribute__((ext_vector_type(4))) short la_s16x4_t;
 union la_pack {
     la_u32x4_t u;
     la_bf16x8_t b;
-    la_u32x2_t h[2];
+    la_s16x4_t h[2];
     unsigned w[4];
 };
 
 #define LA_BK 32      // keys a block
-#define LA_PAD 8      // elements of padding of an LDS row
 #define LA_EMPTY -1e30f
-#define LA_BATCH 6     // requests a thread has in flight while it stages a block
+#define LA_LOG2E 1.4426950408889634f
+
+__device__ __attribute__((aligned(16))) const unsigned la_zero16[4] = {0u, 0u, 0u, 0u};
+
+// four keys of one dim from rows of LDS: see above
+__device__ __forceinline__ la_s16x4_t la_read_transposed(const char* at) {
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) la_s16x4_t*)at);
+}
 
 // SPLIT: all WAVES wavefronts share one tile of 16 rows (decoded tokens): they stage together, each makes the
 // scores again (cheap) and every WAVES-th tile of 16 latent dims of the second product.
 template <int WAVES, int NT, int KS, bool SPLIT>      // rank <= 16 NT, rank + rot <= 32 KS
-__global__ void __launch_bounds__(WAVES* ZI_WAVE)
-latent_attention_cores_kernel(float* __restrict__ out, float* __restrict__ partial, const float* __restrict__ qa,
+__global__ void __launch_bounds__(WAVES* ZI_WAVE, 2)
+latent_attention_cores_kernel(void* __restrict__ out, int out_f32, float* __restrict__ partial, const void* __restrict__ qa, int qa_f32,
                               const zi_bf16* __restrict__ c_cache, const zi_bf16* __restrict__ kr_cache,
                               const int32_t* __restrict__ entry_start, const int32_t* __restrict__ entry_len,
                               const int32_t* __restrict__ entry_past, const int32_t* __restrict__ block_tables,
                               int entries, int max_pages, int num_pages, int heads, int rank, int rot, int page_size,
                               int window, float scale, int chunk_keys, int total_rows) {
-    constexpr int ROWS = SPLIT ? 16 : WAVES * 16, OT = SPLIT ? (NT + WAVES - 1) / WAVES : NT, KD = KS * 32, KP = KD + LA_PAD, RD = NT * 16, CP = LA_BK + LA_PAD;
-    __shared__ __attribute__((aligned(16))) uint16_t krow[LA_BK * KP];
-    __shared__ __attribute__((aligned(16))) uint16_t ct[RD * CP];
+    constexpr int ROWS = SPLIT ? 16 : WAVES * 16, OT = SPLIT ? (NT + WAVES - 1) / WAVES : NT;
+    constexpr int P = KS * 4;                                  // 16-byte pieces of a staged key
+    constexpr int KI = LA_BK * P / (WAVES * ZI_WAVE);          // load instructions a wavefront issues per block
+    static_assert(P % 8 == 0 && (P * 16) % 256 == 128 && KI * WAVES * ZI_WAVE == LA_BK * P, "whole loads, rows half the banks apart");
+    __shared__ __attribute__((aligned(16))) la_u32x4_t buf_a[LA_BK * P];
+    __shared__ __attribute__((aligned(16))) la_u32x4_t buf_b[LA_BK * P];
     int tile = blockIdx.x, e = 0;
     for (; e < entries; ++e) {
         const int tiles = (entry_len[e] * heads + ROWS - 1) / ROWS;
@@ -75,29 +87,33 @@ latent_attention_cores_kernel(float* __restrict__ out, float* __restrict__ parti
         if (k_lo + chunk_keys - 1 < k_hi) k_hi = k_lo + chunk_keys - 1;
     }
 
-    // this lane's row
-    const int row = row0 + (SPLIT ? 0 : wave * 16) + r;
+    // this lane's row; the keys that all rows of the wavefront see are [all_lo, all_hi]
+    const int wave_row0 = row0 + (SPLIT ? 0 : wave * 16);
+    const int row = wave_row0 + r;
     const bool row_ok = row < erows;
     const int rc = row_ok ? row : last_row;
     const int tok = start + rc / heads, head = rc % heads, pos = past + rc / heads;
     const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int wave_last = wave_row0 + 15 < last_row ? wave_row0 + 15 : last_row;
+    const int all_hi = past + (wave_row0 < last_row ? wave_row0 : last_row) / heads, all_pos = past + wave_last / heads;
+    const int all_lo = (window > 0 && all_pos - window + 1 > 0) ? all_pos - window + 1 : 0;
     const int64_t grow = (int64_t)tok * heads + head;
 
     la_pack q[KS];
-    {
-        const float* qr = qa + grow * qw;
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks) {
-            const int d = ks * 32 + 8 * j;
-            if (d < qw) {      // rank + rot is a multiple of 8: a piece of eight lies inside or outside
-                const float4 a = *reinterpret_cast<const float4*>(qr + d), b = *reinterpret_cast<const float4*>(qr + d + 4);
-                q[ks].w[0] = zi_pack_bf16x2(a.x, a.y);
-                q[ks].w[1] = zi_pack_bf16x2(a.z, a.w);
-                q[ks].w[2] = zi_pack_bf16x2(b.x, b.y);
-                q[ks].w[3] = zi_pack_bf16x2(b.z, b.w);
-            } else {
-                q[ks].u = (la_u32x4_t){0u, 0u, 0u, 0u};
-            }
+    for (int ks = 0; ks < KS; ++ks) {
+        const int d = ks * 32 + 8 * j;
+        q[ks].u = (la_u32x4_t){0u, 0u, 0u, 0u};
+        if (d >= qw) continue;      // rank + rot is a multiple of 8: a piece of eight lies inside or outside
+        if (qa_f32) {
+            const float* qr = (const float*)qa + grow * qw + d;
+            const float4 a = *reinterpret_cast<const float4*>(qr), b = *reinterpret_cast<const float4*>(qr + 4);
+            q[ks].w[0] = zi_pack_bf16x2(a.x, a.y);
+            q[ks].w[1] = zi_pack_bf16x2(a.z, a.w);
+            q[ks].w[2] = zi_pack_bf16x2(b.x, b.y);
+            q[ks].w[3] = zi_pack_bf16x2(b.z, b.w);
+        } else {
+            q[ks].u = *reinterpret_cast<const la_u32x4_t*>((const zi_bf16*)qa + grow * qw + d);
         }
     }
 
@@ -106,47 +122,36 @@ latent_attention_cores_kernel(float* __restrict__ out, float* __restrict__ parti
 #pragma unroll
     for (int t = 0; t < OT; ++t) o[t] = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
 
-    constexpr int G = KD / 8;      // pieces of eight of a staged key
-    for (int kb = k_lo; kb <= k_hi; kb += LA_BK) {
-        __syncthreads();
-        // requests in batches of LA_BATCH a thread, all of a batch before the first is put into LDS
-        for (int i0 = threadIdx.x; i0 < LA_BK * G; i0 += WAVES * ZI_WAVE * LA_BATCH) {
-            la_pack val[LA_BATCH];
+    // the place in the pool of key kb + lane % 32, or -1: past the end, or a page that is not held
+    auto places = [&](int kb) {
+        const int kp = kb + (lane & (LA_BK - 1)), kc = kp <= k_hi ? kp : k_hi;
+        const int pi = kc / page_size;
+        const int page = bt[pi < max_pages ? pi : max_pages - 1];
+        return (kp <= k_hi && (unsigned)page < (unsigned)num_pages) ? page * page_size + kc % page_size : -1;
+    };
+    auto issue = [&](int slots, la_u32x4_t* dst) {
+        int ln = lane;      // (what a lane loads is worked out anew every block: kept, it takes the registers of the sums)
+        asm volatile("" : "+v"(ln));
 #pragma unroll
-            for (int u = 0; u < LA_BATCH; ++u) {
-                const int i = i0 + u * WAVES * ZI_WAVE;
-                const int key = i % LA_BK, d = ((i / LA_BK) % G) * 8, kp = kb + key;      // neighbouring lanes, neighbouring keys
-                // addresses are clamped, not guarded (a load under a branch would make every load before it
-                // wait), and what was read for a place that does not exist is masked
-                const bool want = i < LA_BK * G && kp <= k_hi && d < qw;
-                const int kc = kp <= k_hi ? kp : k_hi, dc = d < qw ? d : 0;
-                const int pi = kc / page_size;
-                const int page = bt[pi < max_pages ? pi : max_pages - 1];
-                const bool held = (unsigned)page < (unsigned)num_pages;
-                const int64_t slot = (int64_t)(held ? page : 0) * page_size + kc % page_size;
-                const zi_bf16* src = dc < rank ? c_cache + slot * rank + dc : kr_cache + slot * rot + (dc - rank);
-                const unsigned mask = 0u - (unsigned)(want && held);
-                val[u].u = *reinterpret_cast<const la_u32x4_t*>(src) & mask;
-            }
-#pragma unroll
-            for (int u = 0; u < LA_BATCH; ++u) {
-                const int i = i0 + u * WAVES * ZI_WAVE;
-                if (i >= LA_BK * G) break;
-                const int key = i % LA_BK, d = (i / LA_BK) * 8;
-                *reinterpret_cast<la_u32x4_t*>(&krow[key * KP + d]) = val[u].u;
-                if (d < RD) {
-                    const unsigned keep = d < rank ? 0xffffffffu : 0u;      // the key parts are no values
-#pragma unroll
-                    for (int x = 0; x < 4; ++x) {
-                        const unsigned w = val[u].w[x] & keep;
-                        ct[(d + 2 * x) * CP + key] = (uint16_t)(w & 0xffffu);
-                        ct[(d + 2 * x + 1) * CP + key] = (uint16_t)(w >> 16);
-                    }
-                }
-            }
+        for (int i = 0; i < KI; ++i) {
+            const int L = (wave * KI + i) * ZI_WAVE + ln, key = L / P, d = ((L % P) ^ ((key >> 1) & 7)) * 8;
+            const int slot = __shfl(slots, key, ZI_WAVE);
+            const zi_bf16* src = d < rank ? c_cache + (int64_t)slot * rank + d : kr_cache + (int64_t)slot * rot + (d - rank);
+            if (slot < 0 || d >= qw) src = reinterpret_cast<const zi_bf16*>(la_zero16);
+            __builtin_amdgcn_global_load_lds(src, dst + (wave * KI + i) * ZI_WAVE, 16, 0, 0);
         }
-        __syncthreads();
+    };
+    // where this lane reads in a buffer, in bytes: the keys' rows (k-steps even and odd), and four keys x sixteen dims
+    const int sw = (r >> 1) & 7;      // of rows r and 16 + r
+    const int s_even = (r * P + (j ^ sw)) * 16, s_odd = (r * P + ((4 + j) ^ sw)) * 16;
+    const int vrow = 4 * j + (r >> 2), vsw = (vrow >> 1) & 7;
+    int v_at[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) v_at[t] = (vrow * P + ((t * 2 + ((r & 3) >> 1)) ^ vsw)) * 16 + (r & 1) * 8;
+    const float scale2 = scale * LA_LOG2E;
 
+    auto work = [&](int kb, const la_u32x4_t* buf) {
+        const char* base = reinterpret_cast<const char*>(buf);
         la_f32x4_t s[2];
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
@@ -154,103 +159,161 @@ latent_attention_cores_kernel(float* __restrict__ out, float* __restrict__ parti
 #pragma unroll
             for (int ks = 0; ks < KS; ++ks) {
                 la_pack a;
-                a.u = *reinterpret_cast<const la_u32x4_t*>(&krow[(h * 16 + r) * KP + ks * 32 + 8 * j]);
+                a.u = *reinterpret_cast<const la_u32x4_t*>(base + ((ks & 1) ? s_odd : s_even) + h * (16 * P * 16) + (ks / 2) * 128);
                 s[h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, q[ks].b, s[h], 0, 0, 0);
             }
         }
-        // lane (r, j) holds, of row r, the keys kb + 16 h + 4 j + x
-        bool ok[2][4];
+        // lane (r, j) holds, of row r, the keys kb + 16 h + 4 j + x; in base-2 units from here on
         float mb = LA_EMPTY;
+        const bool whole = kb >= all_lo && kb + LA_BK - 1 <= all_hi && kb + LA_BK - 1 <= k_hi;
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
             for (int x = 0; x < 4; ++x) {
                 const int kp = kb + 16 * h + 4 * j + x;
-                ok[h][x] = row_ok && kp >= lo && kp <= pos && kp <= k_hi;
-                s[h][x] *= scale;
-                if (ok[h][x]) mb = fmaxf(mb, s[h][x]);
+                const bool seen = whole || (row_ok && kp >= lo && kp <= pos && kp <= k_hi);
+                s[h][x] = seen ? s[h][x] * scale2 : -INFINITY;
+                mb = fmaxf(mb, s[h][x]);
             }
         mb = fmaxf(mb, __shfl_xor(mb, 16, ZI_WAVE));
         mb = fmaxf(mb, __shfl_xor(mb, 32, ZI_WAVE));
-        const float m_new = fmaxf(m, mb);
-        const float corr = expf(m - m_new);
-        float p[2][4], sum = 0.f;
+        const float m_new = fmaxf(m, mb);      // (never below LA_EMPTY, so a key that is not seen weighs 2^-inf = 0)
+        const float corr = __builtin_amdgcn_exp2f(m - m_new);
+        float sum = 0.f;
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
             for (int x = 0; x < 4; ++x) {
-                p[h][x] = ok[h][x] ? expf(s[h][x] - m_new) : 0.f;
-                sum += p[h][x];
+                s[h][x] = __builtin_amdgcn_exp2f(s[h][x] - m_new);
+                sum += s[h][x];
             }
-        sum += __shfl_xor(sum, 16, ZI_WAVE);
-        sum += __shfl_xor(sum, 32, ZI_WAVE);
-        l = l * corr + sum;
+        l = l * corr + sum;      // this lane's keys; the row's four lanes are added up at the end
         m = m_new;
         la_pack pb;
-        pb.w[0] = zi_pack_bf16x2(p[0][0], p[0][1]);
-        pb.w[1] = zi_pack_bf16x2(p[0][2], p[0][3]);
-        pb.w[2] = zi_pack_bf16x2(p[1][0], p[1][1]);
-        pb.w[3] = zi_pack_bf16x2(p[1][2], p[1][3]);
+        pb.w[0] = zi_pack_bf16x2(s[0][0], s[0][1]);
+        pb.w[1] = zi_pack_bf16x2(s[0][2], s[0][3]);
+        pb.w[2] = zi_pack_bf16x2(s[1][0], s[1][1]);
+        pb.w[3] = zi_pack_bf16x2(s[1][2], s[1][3]);
+        if (__any(corr != 1.f)) {      // the running maximum seldom moves after the first blocks
+#pragma unroll
+            for (int tq = 0; tq < OT; ++tq) o[tq] *= corr;
+        }
 #pragma unroll
         for (int tq = 0; tq < OT; ++tq) {
-            const int t = SPLIT ? tq * WAVES + wave : tq;
-            if (t * 16 < rank) {
-                o[tq] *= corr;
+            if (SPLIT) {
+                const int t = tq * WAVES + wave;
+                if (t * 16 < rank) {
+                    const char* at = base + (vrow * P + ((t * 2 + ((r & 3) >> 1)) ^ vsw)) * 16 + (r & 1) * 8;
+                    la_pack a;
+                    a.h[0] = la_read_transposed(at);
+                    a.h[1] = la_read_transposed(at + 16 * P * 16);
+                    o[tq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, pb.b, o[tq], 0, 0, 0);
+                }
+            } else if (tq * 16 < rank) {
+                const char* at = base + v_at[tq & 3] + (tq / 4) * 128;
                 la_pack a;
-                a.h[0] = *reinterpret_cast<const la_u32x2_t*>(&ct[(t * 16 + r) * CP + 4 * j]);
-                a.h[1] = *reinterpret_cast<const la_u32x2_t*>(&ct[(t * 16 + r) * CP + 16 + 4 * j]);
+                a.h[0] = la_read_transposed(at);
+                a.h[1] = la_read_transposed(at + 16 * P * 16);
                 o[tq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, pb.b, o[tq], 0, 0, 0);
             }
         }
-    }
-    // lane (r, j) holds, of row r, the dims 16 t + 4 j + x
-    if (!row_ok) return;
-    if (gridDim.y == 1) {
-        const float inv = 1.f / l;
-        float* orow = out + grow * rank;
-#pragma unroll
-        for (int tq = 0; tq < OT; ++tq)
-#pragma unroll
-            for (int x = 0; x < 4; ++x) {
-                const int d = 16 * (SPLIT ? tq * WAVES + wave : tq) + 4 * j + x;
-                if (d < rank) orow[d] = o[tq][x] * inv;
+    };
+    // Two blocks a turn, buffer a then b.  At each barrier the block about to be worked on has arrived (the compiler
+    // waits for all loads into LDS before a barrier) and everyone has finished with the other buffer.
+    if (k_lo <= k_hi) {
+        issue(places(k_lo), buf_a);
+        int next = places(k_lo + LA_BK);
+        int kb = k_lo;
+        while (true) {
+            __syncthreads();
+            if (kb + LA_BK <= k_hi) {
+                issue(next, buf_b);
+                next = places(kb + 2 * LA_BK);
             }
-    } else {
-        float* prow = partial + ((int64_t)blockIdx.y * total_rows + grow) * (rank + 2);
-        if (j == 0 && (!SPLIT || wave == 0)) {
-            prow[0] = m;
-            prow[1] = l;
+            work(kb, buf_a);
+            if (kb + LA_BK > k_hi) break;
+            kb += LA_BK;
+            __syncthreads();
+            if (kb + LA_BK <= k_hi) {
+                issue(next, buf_a);
+                next = places(kb + 2 * LA_BK);
+            }
+            work(kb, buf_b);
+            if (kb + LA_BK > k_hi) break;
+            kb += LA_BK;
         }
+    }
+    l += __shfl_xor(l, 16, ZI_WAVE);
+    l += __shfl_xor(l, 32, ZI_WAVE);
+    // lane (r, j) holds, of row r, the dims 16 t + 4 j + x (rank is a multiple of 8: four dims lie inside or outside)
+    if (!row_ok) return;
+    const bool parts = gridDim.y > 1;
+    const float inv = parts ? 1.f : 1.f / l;
+    const int64_t prow = ((int64_t)blockIdx.y * total_rows + grow) * (rank + 4);      // maximum, sum, two unused, then O
+    if (parts && j == 0 && (!SPLIT || wave == 0)) {
+        partial[prow] = m;
+        partial[prow + 1] = l;
+    }
 #pragma unroll
-        for (int tq = 0; tq < OT; ++tq)
-#pragma unroll
-            for (int x = 0; x < 4; ++x) {
-                const int d = 16 * (SPLIT ? tq * WAVES + wave : tq) + 4 * j + x;
-                if (d < rank) prow[2 + d] = o[tq][x];
-            }
+    for (int tq = 0; tq < OT; ++tq) {
+        const int d = 16 * (SPLIT ? tq * WAVES + wave : tq) + 4 * j;
+        if (d >= rank) continue;
+        const la_f32x4_t v = o[tq] * inv;
+        if (parts) {
+            *reinterpret_cast<la_f32x4_t*>(partial + prow + 4 + d) = v;
+        } else if (out_f32) {
+            *reinterpret_cast<la_f32x4_t*>((float*)out + grow * rank + d) = v;
+        } else {
+            uint2 w;
+            w.x = zi_pack_bf16x2(v[0], v[1]);
+            w.y = zi_pack_bf16x2(v[2], v[3]);
+            *reinterpret_cast<uint2*>((zi_bf16*)out + grow * rank + d) = w;
+        }
     }
 }
 
-// out[row] = sum_c O_c exp(m_c - M) / sum_c l_c exp(m_c - M), chunks in rising order.
-__global__ void __launch_bounds__(256)
-latent_attention_merge_kernel(float* __restrict__ out, const float* __restrict__ partial, int chunks, int total_rows,
+// out[row] = sum_c O_c 2^(m_c - M) / sum_c l_c 2^(m_c - M), chunks in rising order.  A thread owns four dims; the loads of
+// eight chunks travel together.
+#define LA_MAX_CHUNKS 4096
+__global__ void __launch_bounds__(128)
+latent_attention_merge_kernel(void* __restrict__ out, int out_f32, const float* __restrict__ partial, int chunks, int total_rows,
                               int rank) {
-    const int64_t row = blockIdx.x;
+    __shared__ float weight[128];
+    const int64_t row = blockIdx.x, stride = (int64_t)total_rows * (rank + 4);
+    const float* p0 = partial + row * (rank + 4);
+    const int tid = threadIdx.x, lane = tid & (ZI_WAVE - 1);
+    const int d = tid * 4;
+    // every wavefront makes the maximum and the sum: lane c takes chunks c, c + 64, ...
     float M = LA_EMPTY;
-    for (int c = 0; c < chunks; ++c) M = fmaxf(M, partial[((int64_t)c * total_rows + row) * (rank + 2)]);
+    for (int c = lane; c < chunks; c += ZI_WAVE) M = fmaxf(M, p0[c * stride]);
+    M = zi_wave_max(M);
     float L = 0.f;
-    for (int c = 0; c < chunks; ++c) {
-        const float* p = partial + ((int64_t)c * total_rows + row) * (rank + 2);
-        L += p[1] * expf(p[0] - M);
-    }
-    const float inv = 1.f / L;
-    for (int d = threadIdx.x; d < rank; d += blockDim.x) {
-        float acc = 0.f;
-        for (int c = 0; c < chunks; ++c) {
-            const float* p = partial + ((int64_t)c * total_rows + row) * (rank + 2);
-            acc += p[2 + d] * expf(p[0] - M);
+    for (int c = lane; c < chunks; c += ZI_WAVE) L += p0[c * stride + 1] * __builtin_amdgcn_exp2f(p0[c * stride] - M);
+    const float inv = 1.f / zi_wave_sum(L);
+    la_f32x4_t acc = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < chunks; c0 += 128) {
+        __syncthreads();
+        if (c0 + tid < chunks) weight[tid] = __builtin_amdgcn_exp2f(p0[(c0 + tid) * stride] - M);
+        __syncthreads();
+        const int count = chunks - c0 < 128 ? chunks - c0 : 128;
+        if (d >= rank) continue;
+        for (int c = 0; c < count; c += 8) {
+            la_f32x4_t v[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const la_f32x4_t*>(p0 + (c0 + (c + u < count ? c + u : c)) * stride + 4 + d);
+#pragma unroll
+            for (int u = 0; u < 8; ++u) acc += v[u] * (c + u < count ? weight[c + u] : 0.f);
         }
-        out[row * rank + d] = acc * inv;
+    }
+    if (d >= rank) return;
+    acc *= inv;
+    if (out_f32) {
+        *reinterpret_cast<la_f32x4_t*>((float*)out + row * rank + d) = acc;
+    } else {
+        uint2 w;
+        w.x = zi_pack_bf16x2(acc[0], acc[1]);
+        w.y = zi_pack_bf16x2(acc[2], acc[3]);
+        *reinterpret_cast<uint2*>((zi_bf16*)out + row * rank + d) = w;
     }
 }
 
@@ -264,7 +327,8 @@ extern "C" int zi_latent_attention_cores_tiles(int n, int entries, int heads, in
     return (int)(((int64_t)n * heads + rows - 1) / rows) + entries;
 }
 
-extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t partial_floats, const float* qa,
+// qa [n][heads][rank + rot] and out [n][heads][rank], each float32 or bfloat16; partial: chunks * n * heads * (rank + 4) floats.
+extern "C" int zi_latent_attention_cores(void* out, int out_dt, float* partial, int64_t partial_floats, const void* qa, int qa_dt,
                                          const void* c_cache, const void* kr_cache, const int32_t* entry_start,
                                          const int32_t* entry_len, const int32_t* entry_past, const int32_t* block_tables,
                                          int entries, int n, int max_pages, int num_pages, int heads, int rank, int rot,
@@ -272,10 +336,13 @@ extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t par
                                          hipStream_t stream) {
     ZI_REQUIRE(zi_latent_attention_cores_supported(ZI_BF16, rank, rot), "latent_attention_cores: rank %d, rot %d not taken",
                rank, rot);
-    ZI_REQUIRE(n >= 0 && entries > 0 && heads > 0 && page_size > 0 && max_pages > 0 && num_pages > 0 && window >= 0,
-               "latent_attention_cores: bad sizes");
+    ZI_REQUIRE(n >= 0 && entries > 0 && heads > 0 && page_size > 0 && max_pages > 0 && num_pages > 0 && window >= 0 &&
+                   (int64_t)num_pages * page_size < (1ll << 31), "latent_attention_cores: bad sizes");
+    ZI_REQUIRE((out_dt == ZI_F32 || out_dt == ZI_BF16) && (qa_dt == ZI_F32 || qa_dt == ZI_BF16) && ((uintptr_t)qa % 16) == 0 &&
+                   ((uintptr_t)out % 16) == 0 && ((uintptr_t)partial % 16) == 0 && ((uintptr_t)c_cache % 16) == 0 && ((uintptr_t)kr_cache % 16) == 0,
+               "latent_attention_cores: unknown types, or addresses that are not aligned to 16 bytes");
     ZI_REQUIRE(waves == 1 || waves == 4, "latent_attention_cores: 1 or 4 wavefronts a workgroup");
-    ZI_REQUIRE(chunks >= 1 && chunks <= 65535 && (chunks == 1) == (chunk_keys == 0) && chunk_keys >= 0,
+    ZI_REQUIRE(chunks >= 1 && chunks <= LA_MAX_CHUNKS && (chunks == 1) == (chunk_keys == 0) && chunk_keys >= 0,
                "latent_attention_cores: bad cut (%d chunks of %d keys)", chunks, chunk_keys);
     if (chunks > 1) {
         // every key a tile's rows see lies in one of the chunks
@@ -283,7 +350,7 @@ extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t par
         // (without a window the caller sees to it that the chunks reach the last key of every entry)
         ZI_REQUIRE(window == 0 || (int64_t)chunks * chunk_keys >= (int64_t)window + tokens_in_tile,
                    "latent_attention_cores: %d chunks of %d keys do not cover a window of %d", chunks, chunk_keys, window);
-        ZI_REQUIRE(partial && partial_floats >= (int64_t)chunks * n * heads * (rank + 2),
+        ZI_REQUIRE(partial && partial_floats >= (int64_t)chunks * n * heads * (rank + 4),
                    "latent_attention_cores: the workspace is too small");
     }
     if (n == 0) return 0;
@@ -291,8 +358,8 @@ extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t par
     const dim3 grid(zi_latent_attention_cores_tiles(n, entries, heads, waves), chunks);
 #define ZI_LA_LAUNCH(W, NT, KS)                                                                                       \
     latent_attention_cores_kernel<4, NT, KS, W == 1><<<grid, 4 * ZI_WAVE, 0, stream>>>(                                \
-        out, partial, qa, (const zi_bf16*)c_cache, (const zi_bf16*)kr_cache, entry_start, entry_len, entry_past,       \
-        block_tables, entries, max_pages, num_pages, heads, rank, rot, page_size, window, scale, chunk_keys, total_rows)
+        out, out_dt == ZI_F32, partial, qa, qa_dt == ZI_F32, (const zi_bf16*)c_cache, (const zi_bf16*)kr_cache, entry_start, entry_len, \
+        entry_past, block_tables, entries, max_pages, num_pages, heads, rank, rot, page_size, window, scale, chunk_keys, total_rows)
 #define ZI_LA_SIZES(W)                                                       \
     do {                                                                     \
         if (rank <= 128 && rank + rot <= 192) ZI_LA_LAUNCH(W, 8, 6);         \
@@ -305,68 +372,180 @@ extern "C" int zi_latent_attention_cores(float* out, float* partial, int64_t par
 #undef ZI_LA_LAUNCH
     int rc = zi_check_launch("latent_attention_cores");
     if (rc != 0 || chunks == 1) return rc;
-    latent_attention_merge_kernel<<<total_rows, 256, 0, stream>>>(out, partial, chunks, total_rows, rank);
+    latent_attention_merge_kernel<<<total_rows, 128, 0, stream>>>(out, out_dt == ZI_F32, partial, chunks, total_rows, rank);
     return zi_check_launch("latent_attention_merge");
 }
 
 // ---- a product per head on the matrix cores ---------------------------------------------------------------------
-// out[t][h][i] = sum_k w[h][i][k] x[t][h][k]: w bfloat16 [heads][N][K] (k runs fastest), x float32 with row stride
-// ldx and head stride xs (rounded to bfloat16 as it is loaded), out float32 or bfloat16 with row stride ldo and head
-// stride os.  One wavefront per (16 tokens, head, 16 outputs); operands straight from memory.  It carries the
-// queries through W_uk (w = W_uk of the head, transposed at load) and the attended latents through W_uv.
+// out[t][h][i] = sum_k w[h][i][k] x[t][h][k]: w bfloat16 [heads][N][K] (k runs fastest), x float32 (rounded to bfloat16 as
+// it is loaded) or bfloat16 with row stride ldx and head stride xs, out float32 or bfloat16 with row stride ldo and head stride
+// os.  It carries the queries through W_uk (w = W_uk of the head, transposed at load) and the attended latents through W_uv.
 // GATED: out *= sigmoid(gate[t][h * N + i]), the gate bfloat16 or the sum of `splits` float32 terms.
+// Operands straight from memory.  Many tokens: a wavefront owns 32 tokens x 64 outputs (every operand serves several
+// products), the four wavefronts of a workgroup take neighbouring tokens of one head.  Few: 16 x 16, k dealt over the
+// four wavefronts in runs of 32 and added up in their order.
 struct LaGate {
     const void* g;
     int f32, splits;
     int64_t ld, stride;
 };
 
-template <typename TO, bool GATED>
-__global__ void __launch_bounds__(ZI_WAVE)
-headwise_linear_cores_kernel(TO* __restrict__ out, int64_t ldo, int os, const float* __restrict__ x, int64_t ldx, int xs,
-                             const zi_bf16* __restrict__ w, int n, int N, int K, LaGate gt) {
-    const int t0 = blockIdx.x * 16, h = blockIdx.y, n0 = blockIdx.z * 16;
-    const int lane = threadIdx.x, r = lane % 16, j = lane / 16;
-    const zi_bf16* wrow = w + ((int64_t)h * N + (n0 + r < N ? n0 + r : N - 1)) * K;
-    const float* xrow = x + (int64_t)(t0 + r < n ? t0 + r : n - 1) * ldx + (int64_t)h * xs;
-    la_f32x4_t acc = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
-    float gate[4];
-    if constexpr (GATED) {      // asked for before the product, used after it
-        const int64_t at = (int64_t)(t0 + r < n ? t0 + r : n - 1) * gt.ld + (int64_t)h * N;
+__device__ __forceinline__ la_pack la_load8(const float* p) {
+    const float4 lo = *reinterpret_cast<const float4*>(p), hi = *reinterpret_cast<const float4*>(p + 4);
+    la_pack b;
+    b.w[0] = zi_pack_bf16x2(lo.x, lo.y);
+    b.w[1] = zi_pack_bf16x2(lo.z, lo.w);
+    b.w[2] = zi_pack_bf16x2(hi.x, hi.y);
+    b.w[3] = zi_pack_bf16x2(hi.z, hi.w);
+    return b;
+}
+__device__ __forceinline__ la_pack la_load8(const zi_bf16* p) {
+    la_pack b;
+    b.u = *reinterpret_cast<const la_u32x4_t*>(p);
+    return b;
+}
+
+// four gates of one token and head, columns n0 .. n0 + 3 (clamped to the head)
+__device__ __forceinline__ la_f32x4_t la_gates(const LaGate& gt, int64_t t, int h, int n0, int N) {
+    const int64_t at = t * gt.ld + (int64_t)h * N;
+    la_f32x4_t g;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int col = n0 + 4 * j + i < N ? n0 + 4 * j + i : N - 1;
-            gate[i] = gt.f32 ? ((const float*)gt.g)[at + col] : zi_load((const zi_bf16*)gt.g + at + col);
-            for (int s = 1; s < gt.splits; ++s) gate[i] += ((const float*)gt.g)[s * gt.stride + at + col];
+    for (int i = 0; i < 4; ++i) {
+        const int col = n0 + i < N ? n0 + i : N - 1;
+        g[i] = gt.f32 ? ((const float*)gt.g)[at + col] : zi_load((const zi_bf16*)gt.g + at + col);
+    }
+    if (gt.f32) {
+        int s = 1;
+        for (; s + 3 < gt.splits; s += 4) {      // four terms in flight, added in their order
+            la_f32x4_t v[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) v[u][i] = ((const float*)gt.g)[(s + u) * gt.stride + at + (n0 + i < N ? n0 + i : N - 1)];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) g += v[u];
         }
+        for (; s < gt.splits; ++s)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) g[i] += ((const float*)gt.g)[s * gt.stride + at + (n0 + i < N ? n0 + i : N - 1)];
     }
-#pragma unroll 4
-    for (int k0 = 0; k0 < K; k0 += 32) {
-        const int k = k0 + 8 * j;
-        const bool in = k < K;      // K is a multiple of 8
-        const int kc = in ? k : 0;
-        const unsigned mask = 0u - (unsigned)in;
-        la_pack a, b;
-        a.u = *reinterpret_cast<const la_u32x4_t*>(wrow + kc) & mask;
-        const float4 lo = *reinterpret_cast<const float4*>(xrow + kc), hi = *reinterpret_cast<const float4*>(xrow + kc + 4);
-        b.w[0] = zi_pack_bf16x2(lo.x, lo.y) & mask;
-        b.w[1] = zi_pack_bf16x2(lo.z, lo.w) & mask;
-        b.w[2] = zi_pack_bf16x2(hi.x, hi.y) & mask;
-        b.w[3] = zi_pack_bf16x2(hi.z, hi.w) & mask;
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b.b, acc, 0, 0, 0);
-    }
-    if (t0 + r >= n) return;
-    TO* orow = out + (int64_t)(t0 + r) * ldo + (int64_t)h * os + n0 + 4 * j;
+    return g;
+}
+template <typename TO>
+__device__ __forceinline__ void la_store4(TO* orow, la_f32x4_t v, int left) {
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-        if (n0 + 4 * j + i < N) zi_store(orow + i, GATED ? acc[i] / (1.f + expf(-gate[i])) : acc[i]);
+        if (i < left) zi_store(orow + i, v[i]);
+}
+__device__ __forceinline__ void la_gate4(la_f32x4_t& v, const la_f32x4_t& g) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = v[i] / (1.f + expf(-g[i]));
 }
 
+template <typename TX, typename TO, bool GATED>
+__global__ void __launch_bounds__(4 * ZI_WAVE)
+headwise_linear_few_kernel(TO* __restrict__ out, int64_t ldo, int os, const TX* __restrict__ x, int64_t ldx, int xs,
+                           const zi_bf16* __restrict__ w, int n, int N, int K, LaGate gt) {
+    __shared__ la_f32x4_t part[3][ZI_WAVE];
+    const int t0 = blockIdx.x * 16, h = blockIdx.y, n0 = blockIdx.z * 16;
+    const int lane = threadIdx.x % ZI_WAVE, wave = threadIdx.x / ZI_WAVE, r = lane % 16, j = lane / 16;
+    const zi_bf16* wrow = w + ((int64_t)h * N + (n0 + r < N ? n0 + r : N - 1)) * K;
+    const int64_t t = t0 + r < n ? t0 + r : n - 1;
+    const TX* xrow = x + t * ldx + (int64_t)h * xs;
+    la_f32x4_t acc = (la_f32x4_t){0.f, 0.f, 0.f, 0.f}, gate = acc;
+    if (GATED && wave == 0) gate = la_gates(gt, t, h, n0 + 4 * j, N);      // asked for before the product, used after it
+#pragma unroll 4
+    for (int k0 = wave * 32; k0 < K; k0 += 128) {
+        const int k = k0 + 8 * j, kc = k < K ? k : 0;      // K is a multiple of 8
+        const unsigned mask = 0u - (unsigned)(k < K);
+        la_pack a = la_load8(wrow + kc), b = la_load8(xrow + kc);
+        a.u &= mask;
+        b.u &= mask;
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b.b, acc, 0, 0, 0);
+    }
+    if (wave > 0) part[wave - 1][lane] = acc;
+    __syncthreads();
+    if (wave > 0) return;
+#pragma unroll
+    for (int u = 0; u < 3; ++u) acc += part[u][lane];
+    if (t0 + r >= n || n0 + 4 * j >= N) return;
+    if constexpr (GATED) la_gate4(acc, gate);
+    la_store4(out + t * ldo + (int64_t)h * os + n0 + 4 * j, acc, N - n0 - 4 * j);
+}
+
+template <typename TX, typename TO, bool GATED>
+__global__ void __launch_bounds__(4 * ZI_WAVE)
+headwise_linear_many_kernel(TO* __restrict__ out, int64_t ldo, int os, const TX* __restrict__ x, int64_t ldx, int xs,
+                            const zi_bf16* __restrict__ w, int n, int N, int K, LaGate gt) {
+    constexpr int TM = 2, TN = 4;      // tiles of 16 tokens and of 16 outputs
+    const int lane = threadIdx.x % ZI_WAVE, wave = threadIdx.x / ZI_WAVE, r = lane % 16, j = lane / 16;
+    const int t0 = (blockIdx.x * 4 + wave) * (16 * TM), h = blockIdx.y, n0 = blockIdx.z * (16 * TN);
+    if (t0 >= n) return;
+    const zi_bf16* wrow[TN];
+    const TX* xrow[TM];
+#pragma unroll
+    for (int c = 0; c < TN; ++c) {
+        const int i = n0 + c * 16 + r;
+        wrow[c] = w + ((int64_t)h * N + (i < N ? i : N - 1)) * K;
+    }
+#pragma unroll
+    for (int c = 0; c < TM; ++c) {
+        const int t = t0 + c * 16 + r;
+        xrow[c] = x + (int64_t)(t < n ? t : n - 1) * ldx + (int64_t)h * xs;
+    }
+    la_f32x4_t acc[TM][TN];
+#pragma unroll
+    for (int a = 0; a < TM; ++a)
+#pragma unroll
+        for (int c = 0; c < TN; ++c) acc[a][c] = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+    for (int k0 = 0; k0 < K; k0 += 32) {
+        const int k = k0 + 8 * j, kc = k < K ? k : 0;
+        const unsigned mask = 0u - (unsigned)(k < K);
+        la_pack a[TN], b[TM];
+#pragma unroll
+        for (int c = 0; c < TN; ++c) a[c] = la_load8(wrow[c] + kc);
+#pragma unroll
+        for (int c = 0; c < TM; ++c) b[c] = la_load8(xrow[c] + kc);
+#pragma unroll
+        for (int c = 0; c < TN; ++c) a[c].u &= mask;
+#pragma unroll
+        for (int c = 0; c < TM; ++c) b[c].u &= mask;
+#pragma unroll
+        for (int m = 0; m < TM; ++m)
+#pragma unroll
+            for (int c = 0; c < TN; ++c) acc[m][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[c].b, b[m].b, acc[m][c], 0, 0, 0);
+    }
+#pragma unroll
+    for (int m = 0; m < TM; ++m) {
+        const int t = t0 + m * 16 + r;
+        if (t >= n) continue;
+#pragma unroll
+        for (int c = 0; c < TN; ++c) {
+            const int i = n0 + c * 16 + 4 * j;
+            if (i >= N) continue;
+            if constexpr (GATED) la_gate4(acc[m][c], la_gates(gt, t, h, i, N));
+            TO* dst = out + (int64_t)t * ldo + (int64_t)h * os + i;
+            if (sizeof(TO) == 2 && i + 3 < N && ((uintptr_t)dst % 8) == 0) {
+                uint2 p;
+                p.x = zi_pack_bf16x2(acc[m][c][0], acc[m][c][1]);
+                p.y = zi_pack_bf16x2(acc[m][c][2], acc[m][c][3]);
+                *reinterpret_cast<uint2*>(dst) = p;
+            } else {
+                la_store4(dst, acc[m][c], N - i);
+            }
+        }
+    }
+}
+
+// (either storage type of x)
 extern "C" int zi_headwise_linear_supported(int w_dt, int K, int64_t ldx, int xs) {
-    return w_dt == ZI_BF16 && K > 0 && K % 8 == 0 && ldx % 4 == 0 && xs % 4 == 0;
+    return w_dt == ZI_BF16 && K > 0 && K % 8 == 0 && ldx % 8 == 0 && xs % 8 == 0;
 }
 
-extern "C" int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs,
+#define LA_MANY_TOKENS 128      // from this many tokens on the kernel for many
+
+extern "C" int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const void* x, int x_dt, int64_t ldx, int xs,
                                         const void* w, int n, int heads, int N, int K, const void* gate, int g_dt,
                                         int64_t ld_gate, int g_splits, int64_t g_stride, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && heads > 0 && heads <= 65535 && N > 0 && (N + 15) / 16 <= 65535, "headwise_linear: bad sizes");
@@ -377,25 +556,28 @@ extern "C" int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int 
     ZI_REQUIRE(!gate || (ld_gate >= (int64_t)heads * N && g_splits >= 1 && (g_dt == ZI_F32 || (g_dt == ZI_BF16 && g_splits == 1))),
                "headwise_linear: bad gate");
     if (n == 0) return 0;
-    const dim3 grid((n + 15) / 16, heads, (N + 15) / 16);
+    const bool many = n >= LA_MANY_TOKENS;
+    const dim3 grid(many ? (n + 127) / 128 : (n + 15) / 16, heads, many ? (N + 63) / 64 : (N + 15) / 16);
     const LaGate gt = {gate, g_dt == ZI_F32, g_splits, ld_gate, g_stride};
-    ZI_DISPATCH_DTYPE(out_dt, TO, {
-        if (gate)
-            headwise_linear_cores_kernel<TO, true><<<grid, ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, x, ldx, xs, (const zi_bf16*)w, n, N, K, gt);
-        else
-            headwise_linear_cores_kernel<TO, false><<<grid, ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, x, ldx, xs, (const zi_bf16*)w, n, N, K, gt);
-    });
+#define ZI_HW(KERNEL, GATED) KERNEL<TX, TO, GATED><<<grid, 4 * ZI_WAVE, 0, stream>>>((TO*)out, ldo, os, (const TX*)x, ldx, xs, (const zi_bf16*)w, n, N, K, gt)
+    ZI_DISPATCH_DTYPE(x_dt, TX, ZI_DISPATCH_DTYPE(out_dt, TO, {
+        if (many && gate) ZI_HW(headwise_linear_many_kernel, true);
+        else if (many) ZI_HW(headwise_linear_many_kernel, false);
+        else if (gate) ZI_HW(headwise_linear_few_kernel, true);
+        else ZI_HW(headwise_linear_few_kernel, false);
+    }));
+#undef ZI_HW
     return zi_check_launch("headwise_linear");
 }
 
-extern "C" int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs,
+extern "C" int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const void* x, int x_dt, int64_t ldx, int xs,
                                   const void* w, int n, int heads, int N, int K, hipStream_t stream) {
-    return zi_headwise_linear_gated(out, out_dt, ldo, os, x, ldx, xs, w, n, heads, N, K, nullptr, ZI_F32, 0, 1, 0, stream);
+    return zi_headwise_linear_gated(out, out_dt, ldo, os, x, x_dt, ldx, xs, w, n, heads, N, K, nullptr, ZI_F32, 0, 1, 0, stream);
 }
 
 // qa[t][h][rank + ...] = the rotated part of every head's query, turned in neighbouring pairs.
-template <typename T>
-__global__ void latent_query_rot_kernel(float* __restrict__ qa, const T* __restrict__ q, int64_t ldq,
+template <typename T, typename TO>
+__global__ void latent_query_rot_kernel(TO* __restrict__ qa, const T* __restrict__ q, int64_t ldq,
                                         const float* __restrict__ table, int n, int heads, int dim, int rank, int rot) {
     const int half = rot / 2;
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -405,21 +587,21 @@ __global__ void latent_query_rot_kernel(float* __restrict__ qa, const T* __restr
     const T* qr = q + t * ldq + (int64_t)h * (dim + rot) + dim + 2 * p;
     const float u = zi_load(qr), v = zi_load(qr + 1);
     const float c = table[(t * half + p) * 2], s = table[(t * half + p) * 2 + 1];
-    float* o = qa + (t * heads + h) * (rank + rot) + rank + 2 * p;
-    o[0] = u * c - v * s;
-    o[1] = v * c + u * s;
+    TO* o = qa + (t * heads + h) * (rank + rot) + rank + 2 * p;
+    zi_store(o, u * c - v * s);
+    zi_store(o + 1, v * c + u * s);
 }
 
-extern "C" int zi_latent_query_rot(float* qa, const void* q, int dt, int64_t ldq, const float* table, int n, int heads,
+extern "C" int zi_latent_query_rot(void* qa, int qa_dt, const void* q, int dt, int64_t ldq, const float* table, int n, int heads,
                                    int dim, int rank, int rot, hipStream_t stream) {
     ZI_REQUIRE(n >= 0 && heads > 0 && dim > 0 && rank > 0 && rot >= 0 && rot % 2 == 0 && ldq >= (int64_t)heads * (dim + rot),
                "latent_query_rot: bad sizes");
     const int64_t total = (int64_t)n * heads * (rot / 2);
     if (total == 0) return 0;
     ZI_REQUIRE(table, "latent_query_rot: no table of angles");
-    ZI_DISPATCH_DTYPE(dt, T, {
-        latent_query_rot_kernel<T><<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(qa, (const T*)q, ldq, table, n, heads,
-                                                                                         dim, rank, rot);
-    });
+    ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(qa_dt, TO, {
+        latent_query_rot_kernel<T, TO><<<(unsigned)((total + 255) / 256), 256, 0, stream>>>((TO*)qa, (const T*)q, ldq, table, n, heads,
+                                                                                             dim, rank, rot);
+    }));
     return zi_check_launch("latent_query_rot");
 }

@@ -58,7 +58,7 @@ int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* proj, int p_dt
     int n, const void* q_norm, const void* c_norm, int w_dt, float eps, int q_rank, int dkv_at, const float* table,
     const int32_t* slots, void* c_cache, void* kr_cache, int64_t cache_slots, int rank, int rot, hipStream_t stream);
 // latent_cores.hip
-int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs, const void* w,
+int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const void* x, int x_dt, int64_t ldx, int xs, const void* w,
     int n, int heads, int N, int K, const void* gate, int g_dt, int64_t ld_gate, int g_splits, int64_t g_stride,
     hipStream_t stream);
 // attention_prefill.hip
@@ -146,15 +146,15 @@ int zi_latent_attention(float* out, const float* qa, const void* c_cache, const 
     int32_t* tok_index, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* block_tables, int max_pages, int
     num_pages, int heads, int rank, int rot, int page_size, int window, float scale, hipStream_t stream);
 // latent_cores.hip
-int zi_latent_attention_cores(float* out, float* partial, int64_t partial_floats, const float* qa, const void* c_cache,
+int zi_latent_attention_cores(void* out, int out_dt, float* partial, int64_t partial_floats, const void* qa, int qa_dt, const void* c_cache,
     const void* kr_cache, const int32_t* entry_start, const int32_t* entry_len, const int32_t* entry_past, const int32_t*
     block_tables, int entries, int n, int max_pages, int num_pages, int heads, int rank, int rot, int page_size, int
     window, float scale, int waves, int chunk_keys, int chunks, hipStream_t stream);
 // latent_cores.hip
-int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const float* x, int64_t ldx, int xs, const void* w, int
-    n, int heads, int N, int K, hipStream_t stream);
+int zi_headwise_linear(void* out, int out_dt, int64_t ldo, int os, const void* x, int x_dt, int64_t ldx, int xs, const void* w,
+    int n, int heads, int N, int K, hipStream_t stream);
 // latent_cores.hip
-int zi_latent_query_rot(float* qa, const void* q, int dt, int64_t ldq, const float* table, int n, int heads, int dim, int
+int zi_latent_query_rot(void* qa, int qa_dt, const void* q, int dt, int64_t ldq, const float* table, int n, int heads, int dim, int
     rank, int rot, hipStream_t stream);
 // latent.hip
 int zi_latent_value(void* out, int out_dt, int64_t ldo, const float* o, const void* w_uv, int w_dt, int n, int heads,

@@ -20,7 +20,7 @@ from .functional import (add, add_rms_norm, argmax, attention, attention_decode,
                          DECODE_LAYER_SPIN_LIMIT, FEW_ROWS, SUMS_MAX_ROWS)
 from .mixing import (delta_conv_state, delta_prepare, delta_rule, delta_state_floats, gated_act, gated_rms_norm,
                      latent_attention, latent_attention_cores, latent_attention_cores_plan,
-                     latent_attention_cores_supported, latent_attention_cores_workspace, latent_inputs, latent_query, latent_store, latent_value, latent_value_gates,
+                     latent_attention_cores_supported, latent_attention_cores_workspace, latent_inputs, latent_query, latent_query_cores, latent_store, latent_value, latent_value_gates,
                      moe_combine, moe_group, moe_linear,
                      moe_max_tiles, moe_route, moe_tile_rows, rope_pairs)
 from .sublayers import (clamped_glu, clamped_glu_il8, conv_qkv, conv_state_floats, conv_tail, convert, layer_norm, moe_route_top,
@@ -63,6 +63,6 @@ __all__ = [
     "channel_inputs", "channel_state_floats", "delta_channel", "delta_channel_finishes", "input_conv", "lowrank_gates", "norm_input_conv", "norm_input_conv_supported",
     "stream_scale", "attention_decode_merge_gated", "linear_clamped_glu", "clamped_glu_il8",
     "ACTIVATIONS", "activate", "attention_prefill_maps_supported", "difference_heads", "difference_merge", "head_norm_store", "latent_inputs",
-    "latent_value_gates", "stream_mix", "stream_mix_max_streams",
+    "latent_query_cores", "latent_value_gates", "stream_mix", "stream_mix_max_streams",
     "KernelLibraryError", "library_path", "load", "FEW_ROWS", "SUMS_MAX_ROWS",
 ]

@@ -73,12 +73,12 @@ _PROTOTYPES = {
     "zi_latent_store": [P, I, L, I, P, I, F, P, P, P, P, L, I, I, P],
     "zi_latent_query": [P, P, I, L, P, I, P, I, I, I, I, I, P],
     "zi_latent_attention": [P, P, P, P, I, I, P, P, P, P, I, I, I, I, I, I, I, F, P],
-    "zi_latent_attention_cores": [P, P, L, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, F, I, I, I, P],
+    "zi_latent_attention_cores": [P, I, P, L, P, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, F, I, I, I, P],
     "zi_latent_attention_cores_supported": [I, I, I],
     "zi_latent_attention_cores_tiles": [I, I, I, I],
-    "zi_headwise_linear": [P, I, L, I, P, L, I, P, I, I, I, I, P],
+    "zi_headwise_linear": [P, I, L, I, P, I, L, I, P, I, I, I, I, P],
     "zi_headwise_linear_supported": [I, I, L, I],
-    "zi_latent_query_rot": [P, P, I, L, P, I, I, I, I, I, P],
+    "zi_latent_query_rot": [P, I, P, I, L, P, I, I, I, I, I, P],
     "zi_latent_value": [P, I, L, P, P, I, I, I, I, I, P],
     "zi_delta_prepare": [P, P, P, P, L, I, P, P, P, I, P, L, L, P, P, P, I, I, I, I, I, P],
     "zi_delta_conv_state": [P, L, L, P, L, P, P, P, I, I, I, P],
@@ -148,7 +148,7 @@ _PROTOTYPES = {
     "zi_difference_merge": [P, L, P, L, I, P, I, I, I, I, I, F, F, F, P, I, L, I, L, P],
     "zi_activate": [P, I, L, P, I, L, I, L, I, I, I, P],
     "zi_latent_inputs": [P, I, L, P, I, L, I, L, I, P, P, I, F, I, I, P, P, P, P, L, I, I, P],
-    "zi_headwise_linear_gated": [P, I, L, I, P, L, I, P, I, I, I, I, P, I, L, I, L, P],
+    "zi_headwise_linear_gated": [P, I, L, I, P, I, L, I, P, I, I, I, I, P, I, L, I, L, P],
     "zi_tape_record": [P, c_char_p, P, I],
     "zi_tape_record_many": [P, c_char_p, P, P, I],
     "zi_tape_run": [P, P],

@@ -112,9 +112,15 @@ def latent_inputs(proj: torch.Tensor, q_norm: torch.Tensor, eps: float, cq: torc
               _p(kr_cache if c_cache is not None else None), rows, int(rank), int(rot), _stream())
 
 
+def latent_query_cores(w_uk_t: Optional[torch.Tensor], heads: int, dim: int, rot: int, ldq: int = 0) -> bool:
+    """Whether ``latent_query`` runs on the matrix cores (and may leave bfloat16): bfloat16 weights, sizes in eights."""
+    return w_uk_t is not None and w_uk_t.dtype == torch.bfloat16 and w_uk_t.data_ptr() % 16 == 0 \
+        and bool(_lib.load().zi_headwise_linear_supported(1, dim, int(ldq) or heads * (dim + rot), dim + rot))
+
+
 def latent_query(q: torch.Tensor, w_uk: torch.Tensor, table: Optional[torch.Tensor], heads: int, dim: int, rank: int,
                  rot: int, out: torch.Tensor, w_uk_t: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out [n, heads, rank + rot] float32: every head's unrotated query part carried through its block of
+    """out [n, heads, rank + rot] float32 (or, with ``w_uk_t`` where the matrix cores take the sizes, bfloat16): every head's unrotated query part carried through its block of
     ``w_uk`` [heads * dim, rank] (so that it meets latents instead of keys), then its rotated part, turned."""
     _gpu("latent_query", q, w_uk, table, out)
     ldq, width = _rows(q, "latent_query q")
@@ -123,20 +129,21 @@ def latent_query(q: torch.Tensor, w_uk: torch.Tensor, table: Optional[torch.Tens
         raise ValueError(f"latent_query: q must be [n, {heads * (dim + rot)}]")
     if tuple(w_uk.shape) != (heads * dim, rank) or not w_uk.is_contiguous():
         raise ValueError(f"latent_query: w_uk must be a contiguous [{heads * dim}, {rank}] tensor")
-    _f32(out, "latent_query out", (n, heads, rank + rot))
+    if tuple(out.shape) != (n, heads, rank + rot) or not out.is_contiguous():
+        raise ValueError(f"latent_query: out must be a contiguous [n, {heads}, {rank + rot}] tensor")
     if rot:
         _f32(table, "latent_query table", (n, rot // 2, 2))
-    if w_uk_t is not None and q.dtype == torch.float32 and q.data_ptr() % 16 == 0 \
-            and _lib.load().zi_headwise_linear_supported(_code(w_uk_t, "latent_query w_uk_t"), dim, ldq, dim + rot):
+    if w_uk_t is not None and q.data_ptr() % 16 == 0 and latent_query_cores(w_uk_t, heads, dim, rot, ldq):
         # on the matrix cores: the head's block of W_uk, transposed at load, times the unrotated query parts
         if tuple(w_uk_t.shape) != (heads, rank, dim) or not w_uk_t.is_contiguous():
             raise ValueError(f"latent_query: w_uk_t must be a contiguous [{heads}, {rank}, {dim}] tensor")
-        _lib.call("zi_headwise_linear", _p(out), 0, heads * (rank + rot), rank + rot, _p(q), ldq, dim + rot, _p(w_uk_t), n,
-                  heads, rank, dim, _stream())
+        _lib.call("zi_headwise_linear", _p(out), _code(out, "latent_query out"), heads * (rank + rot), rank + rot, _p(q),
+                  _code(q, "latent_query q"), ldq, dim + rot, _p(w_uk_t), n, heads, rank, dim, _stream())
         if rot:
-            _lib.call("zi_latent_query_rot", _p(out), _p(q), _code(q, "latent_query q"), ldq, _p(table), n, heads, dim, rank,
+            _lib.call("zi_latent_query_rot", _p(out), _code(out, "latent_query out"), _p(q), _code(q, "latent_query q"), ldq, _p(table), n, heads, dim, rank,
                       rot, _stream())
         return out
+    _f32(out, "latent_query out")
     _lib.call("zi_latent_query", _p(out), _p(q), _code(q, "latent_query q"), ldq, _p(w_uk), _code(w_uk, "latent_query w_uk"),
               _p(table), n, heads, dim, rank, rot, _stream())
     return out
@@ -207,7 +214,7 @@ def latent_attention_cores_plan(n: int, entries: int, heads: int, window: int, u
 
 def latent_attention_cores_workspace(n: int, heads: int, rank: int, chunks: int) -> int:
     """Floats of workspace for the chunks' partial results (0 without a cut)."""
-    return int(chunks) * int(n) * int(heads) * (int(rank) + 2) if chunks > 1 else 0
+    return int(chunks) * int(n) * int(heads) * (int(rank) + 4) if chunks > 1 else 0
 
 
 def latent_attention_cores(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: torch.Tensor, entry_start: torch.Tensor,
@@ -215,8 +222,8 @@ def latent_attention_cores(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: to
                            window: int, out: torch.Tensor, waves: int = 1, chunk_keys: int = 0, chunks: int = 1,
                            workspace: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``latent_attention`` on the matrix cores, for all tokens of a step (bfloat16 caches): entry e brings the
-    tokens entry_start[e] ... of positions entry_past[e] ...; queries are rounded to bfloat16 for the products,
-    scores, softmax and sums are float32."""
+    tokens entry_start[e] ... of positions entry_past[e] ...; queries (float32 or bfloat16) are rounded to bfloat16 for the products,
+    scores, softmax and sums are float32; out float32 or bfloat16."""
     _gpu("latent_attention_cores", qa, c_cache, kr_cache, entry_start, entry_len, entry_past, block_tables, out, workspace)
     if qa.dim() != 3:
         raise ValueError("latent_attention_cores: qa must be [n, heads, rank + rot]")
@@ -226,8 +233,8 @@ def latent_attention_cores(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: to
     pages, ps = _latent_caches(c_cache, kr_cache, rank, rot, "latent_attention_cores")
     if not latent_attention_cores_supported(c_cache.dtype, rank, rot):
         raise ValueError(f"latent_attention_cores: a {c_cache.dtype} cache with rank {rank} and rot {rot} is not taken")
-    _f32(qa, "latent_attention_cores qa")
-    _f32(out, "latent_attention_cores out", (n, heads, rank))
+    if not qa.is_contiguous() or not out.is_contiguous() or tuple(out.shape) != (n, heads, rank):
+        raise ValueError(f"latent_attention_cores: qa and out [{n}, {heads}, {rank}] must be contiguous")
     E = entry_start.numel()
     for t in (entry_start, entry_len, entry_past):
         _i32(t, "latent_attention_cores entries", E)
@@ -237,25 +244,28 @@ def latent_attention_cores(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: to
     need = latent_attention_cores_workspace(n, heads, rank, chunks)
     if need and (workspace is None or workspace.dtype != torch.float32 or workspace.numel() < need):
         raise ValueError(f"latent_attention_cores: {need} floats of workspace are needed")
-    _lib.call("zi_latent_attention_cores", _p(out), _p(workspace), int(workspace.numel()) if workspace is not None else 0,
-              _p(qa), _p(c_cache), _p(kr_cache), _p(entry_start), _p(entry_len), _p(entry_past), _p(block_tables), E, n,
+    _lib.call("zi_latent_attention_cores", _p(out), _code(out, "latent_attention_cores out"), _p(workspace),
+              int(workspace.numel()) if workspace is not None else 0, _p(qa), _code(qa, "latent_attention_cores qa"), _p(c_cache), _p(kr_cache), _p(entry_start), _p(entry_len), _p(entry_past), _p(block_tables), E, n,
               int(block_tables.shape[1]), pages, heads, rank, rot, ps, int(window), float(scale), int(waves),
               int(chunk_keys), int(chunks), _stream())
     return out
 
 
 def latent_value_gates(w_uv: torch.Tensor, heads: int, rank: int) -> bool:
-    """Whether ``latent_value`` takes a gate itself (else: ``gate_heads`` on its result)."""
+    """Whether ``latent_value`` runs on the matrix cores: it then takes a gate itself (else: ``gate_heads`` on its result) and
+    attended latents in bfloat16."""
     return w_uv.dtype == torch.bfloat16 and w_uv.data_ptr() % 16 == 0 \
         and bool(_lib.load().zi_headwise_linear_supported(1, rank, heads * rank, rank))
 
 
 def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out [n, heads * vdim] = every head's attended latent o [n, heads, rank] through its block of ``w_uv``
+    """out [n, heads * vdim] = every head's attended latent o [n, heads, rank] (float32, or bfloat16 where
+    ``latent_value_gates``) through its block of ``w_uv``
     [heads * vdim, rank]; with ``gate`` ([n, heads * vdim] bfloat16 or float32 with dense rows, or a stack of float32 terms;
     where ``latent_value_gates``) times sigmoid(gate)."""
     _gpu("latent_value", o, w_uv, out, gate)
-    _f32(o, "latent_value o")
+    if o.dim() != 3 or not o.is_contiguous():
+        raise ValueError("latent_value: o must be a contiguous [n, heads, rank] tensor")
     n, heads, rank = o.shape
     if tuple(w_uv.shape) != (heads * vdim, rank) or not w_uv.is_contiguous():
         raise ValueError(f"latent_value: w_uv must be a contiguous [{heads * vdim}, {rank}] tensor")
@@ -263,7 +273,8 @@ def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tens
     if tuple(out.shape) != (n, heads * vdim):
         raise ValueError(f"latent_value: out must be [{n}, {heads * vdim}]")
     if latent_value_gates(w_uv, heads, rank):
-        args = (_p(out), _code(out, "latent_value out"), ldo, vdim, _p(o), heads * rank, rank, _p(w_uv), n, heads, vdim, rank)
+        args = (_p(out), _code(out, "latent_value out"), ldo, vdim, _p(o), _code(o, "latent_value o"), heads * rank, rank, _p(w_uv), n,
+                heads, vdim, rank)
         if gate is None:
             _lib.call("zi_headwise_linear", *args, _stream())
             return out
@@ -276,6 +287,7 @@ def latent_value(o: torch.Tensor, w_uv: torch.Tensor, vdim: int, out: torch.Tens
         return out
     if gate is not None:
         raise ValueError("latent_value: a gate is not taken with these sizes")
+    _f32(o, "latent_value o")
     _lib.call("zi_latent_value", _p(out), _code(out, "latent_value out"), ldo, _p(o), _p(w_uv), _code(w_uv, "latent_value w_uv"),
               n, heads, vdim, rank, _stream())
     return out

@@ -137,7 +137,10 @@ class LatentAttention(Mixer):
                     mats.append(torch.zeros((-at % 8, self.hidden), dtype=self.dq.dtype, device=self.dq.device))
                     at += -at % 8
             self.inputs = torch.cat(mats).contiguous()
-        self.value_gates = self.gate is not None and rt.device.type == "cuda" and ops.latent_value_gates(self.uv, self.nh, self.rank)
+        value_cores = rt.device.type == "cuda" and ops.latent_value_gates(self.uv, self.nh, self.rank)
+        self.value_gates = self.gate is not None and value_cores
+        self.short_query = self.cores and ops.latent_query_cores(self.uk_t, self.nh, self.dim, self.rot)
+        self.short_attended = self.cores and value_cores
 
     def cache_request(self) -> Optional[KVCacheRequest]:
         return latent_cache_request("window" if self.window > 0 else "full", self.rank, self.rot, self.window)
@@ -195,9 +198,10 @@ class LatentAttention(Mixer):
             cq = ops.linear(x, self.dq, out=rt.buffer("latent_cq", (n, self.q_rank), torch.float32))
             x = ops.rms_norm(cq, self.dq_norm, self.eps, out=rt.buffer("latent_cq_normed", (n, self.q_rank)))
         q = ops.linear(x, self.q, out=rt.buffer("latent_q", (n, self.nh * (self.dim + self.rot)), torch.float32))
-        qa = rt.buffer("latent_qa", (n, self.nh, self.rank + self.rot), torch.float32)
+        # between the products on the matrix cores, rows in bfloat16: what the next product would round them to
+        qa = rt.buffer("latent_qa", (n, self.nh, self.rank + self.rot), torch.bfloat16 if self.short_query else torch.float32)
         ops.latent_query(q, self.uk, table, self.nh, self.dim, self.rank, self.rot, out=qa, w_uk_t=self.uk_t)
-        o = rt.buffer("latent_attended", (n, self.nh, self.rank), torch.float32)
+        o = rt.buffer("latent_attended", (n, self.nh, self.rank), torch.bfloat16 if self.short_attended else torch.float32)
         if self.cores:
             max_keys = batch.plans[KEY_BOUND_PLANNER.key].sizes["max_keys"] if self.window <= 0 else 0
             waves, chunk_keys, chunks = ops.latent_attention_cores_plan(n, batch.num_entries, self.nh, self.window, self.units,
