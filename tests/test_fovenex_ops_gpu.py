@@ -389,7 +389,42 @@ def test_query_latents_latents_and_key_parts_from_one_product(qr, rank, rot, pag
     assert torch.equal(alone, cq)
 
 
-@pytest.mark.parametrize("heads, vdim, rank, n", [(3, 40, 64, 5), (12, 128, 512, 40), (2, 18, 24, 17)])
+@pytest.mark.parametrize("heads, dim, rot, rank, n", [(3, 24, 8, 64, 5), (12, 128, 64, 512, 40), (2, 16, 16, 72, 17), (4, 40, 0, 24, 1)])
+def test_queries_carried_through_the_keys_projection_from_partial_sums(heads, dim, rot, rank, n):
+    """The plain product of a query and any key (W_uk c | turned part) is that of the carried query and (c | turned part)."""
+    g = torch.Generator().manual_seed(rank)
+    q = torch.randn((n, heads * (dim + rot)), generator=g).to(BF).float()
+    uk = (torch.randn((heads * dim, rank), generator=g) / dim ** 0.5).to(BF)
+    uk_t = uk.view(heads, dim, rank).transpose(1, 2).contiguous()
+    positions = [2 + 3 * i for i in range(n)]
+    freqs, _ = plain.pair_frequencies(rot, 100.0) if rot else ([], 1.0)
+    table = _table(n, freqs, 1.0, positions) if rot else None
+    per = q.double().view(n, heads, dim + rot)
+    want = torch.einsum("nhd,hdr->nhr", per[..., :dim], uk.double().view(heads, dim, rank))
+    if rot:
+        order = [j // 2 + (j % 2) * (rot // 2) for j in range(rot)]
+        halves = torch.empty_like(per[..., dim:])
+        halves[..., order] = per[..., dim:]
+        want = torch.cat([want, _turned(halves, freqs, 1.0, positions)[..., order]], dim=-1)
+    assert ops.latent_query_cores(uk_t.to(DEV), heads, dim, rot)
+    for S in (1, 3, 8):
+        stack = torch.randn((S, n, q.shape[1]), generator=g)
+        stack[-1] += q - stack.sum(0)
+        for dtype in (F32, BF):
+            out = torch.full((n, heads, rank + rot), float("nan"), dtype=dtype, device=DEV)
+            ops.latent_query(stack.to(DEV), uk.to(DEV), table, heads, dim, rank, rot, out=out, w_uk_t=uk_t.to(DEV))
+            _close(out, want, 1e-2, (S, dtype))
+    for dtype in (F32, BF):      # whole rows, few and many
+        many = torch.cat([q] * 40)
+        t2 = torch.cat([table] * 40) if rot else None
+        out = torch.empty((40 * n, heads, rank + rot), dtype=BF, device=DEV)
+        ops.latent_query(many.to(DEV).to(dtype), uk.to(DEV), t2, heads, dim, rank, rot, out=out, w_uk_t=uk_t.to(DEV))
+        _close(out.view(40, n, heads, -1)[17], want, 1e-2, dtype)
+    two = ops.latent_query(q.to(DEV), uk.to(DEV), table, heads, dim, rank, rot, out=torch.empty((n, heads, rank + rot), device=DEV), w_uk_t=uk_t.to(DEV))
+    _close(two, want, 1e-2, "few")
+
+
+@pytest.mark.parametrize("heads, vdim, rank, n", [(3, 40, 64, 5), (3, 72, 64, 300), (12, 128, 512, 40), (2, 18, 24, 17)])
 def test_values_gated_where_they_are_made(heads, vdim, rank, n):
     g = torch.Generator().manual_seed(rank)
     o = torch.randn((n, heads, rank), generator=g).to(BF).float()

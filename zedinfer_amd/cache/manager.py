@@ -105,6 +105,10 @@ class SequenceCache:
         self.promised: List[int] = [0] * num_groups
         self.closed = False
         self.version = 0          # grows whenever a block table of the sequence changes
+        # what need not be looked at again, per group: the logical pages before ``passed`` that a window has left are
+        # given back; every page from the first one still seen to before ``covered`` is held
+        self.passed: List[int] = [0] * num_groups
+        self.covered: List[int] = [0] * num_groups
 
 
 class CacheManager:
@@ -144,6 +148,7 @@ class CacheManager:
             g = keys[key]
             self.groups[g].caches[cid] = rq
             self.group_of_cache[cid] = g
+        self._window_groups = [(gi, g) for gi, g in enumerate(self.groups) if g.kind == "window"]
         self.slots = IdPool(self.max_requests, "state slot")
         self.live: Dict[object, SequenceCache] = {}
         self.tensors: Dict[int, Dict[str, torch.Tensor]] = {}      # cache id -> name -> [pages, *page shape]
@@ -212,17 +217,19 @@ class CacheManager:
 
     # ---- growth ------------------------------------------------------------------
     def _release_passed(self, seq: SequenceCache) -> None:
-        for gi, g in enumerate(self.groups):
-            if g.kind != "window":
+        for gi, g in self._window_groups:
+            first = g.first_live_page(seq.length)
+            if first <= seq.passed[gi]:
                 continue
-            first = min(g.first_live_page(seq.length), len(seq.pages[gi]))
             table = seq.pages[gi]
-            for i in range(g.kept_pages, first):
+            first = min(first, len(table))
+            for i in range(max(g.kept_pages, seq.passed[gi]), first):
                 if table[i] >= 0:
                     g.pool.give_back(table[i])
                     table[i] = -1
                     seq.held[gi] -= 1
                     seq.version += 1
+            seq.passed[gi] = first
 
     def ensure(self, seq: SequenceCache, new_len: int) -> "Growth":
         """Make sure pages exist for every position below ``new_len`` that a token at or after
@@ -238,15 +245,17 @@ class CacheManager:
         growth = None
         try:
             for gi, g in enumerate(self.groups):
-                table = seq.pages[gi]
-                rows = g.rows_for(new_len)
+                rows = new_len if g.stride == 1 else g.rows_for(new_len)
                 last = (rows - 1) // g.page_size if rows > 0 else -1
+                if last < seq.covered[gi]:
+                    continue                      # most calls: a token inside a page that is held
+                table = seq.pages[gi]
                 if len(table) <= last:
                     if growth is None:
                         growth = Growth(taken=[], grown=[0] * len(self.groups), old_lens=[len(t) for t in seq.pages])
                     while len(table) <= last:
                         table.append(-1)
-                for i in range(g.first_live_page(seq.length), last + 1):
+                for i in range(max(g.first_live_page(seq.length), seq.covered[gi]), last + 1):
                     if table[i] >= 0:
                         continue
                     if growth is None:
@@ -263,6 +272,7 @@ class CacheManager:
                     seq.held[gi] += 1
                     seq.version += 1
                     growth.taken.append((gi, i))
+                seq.covered[gi] = last + 1
         except OutOfPages:
             self.undo(seq, growth)
             raise
@@ -277,11 +287,14 @@ class CacheManager:
             self.groups[gi].pool.give_back(seq.pages[gi][i])
             seq.pages[gi][i] = -1
             seq.held[gi] -= 1
+            seq.covered[gi] = min(seq.covered[gi], i)
         for gi, n in enumerate(growth.grown):
             self.groups[gi].pool.uncommit(n)
             seq.promised[gi] -= n
         for gi, n in enumerate(growth.old_lens):
             del seq.pages[gi][n:]
+            seq.covered[gi] = min(seq.covered[gi], n)
+            seq.passed[gi] = min(seq.passed[gi], n)
         seq.version += 1
 
     def commit(self, seq: SequenceCache, new_len: int) -> None:

@@ -111,8 +111,13 @@ head_norm_store_tile_kernel(zi_bf16* __restrict__ q_out, int64_t ldq, zi_bf16* _
     uint16_t* vt = reinterpret_cast<uint16_t*>(dft_lds + (size_t)DFT_TOKENS * rot * sizeof(float));   // [token][vw]
     const int t0 = blockIdx.x * DFT_TOKENS, tid = threadIdx.x;
     const int nt = (n - t0 < DFT_TOKENS) ? n - t0 : DFT_TOKENS;
+    // the last of the tokens' workgroups (gridDim.y) takes keys and values, the others share the queries; without a cache
+    // all take queries
+    const bool takes_kv = write_kv && blockIdx.y == gridDim.y - 1;
+    const int q_groups = gridDim.y - (write_kv ? 1 : 0), q_per = (nq + q_groups - 1) / q_groups;
+    const int u_first = takes_kv ? 0 : blockIdx.y * q_per, u_end = takes_kv ? nk : (u_first + q_per < nq ? u_first + q_per : nq);
     for (int i = tid; i < nt * rot; i += 256) cs[i] = table[(int64_t)t0 * rot + i];
-    if (write_kv)
+    if (takes_kv)
         for (int i = tid; i < nt * (vw / 8); i += 256) {
             const int tt = i / (vw / 8), c8 = i % (vw / 8);
             *reinterpret_cast<uint4*>(vt + tt * vw + c8 * 8) =
@@ -121,12 +126,11 @@ head_norm_store_tile_kernel(zi_bf16* __restrict__ q_out, int64_t ldq, zi_bf16* _
     __syncthreads();
     // the maps of queries and keys: L lanes each.  Every lane of a wavefront goes round the same number of times (the lanes
     // trade values), those past the end on a map that is not stored.
-    const int units = nt * (nq + (write_kv ? nk : 0)), li = tid % L, swap = half / 8;
+    const int per = u_end - u_first, units = nt * per, li = tid % L, swap = half / 8;
+    const bool is_q = !takes_kv;
     for (int i0 = 0; i0 < units; i0 += 256 / L) {
         const int i = i0 + tid / L, ic = i < units ? i : units - 1;
-        // all query maps of the tokens, then all key maps
-        const bool is_q = ic < nt * nq;
-        const int r = is_q ? ic : ic - nt * nq, per = is_q ? nq : nk, tt = r / per, u = r % per, m = u % maps;
+        const int tt = ic / per, u = u_first + ic % per, m = u % maps;
         float x[8], y[8];
         df_unpack(*reinterpret_cast<const uint4*>(proj + (int64_t)(t0 + tt) * ld + (int64_t)((is_q ? 0 : nq) + u) * dim + li * 8), x);
         const float* gain = is_q ? q_gain : k_gain;
@@ -167,7 +171,7 @@ head_norm_store_tile_kernel(zi_bf16* __restrict__ q_out, int64_t ldq, zi_bf16* _
             for (int c8 = (m * part + dim) / 8 + li; c8 < end / 8; c8 += L) *reinterpret_cast<uint4*>(kr + c8 * 8) = zero;
         }
     }
-    if (!write_kv) return;
+    if (!takes_kv) return;
     // values, transposed; dims from vdim on are nobody's
     bool run = nt == DFT_TOKENS;
     const int s0 = slots[t0];
@@ -230,7 +234,7 @@ extern "C" int zi_head_norm_store(void* q_out, int dt, int64_t ldq, void* kcache
         const size_t lds = (size_t)DFT_TOKENS * (rot * sizeof(float) + (kcache ? (size_t)nkv * vdim * 2 : 0));
         if (fits && lds <= 48 * 1024) {
 #define ZI_DFT(LL)                                                                                                       \
-    head_norm_store_tile_kernel<LL><<<(n + DFT_TOKENS - 1) / DFT_TOKENS, 256, lds, stream>>>(                             \
+    head_norm_store_tile_kernel<LL><<<dim3((n + DFT_TOKENS - 1) / DFT_TOKENS, kcache ? 4 : 3), 256, lds, stream>>>(        \
         (zi_bf16*)q_out, ldq, (zi_bf16*)kcache, (zi_bf16*)vcache, (const zi_bf16*)proj, ld, q_gain, k_gain, eps, table, rot, slots, \
         cache_slots, n, nq, nkv, maps, vdim, d, page_size, pad, kcache != nullptr)
             switch (L) {

@@ -88,13 +88,20 @@ extern "C" int zi_latent_store(const float* dkv, int dt, int64_t ld, int n, cons
 // Rows of proj hold the query latent (q_rank values) from column 0 and, where the layer writes a cache, the token's latent and
 // key part (rank + rot values) from column dkv_at; any storage type, or `splits` float32 partial sums.  Workgroup (token, 0):
 // cq = rms_norm(query latent) * q_norm; workgroup (token, 1): what latent_store does.
+__device__ __forceinline__ float4 li_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 li_load4(const zi_bf16* p) {
+    const uint2 r = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(r.x << 16), __uint_as_float(r.x & 0xffff0000u), __uint_as_float(r.y << 16),
+                       __uint_as_float(r.y & 0xffff0000u));
+}
+
 template <typename T, typename TP, typename TW>
 __global__ void __launch_bounds__(256)
 latent_inputs_kernel(T* __restrict__ cq, int64_t ld_cq, const TP* __restrict__ proj, int64_t ld, int splits, int64_t split_stride,
                      const TW* __restrict__ q_norm, const TW* __restrict__ c_norm, float eps, int q_rank, int dkv_at,
                      const float* __restrict__ table, const int32_t* __restrict__ slots, T* __restrict__ c_cache,
-                     T* __restrict__ kr_cache, int64_t cache_slots, int rank, int rot) {
-    extern __shared__ float xs[];      // [max(q_rank, rank + rot)]
+                     T* __restrict__ kr_cache, int64_t cache_slots, int rank, int rot, int vec) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];      // [max(q_rank, rank + rot)]
     __shared__ float red[16];
     const int t = blockIdx.x;
     const bool query = blockIdx.y == 0;
@@ -103,17 +110,26 @@ latent_inputs_kernel(T* __restrict__ cq, int64_t ld_cq, const TP* __restrict__ p
     const TP* row = proj + (int64_t)t * ld + (query ? 0 : dkv_at);
     const int normed = query ? q_rank : rank, width = query ? q_rank : rank + rot;
     float ss = 0.f;
-    for (int j = threadIdx.x; j < width; j += blockDim.x) {
-        float v = zi_load(row + j);
-        int s = 1;
-        for (; s + 3 < splits; s += 4) {      // four terms' loads in flight, added in their order
-            const float a = zi_load(row + s * split_stride + j), b = zi_load(row + (s + 1) * split_stride + j);
-            const float c = zi_load(row + (s + 2) * split_stride + j), d = zi_load(row + (s + 3) * split_stride + j);
-            v += a; v += b; v += c; v += d;
+    if (vec) {      // four columns at a time, eight terms in flight
+        for (int j = threadIdx.x * 4; j < width; j += blockDim.x * 4) {
+            float4 v = li_load4(row + j);
+            for (int s0 = 1; s0 < splits; s0 += 8) {
+                float4 t[8];
+#pragma unroll
+                for (int u = 0; u < 8; ++u) t[u] = s0 + u < splits ? li_load4(row + (s0 + u) * split_stride + j) : make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+                for (int u = 0; u < 8; ++u) { v.x += t[u].x; v.y += t[u].y; v.z += t[u].z; v.w += t[u].w; }
+            }
+            *reinterpret_cast<float4*>(xs + j) = v;
+            if (j < normed) ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);      // (normed is a multiple of four)
         }
-        for (; s < splits; ++s) v += zi_load(row + s * split_stride + j);
-        xs[j] = v;
-        if (j < normed) ss += v * v;
+    } else {
+        for (int j = threadIdx.x; j < width; j += blockDim.x) {
+            float v = zi_load(row + j);
+            for (int s = 1; s < splits; ++s) v += zi_load(row + s * split_stride + j);
+            xs[j] = v;
+            if (j < normed) ss += v * v;
+        }
     }
     ss = zi_block_sum(ss, red);      // (its barriers also make xs visible to all)
     const float rstd = 1.0f / sqrtf(ss / (float)normed + eps);
@@ -143,10 +159,12 @@ extern "C" int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* pro
     ZI_REQUIRE((size_t)most * sizeof(float) <= 60 * 1024, "latent_inputs: latents of %d values are too large", most);
     if (n == 0) return 0;
     const dim3 grid(n, c_cache ? 2 : 1);
+    const int vec = q_rank % 4 == 0 && (!c_cache || (rank % 4 == 0 && rot % 4 == 0 && dkv_at % 4 == 0)) && ld % 4 == 0 && split_stride % 4 == 0 &&
+                    ((uintptr_t)proj % 16) == 0;
     ZI_DISPATCH_DTYPE(dt, T, ZI_DISPATCH_DTYPE(p_dt, TP, ZI_DISPATCH_DTYPE(w_dt, TW, {
         latent_inputs_kernel<T, TP, TW><<<grid, 256, most * sizeof(float), stream>>>(
             (T*)cq, ld_cq, (const TP*)proj, ld, splits, split_stride, (const TW*)q_norm, (const TW*)c_norm, eps, q_rank, dkv_at, table,
-            slots, (T*)c_cache, (T*)kr_cache, c_cache ? cache_slots : 1, rank, rot);
+            slots, (T*)c_cache, (T*)kr_cache, c_cache ? cache_slots : 1, rank, rot, vec);
     })));
     return zi_check_launch("latent_inputs");
 }

@@ -6,7 +6,8 @@
 //   stage    the block's latents and key parts, [32][rank + rot], from the pages straight into LDS
 //            (global_load_lds_dwordx4), one block ahead, in one of two buffers; where its keys lie in the pool is asked for
 //            two blocks ahead, a lane a key, and traded between lanes.  Rows are not padded but swizzled: the 16-byte
-//            piece c of row k sits at place c xor (k / 2 mod 8), so that neither product's reads meet in a bank
+//            piece c of row k sits at place c xor la_swizzle(k), so that neither product's reads meet in a bank: sixteen
+//            rows' piece c and eight rows' pieces c, c + 1 (c even) lie in different banks
 //   scores   S[key][row] = K . Q^T   v_mfma_f32_16x16x32_bf16: first operand the keys' rows from LDS, second the
 //            queries, held in registers for the whole walk (KS operands a lane)
 //   softmax  a lane holds 8 of a row's 32 scores, the row's other 24 are in 3 lanes: two lane exchanges; running
@@ -42,6 +43,10 @@ union la_pack {
 #define LA_LOG2E 1.4426950408889634f
 
 __device__ __attribute__((aligned(16))) const unsigned la_zero16[4] = {0u, 0u, 0u, 0u};
+
+// of row k (rows k and k + 16 alike): a permutation of 0 .. 7 over eight rows of one parity, its upper two bits one of 0 .. 3
+// over four of them
+__device__ __forceinline__ int la_swizzle(int k) { return ((k & 6)) | ((k >> 3) & 1); }
 
 // four keys of one dim from rows of LDS: see above
 __device__ __forceinline__ la_s16x4_t la_read_transposed(const char* at) {
@@ -134,7 +139,7 @@ latent_attention_cores_kernel(void* __restrict__ out, int out_f32, float* __rest
         asm volatile("" : "+v"(ln));
 #pragma unroll
         for (int i = 0; i < KI; ++i) {
-            const int L = (wave * KI + i) * ZI_WAVE + ln, key = L / P, d = ((L % P) ^ ((key >> 1) & 7)) * 8;
+            const int L = (wave * KI + i) * ZI_WAVE + ln, key = L / P, d = ((L % P) ^ la_swizzle(key)) * 8;
             const int slot = __shfl(slots, key, ZI_WAVE);
             const zi_bf16* src = d < rank ? c_cache + (int64_t)slot * rank + d : kr_cache + (int64_t)slot * rot + (d - rank);
             if (slot < 0 || d >= qw) src = reinterpret_cast<const zi_bf16*>(la_zero16);
@@ -142,9 +147,9 @@ latent_attention_cores_kernel(void* __restrict__ out, int out_f32, float* __rest
         }
     };
     // where this lane reads in a buffer, in bytes: the keys' rows (k-steps even and odd), and four keys x sixteen dims
-    const int sw = (r >> 1) & 7;      // of rows r and 16 + r
+    const int sw = la_swizzle(r);      // of rows r and 16 + r
     const int s_even = (r * P + (j ^ sw)) * 16, s_odd = (r * P + ((4 + j) ^ sw)) * 16;
-    const int vrow = 4 * j + (r >> 2), vsw = (vrow >> 1) & 7;
+    const int vrow = 4 * j + (r >> 2), vsw = la_swizzle(vrow);
     int v_at[4];
 #pragma unroll
     for (int t = 0; t < 4; ++t) v_at[t] = (vrow * P + ((t * 2 + ((r & 3) >> 1)) ^ vsw)) * 16 + (r & 1) * 8;
@@ -498,7 +503,7 @@ headwise_linear_many_kernel(TO* __restrict__ out, int64_t ldo, int os, const TX*
     for (int a = 0; a < TM; ++a)
 #pragma unroll
         for (int c = 0; c < TN; ++c) acc[a][c] = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
     for (int k0 = 0; k0 < K; k0 += 32) {
         const int k = k0 + 8 * j, kc = k < K ? k : 0;
         const unsigned mask = 0u - (unsigned)(k < K);
@@ -604,4 +609,91 @@ extern "C" int zi_latent_query_rot(void* qa, int qa_dt, const void* q, int dt, i
                                                                                              dim, rank, rot);
     }));
     return zi_check_launch("latent_query_rot");
+}
+
+// Few tokens: qa[t][h] = (W_uk[h]^T q_plain, turn(q_rot)) from the query product's float32 partial sums, one launch.
+// x [splits][n][heads * (dim + rot)] (row stride ldx); w bfloat16 [heads][rank][dim].  Workgroups as in
+// headwise_linear_few_kernel (the terms are added as they are loaded); the last of a head's (blockIdx.z) turns the rotated part.
+template <typename TO>
+__global__ void __launch_bounds__(4 * ZI_WAVE)
+latent_query_sums_kernel(TO* __restrict__ qa, const float* __restrict__ x, int splits, int64_t split_stride, int64_t ldx,
+                         const zi_bf16* __restrict__ w, const float* __restrict__ table, int n, int heads, int dim, int rank, int rot) {
+    __shared__ la_f32x4_t part[3][ZI_WAVE];
+    const int t0 = blockIdx.x * 16, h = blockIdx.y;
+    const int out_w = rank + rot, xs = dim + rot;
+    if (blockIdx.z == gridDim.z - 1) {
+        const int half = rot / 2;
+        for (int i = threadIdx.x; i < 16 * half; i += 4 * ZI_WAVE) {
+            const int t = t0 + i / half, p = i % half;
+            if (t >= n) continue;
+            const float* at = x + (int64_t)t * ldx + (int64_t)h * xs + dim + 2 * p;
+            float u = at[0], v = at[1];
+            for (int s = 1; s < splits; ++s) {
+                u += at[s * split_stride];
+                v += at[s * split_stride + 1];
+            }
+            const float c = table[((int64_t)t * half + p) * 2], sn = table[((int64_t)t * half + p) * 2 + 1];
+            TO* o = qa + ((int64_t)t * heads + h) * out_w + rank + 2 * p;
+            zi_store(o, u * c - v * sn);
+            zi_store(o + 1, v * c + u * sn);
+        }
+        return;
+    }
+    const int n0 = blockIdx.z * 16;
+    const int lane = threadIdx.x % ZI_WAVE, wave = threadIdx.x / ZI_WAVE, r = lane % 16, j = lane / 16;
+    const zi_bf16* wrow = w + ((int64_t)h * rank + (n0 + r < rank ? n0 + r : rank - 1)) * dim;
+    const int64_t t = t0 + r < n ? t0 + r : n - 1;
+    const float* xrow = x + t * ldx + (int64_t)h * xs;
+    la_f32x4_t acc = (la_f32x4_t){0.f, 0.f, 0.f, 0.f};
+    for (int k0 = wave * 32; k0 < dim; k0 += 128) {
+        const int k = k0 + 8 * j, kc = k < dim ? k : 0;
+        const unsigned mask = 0u - (unsigned)(k < dim);
+        la_pack a = la_load8(wrow + kc), b;
+        float4 lo = *reinterpret_cast<const float4*>(xrow + kc), hi = *reinterpret_cast<const float4*>(xrow + kc + 4);
+        for (int s0 = 1; s0 < splits; s0 += 4) {      // four terms in flight, added in their order
+            float4 l4[4], h4[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float* at = xrow + (int64_t)(s0 + u < splits ? s0 + u : 0) * split_stride + kc;
+                l4[u] = *reinterpret_cast<const float4*>(at);
+                h4[u] = *reinterpret_cast<const float4*>(at + 4);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                if (s0 + u >= splits) break;
+                lo.x += l4[u].x; lo.y += l4[u].y; lo.z += l4[u].z; lo.w += l4[u].w;
+                hi.x += h4[u].x; hi.y += h4[u].y; hi.z += h4[u].z; hi.w += h4[u].w;
+            }
+        }
+        b.w[0] = zi_pack_bf16x2(lo.x, lo.y);
+        b.w[1] = zi_pack_bf16x2(lo.z, lo.w);
+        b.w[2] = zi_pack_bf16x2(hi.x, hi.y);
+        b.w[3] = zi_pack_bf16x2(hi.z, hi.w);
+        a.u &= mask;
+        b.u &= mask;
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b.b, acc, 0, 0, 0);
+    }
+    if (wave > 0) part[wave - 1][lane] = acc;
+    __syncthreads();
+    if (wave > 0) return;
+#pragma unroll
+    for (int u = 0; u < 3; ++u) acc += part[u][lane];
+    if (t0 + r >= n || n0 + 4 * j >= rank) return;
+    la_store4(qa + (t * heads + h) * out_w + n0 + 4 * j, acc, rank - n0 - 4 * j);
+}
+
+extern "C" int zi_latent_query_sums(void* qa, int qa_dt, const float* x, int splits, int64_t split_stride, int64_t ldx, const void* w,
+                                    const float* table, int n, int heads, int dim, int rank, int rot, hipStream_t stream) {
+    ZI_REQUIRE(n >= 0 && heads > 0 && heads <= 65535 && dim > 0 && rank > 0 && rot >= 0 && rot % 2 == 0 && splits >= 1 &&
+                   ldx >= (int64_t)heads * (dim + rot) && (rank + 15) / 16 < 65535, "latent_query_sums: bad sizes");
+    ZI_REQUIRE(zi_headwise_linear_supported(ZI_BF16, dim, ldx, dim + rot) && split_stride % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0,
+               "latent_query_sums: sizes in eights and aligned rows are needed");
+    ZI_REQUIRE(rot == 0 || table, "latent_query_sums: no table of angles");
+    if (n == 0) return 0;
+    const dim3 grid((n + 15) / 16, heads, (rank + 15) / 16 + 1);
+    ZI_DISPATCH_DTYPE(qa_dt, TO, {
+        latent_query_sums_kernel<TO><<<grid, 4 * ZI_WAVE, 0, stream>>>((TO*)qa, x, splits, split_stride, ldx, (const zi_bf16*)w, table, n,
+                                                                       heads, dim, rank, rot);
+    });
+    return zi_check_launch("latent_query_sums");
 }

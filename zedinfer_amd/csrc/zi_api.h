@@ -58,6 +58,9 @@ int zi_latent_inputs(void* cq, int dt, int64_t ld_cq, const void* proj, int p_dt
     int n, const void* q_norm, const void* c_norm, int w_dt, float eps, int q_rank, int dkv_at, const float* table,
     const int32_t* slots, void* c_cache, void* kr_cache, int64_t cache_slots, int rank, int rot, hipStream_t stream);
 // latent_cores.hip
+int zi_latent_query_sums(void* qa, int qa_dt, const float* x, int splits, int64_t split_stride, int64_t ldx, const void* w,
+    const float* table, int n, int heads, int dim, int rank, int rot, hipStream_t stream);
+// latent_cores.hip
 int zi_headwise_linear_gated(void* out, int out_dt, int64_t ldo, int os, const void* x, int x_dt, int64_t ldx, int xs, const void* w,
     int n, int heads, int N, int K, const void* gate, int g_dt, int64_t ld_gate, int g_splits, int64_t g_stride,
     hipStream_t stream);
@@ -481,5 +484,6 @@ int zi_sample(int32_t* out, const float* logits, int64_t ld, float* work, int ro
     X(zi_activate) \
     X(zi_latent_inputs) \
     X(zi_headwise_linear_gated) \
+    X(zi_latent_query_sums) \
     X(zi_argmax) \
     X(zi_sample)

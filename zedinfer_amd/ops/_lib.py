@@ -148,6 +148,7 @@ _PROTOTYPES = {
     "zi_difference_merge": [P, L, P, L, I, P, I, I, I, I, I, F, F, F, P, I, L, I, L, P],
     "zi_activate": [P, I, L, P, I, L, I, L, I, I, I, P],
     "zi_latent_inputs": [P, I, L, P, I, L, I, L, I, P, P, I, F, I, I, P, P, P, P, L, I, I, P],
+    "zi_latent_query_sums": [P, I, P, I, L, L, P, P, I, I, I, I, I, P],
     "zi_headwise_linear_gated": [P, I, L, I, P, I, L, I, P, I, I, I, I, P, I, L, I, L, P],
     "zi_tape_record": [P, c_char_p, P, I],
     "zi_tape_record_many": [P, c_char_p, P, P, I],

@@ -121,8 +121,19 @@ def latent_query_cores(w_uk_t: Optional[torch.Tensor], heads: int, dim: int, rot
 def latent_query(q: torch.Tensor, w_uk: torch.Tensor, table: Optional[torch.Tensor], heads: int, dim: int, rank: int,
                  rot: int, out: torch.Tensor, w_uk_t: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out [n, heads, rank + rot] float32 (or, with ``w_uk_t`` where the matrix cores take the sizes, bfloat16): every head's unrotated query part carried through its block of
-    ``w_uk`` [heads * dim, rank] (so that it meets latents instead of keys), then its rotated part, turned."""
+    ``w_uk`` [heads * dim, rank] (so that it meets latents instead of keys), then its rotated part, turned.  q [n, heads * (dim +
+    rot)], or (where ``latent_query_cores``) a stack [S, n, ...] of float32 partial sums of it."""
     _gpu("latent_query", q, w_uk, table, out)
+    if q.dim() == 3:
+        S, n, width = q.shape
+        if q.dtype != torch.float32 or not q.is_contiguous() or width != heads * (dim + rot) or tuple(out.shape) != (n, heads, rank + rot) \
+                or not out.is_contiguous() or not latent_query_cores(w_uk_t, heads, dim, rot) or tuple(w_uk_t.shape) != (heads, rank, dim):
+            raise ValueError("latent_query: partial sums must be contiguous float32 [S, n, heads * (dim + rot)], with w_uk_t")
+        if rot:
+            _f32(table, "latent_query table", (n, rot // 2, 2))
+        _lib.call("zi_latent_query_sums", _p(out), _code(out, "latent_query out"), _p(q), S, int(q.stride(0)), width, _p(w_uk_t), _p(table),
+                  n, heads, dim, rank, rot, _stream())
+        return out
     ldq, width = _rows(q, "latent_query q")
     n = q.shape[0]
     if width != heads * (dim + rot):

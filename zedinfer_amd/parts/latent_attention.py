@@ -156,8 +156,12 @@ class LatentAttention(Mixer):
         n = int(num_tokens)
         if self.inputs is not None:
             self.rt.tune_linear(self.rt.buffer("norm_out", (n, self.hidden)), self.inputs, out_dtype=self.inputs_dtype())
-            self.rt.tune_linear(self.rt.buffer("latent_cq_normed", (n, self.q_rank)), self.q, out_dtype=torch.float32)
+            self.rt.tune_linear(self.rt.buffer("latent_cq_normed", (n, self.q_rank)), self.q, out_dtype=self.query_dtype())
             self.rt.tune_linear(self.rt.buffer("latent_heads", (n, self.nh * self.vdim)), self.o)
+
+    def query_dtype(self) -> torch.dtype:
+        """Of the query product for many rows: bfloat16 where the next product would round it to that, float32 elsewhere."""
+        return torch.bfloat16 if self.short_query else torch.float32
 
     def inputs_dtype(self) -> torch.dtype:
         """Of the one product's result for many rows: the activation type, float32 where the gate is a kernel of its own."""
@@ -197,7 +201,12 @@ class LatentAttention(Mixer):
         if self.q_rank and self.inputs is None:
             cq = ops.linear(x, self.dq, out=rt.buffer("latent_cq", (n, self.q_rank), torch.float32))
             x = ops.rms_norm(cq, self.dq_norm, self.eps, out=rt.buffer("latent_cq_normed", (n, self.q_rank)))
-        q = ops.linear(x, self.q, out=rt.buffer("latent_q", (n, self.nh * (self.dim + self.rot)), torch.float32))
+        width = self.nh * (self.dim + self.rot)
+        if self.short_query and ops.linear_sums_supported(x, self.q):      # few rows: the next kernel adds the partial sums
+            S = ops.linear_splits(n, width, self.q.shape[1])
+            q = ops.linear_sums(x, self.q, out=rt.buffer("latent_q_sums", (S, n, width), torch.float32))
+        else:
+            q = ops.linear(x, self.q, out=rt.buffer("latent_q", (n, width), self.query_dtype()))
         # between the products on the matrix cores, rows in bfloat16: what the next product would round them to
         qa = rt.buffer("latent_qa", (n, self.nh, self.rank + self.rot), torch.bfloat16 if self.short_query else torch.float32)
         ops.latent_query(q, self.uk, table, self.nh, self.dim, self.rank, self.rot, out=qa, w_uk_t=self.uk_t)
