@@ -210,9 +210,12 @@ def latent_attention_cores_plan(n: int, entries: int, heads: int, window: int, u
     tiles = lib.zi_latent_attention_cores_tiles(int(n), int(entries), int(heads), waves)
     if window > 0 and tiles < units:
         span = int(window) + -(-16 * waves // int(heads)) + 1
-        chunks = -(-span // LATENT_CHUNK_KEYS)
+        keys = LATENT_CHUNK_KEYS
+        if -(-span // keys) * tiles < units and keys > 32:      # few requests: a walk half as long, twice the workgroups
+            keys //= 2
+        chunks = -(-span // keys)
         if chunks > 1:
-            return waves, LATENT_CHUNK_KEYS, chunks
+            return waves, keys, chunks
     if window <= 0 and max_keys > 0 and tiles < units:
         keys = LATENT_CHUNK_KEYS
         while -(-int(max_keys) // keys) * tiles > 4 * units:      # no more workgroups than four rounds of the chip
