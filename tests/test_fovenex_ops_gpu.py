@@ -458,3 +458,29 @@ def test_the_activation(I, dtype, activation):
         out = ops.activate(src, activation, out=torch.empty((7, I), dtype=dtype, device=DEV))
         _close(out, fn(ref), 1e-6 if dtype == F32 else 5e-3, (activation, terms))
         assert torch.isfinite(out).all()
+
+
+@pytest.mark.parametrize("M,N,K,bias", [(1, 83, 64, True), (16, 256, 200, False), (33, 8960, 256, False), (64, 400, 1536, True)])
+@pytest.mark.parametrize("activation", [a for a in sorted(ops.ACTIVATIONS) if a != "gelu_erf"])
+def test_the_activation_in_the_products_epilogue(M, N, K, bias, activation):
+    g = torch.Generator().manual_seed(M * N)
+    x, w = torch.randn((M, K), generator=g).to(BF), (3 * torch.randn((N, K), generator=g) / K ** 0.5).to(BF)
+    b = torch.randn(N, generator=g).to(BF) if bias else None
+    z = x.double() @ w.double().T + (b.double() if bias else 0.0)
+    fn = {"gelu_tanh": plain.gelu, "silu": lambda t: t * torch.sigmoid(t), "relu2": lambda t: torch.relu(t) ** 2}[activation]
+    out = torch.full((M, N + 5), 9.0, dtype=BF, device=DEV)[:, :N]
+    ops.linear_activated(x.to(DEV), w.to(DEV), activation, bias=None if b is None else b.to(DEV), out=out)
+    _close(out, fn(z), 1e-2, (activation, M, N, K))
+    assert (out.untyped_storage().nbytes() == M * (N + 5) * 2) and bool((torch.as_strided(out, (M, 5), (N + 5, 1), N) == 9.0).all())
+
+
+def test_where_the_products_epilogue_pays():
+    x = lambda M, K: torch.zeros((M, K), dtype=BF, device=DEV)
+    w = lambda N, K: torch.zeros((N, K), dtype=BF, device=DEV)
+    assert ops.linear_activated_supported(x(8, 1536), w(8960, 1536), "gelu_tanh")
+    assert not ops.linear_activated_supported(x(65, 1536), w(8960, 1536), "gelu_tanh")       # more rows than it takes
+    assert not ops.linear_activated_supported(x(8, 8192), w(512, 8192), "gelu_tanh")         # few weight rows, much k: better cut
+    assert not ops.linear_activated_supported(x(8, 1536), w(8960, 1536), "gelu_erf")
+    assert not ops.linear_activated_supported(x(8, 1536).float(), w(8960, 1536).float(), "gelu_tanh")
+    with pytest.raises(ValueError):
+        ops.linear_activated(x(65, 64), w(64, 64), "silu")

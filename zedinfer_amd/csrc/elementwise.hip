@@ -1,6 +1,7 @@
 // Row gathers and elementwise ops: embedding lookup, row gather, residual add,
 // SwiGLU.  Arithmetic is done in float32 and rounded once on store.
 #include "zi_common.h"
+#include "zi_activation.h"
 #include "zi_api.h"
 
 // out[i,:] = table[ids[i],:] * scale   (scale 1: reference: src/backend/ops/embedding/cpu/embedding_cpu.cpp:10-23).
@@ -210,16 +211,6 @@ extern "C" int zi_swiglu(void* out, int out_dt, const void* gate, const void* up
 // out = act(gate) * up, element by element, float32 arithmetic: the gated feed-forward's middle for activations
 // other than the one the SwiGLU kernels above carry.  act: 0 SiLU, 1 GELU in its tanh form
 // 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), 2 GELU with the error function.
-#define ZI_ACT_SILU 0
-#define ZI_ACT_GELU_TANH 1
-#define ZI_ACT_GELU_ERF 2
-
-__device__ __forceinline__ float zi_activation(float z, int act) {
-    if (act == ZI_ACT_GELU_TANH) return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-    if (act == ZI_ACT_GELU_ERF) return 0.5f * z * (1.f + erff(z * 0.70710678118654752440f));
-    return z / (1.f + expf(-z));
-}
-
 template <typename T, typename TO>
 __global__ void gated_act_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ gate, const T* __restrict__ up,
                                  int64_t ld_gate, int64_t ld_up, int n, int inter, int act) {
@@ -332,24 +323,8 @@ extern "C" int zi_relu_squared(void* out, int out_dt, int64_t ldo, const void* z
     return zi_check_launch("relu_squared");
 }
 
-// An activation alone: out = act(z), z [n][inter] with dense rows, possibly as `splits` float32 partial sums.  act: 0 SiLU,
-// 1 GELU in its tanh form, 2 GELU with the error function, 3 relu(z)^2.  The tanh form as z / (1 + e^(-2u)), u = sqrt(2 / pi)
-// (z + 0.044715 z^3), which is the same and loses nothing to cancellation; for bfloat16 results by the chip's exponential and
-// reciprocal.
-#define ZI_ACT_RELU2 3
-template <bool ROUGH>
-__device__ __forceinline__ float ew_activate(float z, int act) {
-    if (act == ZI_ACT_GELU_TANH) {
-        const float w = -2.f * 0.7978845608028654f * z * fmaf(0.044715f * z, z, 1.f);
-        return ROUGH ? z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(w * 1.4426950408889634f)) : z / (1.f + expf(w));
-    }
-    if (act == ZI_ACT_RELU2) {
-        const float p = fmaxf(z, 0.f);
-        return p * p;
-    }
-    return zi_activation(z, act);
-}
-
+// An activation alone: out = act(z), z [n][inter] with dense rows, possibly as `splits` float32 partial sums (the codes are
+// `zi_activate_value`'s).
 template <typename T, typename TO>
 __global__ void activate_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ z, int64_t ldz, int splits,
                                 int64_t split_stride, int n, int inter, int act) {
@@ -358,7 +333,7 @@ __global__ void activate_kernel(TO* __restrict__ out, int64_t ldo, const T* __re
     const int64_t r = i / inter, c = i % inter;
     float v = zi_load(z + r * ldz + c);
     for (int s = 1; s < splits; ++s) v += zi_load(z + s * split_stride + r * ldz + c);
-    zi_store(out + r * ldo + c, ew_activate<sizeof(TO) == 2>(v, act));
+    zi_store(out + r * ldo + c, zi_activate_value<sizeof(TO) == 2>(v, act));
 }
 
 // Four values a thread, the loads of up to SP terms in flight.
@@ -376,8 +351,8 @@ activate_vec_kernel(TO* __restrict__ out, int64_t ldo, const T* __restrict__ z, 
 #pragma unroll
     for (int s = 1; s < SP; ++s) { v.x += t[s].x; v.y += t[s].y; v.z += t[s].z; v.w += t[s].w; }
     constexpr bool rough = sizeof(TO) == 2;
-    ew_store4(out + r * ldo + c, make_float4(ew_activate<rough>(v.x, act), ew_activate<rough>(v.y, act), ew_activate<rough>(v.z, act),
-                                             ew_activate<rough>(v.w, act)));
+    ew_store4(out + r * ldo + c, make_float4(zi_activate_value<rough>(v.x, act), zi_activate_value<rough>(v.y, act), zi_activate_value<rough>(v.z, act),
+                                             zi_activate_value<rough>(v.w, act)));
 }
 
 extern "C" int zi_activate(void* out, int out_dt, int64_t ldo, const void* z, int dt, int64_t ldz, int splits,

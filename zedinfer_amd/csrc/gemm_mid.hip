@@ -10,8 +10,9 @@
 // three register buffers; loads are issued without branches so that they stay in flight).  The k dimension is cut over gridDim.y workgroups when N alone gives too few of them; those
 // leave float32 partial sums [split][M][N] that the consumer adds in rising order.  The cut depends on N
 // and K only.  Epilogues as in the few-rows kernel: plain (bias), partial sums, SwiGLU over gate/up rows
-// interleaved in blocks of 8.
+// interleaved in blocks of 8, an activation of every output.
 #include "zi_common.h"
+#include "zi_activation.h"
 #include <type_traits>
 
 typedef __attribute__((ext_vector_type(8))) __bf16 gm_bf16x8_t;
@@ -29,6 +30,7 @@ typedef __attribute__((ext_vector_type(4))) unsigned gm_u32x4_t;
 #define GM_MODE_PARTIAL 1
 #define GM_MODE_SWIGLU 2
 #define GM_MODE_CLAMPED 3      // like SWIGLU, with biases: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1)
+#define GM_MODE_ACT 4          // + the code of an activation (zi_activate_value), of the sum and the bias
 
 union gm_pack {
     gm_u32x4_t u;
@@ -45,11 +47,12 @@ __device__ __forceinline__ gm_u32x4_t gm_keep(gm_u32x4_t v, bool keep) {
 // What a wavefront does with its sums: C[n = n0 + j*4 + e][m = t*16 + r] in acc[t][e].
 template <int MT>
 __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* __restrict__ out, int mode, int out_f32,
-                                            const zi_bf16* __restrict__ bias, int M, int N, int64_t ldo, int split,
+                                            const zi_bf16* __restrict__ bias_in, int M, int N, int64_t ldo, int split,
                                             int n0, int r, int j, int vec_out, float limit) {
 #pragma unroll
     for (int t = 0; t < MT; ++t) {
         gm_f32x4_t s = acc[t];
+        const zi_bf16* bias = bias_in;
         const int m = t * 16 + r;
         if (mode == GM_MODE_SWIGLU || mode == GM_MODE_CLAMPED) {
             if (mode == GM_MODE_CLAMPED && bias && n0 < N) {
@@ -86,6 +89,12 @@ __device__ __forceinline__ void gm_epilogue(const gm_f32x4_t (&acc)[MT], void* _
         }
         if (m >= M) continue;
         const int nb = n0 + j * 4;
+        if (mode >= GM_MODE_ACT) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                s[e] = zi_activate_value<true, false>(s[e] + (bias && nb + e < N ? zi_load(bias + nb + e) : 0.f), mode - GM_MODE_ACT);
+            bias = nullptr;
+        }
         if (nb + 3 < N && vec_out) {
             if (mode == GM_MODE_PARTIAL) {
                 if (bias && split == 0) {
@@ -389,8 +398,8 @@ gemm_wide_kernel(void* __restrict__ out, int mode, int out_f32, const zi_bf16* _
 // the cuts the cheapest by that measure is taken, then the one with the fewest splits, then the fewest
 // wavefronts.  A matrix with many times more rows than that keeps the units busy whatever the cut (its
 // workgroups follow each other, two to a unit): four wavefronts, no split (measured on the 151,936 rows of
-// the output head: 108 against 119 us with eight).
-void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves) {
+// the output head: 108 against 119 us with eight).  `whole`: the cheapest without a split.  Returns the cost.
+int64_t zi_gemm_mid_plan(int N, int K, int whole, int* splits, int* kb_per_split, int* waves) {
     const int tiles = (N + 15) / 16;
     const int kb_total = (K + GM_KB - 1) / GM_KB;
     int64_t best_cost = -1;
@@ -399,7 +408,7 @@ void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves) 
     const bool many = (tiles + GM_MIN_WAVES - 1) / GM_MIN_WAVES > 4 * cus;
     for (int w = GM_MIN_WAVES; w <= (many ? GM_MIN_WAVES : GM_MAX_WAVES); ++w) {
         const int groups = (tiles + w - 1) / w;
-        for (int s0 = 1; s0 <= (many ? 1 : 16) && s0 <= (kb_total > 1 ? kb_total / 2 : 1); ++s0) {
+        for (int s0 = 1; s0 <= (many || whole ? 1 : 16) && s0 <= (kb_total > 1 ? kb_total / 2 : 1); ++s0) {
             const int per = (kb_total + s0 - 1) / s0;
             const int s = (kb_total + per - 1) / per;
             if (s != s0) continue;      // the same cut under another name
@@ -414,13 +423,14 @@ void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves) 
     *splits = best_s;
     *kb_per_split = best_per;
     *waves = best_w;
+    return best_cost;
 }
 
 // The launch; the checks are the caller's (zi_gemm_skinny).
 int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
                        int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream) {
     int splits, per, waves;
-    zi_gemm_mid_plan(N, K, &splits, &per, &waves);
+    zi_gemm_mid_plan(N, K, mode >= GM_MODE_ACT, &splits, &per, &waves);
     const int tiles = (N + 15) / 16;
     const dim3 grid((tiles + waves - 1) / waves, splits);
     const int mt = (M + 15) / 16;

@@ -12,18 +12,21 @@
 // Epilogues: plain (bias, bfloat16 or float32 out), partial sums, and SwiGLU: when the weight rows are gate
 // and up rows interleaved in blocks of 8 (tile = 8 gate rows, then the 8 up rows of the same columns), the
 // tile's lanes exchange halves and write act = up * gate / (1 + exp(-gate))
-// (reference: src/backend/ops/swiglu/cpu/swiglu_cpu.cpp:9-23).
+// (reference: src/backend/ops/swiglu/cpu/swiglu_cpu.cpp:9-23); and an activation of every output, for products that are made
+// whole.
 //
 // A kernel that kept x in registers and cut k over a workgroup's wavefronts served up to 16 rows before the
 // other one's cut was balanced; since then it was slower at every size from one row on (1.5B gate/up at 8 rows
 // 12.9 against 11.7 us, 32B gate/up 111 against 95 us) and is gone.
 #include "zi_common.h"
+#include "zi_activation.h"
 #include "zi_api.h"
 
 #define SK_MODE_PLAIN 0
 #define SK_MODE_PARTIAL 1
 #define SK_MODE_SWIGLU 2
 #define SK_MODE_CLAMPED 3
+#define SK_MODE_ACT 4              // + the activation's code
 
 // out[m,n] = sum_s partial[s,m,n] + bias[n], splits added in rising order.
 __global__ void gemm_skinny_reduce_kernel(void* __restrict__ out, int out_f32, const float* __restrict__ partial,
@@ -61,7 +64,7 @@ extern "C" int zi_gemm_skinny_pays(int M, int N, int K) {
 }
 
 // The product kernel (gemm_mid.hip): its cut and its launch.
-void zi_gemm_mid_plan(int N, int K, int* splits, int* kb_per_split, int* waves);
+int64_t zi_gemm_mid_plan(int N, int K, int whole, int* splits, int* kb_per_split, int* waves);
 int zi_gemm_mid_launch(void* out, int out_f32, int mode, const zi_bf16* x, const zi_bf16* w, const zi_bf16* bias, int M,
                        int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int vec_out, float limit, hipStream_t stream);
 
@@ -76,7 +79,7 @@ static bool sk_rows32(int M, int mode) { return M > (mode >= SK_MODE_SWIGLU ? SK
 extern "C" int zi_gemm_skinny_splits(int M, int N, int K) {
     int s, per, waves;
     if (sk_rows32(M, SK_MODE_PARTIAL)) zi_gemm_rows32_plan(N, K, M > 128, 0, &s, &per, &waves);
-    else zi_gemm_mid_plan(N, K, &s, &per, &waves);
+    else zi_gemm_mid_plan(N, K, 0, &s, &per, &waves);
     return s;
 }
 
@@ -86,26 +89,40 @@ extern "C" int64_t zi_gemm_skinny_workspace(int M, int N, int K) {
     return s > 1 ? (int64_t)s * M * N : 0;
 }
 
+// 1 when a product with an activation in its epilogue, which is made whole, costs no more than one that may be split and the
+// activation's launch after it: a launch is worth about as much as this many of the cut's wavefront-blocks.
+#define SK_LAUNCH_COST 32
+extern "C" int zi_gemm_skinny_act_pays(int M, int N, int K) {
+    if (M < 1 || M > SK_MID_MAX_ROWS_SWIGLU) return 0;
+    int s, per, waves;
+    const int64_t whole = zi_gemm_mid_plan(N, K, 1, &s, &per, &waves);
+    return whole <= zi_gemm_mid_plan(N, K, 0, &s, &per, &waves) + SK_LAUNCH_COST;
+}
+
 // mode 0: out[M,N] (+ bias), reduced through `workspace` when the product is split.
 // mode 1: out = float32 partial sums [splits][M][N] (splits from zi_gemm_skinny_splits; the bias, if any, is in the first).
 // mode 2: w holds gate and up rows interleaved in blocks of 8; out[M, N/2] (bfloat16) =
 //         up * silu(gate); only for products that are not split.
 // mode 3: the same with g = min(gate + bias, limit), u = clamp(up + bias, -limit, limit), g sigmoid(1.702 g) (u + 1), the
 //         bias [N] (or null) interleaved as the rows are; up to 64 rows.
+// mode 4 + a: out[M,N] (bfloat16) = activation a (0 SiLU, 1 GELU in its tanh form, 3 relu squared) of the product and the bias
+//         [N] (or null); up to 64 rows, the product never split.
 extern "C" int zi_gemm_skinny_act(void* out, int out_dt, int mode, const void* x, const void* w, const void* bias, int M,
                                   int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, float* workspace,
                                   int64_t workspace_floats, float limit, hipStream_t stream) {
     ZI_REQUIRE(zi_gemm_skinny_supported(M, N, K, ldx, ldw),
                "gemm_skinny: unsupported sizes M=%d N=%d K=%d (1 <= M <= 256, K and row strides multiples of 8)", M, N, K);
     ZI_REQUIRE(out_dt == ZI_F32 || out_dt == ZI_BF16, "gemm_skinny: unknown output dtype %d", out_dt);
-    ZI_REQUIRE(mode >= 0 && mode <= 3, "gemm_skinny: unknown mode %d", mode);
+    ZI_REQUIRE(mode >= 0 && mode <= SK_MODE_ACT + ZI_ACT_RELU2 && mode != SK_MODE_ACT + ZI_ACT_GELU_ERF, "gemm_skinny: unknown mode %d", mode);
+    ZI_REQUIRE(mode < SK_MODE_ACT || (M <= SK_MID_MAX_ROWS_SWIGLU && out_dt == ZI_BF16 && ldo >= N),
+               "gemm_skinny: an activation takes up to %d rows and a bfloat16 out of N columns", SK_MID_MAX_ROWS_SWIGLU);
     ZI_REQUIRE(mode != SK_MODE_CLAMPED || (limit > 0.f && M <= SK_MID_MAX_ROWS_SWIGLU), "gemm_skinny: the clamped epilogue takes up to %d rows and a positive limit", SK_MID_MAX_ROWS_SWIGLU);
     ZI_REQUIRE(ldx >= K && ldw >= K, "gemm_skinny: leading dimension too small");
     ZI_REQUIRE(((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0, "gemm_skinny: x and w must be 16-byte aligned");
     int splits, per, waves;
     const bool rows32 = sk_rows32(M, mode);
     if (rows32) zi_gemm_rows32_plan(N, K, M > 128, mode == SK_MODE_SWIGLU, &splits, &per, &waves);
-    else zi_gemm_mid_plan(N, K, &splits, &per, &waves);
+    else zi_gemm_mid_plan(N, K, mode >= SK_MODE_ACT, &splits, &per, &waves);
     void* dst = out;
     int kmode = mode;
     if (mode == SK_MODE_PLAIN) {
@@ -119,13 +136,13 @@ extern "C" int zi_gemm_skinny_act(void* out, int out_dt, int mode, const void* x
         }
     } else if (mode == SK_MODE_PARTIAL) {
         ZI_REQUIRE(out_dt == ZI_F32, "gemm_skinny: partial sums are float32");
-    } else {
+    } else if (mode < SK_MODE_ACT) {
         ZI_REQUIRE(splits == 1, "gemm_skinny: the SwiGLU epilogue needs a product that is not split (N=%d K=%d has %d)",
                    N, K, splits);
         ZI_REQUIRE(N % 16 == 0 && out_dt == ZI_BF16 && ldo >= N / 2,
                    "gemm_skinny: the SwiGLU epilogue needs N %% 16 == 0 and a bfloat16 out of N/2 columns");
     }
-    const zi_bf16* b = (kmode == SK_MODE_PLAIN || mode == SK_MODE_PARTIAL || mode == SK_MODE_CLAMPED) ? (const zi_bf16*)bias : nullptr;
+    const zi_bf16* b = (kmode == SK_MODE_PLAIN || mode == SK_MODE_PARTIAL || mode >= SK_MODE_CLAMPED) ? (const zi_bf16*)bias : nullptr;
     // four columns go out as one store when every row of the destination keeps them aligned
     int vec_out;
     if (kmode == SK_MODE_PARTIAL) vec_out = N % 4 == 0 && ((uintptr_t)dst % 16) == 0;

@@ -36,7 +36,8 @@ from .hybrid import (linear_attention_grouped, moe_route_sigmoid, moe_sum_shared
                      pooled_attention_cores_workspace,
                      rope_table_scaled, ssm_finish, ssm_prepare,
                      ssm_state_floats)
-from .streams import (ACTIVATIONS, activate, difference_heads, difference_merge, head_norm_store, stream_mix, stream_mix_max_streams)
+from .streams import (ACTIVATIONS, activate, difference_heads, difference_merge, head_norm_store, linear_activated, linear_activated_supported,
+                      stream_mix, stream_mix_max_streams)
 from ._lib import KernelLibraryError, library_path, load
 
 __all__ = [
@@ -62,7 +63,7 @@ __all__ = [
     "normed_add_norm", "pool_blocks", "pooled_attention", "pooled_attention_cores", "pooled_attention_cores_cut", "pooled_attention_cores_supported", "pooled_attention_cores_workspace", "rope_table_scaled", "ssm_finish", "ssm_prepare", "ssm_state_floats",
     "channel_inputs", "channel_state_floats", "delta_channel", "delta_channel_finishes", "input_conv", "lowrank_gates", "norm_input_conv", "norm_input_conv_supported",
     "stream_scale", "attention_decode_merge_gated", "linear_clamped_glu", "clamped_glu_il8",
-    "ACTIVATIONS", "activate", "attention_prefill_maps_supported", "difference_heads", "difference_merge", "head_norm_store", "latent_inputs",
+    "ACTIVATIONS", "activate", "attention_prefill_maps_supported", "difference_heads", "difference_merge", "head_norm_store", "latent_inputs", "linear_activated", "linear_activated_supported",
     "latent_query_cores", "latent_value_gates", "stream_mix", "stream_mix_max_streams",
     "KernelLibraryError", "library_path", "load", "FEW_ROWS", "SUMS_MAX_ROWS",
 ]

@@ -1,13 +1,14 @@
 """Checked launches of the kernels behind several residual streams a token, behind attention whose heads are differences
-of two softmax maps, and an activation alone."""
+of two softmax maps, and an activation alone or in a product's epilogue."""
 from __future__ import annotations
 
+from ctypes import c_void_p
 from typing import Optional
 
 import torch
 
 from . import _lib
-from .functional import F32, _angle_table, _check_cache, _code, _gpu, _i32, _p, _rows, _stream, attention_decode_workspace
+from .functional import BF16, F32, FEW_ROWS, _angle_table, _check_cache, _code, _few_rows_operands, _gpu, _i32, _p, _rows, _stream, attention_decode_workspace
 from .mixing import _f32
 from .sublayers import _terms
 
@@ -152,4 +153,31 @@ def activate(z: torch.Tensor, activation: str, out: torch.Tensor) -> torch.Tenso
         raise ValueError(f"activate: unknown activation {activation!r}")
     _lib.call("zi_activate", _p(out), _code(out, "activate out"), ldo, _p(z), _code(z, "activate z"), ldz, splits, split_stride, n, I,
               ACTIVATIONS[activation], _stream())
+    return out
+
+
+def linear_activated_supported(x: torch.Tensor, weight: torch.Tensor, activation: str) -> bool:
+    """Whether ``linear_activated`` takes the operands and is no slower than a product that may be cut and ``activate``."""
+    return (activation in ACTIVATIONS and activation != "gelu_erf" and _few_rows_operands(x, weight, FEW_ROWS)
+            and bool(_lib.load().zi_gemm_skinny_act_pays(int(x.shape[0]), int(weight.shape[0]), int(weight.shape[1]))))
+
+
+def linear_activated(x: torch.Tensor, weight: torch.Tensor, activation: str, bias: Optional[torch.Tensor] = None,
+                     out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """act(x . weight^T + bias) in one kernel for few rows, bfloat16 [M, N]: ``ACTIVATIONS`` but the error function's."""
+    _gpu("linear_activated", x, weight, bias, out)
+    if activation not in ACTIVATIONS or activation == "gelu_erf":
+        raise ValueError(f"linear_activated: no activation {activation!r} in this product")
+    if not _few_rows_operands(x, weight, FEW_ROWS):
+        raise ValueError(f"linear_activated: needs bfloat16 operands of at most {FEW_ROWS} rows, K and row strides multiples of 8")
+    (M, K), N = x.shape, weight.shape[0]
+    if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != N or not bias.is_contiguous()):
+        raise ValueError(f"linear_activated: the bias must be a contiguous bfloat16 [{N}] tensor")
+    if out is None:
+        out = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
+    ldo, _ = _rows(out, "linear_activated out")
+    if tuple(out.shape) != (M, N) or out.dtype != torch.bfloat16:
+        raise ValueError(f"linear_activated: out must be bfloat16 [{M}, {N}]")
+    _lib.call("zi_gemm_skinny_act", _p(out), BF16, 4 + ACTIVATIONS[activation], _p(x), _p(weight), _p(bias), M, N, K, x.stride(0),
+              weight.stride(0), ldo, c_void_p(0), 0, 0.0, _stream())
     return out

@@ -339,8 +339,8 @@ class ReluSquaredMLP(FeedForward):
 @register_feed_forward("activated_mlp")
 class ActivatedMLP(FeedForward):
     """down(act(up(x))), no gate, no biases, the activation one of ``ops.ACTIVATIONS`` ("gelu_tanh", "gelu_erf", "silu",
-    "relu2").  Few rows: the up product leaves partial sums, which the activation's kernel adds; the down product leaves its own
-    for the norm that follows.  params: hidden_size, intermediate_size, activation."""
+    "relu2").  Few rows: the up product has the activation in its epilogue, or, where cutting it is worth a launch, leaves partial
+    sums that the activation's kernel adds; the down product leaves its own for the norm that follows.  params: hidden_size, intermediate_size, activation."""
 
     graph_safe = True
     tape_safe = True
@@ -370,12 +370,15 @@ class ActivatedMLP(FeedForward):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         n, I, rt = x.shape[0], self.inter, self.rt
         act = rt.buffer("ffn_act", (n, I))
-        if ops.linear_sums_supported(x, self.up):
-            S = ops.linear_splits(n, I, self.hidden)
-            z = ops.linear_sums(x, self.up, out=rt.buffer("ffn_up_sums", (S, n, I), torch.float32))
+        if ops.linear_activated_supported(x, self.up, self.activation):
+            ops.linear_activated(x, self.up, self.activation, out=act)
         else:
-            z = ops.linear(x, self.up, out=rt.buffer("ffn_up", (n, I)))
-        ops.activate(z, self.activation, out=act)
+            if ops.linear_sums_supported(x, self.up):
+                S = ops.linear_splits(n, I, self.hidden)
+                z = ops.linear_sums(x, self.up, out=rt.buffer("ffn_up_sums", (S, n, I), torch.float32))
+            else:
+                z = ops.linear(x, self.up, out=rt.buffer("ffn_up", (n, I)))
+            ops.activate(z, self.activation, out=act)
         if ops.linear_sums_supported(act, self.down):
             S = ops.linear_splits(n, self.hidden, I)
             return ops.linear_sums(act, self.down, out=rt.buffer("ffn_out_sums", (S, n, self.hidden), torch.float32))
