@@ -429,6 +429,8 @@ def test_latent_attention_cores_plan_is_a_function_of_the_shape():
     waves, keys, chunks = ops.latent_attention_cores_plan(8, 8, 12, 1024, 256)           # decoded tokens: cut
     assert waves == 1 and keys == ops.mixing.LATENT_CHUNK_KEYS // 2 and chunks * keys >= 1024 + 3
     waves, keys, chunks = ops.latent_attention_cores_plan(64, 64, 12, 1024, 256)         # many requests: longer walks
-    assert waves == 1 and keys == ops.mixing.LATENT_CHUNK_KEYS and chunks * keys >= 1024 + 3
+    assert waves == 1 and keys > ops.mixing.LATENT_CHUNK_KEYS // 2 and 64 * chunks <= 512 and chunks * keys >= 1024 + 3
+    waves, keys, chunks = ops.latent_attention_cores_plan(1, 1, 4, 1 << 20, 256)         # no more chunks than can be merged
+    assert chunks <= 4096 and chunks * keys >= (1 << 20) + 5
     assert ops.latent_attention_cores_plan(8, 8, 12, 0, 256) == (1, 0, 1)                # no window, no cut
     assert ops.latent_attention_cores_plan(8, 8, 12, 40, 256) == (1, 0, 1)               # a window of one chunk

@@ -69,16 +69,29 @@ latent_attention_cores_kernel(void* __restrict__ out, int out_f32, float* __rest
     static_assert(P % 8 == 0 && (P * 16) % 256 == 128 && KI * WAVES * ZI_WAVE == LA_BK * P, "whole loads, rows half the banks apart");
     __shared__ __attribute__((aligned(16))) la_u32x4_t buf_a[LA_BK * P];
     __shared__ __attribute__((aligned(16))) la_u32x4_t buf_b[LA_BK * P];
-    int tile = blockIdx.x, e = 0;
-    for (; e < entries; ++e) {
-        const int tiles = (entry_len[e] * heads + ROWS - 1) / ROWS;
-        if (tile < tiles) break;
-        tile -= tiles;
+    const int lane = threadIdx.x % ZI_WAVE, wave = threadIdx.x / ZI_WAVE, r = lane % 16, j = lane / 16;
+    // the entry whose tiles this one is among: 64 entries at a time, a lane each, their tiles summed up over the lanes
+    int tile = blockIdx.x, e = entries;
+    for (int e0 = 0; e0 < entries; e0 += ZI_WAVE) {
+        const int mine = e0 + lane < entries ? (entry_len[e0 + lane] * heads + ROWS - 1) / ROWS : 0;
+        int upto = mine;
+#pragma unroll
+        for (int d = 1; d < ZI_WAVE; d *= 2) {
+            const int below = __shfl_up(upto, d, ZI_WAVE);
+            if (lane >= d) upto += below;
+        }
+        const uint64_t past_it = __ballot(upto > tile);
+        if (past_it) {
+            const int at = __builtin_ctzll(past_it);
+            e = e0 + at;
+            tile -= __builtin_amdgcn_readlane(upto - mine, at);
+            break;
+        }
+        tile -= __builtin_amdgcn_readlane(upto, ZI_WAVE - 1);
     }
     if (e >= entries) return;      // the launch is sized for the worst case: the whole workgroup leaves
     const int len = entry_len[e], past = entry_past[e], start = entry_start[e];
     const int erows = len * heads, row0 = tile * ROWS;
-    const int lane = threadIdx.x % ZI_WAVE, wave = threadIdx.x / ZI_WAVE, r = lane % 16, j = lane / 16;
     const int32_t* bt = block_tables + (int64_t)e * max_pages;
     const int qw = rank + rot;
 
@@ -328,8 +341,9 @@ extern "C" int zi_latent_attention_cores_supported(int dt, int rank, int rot) {
 
 // Rows of a tile for `waves` wavefronts, and the most tiles a step of n tokens in `entries` entries has.
 extern "C" int zi_latent_attention_cores_tiles(int n, int entries, int heads, int waves) {
-    const int rows = 16 * waves;
-    return (int)(((int64_t)n * heads + rows - 1) / rows) + entries;
+    const int64_t rows = 16 * waves;
+    const int64_t by_entry = ((int64_t)n * heads + rows - 1) / rows + entries, by_token = (int64_t)n * ((heads + rows - 1) / rows);
+    return (int)(by_entry < by_token ? by_entry : by_token);
 }
 
 // qa [n][heads][rank + rot] and out [n][heads][rank], each float32 or bfloat16; partial: chunks * n * heads * (rank + 4) floats.

@@ -189,8 +189,10 @@ def latent_attention(qa: torch.Tensor, c_cache: torch.Tensor, kr_cache: torch.Te
     return out
 
 
-# keys of a chunk when a tile's keys are cut over workgroups (a multiple of the kernel's block of 32)
+# keys of a chunk when a tile's keys are cut over workgroups (a multiple of the kernel's block of 32): half as many at least
+# under a window, this many at least without one
 LATENT_CHUNK_KEYS = max(32, int(os.environ.get("ZEDINFER_LATENT_CHUNK_KEYS", "128") or 128) // 32 * 32)
+LATENT_MAX_CHUNKS = 4096     # what the kernel that merges them takes
 
 
 def latent_attention_cores_supported(cache_dtype: torch.dtype, rank: int, rot: int) -> bool:
@@ -210,9 +212,10 @@ def latent_attention_cores_plan(n: int, entries: int, heads: int, window: int, u
     tiles = lib.zi_latent_attention_cores_tiles(int(n), int(entries), int(heads), waves)
     if window > 0 and tiles < units:
         span = int(window) + -(-16 * waves // int(heads)) + 1
-        keys = LATENT_CHUNK_KEYS
-        if -(-span // keys) * tiles < units and keys > 32:      # few requests: a walk half as long, twice the workgroups
-            keys //= 2
+        # as many chunks as there is room for on the chip at once (two workgroups a compute unit), none of them nearly empty
+        most = max(1, min(2 * int(units) // tiles, LATENT_MAX_CHUNKS))
+        keys = max(LATENT_CHUNK_KEYS // 2, 32, -(-span // most))
+        keys = -(-keys // 32) * 32
         chunks = -(-span // keys)
         if chunks > 1:
             return waves, keys, chunks
